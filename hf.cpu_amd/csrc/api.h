@@ -101,14 +101,16 @@ int hfa_attention_prompt_rows(void);
 // of head h being its weights on the values of group (h's group + r) mod G (see hfa_talk_mix; on the matrix cores one pass a round).
 // `softcap` > 0: score <- softcap tanh(score / softcap) before the weights are formed. `weights` 0: softmax; 1: no softmax, a
 // visible key weighs sigmoid(score + head_bias[h]) (head_bias: one fp32 per query head, or null), not normalised over the keys.
-// Sigmoid weights (with or without a cap) run on the matrix cores under the same conditions as the softmax; a cap under a softmax goes the plain way.
+// `sink_w` (with `sink`): the extra term's score is sink_w[h] (one fp32 per query head) instead of 0. `dist_scale` and `dist_rate`
+// (one fp32 per query head each, or both null; softmax only): after scale and cap a score is lowered by dist_scale[h] ln(1 + dist_rate[h] (i - j)).
+// Sigmoid weights, caps and distance terms run on the matrix cores under the same conditions as the plain softmax.
 int hfa_paged_attention(const void* q, int dtype, int ldq, const void* k_cache, const void* v_cache,
                         int kv_width, int v_width, const int* block_table, int max_blocks, const int* token_slot,
                         const int* positions, const int* q_start, int n_seqs, int max_q_len, int max_seq_len,
                         void* out, int ldo, int n_tokens, int n_heads, int n_kv_heads, int head_dim, int v_head_dim,
                         int page_tokens, int window, int mask_chunk, float scale, const float* slopes, int sink, int cross_values,
-                        float softcap, int weights, const float* head_bias,
-                        void* workspace, size_t workspace_bytes, int force_plain, hipStream_t stream);
+                        float softcap, int weights, const float* head_bias, const float* sink_w, const float* dist_scale,
+                        const float* dist_rate, void* workspace, size_t workspace_bytes, int force_plain, hipStream_t stream);
 
 // Decoded tokens (one a request) whose queries, new keys and new values are still the 32-bit rows [q | k | v] that
 // the product left (`raw`, bias added): rotation of queries and keys (cos_sin: hfa_rope_table's output for the step's
@@ -124,7 +126,8 @@ int hfa_decode_attention(const float* raw, int ld_raw, const float* cos_sin, voi
                          const int* slot_map, const int* block_table, int max_blocks, const int* token_slot,
                          const int* positions, const int* q_start, int n_seqs, int max_seq_len, void* out, int ldo,
                          int n_heads, int n_kv_heads, int head_dim, int page_tokens, int window, int mask_chunk, float scale,
-                         void* workspace, size_t workspace_bytes, hipStream_t stream);
+                         float softcap, const float* dist_scale, const float* dist_rate, void* workspace, size_t workspace_bytes,
+                         hipStream_t stream);
 
 // Layer norm: out[r, :] = (x[rows ? rows[r] : r, :] - mean) / sqrt(var + eps) * w + b (b null: no shift), var the mean
 // squared deviation, all in fp32. With splits > 0 (and no rows) a deferred product's partial sums
@@ -152,7 +155,7 @@ int hfa_qkv_prepare(void* qkv, int dtype, int ld, const int* positions, const fl
 
 // Mixers with per-request state (recurrent.hip). A request's tokens of a step are rows q_start[s] .. q_start[s + 1] - 1;
 // its state is row seq_slot[s] of `state` (fp32, state_ld floats a row).
-// hfa_causal_conv: out[t, c] = act(bias[c] + sum_j taps[c, j] in[t - (K - 1) + j, c]) (fp32 out; act HFA_ACT_SILU or none);
+// hfa_causal_conv: out[t, c] = act(bias[c] + sum_j taps[c, j] in[t - (K - 1) + j, c]) (formed in fp32; act HFA_ACT_SILU or none);
 // inputs before the step's first token come from the state row ([K - 1][C], oldest first), which then receives the
 // step's last K - 1 inputs.
 // hfa_linear_scan: per head h (keys and queries of head h / (n_heads / qk_heads)), S [qk_dim][v_dim] in the state row (in the
@@ -169,8 +172,8 @@ int hfa_qkv_prepare(void* qkv, int dtype, int ld, const int* positions, const fl
 // with k_t, q_t first divided by sqrt(sum of squares + unit_eps) and q_t multiplied by q_scale. max_q_len: the most tokens of a
 // request (an upper bound will do; it only chooses between a walk for prompt portions and one for single tokens).
 int hfa_causal_conv(const void* in, int dtype, int ld_in, const float* taps, const float* bias, int n_channels, int n_taps,
-                    float* state, size_t state_ld, const int* q_start, const int* seq_slot, int n_seqs, int max_q_len, float* out,
-                    int ldo, int act, hipStream_t stream);
+                    float* state, size_t state_ld, const int* q_start, const int* seq_slot, int n_seqs, int max_q_len, void* out,
+                    int out_dtype, int ldo, int act, hipStream_t stream);
 size_t hfa_linear_scan_state_floats(int n_heads, int qk_dim, int v_dim);
 int hfa_linear_scan(const void* q, int ldq, const void* k, int ldk, int qk_heads, int qk_dim, const void* v, int ldv, int n_heads,
                     int v_dim, int dtype, int gate, const float* decay, const void* step, int step_dtype, int ld_step,
@@ -212,15 +215,32 @@ int hfa_scale_add(const float* y, int ldy, const float* col, float scale, float*
 int hfa_gate_mul(const void* x, int x_dtype, int ldx, const void* gate, int gate_dtype, int ldg, void* out, int out_dtype,
                  int ldo, int n_rows, int width, int act, hipStream_t stream);
 
-// Attention through latents (latent.hip). hfa_latent_pack lays a step's rows out for hfa_rope_store and hfa_paged_attention with one
-// key/value head whose key is [rotated part: R | latent: C] and whose value is the latent: from `down` ([T, >= C + R] fp32: the
-// latent before its norm, then the rotated key part) and `q` ([T, H (D + R)], head by head [D unrotated | R to be rotated]) it
-// writes packed[t] = [H heads of (R | C: left alone) | R | C | C]: the queries' parts to be rotated, the key's part to be rotated,
-// and the latent c = down[:C] / sqrt(mean(down[:C]^2) + eps) * w twice (as the key's rest and as the value). Sums in fp32.
-// `folded` ([T, H C] of q's type, or null): the heads' C parts are copied from there (else they are left alone).
-int hfa_latent_pack(const float* down, int ld_down, const void* q, int q_dtype, int ldq, const float* w, float eps, void* packed,
-                    int out_dtype, int ld_packed, int n_tokens, int n_heads, int dim, int rot, int latent, const void* folded,
-                    int ld_folded, hipStream_t stream);
+// Attention through latents (latent.hip). hfa_latent_store: what lies between the projections and the attention kernels. Rows of the
+// latent before its norm and the rotated key part (`down`, [T, >= C + R] fp32) and the heads' queries (`q`, [T, H (D + R)]): c = down[:C] / sqrt(mean^2 +
+// eps) * w; the first rot_dim of the R rotated values are turned (pairing as in hfa_qkv_prepare); the key row [rotated: R | c] goes to
+// k_cache row slot_map[t], the value c to v_cache (transposed inside its page), and every head's rotated part to q_out, whose rows
+// hold H heads of [R | C] (their C parts are left alone: the products that fold the keys' expansion write them).
+// hfa_head_rows: out[t, h, :N] = W_h a[t, h, :K] (* sigmoid(gate[t, h, :])) for few rows t, every head with a matrix of its own
+// (w [H][N][K] bf16, a fp32 or bf16 rounded to bf16 as it is read, out bf16): one block 32 outputs of one head and 32 rows.
+// K a multiple of 16, N of 32, strides of a in 16-byte, of out in 8-byte steps.
+int hfa_latent_store(const float* down, int ld_down, const void* q, int q_dtype, int ldq, const float* w, float eps, const int* positions,
+                     const float* inv_freq, int rot_dim, int pairing, void* q_out, int ld_out, void* k_cache, void* v_cache, int dtype,
+                     const int* slot_map, int page_tokens, int n_tokens, int n_heads, int dim, int rot, int latent, hipStream_t stream);
+int hfa_head_rows(const void* a, int a_dtype, int lda, int a_head, const void* w, void* out, int ldo, int out_head, const float* gate,
+                  int ldg, int n_rows, int n_heads, int N, int K, hipStream_t stream);
+
+// Residuals of several streams (streams.hip). x: [n_rows][n_streams][width] fp32. mode 0: the streams as stored; 1: every stream
+// becomes y[t]; 2: new_b = sum_a mix[a * n_streams + b] old_a + out_w[b] y[t]. y is fp32 rows, or with splits > 0 the partial sums
+// ([splits][n_rows][width]) of a product that hfa_gemm deferred. hfa_stream_step writes the new streams (modes 1 and 2) and, with
+// in_w, out[t] = conv(n), n = u / sqrt(mean(u^2) + eps) * norm_w, u = sum_b in_w[b] new_b; taps ([width][n_taps], null: out = n): a
+// causal convolution for steps in which every row is a request's only token, its earlier inputs in state row slots[t] ([n_taps - 1]
+// [width], oldest first), which moves on. hfa_stream_sum: out[r] = sum_b new_b of row rows[r] (null: r); nothing is written back.
+int hfa_stream_step(float* x, int n_streams, int width, int mode, const float* y, int ldy, const float* partial, int splits,
+                    const float* mix, const float* out_w, const float* in_w, const float* norm_w, float eps, void* out, int out_dtype,
+                    int ldo, const float* taps, int n_taps, float* state, size_t state_ld, const int* slots, int n_rows,
+                    hipStream_t stream);
+int hfa_stream_sum(const float* x, int n_streams, int width, int mode, const float* y, int ldy, const float* partial, int splits,
+                   const float* mix, const float* out_w, const int* rows, float* out, int n_out, int n_rows, hipStream_t stream);
 
 // hfa_channel_scan (recurrent.hip): per head, S [qk_dim][v_dim] in hfa_linear_scan's layout: S <- diag(a_t) S + k_t v_t^T, y_t = S^T
 // (q_scale q_t), with a decay per key channel a_t = decay[t, h qk_dim + n] (fp32); kcomp 1: k_t = 1 - a_t (k is not read), else k_t

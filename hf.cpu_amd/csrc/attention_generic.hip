@@ -48,14 +48,16 @@ __device__ __forceinline__ float dot_row(const float* __restrict__ q_s, const fl
 // group (h's group + r) mod G. A design that mixes the heads' weights after the softmax sums these (hfa_talk_mix).
 #define ATT_MAX_CROSS 1024
 // softcap > 0: score <- softcap tanh(score / softcap). weights 1: no softmax; a visible key weighs sigmoid(score + head_bias[h])
-// (head_bias null: 0), and the weights are not normalised over the keys.
+// (head_bias null: 0), and the weights are not normalised over the keys. dist_scale (null: none): the score is lowered by
+// dist_scale[h] ln(1 + dist_rate[h] (i - j)) after the cap. sink with sink_w: the extra term's score is sink_w[h] instead of 0.
 template <typename T, bool CROSS, int MAXD>
 __global__ __launch_bounds__(WAVE) void attn_generic_kernel(
     const T* __restrict__ q, int ldq, const T* __restrict__ kc, const T* __restrict__ vc, int kvw, int vw,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ token_slot,
     const int* __restrict__ positions, T* __restrict__ out, int ldo, int H, int G, int D, int Dv, int page_tokens,
     int window, int mask_chunk, float scale, const float* __restrict__ slopes, int sink, float softcap, int weights,
-    const float* __restrict__ head_bias) {
+    const float* __restrict__ head_bias, const float* __restrict__ sink_w, const float* __restrict__ dist_scale,
+    const float* __restrict__ dist_rate) {
     __shared__ float q_s[MAXD];
     __shared__ float p_s[WAVE];
     __shared__ int row_s[WAVE];
@@ -71,6 +73,7 @@ __global__ __launch_bounds__(WAVE) void attn_generic_kernel(
     constexpr int NACC = (CROSS ? ATT_MAX_CROSS : MAXD) / WAVE;
     const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
     const float hb = (weights == 1 && head_bias) ? head_bias[h] : 0.f;
+    const float r1 = dist_scale ? dist_scale[h] : 0.f, r2 = dist_scale ? dist_rate[h] : 0.f;
     const int v_first = CROSS ? 0 : kvh * Dv, v_cols = CROSS ? G * Dv : Dv;      // the columns of a value row that this head reads
     float acc[NACC];
 #pragma unroll
@@ -86,6 +89,7 @@ __global__ __launch_bounds__(WAVE) void attn_generic_kernel(
             s = dot_row(q_s, kc + (size_t)row * kvw + kvh * D, D) * scale;
             if (slopes) s += slope * (float)(j - pos);
             if (softcap > 0.f) s = softcap * tanhf(s * inv_cap);
+            if (dist_scale) s -= r1 * log1pf(r2 * (float)(pos - j));
         }
         float corr = 1.f, p;
         if (weights == 1) {
@@ -119,7 +123,8 @@ __global__ __launch_bounds__(WAVE) void attn_generic_kernel(
         }
         __syncthreads();
     }
-    const float inv = weights == 1 ? 1.f : 1.0f / (sink ? l + expf(-m) : l);      // the term of score 0 that has no value
+    // the term that has no value: its score is the head's number, or 0
+    const float inv = weights == 1 ? 1.f : 1.0f / (sink ? l + expf((sink_w ? sink_w[h] : 0.f) - m) : l);
 #pragma unroll
     for (int i = 0; i < NACC; i++) {
         const int d = lane + WAVE * i;
@@ -137,7 +142,8 @@ int attn_generic_launch(const void* q, int dtype, int ldq, const void* k_cache, 
                         int v_width, const int* block_table, int max_blocks, const int* token_slot, const int* positions,
                         void* out, int ldo, int n_tokens, int n_heads, int n_kv_heads, int head_dim, int v_head_dim,
                         int page_tokens, int window, int mask_chunk, float scale, const float* slopes, int sink, int cross, float softcap,
-                        int weights, const float* head_bias, hipStream_t stream) {
+                        int weights, const float* head_bias, const float* sink_w, const float* dist_scale, const float* dist_rate,
+                        hipStream_t stream) {
     HFA_REQUIRE(!cross || n_kv_heads * v_head_dim <= ATT_MAX_CROSS, "paged_attention: a value row of %d columns exceeds what one wave "
                 "applies its weights to (%d)", n_kv_heads * v_head_dim, ATT_MAX_CROSS);
     const bool wide = head_dim > ATT_MAX_D || v_head_dim > ATT_MAX_D;
@@ -150,7 +156,7 @@ int attn_generic_launch(const void* q, int dtype, int ldq, const void* k_cache, 
     attn_generic_kernel<T, CROSS, MAXD><<<grid, WAVE, 0, stream>>>(                                                               \
         (const T*)q, ldq, (const T*)k_cache, (const T*)v_cache, kv_width, v_width, block_table, max_blocks, token_slot, positions, \
         (T*)out, ldo, n_heads, n_kv_heads, head_dim, v_head_dim, page_tokens, window, mask_chunk, scale, slopes, sink, softcap,   \
-        weights, head_bias)
+        weights, head_bias, sink_w, dist_scale, dist_rate)
     if (dtype == HFA_F32) { if (cross) ATT_GO(float, true, ATT_MAX_D); else if (wide) ATT_GO(float, false, ATT_MAX_D_WIDE); else ATT_GO(float, false, ATT_MAX_D); }
     else { if (cross) ATT_GO(bf16, true, ATT_MAX_D); else if (wide) ATT_GO(bf16, false, ATT_MAX_D_WIDE); else ATT_GO(bf16, false, ATT_MAX_D); }
 #undef ATT_GO
@@ -200,8 +206,10 @@ extern "C" int hfa_decode_attention(const float* raw, int ld_raw, const float* c
                                     int kv_width, const int* slot_map, const int* block_table, int max_blocks,
                                     const int* token_slot, const int* positions, const int* q_start, int n_seqs,
                                     int max_seq_len, void* out, int ldo, int n_heads, int n_kv_heads, int head_dim,
-                                    int page_tokens, int window, int mask_chunk, float scale, void* workspace,
+                                    int page_tokens, int window, int mask_chunk, float scale, float softcap,
+                                    const float* dist_scale, const float* dist_rate, void* workspace,
                                     size_t workspace_bytes, hipStream_t stream) {
+    HFA_REQUIRE(softcap >= 0.f && (!dist_scale) == (!dist_rate), "decode_attention: a negative soft cap, or half of a distance term");
     HFA_REQUIRE(raw && k_cache && v_cache && block_table && token_slot && positions && q_start && out,
                 "decode_attention: a null argument");
     HFA_REQUIRE(n_seqs > 0 && max_seq_len > 0 && max_blocks > 0 && window >= 0 && mask_chunk >= 0, "decode_attention: bad sizes");
@@ -209,7 +217,8 @@ extern "C" int hfa_decode_attention(const float* raw, int ld_raw, const float* c
                 "decode_attention: a row stride is smaller than its row");
     AttnArgs a = {nullptr, 8, k_cache, v_cache, kv_width, block_table, max_blocks, token_slot, positions, q_start,
                   n_seqs, 1, max_seq_len, out, ldo, n_seqs, n_heads, n_kv_heads, head_dim, page_tokens,
-                  window, scale, workspace, workspace_bytes, stream, raw, ld_raw, cos_sin, slot_map, mask_chunk, 0, 0};
+                  window, scale, workspace, workspace_bytes, stream, raw, ld_raw, cos_sin, slot_map, mask_chunk, 0, 0,
+                  softcap, 0, nullptr, nullptr, dist_scale, dist_rate};
     HFA_REQUIRE(((uintptr_t)raw & 15) == 0 && (cos_sin == nullptr || ((uintptr_t)cos_sin & 15) == 0) && attn_mfma_supports(a),
                 "decode_attention: this shape is not taken (see hfa_decode_attention_supports)");
     return attn_mfma_launch(a);
@@ -221,7 +230,8 @@ extern "C" int hfa_paged_attention(const void* q, int dtype, int ldq, const void
                                    int max_seq_len, void* out, int ldo, int n_tokens, int n_heads, int n_kv_heads,
                                    int head_dim, int v_head_dim, int page_tokens, int window, int mask_chunk, float scale,
                                    const float* slopes, int sink, int cross_values, float softcap, int weights,
-                                   const float* head_bias, void* workspace, size_t workspace_bytes,
+                                   const float* head_bias, const float* sink_w, const float* dist_scale, const float* dist_rate,
+                                   void* workspace, size_t workspace_bytes,
                                    int force_plain, hipStream_t stream) {
     HFA_REQUIRE(n_tokens > 0 && n_heads > 0 && n_kv_heads > 0 && head_dim > 0 && v_head_dim > 0 && page_tokens > 0 && max_blocks > 0,
                 "paged_attention: bad sizes");
@@ -235,12 +245,14 @@ extern "C" int hfa_paged_attention(const void* q, int dtype, int ldq, const void
     AttnArgs a = {q, ldq, k_cache, v_cache, kv_width, block_table, max_blocks, token_slot, positions, q_start,
                   n_seqs, max_q_len, max_seq_len, out, ldo, n_tokens, n_heads, n_kv_heads, head_dim, page_tokens,
                   window, scale, workspace, workspace_bytes, stream, nullptr, 0, nullptr, nullptr, mask_chunk, sink ? 1 : 0, 0,
-                  softcap, weights, head_bias};
-    // the matrix-core kernels take no slopes: scores with a position term go the plain way
+                  softcap, weights, head_bias, sink ? sink_w : nullptr, dist_scale, dist_rate};
+    // the matrix-core kernels take no slopes: scores with a linear position term go the plain way,
     // and they know one head size and one row width for keys and values
     HFA_REQUIRE(softcap >= 0.f && (weights == 0 || weights == 1), "paged_attention: a negative soft cap or an unknown kind of weights");
-    // nor a soft cap on the scores under a softmax; sigmoid weights (with or without a cap) they take, for a head's own values
-    if (!force_plain && !slopes && (weights == 1 ? !cross_values && !sink : softcap == 0.f) && dtype == HFA_BF16 && v_head_dim == head_dim && v_width == kv_width && attn_mfma_supports(a)) {
+    HFA_REQUIRE((!dist_scale) == (!dist_rate) && (!dist_scale || (weights == 0 && !slopes && !cross_values)) && (!sink_w || (sink && !cross_values)),
+                "paged_attention: a distance term has two numbers a head and goes with a softmax over a head's own values, a sink's scores with a sink");
+    // sigmoid weights and shaped scores (a soft cap, a distance term) they take for a head's own values
+    if (!force_plain && !slopes && (weights == 1 ? !cross_values && !sink : !cross_values || softcap == 0.f) && dtype == HFA_BF16 && v_head_dim == head_dim && v_width == kv_width && attn_mfma_supports(a)) {
         if (!cross_values) return attn_mfma_launch(a);
         // single tokens: one pass over the cache for all rounds
         int chunk_keys = 0, n_chunks = 0;
@@ -262,5 +274,6 @@ extern "C" int hfa_paged_attention(const void* q, int dtype, int ldq, const void
         return attn_shared_launch(a, v_head_dim);
     return attn_generic_launch(q, dtype, ldq, k_cache, v_cache, kv_width, v_width, block_table, max_blocks, token_slot,
                                positions, out, ldo, n_tokens, n_heads, n_kv_heads, head_dim, v_head_dim, page_tokens, window,
-                               mask_chunk, scale, slopes, sink ? 1 : 0, cross_values ? 1 : 0, softcap, weights, head_bias, stream);
+                               mask_chunk, scale, slopes, sink ? 1 : 0, cross_values ? 1 : 0, softcap, weights, head_bias, sink ? sink_w : nullptr,
+                               dist_scale, dist_rate, stream);
 }

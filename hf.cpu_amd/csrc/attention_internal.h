@@ -21,10 +21,20 @@ struct AttnArgs {
     int mask_chunk;                // > 0: a query sees only the keys of its own run of mask_chunk positions, counted from 0
     int sink;                      // 1: the softmax's denominator holds one more term of score 0 that has no value
     int v_rot;                     // the weights of a head of group c are applied to the values of group (c + v_rot) mod G (0: its own)
-    float softcap;                 // > 0 (with weights 1 only): score <- softcap tanh(score / softcap)
+    float softcap;                 // > 0: score <- softcap tanh(score / softcap)
     int weights;                   // 0: softmax; 1: sigmoid(score + head_bias[head]), not normalised over the keys
     const float* head_bias;        // one number a query head, or null
+    const float* sink_w;           // with sink: the extra term's score per query head (null: 0)
+    const float* dist_scale;       // per query head, or null: a softmax's score is lowered by dist_scale[h] ln(1 + dist_rate[h] (i - j))
+    const float* dist_rate;
 };
+
+// Whether a softmax's scores are more than a scaled product (a soft cap, a term of the distance): the matrix-core kernels
+// then run an instantiation of their own.
+inline bool attn_shaped_scores(const AttnArgs& a) { return a.weights == 0 && (a.softcap > 0.f || a.dist_scale != nullptr); }
+
+// Whether a query sees a bounded run of keys only: cuts of the keys are then counted from the first key block of a tile.
+__host__ __device__ __forceinline__ bool attn_bounded(int window, int mask_chunk) { return window > 0 || mask_chunk > 0; }
 
 // The first key that the query at `pos` sees: a window of the last `window` positions (0: none) and/or the start
 // of the query's own masking chunk (0: none). It never falls as pos grows.
@@ -41,7 +51,8 @@ int attn_generic_launch(const void* q, int dtype, int ldq, const void* k_cache, 
                         int v_width, const int* block_table, int max_blocks, const int* token_slot, const int* positions,
                         void* out, int ldo, int n_tokens, int n_heads, int n_kv_heads, int head_dim, int v_head_dim,
                         int page_tokens, int window, int mask_chunk, float scale, const float* slopes, int sink, int cross, float softcap,
-                        int weights, const float* head_bias, hipStream_t stream);
+                        int weights, const float* head_bias, const float* sink_w, const float* dist_scale, const float* dist_rate,
+                        hipStream_t stream);
 
 // Single tokens of a mixer that mixes its heads' weights after the softmax: every head's weights on the values of every
 // group in one pass over the cache, written in rounds of groups (see attention_cross.hip). `supports` leaves the cut

@@ -71,9 +71,25 @@ union Frag {
 // new key, stores it and the new value into the cache (rows slot_map[token]) for the steps to come, and uses them
 // from LDS itself, since what the cache row held before is not the token's. What rope_store would have done in a
 // kernel and a pass over memory of its own.
-// SIG: the weights are no softmax but sigmoid(capped score + head_bias[head]) (see hfa_paged_attention); records of key
+// MODE ATT_SIGMOID: the weights are no softmax but sigmoid(capped score + head_bias[head]) (see hfa_paged_attention); records of key
 // chunks then carry maximum 0 and sum 1 in the first chunk and 0 in the others, so that the merge adds the chunks up.
-template <int NDB, bool SPLIT, bool FUSED, bool SIG = false>
+// MODE ATT_SHAPED: a softmax whose scores are soft-capped and/or lowered by a term of the distance first.
+#define ATT_PLAIN 0
+#define ATT_SIGMOID 1
+#define ATT_SHAPED 2
+#define LOG2E 1.4426950408889634f
+
+// A score in powers of two from the product `dot`: dot * scale (natural; sc = the scale), capped by c tanh(s / c) = c (1 - 2 / (1 +
+// exp(2 s / c))) where c > 0 (cap2 = 2 log2(e) / c), lowered by r1 ln(1 + r2 d).
+__device__ __forceinline__ float shaped_score(float dot, float sc, float softcap, float cap2, bool dist, float r1, float r2, float d) {
+    float sv = dot * sc;
+    if (softcap > 0.f) sv = softcap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + fast_exp2(sv * cap2)));
+    sv *= LOG2E;
+    if (dist) sv = fmaf(-r1, __builtin_amdgcn_logf(fmaf(r2, d, 1.0f)), sv);       // r1 ln(x) log2(e) = r1 log2(x)
+    return sv;
+}
+
+template <int NDB, bool SPLIT, bool FUSED, int MODE = ATT_PLAIN>
 __global__ __launch_bounds__(WAVE) void attn_mfma_kernel(
     const uint16_t* __restrict__ q, int ldq, const uint16_t* __restrict__ kc, const uint16_t* __restrict__ vc, int kvw,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ token_slot,
@@ -81,8 +97,10 @@ __global__ __launch_bounds__(WAVE) void attn_mfma_kernel(
     int ldo, float* __restrict__ partial, int H, int psh, int window, int mask_chunk, float scale_log2e, int tpt, int cpt,
     int chunk_keys, int n_chunks, int one_tile_each, const float* __restrict__ raw, int ld_raw,
     const float* __restrict__ cs, const int* __restrict__ slot_map, int G, int sink, int v_rot, float softcap = 0.f,
-    const float* __restrict__ head_bias = nullptr) {
+    const float* __restrict__ head_bias = nullptr, const float* __restrict__ sink_w = nullptr,
+    const float* __restrict__ dist_scale = nullptr, const float* __restrict__ dist_rate = nullptr) {
     constexpr int D = NDB * 32, KS = D / 16;
+    constexpr bool SIG = MODE == ATT_SIGMOID;
     const int P = 1 << psh;                                // tokens per page, a power of two
     const int lane = threadIdx.x, col = lane & 31, half = lane >> 5;
     const int g = blockIdx.y, chunk = blockIdx.z;
@@ -115,14 +133,16 @@ __global__ __launch_bounds__(WAVE) void attn_mfma_kernel(
     const int my_tok = col_ok ? t0 + col / cpt : t0;
     const int my_head = g * cpt + (col_ok ? col % cpt : 0);
     const float hb = (SIG && head_bias) ? head_bias[my_head] : 0.f;
+    const bool dist = MODE == ATT_SHAPED && dist_scale != nullptr;
+    const float r1 = dist ? dist_scale[my_head] : 0.f, r2 = dist ? dist_rate[my_head] : 0.f;
     const int pos = positions[my_tok];
     const int pos_first = positions[t0], hi = positions[t_end - 1];
     int k_begin = first_visible(pos_first, window, mask_chunk);
     int k_end = hi;
     if (SPLIT) {
-        // Under a mask by chunks the tile's keys begin far into the sequence: the cuts are then counted from the first
-        // key block that the tile sees, not from key 0 (whose chunks would mostly hold nothing).
-        const int c_lo = (mask_chunk > 0 ? k_begin / KB * KB : 0) + chunk * chunk_keys;
+        // Under a window or a mask by chunks the tile's keys begin far into the sequence: the cuts are then counted from the
+        // first key block that the tile sees, not from key 0 (whose chunks would mostly hold nothing).
+        const int c_lo = (attn_bounded(window, mask_chunk) ? k_begin / KB * KB : 0) + chunk * chunk_keys;
         k_begin = k_begin > c_lo ? k_begin : c_lo;
         k_end = k_end < c_lo + chunk_keys - 1 ? k_end : c_lo + chunk_keys - 1;
     }
@@ -312,7 +332,7 @@ __global__ __launch_bounds__(WAVE) void attn_mfma_kernel(
                 st[r] = (kr >= vlo && kr <= vhi) ? __builtin_amdgcn_rcpf(1.0f + fast_exp2(-1.4426950408889634f * (sv + hb))) : 0.f;
             }
         } else {
-            const bool inside = __all(!col_ok || (key0 >= vlo && key0 + KB - 1 <= vhi)) != 0;
+            const bool inside = MODE == ATT_PLAIN && __all(!col_ok || (key0 >= vlo && key0 + KB - 1 <= vhi)) != 0;
             float mx = NEG_BIG, mn, corr, psum = 0.f;
             if (inside) {
 #pragma unroll
@@ -326,11 +346,14 @@ __global__ __launch_bounds__(WAVE) void attn_mfma_kernel(
                     psum += st[r];
                 }
             } else {
+                const float cap2 = MODE == ATT_SHAPED && softcap > 0.f ? 2.0f * LOG2E / softcap : 0.f;
 #pragma unroll
                 for (int r = 0; r < 16; r++) {
                     const int kr = key0 + 8 * (r / 4) + 4 * half + (r % 4);
                     const bool vis = kr >= vlo && kr <= vhi;
-                    st[r] = vis ? st[r] * scale_log2e : NEG_BIG;
+                    const float sv = MODE == ATT_SHAPED ? shaped_score(st[r], scale_log2e * 0.6931471805599453f, softcap, cap2, dist, r1, r2, (float)(pos - kr))
+                                                        : st[r] * scale_log2e;
+                    st[r] = vis ? sv : NEG_BIG;
                     mx = fmaxf(mx, st[r]);
                 }
                 mx = pair_max(mx);
@@ -478,7 +501,7 @@ __global__ __launch_bounds__(WAVE) void attn_mfma_kernel(
                 *reinterpret_cast<float4*>(dst + 2 + 32 * db + 8 * rg + 4 * half) = v;
             }
     } else {
-        const float inv = 1.0f / (sink ? l + exp2f(-m) : l);      // the term of score 0 and no value: 2^(0 - m)
+        const float inv = 1.0f / (sink ? l + exp2f((sink_w ? sink_w[my_head] * LOG2E : 0.f) - m) : l);      // the term that has no value
         uint16_t* dst = out + (size_t)my_tok * ldo + my_head * D;
 #pragma unroll
         for (int db = 0; db < NDB; db++)
@@ -503,15 +526,17 @@ __global__ __launch_bounds__(WAVE) void attn_mfma_kernel(
 // are numbered from the end of each request backwards, so the longest ones start first.
 #define PVS 36       // LDS row of a value dimension: 32 keys + 4 pad (elements)
 
-template <int NDB, bool SMALL_PAGES, bool SIG = false>
+template <int NDB, bool SMALL_PAGES, int MODE = ATT_PLAIN>
 __global__ __launch_bounds__(4 * WAVE) __attribute__((amdgpu_waves_per_eu(2))) void attn_prefill_kernel(
     const uint16_t* __restrict__ q, int ldq, const uint16_t* __restrict__ kc, const uint16_t* __restrict__ vc, int kvw,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ token_slot,
     const int* __restrict__ positions, const int* __restrict__ q_start, int n_seqs, uint16_t* __restrict__ out,
     int ldo, int psh, int window, int mask_chunk, float scale_log2e, int tpt, int cpt, int n_tiles, int pair_from,
     float* __restrict__ partial, int H, int chunk_keys, int n_chunks, int sink, int v_rot, float softcap = 0.f,
-    const float* __restrict__ head_bias = nullptr) {
+    const float* __restrict__ head_bias = nullptr, const float* __restrict__ sink_w = nullptr,
+    const float* __restrict__ dist_scale = nullptr, const float* __restrict__ dist_rate = nullptr) {
     constexpr int D = NDB * 32, KS = D / 16, KROW = D + 8;
+    constexpr bool SIG = MODE == ATT_SIGMOID;
     const int P = 1 << psh;                                // tokens per page, a power of two
     __shared__ __attribute__((aligned(16))) uint16_t k_s[2][KB * KROW];
     __shared__ __attribute__((aligned(16))) uint16_t v_s[2][D * PVS];
@@ -560,6 +585,8 @@ __global__ __launch_bounds__(4 * WAVE) __attribute__((amdgpu_waves_per_eu(2))) v
     const int my_tok = col_ok ? w0 + col / cpt : t0;
     const int my_head = g * cpt + (col_ok ? col % cpt : 0);
     const float hb = (SIG && head_bias) ? head_bias[my_head] : 0.f;
+    const bool dist = MODE == ATT_SHAPED && dist_scale != nullptr;
+    const float r1 = dist ? dist_scale[my_head] : 0.f, r2 = dist ? dist_rate[my_head] : 0.f;
     const int pos = positions[my_tok];
     const int pos_first = positions[t0];
     int hi = positions[t_end - 1];
@@ -568,8 +595,8 @@ __global__ __launch_bounds__(4 * WAVE) __attribute__((amdgpu_waves_per_eu(2))) v
     // of the key block) and leaves maximum, sum and unscaled output for attn_merge_kernel; a chunk
     // that holds none of the tile's keys leaves an empty record.
     if (n_chunks > 1) {
-        // (under a mask by chunks, counted from the first key block that the tile sees: see attn_mfma_kernel)
-        const int c_lo = (mask_chunk > 0 ? k_begin / KB * KB : 0) + blockIdx.z * chunk_keys, c_hi = c_lo + chunk_keys - 1;
+        // (under a window or a mask by chunks, counted from the first key block that the tile sees: see attn_mfma_kernel)
+        const int c_lo = (attn_bounded(window, mask_chunk) ? k_begin / KB * KB : 0) + blockIdx.z * chunk_keys, c_hi = c_lo + chunk_keys - 1;
         k_begin = k_begin > c_lo ? k_begin : c_lo;
         hi = hi < c_hi ? hi : c_hi;
     }
@@ -749,7 +776,7 @@ __global__ __launch_bounds__(4 * WAVE) __attribute__((amdgpu_waves_per_eu(2))) v
                         st[r] = (kr >= vlo && kr <= vhi) ? __builtin_amdgcn_rcpf(1.0f + fast_exp2(-1.4426950408889634f * (sv + hb))) : 0.f;
                     }
                 } else {
-                    const bool inside = __all(!col_ok || (key0 >= vlo && key0 + KB - 1 <= vhi)) != 0;
+                    const bool inside = MODE == ATT_PLAIN && __all(!col_ok || (key0 >= vlo && key0 + KB - 1 <= vhi)) != 0;
                     float mx = NEG_BIG, mn, corr, psum = 0.f;
                     if (inside) {                                   // the scale (positive) moves into the exponent's fma
 #pragma unroll
@@ -763,11 +790,14 @@ __global__ __launch_bounds__(4 * WAVE) __attribute__((amdgpu_waves_per_eu(2))) v
                             psum += st[r];
                         }
                     } else {
+                        const float cap2 = MODE == ATT_SHAPED && softcap > 0.f ? 2.0f * LOG2E / softcap : 0.f;
 #pragma unroll
                         for (int r = 0; r < 16; r++) {
                             const int kr = key0 + 8 * (r / 4) + 4 * half + (r % 4);
                             const bool vis = kr >= vlo && kr <= vhi;
-                            st[r] = vis ? st[r] * scale_log2e : NEG_BIG;
+                            const float sv = MODE == ATT_SHAPED ? shaped_score(st[r], scale_log2e * 0.6931471805599453f, softcap, cap2, dist, r1, r2, (float)(pos - kr))
+                                                                : st[r] * scale_log2e;
+                            st[r] = vis ? sv : NEG_BIG;
                             mx = fmaxf(mx, st[r]);
                         }
                         mx = pair_max(mx);
@@ -839,7 +869,7 @@ __global__ __launch_bounds__(4 * WAVE) __attribute__((amdgpu_waves_per_eu(2))) v
                     make_float4(o[db][4 * rg], o[db][4 * rg + 1], o[db][4 * rg + 2], o[db][4 * rg + 3]);
         return;
     }
-    const float inv = 1.0f / (sink ? l + exp2f(-m) : l);          // the term of score 0 and no value: 2^(0 - m)
+    const float inv = 1.0f / (sink ? l + exp2f((sink_w ? sink_w[my_head] * LOG2E : 0.f) - m) : l);          // the term that has no value
     uint16_t* dst = out + (size_t)my_tok * ldo + my_head * D;
 #pragma unroll
     for (int db = 0; db < NDB; db++)
@@ -860,7 +890,8 @@ __global__ __launch_bounds__(4 * WAVE) __attribute__((amdgpu_waves_per_eu(2))) v
 #define MERGE_MAX_CHUNKS 512
 #define MERGE_GROUP 16
 __global__ __launch_bounds__(WAVE) void attn_merge_kernel(const float* __restrict__ partial, uint16_t* __restrict__ out,
-                                                          int ldo, int H, int D, int n_chunks, int sink) {
+                                                          int ldo, int H, int D, int n_chunks, int sink,
+                                                          const float* __restrict__ sink_w) {
     __shared__ float w_s[MERGE_MAX_CHUNKS];
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const size_t row = D + 2;
@@ -888,7 +919,7 @@ __global__ __launch_bounds__(WAVE) void attn_merge_kernel(const float* __restric
         L += ml.y * w;
     }
     L = wave_sum(L);
-    if (sink) L += exp2f(-M);                            // once for all chunks: the term of score 0 and no value
+    if (sink) L += exp2f((sink_w ? sink_w[h] * LOG2E : 0.f) - M);       // once for all chunks: the term that has no value
     __syncthreads();
     if (!has) return;
     float ax = 0.f, ay = 0.f;
@@ -939,17 +970,19 @@ static int launch_ndb(const AttnArgs& a, int tiles, int tpt, int cpt, int chunk_
     (const uint16_t*)a.q, a.ldq, (const uint16_t*)a.k_cache, (const uint16_t*)a.v_cache, a.kv_width, a.block_table,      \
         a.max_blocks, a.token_slot, a.positions, a.q_start, a.n_seqs, (uint16_t*)a.out, a.ldo, PARTIAL, a.n_heads,         \
         page_shift(a.page_tokens), a.window, a.mask_chunk, sl, tpt, cpt, chunk_keys, n_chunks, a.max_q_len <= tpt, a.raw, a.ld_raw,      \
-        a.cos_sin, a.slot_map, a.n_kv_heads, a.sink, a.v_rot
-    if (a.weights == 1) {
-        if (n_chunks > 1) attn_mfma_kernel<NDB, true, false, true><<<grid, WAVE, 0, a.stream>>>(ATTN_ARGS((float*)a.workspace), a.softcap, a.head_bias);
-        else attn_mfma_kernel<NDB, false, false, true><<<grid, WAVE, 0, a.stream>>>(ATTN_ARGS(nullptr), a.softcap, a.head_bias);
-    } else if (a.raw) {
-        if (n_chunks > 1) attn_mfma_kernel<NDB, true, true><<<grid, WAVE, 0, a.stream>>>(ATTN_ARGS((float*)a.workspace));
-        else attn_mfma_kernel<NDB, false, true><<<grid, WAVE, 0, a.stream>>>(ATTN_ARGS(nullptr));
-    } else {
-        if (n_chunks > 1) attn_mfma_kernel<NDB, true, false><<<grid, WAVE, 0, a.stream>>>(ATTN_ARGS((float*)a.workspace));
-        else attn_mfma_kernel<NDB, false, false><<<grid, WAVE, 0, a.stream>>>(ATTN_ARGS(nullptr));
-    }
+        a.cos_sin, a.slot_map, a.n_kv_heads, a.sink, a.v_rot, a.softcap, a.head_bias, a.sink_w, a.dist_scale, a.dist_rate
+#define ATTN_GO(FUSED, MODE)                                                                                               \
+    do {                                                                                                                   \
+        if (n_chunks > 1) attn_mfma_kernel<NDB, true, FUSED, MODE><<<grid, WAVE, 0, a.stream>>>(ATTN_ARGS((float*)a.workspace)); \
+        else attn_mfma_kernel<NDB, false, FUSED, MODE><<<grid, WAVE, 0, a.stream>>>(ATTN_ARGS(nullptr));                    \
+    } while (0)
+    const bool shaped = attn_shaped_scores(a);
+    if (a.weights == 1) ATTN_GO(false, ATT_SIGMOID);
+    else if (a.raw && shaped) ATTN_GO(true, ATT_SHAPED);
+    else if (a.raw) ATTN_GO(true, ATT_PLAIN);
+    else if (shaped) ATTN_GO(false, ATT_SHAPED);
+    else ATTN_GO(false, ATT_PLAIN);
+#undef ATTN_GO
 #undef ATTN_ARGS
     HFA_LAUNCH_CHECK("attn_mfma");
     return 0;
@@ -978,10 +1011,11 @@ static int launch_prefill(const AttnArgs& a, int tpt, int cpt) {
     // chunks' results together (portions of a few hundred tokens far into a long prompt).
     int n_chunks = 1, chunk_keys = a.max_seq_len;
     const long blocks = (long)a.n_kv_heads * ((a.n_tokens + tile_tokens - 1) / tile_tokens);
-    // the keys that one tile can see: all of the sequence, or a masking chunk and the tile's own tokens (and the key
+    // the keys that one tile can see: all of the sequence, or a window or masking chunk and the tile's own tokens (and the key
     // block that the cuts are aligned to); the cuts are made over these
     int reach = a.max_seq_len;
     if (a.mask_chunk > 0 && a.mask_chunk + tile_tokens + KB < reach) reach = a.mask_chunk + tile_tokens + KB;
+    if (a.window > 0 && a.window + tile_tokens + KB < reach) reach = a.window + tile_tokens + KB;
     if (blocks < 2 * cus && reach >= 512 && a.workspace != nullptr) {
         long want = (2 * cus + blocks - 1) / blocks;
         if (want > reach / 256) want = reach / 256;
@@ -1001,19 +1035,21 @@ static int launch_prefill(const AttnArgs& a, int tpt, int cpt) {
     (const uint16_t*)a.q, a.ldq, (const uint16_t*)a.k_cache, (const uint16_t*)a.v_cache, a.kv_width, a.block_table,            \
         a.max_blocks, a.token_slot, a.positions, a.q_start, a.n_seqs, (uint16_t*)a.out, a.ldo, page_shift(a.page_tokens),      \
         a.window, a.mask_chunk, a.scale * 1.4426950408889634f, tpt, cpt, n_tiles, pair_from, (float*)a.workspace, a.n_heads,   \
-        chunk_keys, n_chunks, a.sink, a.v_rot
-    if (a.weights == 1) {
-        if (a.page_tokens <= 32) attn_prefill_kernel<NDB, true, true><<<grid, 4 * WAVE, 0, a.stream>>>(PREFILL_ARGS, a.softcap, a.head_bias);
-        else attn_prefill_kernel<NDB, false, true><<<grid, 4 * WAVE, 0, a.stream>>>(PREFILL_ARGS, a.softcap, a.head_bias);
-    } else if (a.page_tokens <= 32)
-        attn_prefill_kernel<NDB, true><<<grid, 4 * WAVE, 0, a.stream>>>(PREFILL_ARGS);
-    else
-        attn_prefill_kernel<NDB, false><<<grid, 4 * WAVE, 0, a.stream>>>(PREFILL_ARGS);
+        chunk_keys, n_chunks, a.sink, a.v_rot, a.softcap, a.head_bias, a.sink_w, a.dist_scale, a.dist_rate
+#define PREFILL_GO(MODE)                                                                                   \
+    do {                                                                                                   \
+        if (a.page_tokens <= 32) attn_prefill_kernel<NDB, true, MODE><<<grid, 4 * WAVE, 0, a.stream>>>(PREFILL_ARGS); \
+        else attn_prefill_kernel<NDB, false, MODE><<<grid, 4 * WAVE, 0, a.stream>>>(PREFILL_ARGS);          \
+    } while (0)
+    if (a.weights == 1) PREFILL_GO(ATT_SIGMOID);
+    else if (attn_shaped_scores(a)) PREFILL_GO(ATT_SHAPED);
+    else PREFILL_GO(ATT_PLAIN);
+#undef PREFILL_GO
 #undef PREFILL_ARGS
     HFA_LAUNCH_CHECK("attn_prefill");
     if (n_chunks > 1) {
         attn_merge_kernel<<<dim3(a.n_tokens, a.n_heads), WAVE, 0, a.stream>>>((const float*)a.workspace, (uint16_t*)a.out, a.ldo,
-                                                                            a.n_heads, a.head_dim, n_chunks, a.sink);
+                                                                            a.n_heads, a.head_dim, n_chunks, a.sink, a.sink_w);
         HFA_LAUNCH_CHECK("attn_merge");
     }
     return 0;
@@ -1059,8 +1095,8 @@ int attn_mfma_launch(const AttnArgs& a) {
         int want = (int)((fill + waves - 1) / waves);
         const int most = (span + 127) / 128;
         if (want > most) want = most;
-        // under a mask by chunks the cuts are counted from the tile's first key block: they cover what a tile can see
-        const int reach = a.mask_chunk > 0 && span + KB < a.max_seq_len ? span + KB : a.max_seq_len;
+        // under a window or a mask by chunks the cuts are counted from the tile's first key block: they cover what a tile can see
+        const int reach = attn_bounded(a.window, a.mask_chunk) && span + KB < a.max_seq_len ? span + KB : a.max_seq_len;
         chunk_keys = ((reach + want - 1) / want + KB - 1) / KB * KB;
         if (chunk_keys < 64) chunk_keys = 64;
         n_chunks = (reach + chunk_keys - 1) / chunk_keys;
@@ -1080,7 +1116,7 @@ int attn_mfma_launch(const AttnArgs& a) {
     if (rc || n_chunks == 1) return rc;
     dim3 grid(a.n_tokens, a.n_heads);
     attn_merge_kernel<<<grid, WAVE, 0, a.stream>>>((const float*)a.workspace, (uint16_t*)a.out, a.ldo, a.n_heads,
-                                                  a.head_dim, n_chunks, a.sink);
+                                                  a.head_dim, n_chunks, a.sink, a.sink_w);
     HFA_LAUNCH_CHECK("attn_merge");
     return 0;
 }

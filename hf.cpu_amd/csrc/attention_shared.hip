@@ -54,7 +54,8 @@ __global__ __launch_bounds__(4 * WAVE) void attn_shared_kernel(
     const uint16_t* __restrict__ q, int ldq, const uint16_t* __restrict__ kc, const uint16_t* __restrict__ vc, int DK, int C,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ token_slot, const int* __restrict__ positions,
     const int* __restrict__ q_start, int n_seqs, uint16_t* __restrict__ out, int ldo, float* __restrict__ partial, int H, int psh,
-    float scale_log2e, int tpt, int cpt, int chunk_keys, int n_chunks, int one_tile_each) {
+    float scale_log2e, int tpt, int cpt, int chunk_keys, int n_chunks, int one_tile_each, int window, int mask_chunk,
+    int sink, const float* __restrict__ sink_w) {
     __shared__ float part_s[2][4][16][WAVE];
     const int P = 1 << psh;
     const int tid = threadIdx.x, lane = tid & (WAVE - 1), wave = tid / WAVE, col = lane & 31, half = lane >> 5;
@@ -84,12 +85,15 @@ __global__ __launch_bounds__(4 * WAVE) void attn_shared_kernel(
     const int my_tok = col_ok ? t0 + col / cpt : t0;
     const int pos = positions[my_tok];
     const int hi = positions[t_end - 1];
-    int k_begin = 0, k_end = hi;
+    int k_begin = first_visible(positions[t0], window, mask_chunk), k_end = hi;
     if (SPLIT) {
-        k_begin = chunk * chunk_keys;
-        k_end = k_end < k_begin + chunk_keys - 1 ? k_end : k_begin + chunk_keys - 1;
+        // under a window or a mask by chunks the cuts are counted from the first key block that the tile sees
+        const int c_lo = (attn_bounded(window, mask_chunk) ? k_begin / SH_KB * SH_KB : 0) + chunk * chunk_keys;
+        k_begin = k_begin > c_lo ? k_begin : c_lo;
+        k_end = k_end < c_lo + chunk_keys - 1 ? k_end : c_lo + chunk_keys - 1;
     }
-    const int vlo = k_begin, vhi = col_ok ? (pos < k_end ? pos : k_end) : -1;
+    const int my_first = first_visible(pos, window, mask_chunk);
+    const int vlo = my_first > k_begin ? my_first : k_begin, vhi = col_ok ? (pos < k_end ? pos : k_end) : -1;
     const int* bt = block_table + (size_t)token_slot[t0] * max_blocks;
 
     ShFrag qf[KSW];
@@ -235,7 +239,7 @@ __global__ __launch_bounds__(4 * WAVE) void attn_shared_kernel(
                 for (int e = 0; e < 4; e++) dst[2 + 32 * db + 8 * rg + 4 * half + e] = o[j][4 * rg + e];
         }
     } else {
-        const float inv = 1.0f / l;
+        const float inv = 1.0f / (sink ? l + exp2f((sink_w ? sink_w[my_head] * 1.4426950408889634f : 0.f) - m) : l);   // the term that has no value
         uint16_t* dst = out + (size_t)my_tok * ldo + (size_t)my_head * C;
 #pragma unroll
         for (int j = 0; j < NDBW; j++) {
@@ -256,7 +260,7 @@ __global__ __launch_bounds__(4 * WAVE) void attn_shared_kernel(
 // a chain of trips to memory and little else: the chunks' maxima and sums are fetched by one thread each, at once, and a thread's
 // values of all chunks are asked for eight at a time before they are added.
 __global__ __launch_bounds__(256) void attn_shared_merge_kernel(const float* __restrict__ partial, uint16_t* __restrict__ out, int ldo, int H,
-                                                                int C, int n_chunks) {
+                                                                int C, int n_chunks, int sink, const float* __restrict__ sink_w) {
     __shared__ float m_s[SH_MAX_CHUNKS], l_s[SH_MAX_CHUNKS], w_s[SH_MAX_CHUNKS];
     const int t = blockIdx.x, h = blockIdx.y;
     const size_t row = C + 2;
@@ -276,6 +280,7 @@ __global__ __launch_bounds__(256) void attn_shared_merge_kernel(const float* __r
         L = fmaf(l_s[c], w, L);
     }
     __syncthreads();
+    if (sink) L += exp2f((sink_w ? sink_w[h] * 1.4426950408889634f : 0.f) - M);     // once for all chunks: the term that has no value
     const float inv = 1.0f / L;
     for (int d = threadIdx.x; d < C; d += blockDim.x) {
         float acc = 0.f;
@@ -300,7 +305,7 @@ static int sh_page_shift(int page_tokens) {
 bool attn_shared_supports(const AttnArgs& a, int v_head_dim, int v_width) {
     return a.n_kv_heads == 1 && a.head_dim % 16 == 0 && a.head_dim <= 576 && v_head_dim % 32 == 0 && v_head_dim <= 512 &&
            a.kv_width == a.head_dim && v_width == v_head_dim && a.page_tokens >= 4 && sh_page_shift(a.page_tokens) >= 0 && a.scale > 0.f &&
-           a.window == 0 && a.mask_chunk == 0 && !a.sink && a.v_rot == 0 && a.weights == 0 && a.softcap == 0.f && a.q_start != nullptr &&
+           a.v_rot == 0 && a.weights == 0 && !attn_shaped_scores(a) && a.q_start != nullptr &&
            a.raw == nullptr && a.ldq % 8 == 0 && a.ldo % 4 == 0 && ((uintptr_t)a.q & 15) == 0 && ((uintptr_t)a.out & 7) == 0 &&
            ((uintptr_t)a.k_cache & 15) == 0 && ((uintptr_t)a.v_cache & 15) == 0 && (size_t)a.n_tokens * a.n_heads < ((size_t)1 << 31) / 600;
 }
@@ -314,13 +319,18 @@ int attn_shared_launch(const AttnArgs& a, int v_head_dim) {
     // few blocks and long contexts: cut the keys into chunks so that the machine is full
     int n_chunks = 1, chunk_keys = a.max_seq_len;
     const long blocks = (long)(one_each ? a.n_seqs : (a.n_tokens + tpt - 1) / tpt) * head_blocks;
-    if (blocks < 512 && a.max_seq_len > 256 && a.workspace) {
+    // the keys that one tile can see: all of the sequence, or a window or masking chunk, the tile's own tokens and the key block
+    // that the cuts are aligned to
+    int reach = a.max_seq_len;
+    if (a.window > 0 && a.window + tpt + SH_KB < reach) reach = a.window + tpt + SH_KB;
+    if (a.mask_chunk > 0 && a.mask_chunk + tpt + SH_KB < reach) reach = a.mask_chunk + tpt + SH_KB;
+    if (blocks < 512 && reach > 256 && a.workspace) {
         long want = (512 + blocks - 1) / blocks;
-        const long most = (a.max_seq_len + 127) / 128;        // no chunk of fewer than 128 keys (64 were measured: no gain)
+        const long most = (reach + 127) / 128;                // no chunk of fewer than 128 keys (64 were measured: no gain)
         if (want > most) want = most;
         if (want > SH_MAX_CHUNKS) want = SH_MAX_CHUNKS;
-        chunk_keys = (int)(((a.max_seq_len + want - 1) / want + SH_KB - 1) / SH_KB * SH_KB);
-        n_chunks = (a.max_seq_len + chunk_keys - 1) / chunk_keys;
+        chunk_keys = (int)(((reach + want - 1) / want + SH_KB - 1) / SH_KB * SH_KB);
+        n_chunks = (reach + chunk_keys - 1) / chunk_keys;
         const size_t need = (size_t)a.n_tokens * H * n_chunks * (C + 2) * sizeof(float);
         if (n_chunks < 2 || n_chunks > SH_MAX_CHUNKS || need > a.workspace_bytes) {
             n_chunks = 1;
@@ -332,7 +342,7 @@ int attn_shared_launch(const AttnArgs& a, int v_head_dim) {
 #define SH_ARGS                                                                                                                     \
     (const uint16_t*)a.q, a.ldq, (const uint16_t*)a.k_cache, (const uint16_t*)a.v_cache, DK, C, a.block_table, a.max_blocks,          \
         a.token_slot, a.positions, a.q_start, a.n_seqs, (uint16_t*)a.out, a.ldo, (float*)a.workspace, H, sh_page_shift(a.page_tokens), \
-        sl, tpt, cpt, chunk_keys, n_chunks, one_each
+        sl, tpt, cpt, chunk_keys, n_chunks, one_each, a.window, a.mask_chunk, a.sink, a.sink_w
 #define SH_GO(KSW, NDBW)                                                                               \
     do {                                                                                               \
         if (n_chunks > 1) attn_shared_kernel<KSW, NDBW, true><<<grid, 4 * WAVE, 0, a.stream>>>(SH_ARGS); \
@@ -345,7 +355,7 @@ int attn_shared_launch(const AttnArgs& a, int v_head_dim) {
 #undef SH_ARGS
     HFA_LAUNCH_CHECK("attn_shared");
     if (n_chunks > 1) {
-        attn_shared_merge_kernel<<<dim3(a.n_tokens, H), 256, 0, a.stream>>>((const float*)a.workspace, (uint16_t*)a.out, a.ldo, H, C, n_chunks);
+        attn_shared_merge_kernel<<<dim3(a.n_tokens, H), 256, 0, a.stream>>>((const float*)a.workspace, (uint16_t*)a.out, a.ldo, H, C, n_chunks, a.sink, a.sink_w);
         HFA_LAUNCH_CHECK("attn_shared_merge");
     }
     return 0;

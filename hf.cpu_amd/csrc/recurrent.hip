@@ -16,12 +16,12 @@
 #define CONV_SEG 64              // tokens that one thread walks
 
 // One thread a (request, run of CONV_SEG tokens, channel). state row: [K - 1][C] inputs, oldest first.
-template <typename T>
+template <typename T, typename TO>
 __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ in, int ld_in, const float* __restrict__ taps,
                                                          const float* __restrict__ bias, int C, int K,
                                                          float* __restrict__ state, size_t state_ld,
                                                          const int* __restrict__ q_start, const int* __restrict__ seq_slot,
-                                                         float* __restrict__ out, int ldo, int act) {
+                                                         TO* __restrict__ out, int ldo, int act) {
     const int c = blockIdx.x * blockDim.x + threadIdx.x, s = blockIdx.z;
     if (c >= C) return;
     const int q0 = q_start[s], n = q_start[s + 1] - q0, t0 = blockIdx.y * CONV_SEG;
@@ -52,7 +52,7 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
 #pragma unroll
         for (int j = 0; j < CONV_MAX_TAPS; j++)
             if (j < K) acc = fmaf(w[j], win[j], acc);
-        out[(size_t)(q0 + t) * ldo + c] = act == HFA_ACT_SILU ? acc / (1.0f + expf(-acc)) : acc;
+        out[(size_t)(q0 + t) * ldo + c] = from_f32<TO>(act == HFA_ACT_SILU ? acc / (1.0f + expf(-acc)) : acc);
 #pragma unroll
         for (int j = 0; j < CONV_MAX_TAPS - 1; j++) win[j] = win[j + 1];
     }
@@ -60,22 +60,22 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
 
 extern "C" int hfa_causal_conv(const void* in, int dtype, int ld_in, const float* taps, const float* bias, int n_channels,
                                int n_taps, float* state, size_t state_ld, const int* q_start, const int* seq_slot, int n_seqs,
-                               int max_q_len, float* out, int ldo, int act, hipStream_t stream) {
+                               int max_q_len, void* out, int out_dtype, int ldo, int act, hipStream_t stream) {
     HFA_REQUIRE(in && taps && (state || n_taps == 1) && q_start && seq_slot && out && n_channels > 0 && n_seqs > 0 && max_q_len > 0,
                 "causal_conv: bad arguments");
     HFA_REQUIRE(n_taps >= 1 && n_taps <= CONV_MAX_TAPS, "causal_conv: %d taps (1 to %d)", n_taps, CONV_MAX_TAPS);
     HFA_REQUIRE(ld_in >= n_channels && ldo >= n_channels && state_ld >= (size_t)(n_taps - 1) * n_channels,
                 "causal_conv: a row is shorter than its channels");
     HFA_REQUIRE(act == HFA_ACT_NONE || act == HFA_ACT_SILU, "causal_conv: the activation is silu or none");
-    HFA_REQUIRE(dtype == HFA_F32 || dtype == HFA_BF16, "causal_conv: unknown dtype %d", dtype);
+    HFA_REQUIRE((dtype == HFA_F32 || dtype == HFA_BF16) && (out_dtype == HFA_F32 || out_dtype == HFA_BF16), "causal_conv: unknown dtype %d or %d", dtype, out_dtype);
     HFA_REQUIRE(n_seqs <= 65535 && (max_q_len + CONV_SEG - 1) / CONV_SEG <= 65535, "causal_conv: the step exceeds the grid");
     dim3 grid((n_channels + 255) / 256, (max_q_len + CONV_SEG - 1) / CONV_SEG, n_seqs);
-    if (dtype == HFA_F32)
-        causal_conv_kernel<float><<<grid, 256, 0, stream>>>((const float*)in, ld_in, taps, bias, n_channels, n_taps, state, state_ld,
-                                                            q_start, seq_slot, out, ldo, act);
-    else
-        causal_conv_kernel<bf16><<<grid, 256, 0, stream>>>((const bf16*)in, ld_in, taps, bias, n_channels, n_taps, state, state_ld,
-                                                           q_start, seq_slot, out, ldo, act);
+#define CONV_GO(T, TO)                                                                                                                    \
+    causal_conv_kernel<T, TO><<<grid, 256, 0, stream>>>((const T*)in, ld_in, taps, bias, n_channels, n_taps, state, state_ld, q_start, seq_slot, \
+                                                        (TO*)out, ldo, act)
+    if (dtype == HFA_F32) { if (out_dtype == HFA_F32) CONV_GO(float, float); else CONV_GO(float, bf16); }
+    else { if (out_dtype == HFA_F32) CONV_GO(bf16, float); else CONV_GO(bf16, bf16); }
+#undef CONV_GO
     HFA_LAUNCH_CHECK("causal_conv");
     return 0;
 }

@@ -92,6 +92,16 @@ class Scaled:
     source_changed: bool = False       # x has gone on since: products may still read `out`, nothing can make it whole
 
 
+@dataclass
+class StreamUpdate:
+    """What a sublayer leaves undone on a residual of several streams: its result ``y`` has yet to go into them. ``mix`` None:
+    every stream becomes ``y`` (the copies of the embedding at the start)."""
+    x: torch.Tensor          # [T, streams, width]
+    y: torch.Tensor          # [T, width] (or a product into it that is still pending)
+    mix: object
+    out: object
+
+
 class _NoSection:
     def __enter__(self):
         return self
@@ -145,6 +155,8 @@ class Ops:
         self._pending = None
         self._lazy = None                    # a LazyProduct
         self._lazy_rope = None               # a LazyRope
+        self._stream_undone = None           # a StreamUpdate
+        self._head_plans = {}                # (rows, heads, tile) -> tiles of the heads' products, made once a pass
         self._rope_tables = {}               # (positions, frequencies, tokens) -> cosines and sines of a pass's angles
         self._scaled = {}                    # data_ptr of a norm's output -> Scaled
         self.rows_parts = int(self.lib.hfa_gemm_rows_parts())
@@ -193,6 +205,7 @@ class Ops:
         self._stream_handle = torch.cuda.current_stream(self.device).cuda_stream
         self._scaled.clear()                 # what an earlier pass left in its work buffers is of no use to this one
         self._rope_tables.clear()
+        self._head_plans.clear()
         try:
             yield self
         finally:
@@ -398,6 +411,7 @@ class Ops:
         self._pending = None
         self._lazy = None
         self._lazy_rope = None
+        self._stream_undone = None
         self._scaled.clear()
 
     # ---- products of few rows that finish their outputs themselves (csrc/gemm_rows.hip) -----------------------
@@ -486,6 +500,10 @@ class Ops:
             self._rows_resid(z)
         if tensor is not None:
             self._whole(tensor)
+        su = self._stream_undone
+        if su is not None and (tensor is None or su.x.data_ptr() == tensor.data_ptr()):
+            self._stream_undone = None
+            self._stream_step(su, su.x)
         p = self._pending
         if p is None or (tensor is not None and p.out.data_ptr() != tensor.data_ptr()):
             return
@@ -621,7 +639,8 @@ class Ops:
             None if pend is None or pend.bias is None else pend.bias.data_ptr(), self._stream()))
 
     def paged_attention(self, q, n_heads, n_kv_heads, head_dim, cache, step, window, scale, out, slopes=None,
-                        v_head_dim=None, mask_chunk=0, sink=False, cross_values=False, softcap=0.0, weights="softmax", head_bias=None):
+                        v_head_dim=None, mask_chunk=0, sink=False, cross_values=False, softcap=0.0, weights="softmax", head_bias=None,
+                        sink_scores=None, distance=None):
         """Attention of the first ``n_heads * head_dim`` columns of ``q`` over ``cache``. ``slopes``
         (fp32, one per query head): the score of key j for the query at p gets ``slopes[h] * (j - p)``
         added, for position encodings that enter the scores; the plain kernel then runs, as it does when
@@ -632,7 +651,9 @@ class Ops:
         round r of head h (at ``(r * heads + h) * v_head_dim``) being its weights on the values of group (h's group + r) mod
         groups (see ``talk_mix``). ``softcap`` c > 0: a score becomes ``c tanh(score / c)`` before the weights are formed.
         ``weights`` ``"sigmoid"``: no softmax; a visible key weighs ``sigmoid(score + head_bias[h])`` (``head_bias``: fp32, one per
-        query head, or None), and the weights are not normalised over the keys (on the matrix cores where a softmax would be; a cap under a softmax takes the plain kernel)."""
+        query head, or None), and the weights are not normalised over the keys. ``sink_scores`` (fp32, one per query head; with
+        ``sink``): the extra term's score is the head's number instead of 0. ``distance`` = (a, b) (fp32, one per query head each;
+        softmax only): after scale and cap the score of key j for the query at p is lowered by ``a[h] ln(1 + b[h] (p - j))``."""
         v_head_dim = head_dim if v_head_dim is None else int(v_head_dim)
         mask_chunk = int(mask_chunk)
         if weights not in ("softmax", "sigmoid") or (weights == "sigmoid" and (sink or cross_values)):
@@ -641,17 +662,21 @@ class Ops:
                                       or not head_bias.is_contiguous() or head_bias.device != q.device):
             fail(EINVAL, "paged_attention: head_bias goes with sigmoid weights and is contiguous fp32 on the device, one per query head")
         softcap = float(softcap or 0.0)
-        shaped_scores = softcap != 0.0 or weights != "softmax"
-        plain_scores = softcap != 0.0 and weights == "softmax"        # what only the plain kernel computes
+        for t, what in ((sink_scores, "sink_scores"),) + tuple((t, "distance") for t in (distance or ())):
+            if t is not None and (t.dtype != torch.float32 or t.numel() != n_heads or not t.is_contiguous() or t.device != q.device):
+                fail(EINVAL, f"paged_attention: {what} is contiguous fp32 on the device, one number per query head")
+        if (sink_scores is not None and not sink) or (distance is not None and (weights != "softmax" or slopes is not None or cross_values)):
+            fail(EINVAL, "paged_attention: sink_scores go with a sink term, a distance term with a softmax over a head's own values")
+        dist_a, dist_b = (None, None) if distance is None else (distance[0].data_ptr(), distance[1].data_ptr())
         self._scaled.pop(out.data_ptr(), None)               # whatever `out` held, it is no norm's lazy output any more
         lr = self._lazy_rope
         if lr is not None and lr.qkv.data_ptr() == q.data_ptr() and lr.cache is cache and slopes is None and not sink \
-                and not cross_values and not shaped_scores \
+                and not cross_values and weights == "softmax" \
                 and step.max_q_len == 1 and step.n_seqs == q.shape[0] and not self.force_plain_attention \
                 and out.dtype == torch.bfloat16 and v_head_dim == head_dim and lr.args[4] == n_heads and lr.args[6] == head_dim \
                 and lr.args[5] in (0, n_kv_heads) and cache.k.shape[1] == n_kv_heads * head_dim \
                 and cache.k.numel() < 1 << 32 and cache.k.shape[0] < 1 << 24:
-            return self._decode_attention(lr, step, window, scale, out, mask_chunk, n_kv_heads)
+            return self._decode_attention(lr, step, window, scale, out, mask_chunk, n_kv_heads, softcap, dist_a, dist_b)
         self.settle()
         if slopes is not None and (slopes.dtype != torch.float32 or slopes.numel() != n_heads or not slopes.is_contiguous()
                                    or slopes.device != q.device):
@@ -685,7 +710,8 @@ class Ops:
                 max_q_len, step.max_seq_len, out.data_ptr() + first * ldo * out.element_size(), ldo, n_tokens, n_heads,
                 n_kv_heads, head_dim, v_head_dim, cache.page_tokens, int(window), mask_chunk, float(scale),
                 None if slopes is None else slopes.data_ptr(), 1 if sink else 0, 1 if cross_values else 0, softcap,
-                1 if weights == "sigmoid" else 0, None if head_bias is None else head_bias.data_ptr(), self.attn_workspace.data_ptr(),
+                1 if weights == "sigmoid" else 0, None if head_bias is None else head_bias.data_ptr(),
+                None if sink_scores is None else sink_scores.data_ptr(), dist_a, dist_b, self.attn_workspace.data_ptr(),
                 self.attn_workspace.numel(), 1 if plain else 0, self._stream()))
 
         # Decoded tokens beside prompt portions: one call would send all of them to the kernel for prompt
@@ -693,7 +719,7 @@ class Ops:
         # take as long as thousands of prompt tokens). The step lays requests with few tokens first, so
         # each part is a step of its own: the first goes to the kernel that cuts the keys into chunks.
         n_short = getattr(step, "n_short_seqs", 0)
-        if not plain and not plain_scores and v_head_dim == head_dim and q.dtype == torch.bfloat16 \
+        if not plain and v_head_dim == head_dim and q.dtype == torch.bfloat16 \
                 and step.max_q_len >= self.prompt_rows and 0 < n_short < step.n_seqs:
             ts = step.n_short_tokens
             _ints(step.q_start_long, "q_start_long", step.n_seqs - n_short + 1)
@@ -702,7 +728,7 @@ class Ops:
         else:
             call(0, T, step.q_start, step.n_seqs, step.max_q_len)
 
-    def _decode_attention(self, lr, step, window, scale, out, mask_chunk=0, kv_heads=None):
+    def _decode_attention(self, lr, step, window, scale, out, mask_chunk=0, kv_heads=None, softcap=0.0, dist_a=None, dist_b=None):
         """Rotation, the store of the new keys and values and attention over the cache for decoded tokens, in one
         kernel: the queued ``rope_store`` (``lr``) and this call together."""
         qkv, positions, inv_freq, rot_dim, n_heads, n_kv_heads, head_dim, cache, slot_map, _ = lr.args
@@ -725,7 +751,7 @@ class Ops:
             cache.v.data_ptr(), cache.k.shape[1], None if slot_map is None else _ints(slot_map, "slot_map", T), g.block_table.data_ptr(),
             g.block_table.shape[1], _ints(step.token_slot, "token_slot", T), _ints(step.positions, "positions", T),
             _ints(step.q_start, "q_start", T + 1), T, step.max_seq_len, out.data_ptr(), _rows(out, "attention out"),
-            n_heads, n_kv_heads, head_dim, cache.page_tokens, int(window), int(mask_chunk), float(scale),
+            n_heads, n_kv_heads, head_dim, cache.page_tokens, int(window), int(mask_chunk), float(scale), softcap, dist_a, dist_b,
             self.attn_workspace.data_ptr(),
             self.attn_workspace.numel(), self._stream()))
 
@@ -811,7 +837,7 @@ class Ops:
             None if slot_map is None else _ints(slot_map, "slot_map", T), getattr(cache, "page_tokens", 0) or 0, T, self._stream()))
 
     def causal_conv(self, x, taps, bias, state, step, out, activation=None):
-        """``out[t, c] = act(bias[c] + sum_j taps[c, j] x[t - (K - 1) + j, c])`` along each request's tokens (fp32 out);
+        """``out[t, c] = act(bias[c] + sum_j taps[c, j] x[t - (K - 1) + j, c])`` along each request's tokens (formed in fp32);
         the K - 1 inputs before a request's first token of this step come from its row of ``state`` ([slots, >= (K - 1) C]
         fp32, oldest input first), which then receives the step's last K - 1 inputs. ``activation``: ``silu`` or None."""
         self.settle()
@@ -819,15 +845,16 @@ class Ops:
         T, C = out.shape
         K = taps.shape[1]
         if taps.dtype != torch.float32 or not taps.is_contiguous() or taps.shape[0] != C or x.shape[0] != T or x.shape[1] != C \
-                or out.dtype != torch.float32 or state.dtype != torch.float32 or state.stride(1) != 1 or state.shape[1] < (K - 1) * C \
+                or state.dtype != torch.float32 or state.stride(1) != 1 or state.shape[1] < (K - 1) * C \
                 or (bias is not None and (bias.dtype != torch.float32 or bias.numel() != C or not bias.is_contiguous())):
-            fail(EINVAL, "causal_conv: taps [channels, taps] and bias fp32, fp32 output and state, one width for all")
+            fail(EINVAL, "causal_conv: taps [channels, taps] and bias fp32, fp32 state, one width for all")
         if activation not in (None, "silu"):
             fail(ENOTSUP, f"causal_conv: activation '{activation}' is neither silu nor None")
+        self._scaled.pop(out.data_ptr(), None)
         self._check(self.lib.hfa_causal_conv(
             x.data_ptr(), _code(x), _rows(x, "conv in"), taps.data_ptr(), None if bias is None else bias.data_ptr(), C, K,
             state.data_ptr(), state.stride(0), _ints(step.q_start, "q_start", step.n_seqs + 1),
-            _ints(step.seq_slot, "seq_slot", step.n_seqs), step.n_seqs, step.max_q_len, out.data_ptr(), _rows(out, "conv out"),
+            _ints(step.seq_slot, "seq_slot", step.n_seqs), step.n_seqs, step.max_q_len, out.data_ptr(), _code(out), _rows(out, "conv out"),
             self.ACTIVATIONS["silu"] if activation else 0, self._stream()))
 
     @staticmethod
@@ -998,7 +1025,8 @@ class Ops:
             fail(EINVAL, "head_products: a [T * heads, >= K], w [heads, N, K] contiguous, out [T * heads, >= N]")
         N, K = int(w.shape[1]), int(w.shape[2])
         code, wcode = _code(a), _code(w)
-        plain = 1 if self.force_plain_gemm else 0
+        # (rows that do not start on 16 bytes: the plain products, in tiles that they take)
+        plain = 1 if self.force_plain_gemm or (code == BF16 and (_rows(a, "head rows") % 8 or (a.data_ptr() | w.data_ptr()) & 15)) else 0
         tile_rows = 32 if plain else int(self.lib.hfa_moe_tile_rows(code, wcode, R, H, N, K))
         max_tiles = R // tile_rows + H
         key = ("head ids", H)
@@ -1011,34 +1039,148 @@ class Ops:
                 self._shared[key + (ids.shape[0],)] = ids
             ids = memory.to_device(torch.arange(H, dtype=torch.int32).repeat(rows, 1), self.device, "the heads as choices of every token")
             self._shared[key] = ids
-        row_pair = self.scratch("heads_row_pair", (R,), torch.int32)
-        tiles = self.scratch("heads_tiles", (3 * max_tiles + 1,), torch.int32)
-        n_tiles = tiles[3 * max_tiles:]
-        self._check(self.lib.hfa_moe_plan(ids.data_ptr(), R, H, tile_rows, row_pair.data_ptr(), tiles.data_ptr(), n_tiles.data_ptr(),
-                                          self._stream()))
+        # the tiles follow from these three numbers alone: one plan serves every such product of a pass
+        hit = self._head_plans.get((R, H, tile_rows))
+        if hit is None:
+            row_pair = self.scratch(f"heads_row_pair@{H},{tile_rows}", (R,), torch.int32)
+            tiles = self.scratch(f"heads_tiles@{H},{tile_rows}", (3 * max_tiles + 1,), torch.int32)
+            n_tiles = tiles[3 * max_tiles:]
+            self._check(self.lib.hfa_moe_plan(ids.data_ptr(), R, H, tile_rows, row_pair.data_ptr(), tiles.data_ptr(), n_tiles.data_ptr(),
+                                              self._stream()))
+            if self._stream_handle is not None:              # inside a pass
+                self._head_plans[(R, H, tile_rows)] = (row_pair, tiles, n_tiles)
+        else:
+            row_pair, tiles, n_tiles = hit
         self._check(self.lib.hfa_moe_gemm(a.data_ptr(), _rows(a, "head rows"), code, 1, w.data_ptr(), wcode, row_pair.data_ptr(),
                                           tiles.data_ptr(), n_tiles.data_ptr(), max_tiles, tile_rows, out.data_ptr(), _rows(out, "head out"),
                                           _code(out), 1, None, 0, N, K, plain, 0, 0.0, 0.0, 0.0, self._stream()))
 
-    def latent_pack(self, down, q, weight, eps, packed, n_heads, dim, rot, latent, folded=None):
-        """The rows that ``rope_store`` and ``paged_attention`` take for attention through latents with one key/value head
-        (key ``[rotated part | latent]``, value the latent): from ``down`` (fp32 [T, latent + rot]: the latent before its norm, then
-        the key's part to be rotated) and ``q`` ([T, heads * (dim + rot)], a head being ``[dim | rot]``) it writes
-        ``packed[t] = [heads x (rot | latent: left alone) | rot | latent | latent]``, the latent RMS-normed with ``weight``. ``folded``
-        (``[T, heads * latent]``): the heads' queries with the keys' expansion folded in, copied into the heads' latent parts."""
+    def head_rows(self, a, w, out, a_head, out_head, gate=None):
+        """``out[t, h out_head + n] = sum_k w[h, n, k] a[t, h a_head + k]`` (times ``sigmoid(gate[t, h N + n])`` with ``gate``, fp32) for
+        the few rows of a decode step: ``head_products`` in one launch, without a plan. ``a`` is fp32 or bf16 (rounded to bf16 as it
+        is read), ``w`` [heads, N, K] and ``out`` bf16; N is a multiple of 32 and K of 16, operands start on 16 bytes, results on 8."""
+        self.settle()
+        self._whole(a)
+        self._scaled.pop(out.data_ptr(), None)
+        T = a.shape[0]
+        H, N, K = w.shape
+        if w.dtype != torch.bfloat16 or out.dtype != torch.bfloat16 or not w.is_contiguous() or out.shape[0] != T or a.shape[1] < (H - 1) * a_head + K or out.shape[1] < (H - 1) * out_head + N \
+                or (gate is not None and (gate.dtype != torch.float32 or gate.shape[0] != T or gate.shape[1] < H * N)):
+            fail(EINVAL, "head_rows: rows of heads in and out, an fp32 gate of the results' width")
+        self._check(self.lib.hfa_head_rows(a.data_ptr(), _code(a), _rows(a, "head rows"), int(a_head), w.data_ptr(), out.data_ptr(),
+                                           _rows(out, "head out"), int(out_head), None if gate is None else gate.data_ptr(),
+                                           0 if gate is None else _rows(gate, "gate"), T, H, N, K, self._stream()))
+
+    def latent_store(self, down, q, weight, eps, positions, inv_freq, rot_dim, pairing, q_out, cache, slot_map, n_heads, dim, rot, latent):
+        """Attention through latents between the projections and ``paged_attention``, one key/value head a token (key ``[rotated
+        part: rot | latent]``, value the latent): from ``down`` (fp32 [T, latent + rot]: the latent before its norm, then the key's
+        part to be rotated) and ``q`` ([T, heads * (dim + rot)], a head being ``[dim | rot]``) the latent, RMS-normed with ``weight``,
+        goes to the cache with the rotated key part, and the queries' rotated parts to ``q_out`` ([T, heads * (rot + latent)]), whose
+        latent parts are left alone. ``rot_dim`` of the ``rot`` values are turned, paired as in ``qkv_prepare``."""
         self.settle()
         self._whole(q)
-        if folded is not None and (folded.shape[0] != down.shape[0] or folded.shape[1] < n_heads * latent or folded.dtype != q.dtype):
-            fail(EINVAL, "latent_pack: the folded queries are [T, heads * latent] of the queries' dtype")
+        self._scaled.pop(q_out.data_ptr(), None)
         T = down.shape[0]
+        if pairing not in self.PAIRINGS:
+            fail(ENOTSUP, f"rotary pairing '{pairing}' is not one of {', '.join(self.PAIRINGS)}")
         if down.dtype != torch.float32 or down.shape[1] < latent + rot or q.shape[0] != T or q.shape[1] < n_heads * (dim + rot) \
-                or packed.shape[0] != T or packed.shape[1] < n_heads * (rot + latent) + rot + 2 * latent \
+                or q_out.shape[0] != T or q_out.shape[1] < n_heads * (rot + latent) or q_out.dtype != cache.k.dtype \
                 or weight.dtype != torch.float32 or weight.numel() != latent or not weight.is_contiguous():
-            fail(EINVAL, "latent_pack: rows of the latent and the rotated part (fp32), the heads' queries, an fp32 weight of the latent's size")
-        self._check(self.lib.hfa_latent_pack(down.data_ptr(), _rows(down, "latent rows"), q.data_ptr(), _code(q), _rows(q, "queries"),
-                                             weight.data_ptr(), float(eps), packed.data_ptr(), _code(packed), _rows(packed, "packed rows"),
-                                             T, n_heads, dim, rot, latent, None if folded is None else folded.data_ptr(),
-                                             0 if folded is None else _rows(folded, "folded queries"), self._stream()))
+            fail(EINVAL, "latent_store: rows of the latent and the rotated part (fp32), the heads' queries, an fp32 weight of the latent's size")
+        for c, width in ((cache.k, rot + latent), (cache.v, latent)):
+            if c.dim() != 2 or c.shape[1] != width or not c.is_contiguous() or c.dtype != q_out.dtype:
+                fail(EINVAL, f"latent_store: the cache must have one row of {width} values per token")
+        if rot_dim and (inv_freq is None or inv_freq.dtype != torch.float32 or inv_freq.numel() < rot_dim // 2):
+            fail(EINVAL, "latent_store: a rotation needs one fp32 frequency a pair")
+        self._check(self.lib.hfa_latent_store(
+            down.data_ptr(), _rows(down, "latent rows"), q.data_ptr(), _code(q), _rows(q, "queries"), weight.data_ptr(), float(eps),
+            None if not rot_dim else _ints(positions, "positions", T), None if not rot_dim else inv_freq.data_ptr(), int(rot_dim),
+            self.PAIRINGS[pairing], q_out.data_ptr(), _rows(q_out, "queries out"), cache.k.data_ptr(), cache.v.data_ptr(), _code(q_out),
+            _ints(slot_map, "slot_map", T), cache.page_tokens, T, n_heads, dim, rot, latent, self._stream()))
+
+    # ---- residuals of several streams ---------------------------------------------------------------------------
+    def _stream_source(self, su):
+        """(mode, y, its stride, partial sums, splits) of an update, taking a product into ``y`` that is still pending along."""
+        p = self._pending
+        if p is not None and p.out.data_ptr() == su.y.data_ptr():
+            if not p.accumulate and p.bias is None and p.out.shape == su.y.shape:
+                self._pending = None
+                return (1 if su.mix is None else 2), None, 0, self.workspace.data_ptr(), p.splits
+            self.settle(su.y)
+        return (1 if su.mix is None else 2), su.y.data_ptr(), _rows(su.y, "a sublayer's result"), None, 0
+
+    def _stream_check(self, x, what):
+        if x.dtype != torch.float32 or x.dim() != 3 or not x.is_contiguous():
+            fail(EINVAL, f"{what}: the residual is contiguous fp32 [T, streams, width]")
+        return x.shape
+
+    def _stream_step(self, su, x, in_w=None, weight=None, eps=0.0, out=None, taps=None, state=None, slots=None):
+        T, S, E = x.shape
+        mode, y, ldy, partial, splits = (0, None, 0, None, 0) if su is None else self._stream_source(su)
+
+        def ptr(t):
+            return None if t is None else t.data_ptr()
+        self._check(self.lib.hfa_stream_step(
+            x.data_ptr(), S, E, mode, y, ldy, partial, splits, None if su is None else ptr(su.mix), None if su is None else ptr(su.out),
+            ptr(in_w), ptr(weight), float(eps), ptr(out), F32 if out is None else _code(out), 0 if out is None else _rows(out, "norm out"),
+            ptr(taps), 0 if taps is None else taps.shape[1], ptr(state), 0 if state is None else state.stride(0), ptr(slots), T, self._stream()))
+
+    def stream_update(self, x, y, mix=None, out=None):
+        """``x[t, b] <- sum_a mix[a, b] x[t, a] + out[b] y[t]`` (all from the old streams), left undone until ``stream_input`` or
+        ``stream_sum`` asks for ``x``: one kernel then does both. A product into ``y`` may still be pending (``gemm(..., defer=True)``).
+        ``mix`` None: every stream becomes ``y[t]``."""
+        T, S, E = self._stream_check(x, "stream_update")
+        if self._stream_undone is not None:
+            self.settle(self._stream_undone.x)
+        for t, shape in ((mix, (S, S)), (out, (S,))):
+            if t is not None and (t.dtype != torch.float32 or tuple(t.shape) != shape or not t.is_contiguous()):
+                fail(EINVAL, f"stream_update: weights of {S} streams are contiguous fp32 [streams, streams] and [streams]")
+        if (mix is None) != (out is None) or y.dtype != torch.float32 or tuple(y.shape) != (T, E):
+            fail(EINVAL, "stream_update: the sublayer's result is fp32 [T, width]; mix and out go together")
+        self._stream_undone = StreamUpdate(x, y, mix, out)
+
+    def stream_input(self, x, in_w, weight, eps, out, taps=None, state=None, slots=None):
+        """``out[t] = rmsnorm(sum_b in_w[b] x[t, b]) * weight``, after an update of ``x`` that was left undone. ``taps`` (fp32 [width,
+        taps]): ``out`` is the causal convolution of the normed rows, for steps in which every row is a request's only token; the
+        inputs before it are rows ``slots[t]`` of ``state``, which move on (otherwise: ``causal_conv`` on ``out``)."""
+        T, S, E = self._stream_check(x, "stream_input")
+        if tuple(in_w.shape) != (S,) or in_w.dtype != torch.float32 or weight.dtype != torch.float32 or weight.numel() != E \
+                or not weight.is_contiguous() or not in_w.is_contiguous() or tuple(out.shape) != (T, E):
+            fail(EINVAL, "stream_input: one fp32 weight a stream, a norm's weight and an output of the streams' width")
+        if taps is not None:
+            K = taps.shape[1]
+            if taps.dtype != torch.float32 or not taps.is_contiguous() or taps.shape[0] != E or (K > 1 and (
+                    state is None or state.dtype != torch.float32 or state.stride(1) != 1 or state.shape[1] < (K - 1) * E)):
+                fail(EINVAL, "stream_input: taps [width, taps] and the state of their earlier inputs, fp32")
+            if K > 1:
+                _ints(slots, "slots", T)
+        su = self._stream_undone
+        if su is not None and su.x.data_ptr() == x.data_ptr() and su.x.shape == x.shape:
+            self._stream_undone = None
+        else:
+            su = None
+            self.settle()
+        self._scaled.pop(out.data_ptr(), None)
+        self._stream_step(su, x, in_w, weight, eps, out, taps, state, slots)
+
+    def stream_sum(self, x, out, rows=None):
+        """``out[r] = sum_b x[rows[r], b]`` (``rows`` None: every row in order), with an update of ``x`` that was left undone, which
+        thereby is dropped: ``x`` itself stays as it was."""
+        T, S, E = self._stream_check(x, "stream_sum")
+        R = out.shape[0]
+        if out.dtype != torch.float32 or tuple(out.shape) != (R, E) or not out.is_contiguous() or (rows is None and R != T):
+            fail(EINVAL, "stream_sum: contiguous fp32 rows of the streams' width")
+        su = self._stream_undone
+        if su is not None and su.x.data_ptr() == x.data_ptr() and su.x.shape == x.shape:
+            self._stream_undone = None
+        else:
+            su = None
+            self.settle()
+        mode, y, ldy, partial, splits = (0, None, 0, None, 0) if su is None else self._stream_source(su)
+        self._source_changes(out)
+        self._check(self.lib.hfa_stream_sum(x.data_ptr(), S, E, mode, y, ldy, partial, splits, None if su is None or su.mix is None else su.mix.data_ptr(),
+                                            None if su is None or su.out is None else su.out.data_ptr(), None if rows is None else _ints(rows, "rows", R),
+                                            out.data_ptr(), R, T, self._stream()))
 
     # ---- layer norm, plain activations, soft cap -----------------------------------------------------------------
     def layernorm(self, x, weight, bias, eps, out, rows=None):

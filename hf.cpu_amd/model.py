@@ -139,18 +139,21 @@ class Model:
     def cache_needs(self):
         """One entry for every (schedule entry, part of its layer that keeps a cache): PagedKV,
         FixedState, or None (an entry that reads another entry's cache keeps none of its own).
-        ``cache_slots[i]`` says which of them schedule entry ``i`` uses: {part name: index}."""
+        ``cache_slots[i]`` says which of them schedule entry ``i`` uses, its own or another entry's: {part name: index}."""
         needs, self.cache_slots = [], []
         for e in self.schedule:
             slots = {}
             for name, part in self.layers[e.layer].cache_parts():
-                need = part.cache_need() if e.cache_of is None else None
-                slots[name] = _number_needs(need, needs)
-                if e.cache_of is not None and hasattr(part, "reads_cache"):
+                if e.cache_of is None or not getattr(part, "shares_cache", True):
+                    slots[name] = _number_needs(part.cache_need(), needs)
+                    continue
+                needs.append(None)                           # the entry keeps none of its own for this part
+                k = self.cache_slots[e.cache_of].get(name)
+                if k is not None:
+                    slots[name] = k
+                if hasattr(part, "reads_cache") and isinstance(k, int) and isinstance(needs[k], PagedKV):
                     # what the reader sees of the other entry's storage decides with it how long rows are kept
-                    k = self.cache_slots[e.cache_of].get(name)
-                    if isinstance(k, int) and isinstance(needs[k], PagedKV):
-                        needs[k] = part.reads_cache(needs[k])
+                    needs[k] = part.reads_cache(needs[k])
             self.cache_slots.append(slots)
         return needs
 
@@ -165,19 +168,31 @@ class Model:
 
     def _forward(self, ops, step, caches, logits_out):
         T = step.n_tokens
-        x = ops.scratch("residual", (T, self.hidden_size), torch.float32)
-        self.embedding.forward(ops, step, x)
+        S = self.plan.streams
+        if S:                                     # several streams, all of them the embedding at the start
+            x = ops.scratch("residual", (T, S, self.hidden_size), torch.float32)
+            e = ops.scratch("embedded", (T, self.hidden_size), torch.float32)
+            self.embedding.forward(ops, step, e)
+            ops.stream_update(x, e)
+        else:
+            x = ops.scratch("residual", (T, self.hidden_size), torch.float32)
+            self.embedding.forward(ops, step, x)
         if not hasattr(self, "cache_slots"):
             self.cache_needs()
         for i, e in enumerate(self.schedule):
             layer = self.layers[e.layer]
             own = e.cache_of is None
-            mine = {name: _views_of(k, caches) for name, k in self.cache_slots[i if own else e.cache_of].items()}
+            mine = {name: _views_of(k, caches) for name, k in self.cache_slots[i].items()}
             layer.block.forward(ops, step, x, layer.named, mine, write_cache=own)
         R = step.n_logit_rows
         if R:
             h = ops.scratch("head_in", (R, self.hidden_size), ops.act_dtype)
-            if getattr(step, "rows_in_order", False):         # every token's logits, in order: no rows to gather
+            if S:                                 # the streams' sum at the wanted rows
+                total = ops.scratch("streams_sum", (R, self.hidden_size), torch.float32)
+                with ops.section("streams"):
+                    ops.stream_sum(x, total, None if getattr(step, "rows_in_order", False) else step.logit_rows)
+                norm_for(ops, self.final_norm, self.head, total, h)
+            elif getattr(step, "rows_in_order", False):         # every token's logits, in order: no rows to gather
                 norm_for(ops, self.final_norm, self.head, x, h)
             else:
                 self.final_norm.forward(ops, x, h, rows=step.logit_rows)      # src/model.c:629-636

@@ -33,10 +33,9 @@ def _rotary(rot, head_dim):
 def _mixer(cfg, lc, prefix):
     E, m = cfg.width, lc.mixer
     if lc.type == "latent_attention":
-        # attention sees a head as [rotated part | latent]: the rotation acts on the first dimensions of such a head
         return PartSpec("latent_attention", dict(
             hidden_size=E, n_heads=m.heads, head_dim=m.dim, rot_dim=m.rot_dim, v_head_dim=m.vdim, kv_rank=m.kv_rank,
-            q_rank=m.q_rank or None, scale=m.scale, eps=cfg.norm_eps, position=_rotary(m.rot, m.rot_dim + m.kv_rank), prefix=prefix))
+            q_rank=m.q_rank or None, scale=m.scale, eps=cfg.norm_eps, position=_rotary(m.rot, m.rot_dim), prefix=prefix))
     if lc.type == "hgrn2":
         return PartSpec("hgrn2", dict(hidden_size=E, n_heads=m.heads, head_dim=m.dim, v_head_dim=m.vdim, eps=cfg.norm_eps, prefix=prefix))
     lt, rt = m.left, m.right

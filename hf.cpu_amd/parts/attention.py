@@ -52,7 +52,9 @@ class Attention(Part):
 
     ``softcap`` c > 0: a score becomes ``c tanh(score / c)`` after the scale. ``weights="sigmoid"``: no softmax; a visible key
     weighs ``sigmoid(score + b_h)`` with one number a head (the tensor ``head_bias`` in ``names``, [heads]), and the weights are
-    not normalised over the keys.
+    not normalised over the keys. ``sink="learned"``: the extra term's score is one number a head (the tensor ``sink``) instead of
+    0. ``distance``: after scale and cap a score is lowered by ``a_h ln(1 + b_h (i - j))`` with two numbers a head (the tensors
+    ``dist_scale`` and ``dist_rate``).
     """
     graph_safe = True
     lazy_input_ok = True
@@ -62,7 +64,7 @@ class Attention(Part):
     def __init__(self, hidden_size, n_heads, n_kv_heads, head_dim, qkv_bias, window, position,
                  scale=None, out_bias=False, v_head_dim=None, prefix="", mask_chunk=0, own_kv=True, names=None,
                  qk_norm=None, sink=False, v_mix=None, conv_taps=0, head_norm=None, talk=False, out_gate=False,
-                 softcap=None, weights="softmax"):
+                 softcap=None, weights="softmax", distance=False):
         """``v_head_dim``: the size of a value head where it is not ``head_dim`` (key rows of the cache are
         then ``n_kv_heads * head_dim`` wide, value rows ``n_kv_heads * v_head_dim``, and the output
         projection reads ``n_heads * v_head_dim`` columns; such a mixer runs the plain kernels)."""
@@ -81,7 +83,8 @@ class Attention(Part):
         self.names = {n: f"{n}_proj.weight" for n in "qkvo"}
         self.names.update({f"{n}_bias": f"{n}_proj.bias" for n in "qkvo"})
         self.names.update(q_norm="q_norm.weight", k_norm="k_norm.weight", v_mix="v_mix", talk="talk", g="g_proj.weight",
-                          q_conv="q_conv.weight", k_conv="k_conv.weight", v_conv="v_conv.weight", head_bias="head_bias")
+                          q_conv="q_conv.weight", k_conv="k_conv.weight", v_conv="v_conv.weight", head_bias="head_bias",
+                          sink="sink", dist_scale="dist_scale", dist_rate="dist_rate")
         self.names.update(names or {})
         self.conv_taps = int(conv_taps)
         self.head_norm = None if head_norm is None else float(head_norm)
@@ -92,10 +95,14 @@ class Attention(Part):
             fail(EINVAL, f"attention: weights '{weights}' (softmax, or sigmoid without a sink term) and a soft cap of {softcap}")
         self.weights = weights
         self.head_bias = None
+        self.distance, self.learned_sink = bool(distance), sink == "learned"
+        if self.distance and weights != "softmax":
+            fail(EINVAL, "attention: a distance term goes with softmax weights")
+        self.dist_w = self.sink_w = None
         if self.out_gate and not own_kv:
             fail(EINVAL, "attention: an output gate goes with a mixer that has projections of its own")
         if self.shaped and (position.kind != "none" or not own_kv or qk_norm is not None or sink or v_mix or qkv_bias or window
-                            or mask_chunk or self.softcap or weights != "softmax"):
+                            or mask_chunk or self.softcap or weights != "softmax" or distance):
             fail(EINVAL, "attention: a convolution, per-head norms, mixed heads and an output gate go without rotation, biases, "
                          "windows and the other options")
         if not 0 <= self.conv_taps <= 8:
@@ -141,6 +148,10 @@ class Attention(Part):
             specs.append(ParamSpec(p + nm["g"], (self.OD, self.E)))
         if self.weights == "sigmoid":
             specs.append(ParamSpec(p + nm["head_bias"], (self.H,), "vector", ("normal", 0.5)))
+        if self.learned_sink:
+            specs.append(ParamSpec(p + nm["sink"], (self.H,), "vector", ("normal", 0.5)))
+        if self.distance:
+            specs += [ParamSpec(p + nm[n], (self.H,), "vector", ("one_plus_normal", 0.1)) for n in ("dist_scale", "dist_rate")]
         return specs
 
     def _projections(self):
@@ -174,6 +185,10 @@ class Attention(Part):
             self.b_qkv = memory.cat(biases, 0, f"{p}q, k and v biases in one vector")
         if self.weights == "sigmoid":
             self.head_bias = params[p + nm["head_bias"]].contiguous()
+        if self.learned_sink:
+            self.sink_w = params[p + nm["sink"]].contiguous()
+        if self.distance:
+            self.dist_w = tuple(params[p + nm[n]].contiguous() for n in ("dist_scale", "dist_rate"))
         self.w_o = params[p + nm["o"]]
         self.short_request_rows = ops.prompt_rows     # where the attention kernels for decoded tokens and for prompt portions part
         if self.out_bias:
@@ -218,10 +233,7 @@ class Attention(Part):
                 ops.paged_attention(q, self.H, self.G, self.D, kv, step, 0, self.scale, cross, v_head_dim=self.Dv, cross_values=True)
                 ops.talk_mix(cross, self.talk_w, self.H, self.G, self.Dv, att, gate=proj[:, C:] if self.out_gate else None)
         with ops.section("wo"):
-            if accumulate:
-                ops.gemm(att, self.w_o, x, accumulate=True, defer=True)
-            else:
-                ops.gemm(att, self.w_o, x)
+            ops.gemm(att, self.w_o, x, accumulate=accumulate, defer=True)
 
     def forward(self, ops, step, h, cache, x, write_cache=True, accumulate=True):
         if self.shaped:
@@ -269,52 +281,62 @@ class Attention(Part):
             ops.paged_attention(qkv, self.H, self.G, self.D, cache, step, self.window, self.scale, att,
                                 slopes=getattr(self.position, "score_slopes", None), v_head_dim=self.Dv,
                                 mask_chunk=self.mask_chunk, sink=self.sink, softcap=self.softcap, weights=self.weights,
-                                head_bias=self.head_bias)
+                                head_bias=self.head_bias, sink_scores=self.sink_w, distance=self.dist_w)
             if gate is not None:
                 ops.gate_mul(att, gate, att, "sigmoid")
         with ops.section("wo"):
-            if accumulate:
-                ops.gemm(att, self.w_o, x, bias=self.b_o, accumulate=True, defer=True)
-            else:
-                ops.gemm(att, self.w_o, x, bias=self.b_o)
+            ops.gemm(att, self.w_o, x, bias=self.b_o, accumulate=accumulate, defer=True)
 
 
 @register_part("mixer", "latent_attention")
 class LatentAttention(Part):
-    """Causal softmax attention whose queries, keys and values come through latents. With H = ``n_heads``, D = ``head_dim`` (the
-    unrotated dimensions of a query/key head), R = ``rot_dim`` (the rotated ones), Dv = ``v_head_dim``, C = ``kv_rank``:
+    """Causal softmax attention whose keys and values (and, optionally, queries) come through latents. With H = ``n_heads``, D =
+    ``head_dim`` (the unrotated dimensions of a query/key head), R = ``rot_dim`` (the rotated ones), Dv = ``v_head_dim``, C = ``kv_rank``:
 
-    * ``c_q = rmsnorm(Wdq h) * q_norm``; ``q = Wuq c_q``, head by head ``[D unrotated | R rotated]``;
+    * ``q = Wuq (rmsnorm(Wdq h) * q_norm)``, or ``q = Wq h`` (``q_latent`` False); head by head ``[D unrotated | R rotated]``;
     * ``Wdkv h`` has ``C + R`` rows: the first C, RMS-normed with ``kv_norm``, are the latent ``c``; the last R are one key part
       that all heads share and that is rotated like the queries' R parts (``position``: a rotary PartSpec over R dimensions);
-    * per head ``k = [Wuk c | rotated part]``, ``v = Wuv c``; ``score = q . k * scale``; softmax over the keys ``j <= i``;
+    * per head ``k = [Wuk c | rotated part]``, ``v = Wuv c``; ``score = q . k * scale``; softmax over the keys ``j <= i``, with
+      ``window > 0`` over the last ``window`` of them; ``sink``: a head's denominator has one more term ``exp(sink_h)`` (the tensor
+      ``sink``, [heads]) that has no value;
     * the concatenated heads are multiplied by ``sigmoid(Wg h)`` (``out_gate``) and projected by ``Wo``.
 
     The cache holds one row a token: the rotated part and the latent as the key of one shared head, the latent as its value. The
     keys' expansion is folded into the queries, ``q' = Wuk_h^T q_h`` (``score = q' . c + q_rot . k_rot``), and the values' is
     applied after the weighted sum, ``o_h = Wuv_h (sum_j p_j c_j)``: attention itself is the engine's, with H query heads on one
     key/value head of ``R + C`` key and ``C`` value dimensions. The latents' norms are fp32 over the 32-bit sums of their products.
-    ``names``: the tensors' names after ``prefix`` (keys dq, q_norm, uq, dkv, kv_norm, uk, uv, g, o).
-    ``forward(..., accumulate=False)`` writes ``x = ...`` instead of adding."""
+    ``names``: the tensors' names after ``prefix`` (keys dq, q_norm, uq or q; dkv, kv_norm, uk, uv, g, o, sink).
+    ``forward(..., accumulate=False)`` writes ``x = ...`` instead of adding.
+
+    The products that read the mixer's input are held as one matrix (queries or their latent first, then ``Wdkv``, then the gate):
+    a step of few rows runs it as one product with 32-bit sums, from which the heads' products (``Ops.head_rows``) and the store
+    read; a prompt portion runs its parts with the output type that each wants."""
     graph_safe = True
     can_overwrite = True
 
+    FEW_ROWS = 64                # rows up to which the heads' products run as one launch without a plan
+
     def __init__(self, hidden_size, n_heads, head_dim, rot_dim, v_head_dim, kv_rank, position, scale=None, q_rank=None, eps=1e-6,
-                 out_gate=True, prefix="", names=None):
+                 out_gate=True, prefix="", names=None, q_latent=True, window=0, sink=False):
         """``q_rank`` None: the query latent's size is the tensors'."""
         super().__init__(prefix)
         self.E, self.H, self.D, self.R, self.Dv, self.C = hidden_size, n_heads, head_dim, rot_dim, v_head_dim, kv_rank
-        self.q_rank = q_rank or None
+        self.q_latent = bool(q_latent)
+        self.q_rank = (q_rank or None) if self.q_latent else None
         self.eps = float(eps)
+        self.window, self.sink = int(window), bool(sink)
+        if self.window < 0:
+            fail(EINVAL, "latent_attention: a window is counted in tokens, 0 for none")
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(head_dim + rot_dim)
         self.out_gate = bool(out_gate)
         self.position = make_part("position", position)
-        if getattr(self.position, "head_dim", rot_dim) != rot_dim + kv_rank:
-            fail(EINVAL, f"latent_attention: the position part acts on heads of {rot_dim} + {kv_rank} dimensions, the rotated part first")
-        self.names = dict(dq="dq", q_norm="dq.norm", uq="uq", dkv="dkv", kv_norm="dkv.norm", uk="uk", uv="uv", g="g", o="o")
+        if getattr(self.position, "score_slopes", None) is not None or getattr(self.position, "rot_dim", 0) > rot_dim:
+            fail(EINVAL, f"latent_attention: the position part turns at most the {rot_dim} rotated dimensions")
+        self.names = dict(dq="dq", q_norm="dq.norm", uq="uq", q="q", dkv="dkv", kv_norm="dkv.norm", uk="uk", uv="uv", g="g", o="o", sink="sink")
         self.names.update(names or {})
         self.HD = rot_dim + kv_rank                          # a head as attention sees it: [rotated part | latent]
-        self.w_down = self.w_uq = self.w_uk_t = self.w_uv = self.w_o = self.q_norm_w = self.kv_norm_w = None
+        self.w_in = self.w_uq = self.w_uk_t = self.w_uv = self.w_o = self.q_norm_w = self.kv_norm_w = self.sink_w = None
+        self.q_cols, self.few_ok = 0, False
 
     def sub_parts(self):
         return [self.position]
@@ -322,73 +344,107 @@ class LatentAttention(Part):
     def param_specs(self):
         p, nm = self.prefix, self.names
         rq = self.q_rank or 0                                # 0: any size (the loader takes the tensor's)
-        specs = [ParamSpec(p + nm["dq"], (rq, self.E)), ParamSpec(p + nm["q_norm"], (rq,), "vector", ("one_plus_normal", 0.1)),
-                 ParamSpec(p + nm["uq"], (self.H * (self.D + self.R), rq), "matrix", ("normal", 0.1)),
-                 ParamSpec(p + nm["dkv"], (self.C + self.R, self.E)),
-                 ParamSpec(p + nm["kv_norm"], (self.C,), "vector", ("one_plus_normal", 0.1)),
-                 ParamSpec(p + nm["uk"], (self.H * self.D, self.C), "matrix", ("normal", 0.1)),
-                 ParamSpec(p + nm["uv"], (self.H * self.Dv, self.C), "matrix", ("normal", 0.1)),
-                 ParamSpec(p + nm["o"], (self.E, self.H * self.Dv))]
+        q_rows = self.H * (self.D + self.R)
+        if self.q_latent:
+            specs = [ParamSpec(p + nm["dq"], (rq, self.E)), ParamSpec(p + nm["q_norm"], (rq,), "vector", ("one_plus_normal", 0.1)),
+                     ParamSpec(p + nm["uq"], (q_rows, rq), "matrix", ("normal", 0.1))]
+        else:
+            specs = [ParamSpec(p + nm["q"], (q_rows, self.E))]
+        specs += [ParamSpec(p + nm["dkv"], (self.C + self.R, self.E)),
+                  ParamSpec(p + nm["kv_norm"], (self.C,), "vector", ("one_plus_normal", 0.1)),
+                  ParamSpec(p + nm["uk"], (self.H * self.D, self.C), "matrix", ("normal", 0.1)),
+                  ParamSpec(p + nm["uv"], (self.H * self.Dv, self.C), "matrix", ("normal", 0.1)),
+                  ParamSpec(p + nm["o"], (self.E, self.H * self.Dv))]
         if self.out_gate:
             specs.append(ParamSpec(p + nm["g"], (self.H * self.Dv, self.E)))
+        if self.sink:
+            specs.append(ParamSpec(p + nm["sink"], (self.H,), "vector", ("normal", 0.5)))
         return specs
 
     def cache_need(self):
-        return PagedKV(self.HD, self.C)
+        return PagedKV(self.HD, self.C, self.window)
 
     def bind(self, params, ops):
         p, nm = self.prefix, self.names
-        mats = [params[p + nm["dq"]], params[p + nm["dkv"]]]
-        self.q_rank = mats[0].shape[0]
+        mats = [params[p + nm["dq" if self.q_latent else "q"]], params[p + nm["dkv"]]]
         if self.out_gate:
-            self.w_gate = params[p + nm["g"]]
+            mats.append(params[p + nm["g"]])
         dt = torch.float32 if any(m.dtype == torch.float32 for m in mats) else mats[0].dtype
-        # the two projections into latents share their input: one product, whose 32-bit sums the norms read
-        self.w_down = memory.cat([m.to(dt) for m in mats], 0, f"{p}both projections into latents in one matrix")
-        self.w_uq, self.w_uv, self.w_o = params[p + nm["uq"]], params[p + nm["uv"]], params[p + nm["o"]]
-        if self.w_uq.shape[1] != self.q_rank or params[p + nm["q_norm"]].numel() != self.q_rank:
-            fail(EINVAL, f"latent_attention '{p}': the query latent's sizes do not match")
+        self.w_in = memory.cat([m.to(dt) for m in mats], 0, f"{p}the products that read the mixer's input in one matrix")
+        self.q_cols = mats[0].shape[0]                       # of the queries, or of their latent
+        self.w_uv, self.w_o = params[p + nm["uv"]].view(self.H, self.Dv, self.C), params[p + nm["o"]]
+        if self.q_latent:
+            self.w_uq, self.q_norm_w = params[p + nm["uq"]], params[p + nm["q_norm"]].contiguous()
+            self.q_rank = self.q_cols
+            if self.w_uq.shape[1] != self.q_rank or self.q_norm_w.numel() != self.q_rank:
+                fail(EINVAL, f"latent_attention '{p}': the query latent's sizes do not match")
         # q' = Wuk_h^T q_h: the product reads Wuk_h [D, C] as [C, D] rows
         uk = params[p + nm["uk"]]
         self.w_uk_t = memory.to_device(uk.reshape(self.H, self.D, self.C).transpose(1, 2), ops.device,
                                        f"{p}the keys' expansion, transposed head by head")
-        self.q_norm_w, self.kv_norm_w = params[p + nm["q_norm"]].contiguous(), params[p + nm["kv_norm"]].contiguous()
+        self.kv_norm_w = params[p + nm["kv_norm"]].contiguous()
+        if self.sink:
+            self.sink_w = params[p + nm["sink"]].contiguous()
         self.short_request_rows = ops.prompt_rows
+        # whether the one-launch products take these sizes and types (16-byte reads of operands, 8-byte stores of results)
+        self.few_ok = (ops.act_dtype == torch.bfloat16 and all(m.dtype == torch.bfloat16 for m in (self.w_in, self.w_uk_t, self.w_uv))
+                       and self.D % 16 == 0 and self.C % 32 == 0 and self.Dv % 32 == 0 and self.R % 8 == 0)
 
     def forward(self, ops, step, h, cache, x, write_cache=True, accumulate=True):
         if not write_cache:
             fail(EINVAL, f"latent_attention '{self.prefix}': this mixer cannot read another entry's cache")
         T, H, D, R, C, Dv, HD = h.shape[0], self.H, self.D, self.R, self.C, self.Dv, self.HD
-        rq = self.q_rank
-        down = ops.scratch("latent_down", (T, rq + C + R), torch.float32)
+        Q, CR = self.q_cols, C + R
+        few = self.few_ok and T <= self.FEW_ROWS and not ops.force_plain_gemm
+        gate = None
         with ops.section("latent_down"):
-            ops.gemm(h, self.w_down, down)
-            if self.out_gate:
-                gate = ops.scratch("att_gate", (T, H * Dv), ops.act_dtype)
-                ops.gemm(h, self.w_gate, gate)
-        cq = ops.scratch("latent_q", (T, rq), ops.act_dtype)
-        q = ops.scratch("latent_q_up", (T, H * (D + R)), ops.act_dtype)
-        with ops.section("latent_q"):
-            ops.group_rmsnorm(down[:, :rq], self.q_norm_w, self.eps, 1, cq)
-            ops.gemm(cq, self.w_uq, q)
-        packed = ops.scratch("qkv", (T, H * HD + HD + C), ops.act_dtype)
-        folded = ops.scratch("latent_q_folded", (T, H * C), ops.act_dtype)
+            if few:                                          # one product: 32-bit rows [queries or their latent | dkv | gate]
+                rows = ops.scratch("latent_rows", (T, self.w_in.shape[0]), torch.float32)
+                ops.gemm(h, self.w_in, rows)
+                q, down = rows[:, :Q], rows[:, Q:Q + CR]
+                if self.out_gate:
+                    gate = rows[:, Q + CR:]
+            else:
+                if self.q_latent:
+                    rows = ops.scratch("latent_rows", (T, Q + CR), torch.float32)
+                    ops.gemm(h, self.w_in[:Q + CR], rows)
+                    q, down = rows[:, :Q], rows[:, Q:]
+                else:
+                    q = ops.scratch("latent_q_up", (T, Q), ops.act_dtype)
+                    down = ops.scratch("latent_rows", (T, CR), torch.float32)
+                    ops.gemm(h, self.w_in[:Q], q)
+                    ops.gemm(h, self.w_in[Q:Q + CR], down)
+                if self.out_gate:
+                    gate = ops.scratch("att_gate", (T, H * Dv), ops.act_dtype)
+                    ops.gemm(h, self.w_in[Q + CR:], gate)
+        if self.q_latent:
+            cq = ops.scratch("latent_q", (T, Q), ops.act_dtype)
+            up = ops.scratch("latent_q_up", (T, H * (D + R)), ops.act_dtype)
+            with ops.section("latent_q"):
+                ops.group_rmsnorm(q, self.q_norm_w, self.eps, 1, cq)
+                ops.gemm(cq, self.w_uq, up)
+            q = up
+        # a head's query as attention sees it: [rotated part | the keys' expansion folded in]
+        folded = ops.scratch("latent_queries", (T, H * HD), ops.act_dtype)
         with ops.section("latent_pack"):
-            # the keys' expansion, folded into each head's query: one grouped product over the heads
-            ops.head_products(q.view(T * H, D + R), self.w_uk_t, folded.view(T * H, C), H)
-            ops.latent_pack(down[:, rq:], q, self.kv_norm_w, self.eps, packed, H, D, R, C, folded=folded)
-            self.position.store(ops, step, packed, H, 1, cache, True, v_head_dim=C)
+            if few:
+                ops.head_rows(q, self.w_uk_t, folded[:, R:], D + R, HD)
+            else:
+                ops.head_products(q.view(T * H, D + R), self.w_uk_t, folded.view(T * H, HD)[:, R:], H)
+            pos = self.position
+            ops.latent_store(down, q, self.kv_norm_w, self.eps, step.positions, getattr(pos, "inv_freq", None), getattr(pos, "rot_dim", 0),
+                             getattr(pos, "pairing", "split_half"), folded, cache, step.group(cache.group).slot_map, H, D, R, C)
         att = ops.scratch("latent_att", (T, H * C), ops.act_dtype)
         with ops.section("latent_attn"):
-            ops.paged_attention(packed, H, 1, HD, cache, step, 0, self.scale, att, v_head_dim=C)
+            ops.paged_attention(folded, H, 1, HD, cache, step, self.window, self.scale, att, v_head_dim=C, sink=self.sink, sink_scores=self.sink_w)
         heads = ops.scratch("att", (T, H * Dv), ops.act_dtype)
         with ops.section("latent_v"):
             # the values' expansion of each head's weighted sum of latents
-            ops.head_products(att.view(T * H, C), self.w_uv.view(H, Dv, C), heads.view(T * H, Dv), H)
-            if self.out_gate:
-                ops.gate_mul(heads, gate, heads, "sigmoid")
-        with ops.section("latent_wo"):
-            if accumulate:
-                ops.gemm(heads, self.w_o, x, accumulate=True, defer=True)
+            if few:
+                ops.head_rows(att, self.w_uv, heads, C, Dv, gate=gate)
             else:
-                ops.gemm(heads, self.w_o, x)
+                ops.head_products(att.view(T * H, C), self.w_uv, heads.view(T * H, Dv), H)
+                if gate is not None:
+                    ops.gate_mul(heads, gate, heads, "sigmoid")
+        with ops.section("latent_wo"):
+            ops.gemm(heads, self.w_o, x, accumulate=accumulate, defer=True)

@@ -9,6 +9,7 @@ Interfaces by role (``step`` is the engine's StepInputs, ``ops`` its kernels):
 
   embedding     forward(ops, step, out_x)                    tokens -> fp32 residual stream [T, E]
   norm          forward(ops, x, out, rows=None)              fp32 [T, E] -> activation dtype [T or R, E]
+  input         cache_need(); forward(ops, step, n, cache, out)   what a sublayer reads, made from its normed input (fp32 [T, E])
   position      store(ops, step, qkv, heads, kv_heads, cache, write[, v_head_dim=...])    acts on packed q | k | v rows
   mixer         cache_need(); forward(ops, step, h, cache, x, write_cache=True)     x += mixer(h)
   feed_forward  forward(ops, step, h, x)                                             x += ffn(h)
@@ -76,6 +77,9 @@ class Part:
     # others (decoded tokens beside prompt portions) says so here: the step function then lays those requests first
     # (``StepInputs.n_short_seqs``), so that the part can take the two groups as steps of their own. 0: no such line.
     short_request_rows = 0
+    # A schedule entry that reads another entry's cache (``ScheduleEntry.cache_of``) shares the cache of the part of the same
+    # name there; a part that keeps one of its own all the same (state that does not come from keys and values) says False.
+    shares_cache = True
 
     def __init__(self, prefix=""):
         self.prefix = prefix

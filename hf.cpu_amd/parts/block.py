@@ -2,6 +2,7 @@
 import torch
 
 from ..registry import register_part
+from ..status import EINVAL, fail
 from .base import ParamSpec, Part
 
 
@@ -162,6 +163,71 @@ class SandwichBlock(Part):
             else:
                 ff.forward(ops, step, h, y)
         self._sublayer(ops, step, x, h, "feed_forward", ff, parts["norm2b"], run_ff)
+
+
+@register_part("block", "hyper")
+class HyperBlock(Part):
+    """Hyper-connections: the residual is ``streams`` streams side by side (fp32 [T, streams, width]; the plan's ``streams``).
+    For each sublayer (mixer; feed-forward, where the layer has one) with weights ``in`` [streams], ``out`` [streams] and ``mix``
+    [streams, streams] (indexed [from, to]): ``y = sublayer(input(norm(sum_s in[s] x_s)))``, then, all streams at once from the old
+    ones, ``x_t <- sum_s mix[s, t] x_s + out[t] y``. ``names`` = {"mixer": prefix, "feed_forward": prefix} of the weights' tensors
+    (``<prefix>in``, ``<prefix>out``, ``<prefix>mix``) after ``prefix``.
+
+    Parts: norm1, mixer and, where the layer has it, norm2, feed_forward; ``input1`` and ``input2`` (optional, role ``input``)
+    stand between a norm and its sublayer. The norms are ``rmsnorm`` parts. Streams, sums, norms and a sublayer's result are
+    fp32. A sublayer's update waits for the next sublayer (or the model's last norm), whose kernel takes it along; where every
+    request brings one token, the input convolution is done there too. ``unused``: names of tensors after ``prefix`` with their
+    shapes that a checkpoint may hold although this layer reads none of them (a layer without a feed-forward)."""
+    graph_safe = True
+
+    def __init__(self, hidden_size, streams, names, prefix="", unused=()):
+        super().__init__(prefix)
+        if streams < 1:
+            fail(EINVAL, f"hyper: {streams} streams")
+        self.E, self.S, self.names = hidden_size, int(streams), dict(names)
+        self.unused = tuple(unused)
+        self.weights = {}
+
+    def param_specs(self):
+        S, specs = self.S, []
+        for n in self.names.values():
+            p = self.prefix + n
+            specs += [ParamSpec(p + "in", (S,), "vector", ("normal", 0.5)), ParamSpec(p + "out", (S,), "vector", ("one_plus_normal", 0.1)),
+                      ParamSpec(p + "mix", (S, S), "vector", ("normal", 0.8 / S ** 0.5))]
+        return specs + [ParamSpec(self.prefix + n, tuple(shape), "vector", ("normal", 0.1), optional=True) for n, shape in self.unused]
+
+    def bind(self, params, ops):
+        self.weights = {k: tuple(params[self.prefix + n + w].contiguous() for w in ("in", "mix", "out")) for k, n in self.names.items()}
+
+    def _sublayer(self, ops, step, x, which, norm, conv, conv_cache, part, run):
+        T = x.shape[0]
+        w_in, mix, out = self.weights[which]
+        h = ops.scratch("normed", (T, self.E), ops.act_dtype)
+        with ops.section("streams"):
+            if conv is None:
+                ops.stream_input(x, w_in, norm.weight, norm.eps, h)
+            elif step.max_q_len == 1 and step.n_seqs == T:
+                ops.stream_input(x, w_in, norm.weight, norm.eps, h, **conv.single_token(step, conv_cache))
+            else:
+                n = ops.scratch("normed32", (T, self.E), torch.float32)
+                ops.stream_input(x, w_in, norm.weight, norm.eps, n)
+                conv.forward(ops, step, n, conv_cache, h)
+        y = ops.scratch("branch", (T, self.E), torch.float32)
+        if getattr(part, "can_overwrite", False):
+            run(h, y, dict(accumulate=False))
+        else:                                  # a part that only knows how to add: into zeros
+            ops.settle()
+            y.zero_()
+            run(h, y, {})
+        ops.stream_update(x, y, mix, out)
+
+    def forward(self, ops, step, x, parts, caches, write_cache=True):
+        mixer, ff = parts["mixer"], parts.get("feed_forward")
+        self._sublayer(ops, step, x, "mixer", parts["norm1"], parts.get("input1"), caches.get("input1"), mixer,
+                       lambda h, y, kw: mixer.forward(ops, step, h, caches.get("mixer"), y, write_cache, **kw))
+        if ff is not None:
+            self._sublayer(ops, step, x, "feed_forward", parts["norm2"], parts.get("input2"), caches.get("input2"), ff,
+                           lambda h, y, kw: ff.forward(ops, step, h, y, **kw))
 
 
 def norm_for(ops, norm, reader, x, out, rows=None):

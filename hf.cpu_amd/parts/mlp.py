@@ -112,7 +112,4 @@ class PlainMLP(Part):
             with ops.section("up"):
                 ops.gemm(h, self.w_up, act, activation=self.activation)
         with ops.section("down"):
-            if accumulate:
-                ops.gemm(act, self.w_down, x, accumulate=True, defer=True)
-            else:
-                ops.gemm(act, self.w_down, x)
+            ops.gemm(act, self.w_down, x, accumulate=accumulate, defer=True)

@@ -14,21 +14,27 @@ class RMSNorm(Part):
     can_be_lazy = True          # forward(..., lazy=True) may leave the division to the products that read the output
 
 
-    def __init__(self, size, eps, prefix="", weight="weight", scalar=False):
+    def __init__(self, size, eps, prefix="", weight="weight", scalar=False, offset=0.0):
         """The scale is the tensor ``prefix + weight``; ``scalar``: a single number for all coordinates (a tensor without
-        dimensions), held as a vector of that number."""
+        dimensions), held as a vector of that number. ``offset``: the scale is the tensor plus this number (1 where a checkpoint
+        stores its distance from 1); the sum is formed once, in fp32."""
         super().__init__(prefix)
         self.size = size
         self.eps = float(eps)
         self.name = prefix + weight
         self.scalar = bool(scalar)
+        self.offset = float(offset)
         self.weight = None
 
     def param_specs(self):
-        return [ParamSpec(self.name, () if self.scalar else (self.size,), "vector", ("one_plus_normal", 0.1))]
+        rule = ("normal", 0.1) if self.offset else ("one_plus_normal", 0.1)
+        return [ParamSpec(self.name, () if self.scalar else (self.size,), "vector", rule)]
 
     def bind(self, params, ops):
         self.weight = params[self.name]
+        if self.offset:
+            memory.note(f"{self.name}, with its offset")
+            self.weight = self.weight + self.offset
         if self.scalar:
             self.weight = memory.to_device(self.weight.reshape(1).expand(self.size).contiguous(), ops.device,
                                            f"{self.name}, once a coordinate")

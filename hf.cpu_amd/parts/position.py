@@ -89,6 +89,6 @@ class NoPosition(Part):
                             self.head_dim if v_head_dim is None else v_head_dim, cache,
                             step.group(cache.group).slot_map if write else None, **prepare)
             return
-        if write:
-            ops.rope_store(qkv, step.positions, None, 0, n_heads, n_kv_heads, self.head_dim,
-                           cache, step.group(cache.group).slot_map, v_head_dim=v_head_dim)
+        # (a layer that only reads has nothing to store, but attention may take its queries as the product left them)
+        ops.rope_store(qkv, step.positions, None, 0, n_heads, n_kv_heads, self.head_dim,
+                       cache, step.group(cache.group).slot_map if write else None, v_head_dim=v_head_dim)

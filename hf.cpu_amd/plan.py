@@ -34,14 +34,14 @@ class LayerPlan:
 
     @classmethod
     def of(cls, label, block, **named):
-        """Parts by keyword; the role follows from the name: ``mixer*``, ``feed_forward*``, ``norm*``,
+        """Parts by keyword; the role follows from the name: ``mixer*``, ``feed_forward*``, ``norm*``, ``input*``,
         ``position*``, or give ``name=(role, spec)``."""
         parts = []
         for name, spec in named.items():
             if isinstance(spec, tuple):
                 role, spec = spec
             else:
-                role = next((r for r in ("mixer", "feed_forward", "norm", "position") if name.startswith(r)), None)
+                role = next((r for r in ("mixer", "feed_forward", "norm", "input", "position") if name.startswith(r)), None)
                 if role is None:
                     raise ValueError(f"layer {label!r}: the role of part '{name}' does not follow from its name; "
                                      f"give {name}=(role, spec)")
@@ -67,7 +67,8 @@ class LayerPlan:
 class ScheduleEntry:
     """One execution of a layer. Entries run in list order; a layer may appear more
     than once (each appearance has a cache of its own), and an entry with
-    ``cache_of`` set keeps no cache but reads the one of that earlier entry."""
+    ``cache_of`` set keeps no cache but reads the one of that earlier entry (except for parts
+    whose ``shares_cache`` is False, which keep their own)."""
     layer: int
     cache_of: Optional[int] = None
 
@@ -83,6 +84,7 @@ class ModelPlan:
     head: PartSpec               # role "head"
     max_context: int = 0         # trained context, informational (src/model.c:128-129)
     eos_token_ids: tuple = ()
+    streams: int = 0             # > 0: the residual is that many streams side by side ([T, streams, width], see the block "hyper")
 
     def check(self):
         n = len(self.layers)

@@ -7,7 +7,7 @@ unknown one is refused by name, as the reference refuses an unknown
 """
 from .status import ENOTSUP, fail
 
-ROLES = ("embedding", "norm", "position", "mixer", "feed_forward", "block", "head")
+ROLES = ("embedding", "norm", "input", "position", "mixer", "feed_forward", "block", "head")
 
 _architectures = {}
 _parts = {role: {} for role in ROLES}

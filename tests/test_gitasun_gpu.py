@@ -10,6 +10,7 @@ import torch
 import helpers
 import gitasun_helpers as gh
 import plain_gitasun as pg
+from hf_cpu_amd.cache.storage import PagedView
 from test_kernels_gpu import FakeCache, FakeStep, dev, ints, rounded, to_value_layout
 
 pytestmark = pytest.mark.gpu
@@ -334,27 +335,47 @@ def test_many_heads_on_one_wide_key_value_head(ops16, H, DK, C, page, lengths, q
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("H,D,R,C", [(3, 6, 4, 10), (1, 8, 8, 5), (4, 64, 64, 96), (2, 32, 64, 64), (16, 128, 64, 512)])
-def test_rows_for_attention_through_latents(ops32, dtype, H, D, R, C):
+@pytest.mark.parametrize("pairing", ["split_half", "interleaved"])
+@pytest.mark.parametrize("H,D,R,C,rot_dim", [(3, 6, 4, 10, 4), (1, 8, 8, 5, 6), (4, 64, 64, 96, 64), (2, 32, 64, 64, 32), (16, 128, 64, 512, 64)])
+def test_store_for_attention_through_latents(ops32, dtype, pairing, H, D, R, C, rot_dim):
+    """The latent's norm, the rotation of both rotated parts and the store, in one kernel; queries as 32-bit rows too."""
     rng = np.random.default_rng(H + D + C)
-    T = 11
+    T, P, pages = 11, 8, 5
+    HD = R + C
     down = (rng.standard_normal((T, C + R)) * rng.uniform(0.1, 9.0, (T, 1))).astype(np.float32)
     q = rounded(rng.standard_normal((T, H * (D + R))), dtype)
     w = (1.0 + 0.2 * rng.standard_normal(C)).astype(np.float32)
-    HD = R + C
-    packed = torch.full((T, H * HD + HD + C + 3), 7.0, dtype=dtype, device="cuda")
+    positions = rng.integers(0, 3000, T).astype(np.int32)
+    inv = (500.0 ** (-2.0 * np.arange(rot_dim // 2) / rot_dim)).astype(np.float32)
+    slots = rng.permutation(pages * P)[:T].astype(np.int32)
     wide = dev(np.concatenate([np.zeros((T, 2), np.float32), down], axis=1))
-    ops32.latent_pack(wide[:, 2:], dev(q, dtype), dev(w), 1e-5, packed, H, D, R, C)
-    got = packed.float().cpu().numpy()
+
+    def turn(x):                                   # [T, .., R]
+        out = x.copy()
+        ang = positions.astype(np.float32)[:, None] * inv
+        cs, sn = (f(ang).reshape((T,) + (1,) * (x.ndim - 2) + (-1,)) for f in (np.cos, np.sin))
+        i0, i1 = (slice(0, rot_dim, 2), slice(1, rot_dim, 2)) if pairing == "interleaved" else (slice(0, rot_dim // 2), slice(rot_dim // 2, rot_dim))
+        out[..., i0] = x[..., i0] * cs - x[..., i1] * sn
+        out[..., i1] = x[..., i1] * cs + x[..., i0] * sn
+        return out
     c = pg.rms_norm(down[:, :C].astype(np.float64), w, 1e-5)
-    tol = 1e-6 if dtype == torch.float32 else 1e-2
-    for hd in range(H):
-        assert np.array_equal(got[:, hd * HD:hd * HD + R], q[:, hd * (D + R) + D:(hd + 1) * (D + R)].astype(np.float32))
-        assert np.all(got[:, hd * HD + R:(hd + 1) * HD] == 7.0)                                  # left for the folded queries
-    key = got[:, H * HD:]
-    assert np.max(np.abs(key[:, :R] - rounded(down[:, C:], dtype))) == 0.0
-    assert np.max(np.abs(key[:, R:HD] - c) / (np.abs(c) + 1.0)) <= tol and np.array_equal(key[:, R:HD], key[:, HD:HD + C])
-    assert np.all(key[:, HD + C:] == 7.0)
+    k_rot = turn(down[:, C:].astype(np.float64))
+    tol = 1e-5 if dtype == torch.float32 else 1e-2
+    for q_dtype in {dtype, torch.float32}:
+        cache = PagedView(0, torch.zeros((pages * P, HD), dtype=dtype, device="cuda"), torch.zeros((pages * P, C), dtype=dtype, device="cuda"), P, 0)
+        q_out = torch.full((T, H * HD), 7.0, dtype=dtype, device="cuda")
+        ops32.latent_store(wide[:, 2:], dev(q, q_dtype), dev(w), 1e-5, ints(positions), dev(inv), rot_dim, pairing, q_out, cache,
+                           ints(slots), H, D, R, C)
+        got = q_out.float().cpu().numpy().reshape(T, H, HD)
+        q_rot = turn(q.reshape(T, H, D + R)[..., D:].astype(np.float64))
+        assert np.max(np.abs(got[..., :R] - q_rot) / (np.abs(q_rot) + 1.0)) <= tol
+        assert np.all(got[..., R:] == 7.0)                                                       # left for the folded queries
+        key = cache.k.float().cpu().numpy()[slots]
+        val = cache.v.float().cpu().numpy().reshape(pages, C, P)[slots // P, :, slots % P]
+        assert np.max(np.abs(key[:, :R] - k_rot) / (np.abs(k_rot) + 1.0)) <= tol
+        assert np.max(np.abs(key[:, R:] - c) / (np.abs(c) + 1.0)) <= tol and np.array_equal(key[:, R:], val)
+        others = np.setdiff1d(np.arange(pages * P), slots)
+        assert np.all(cache.k.float().cpu().numpy()[others] == 0.0)
 
 
 @pytest.mark.parametrize("E,top", [(5, 2), (10, 2), (4, 1), (3, 3), (64, 8), (256, 6)])
