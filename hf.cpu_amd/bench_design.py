@@ -1,6 +1,6 @@
-"""``bench.py --design goridra | tobozen | mobupel | gitasun``: prefill and decode of a design at sizes that resemble a real model's layers
+"""``bench.py --design goridra | tobozen | mobupel | gitasun | fugevik``: prefill and decode of a design at sizes that resemble a real model's layers
 (random weights), beside the closest other design at equal width, heads and layer count (Goridra beside Qwen2 dense,
-Tobozen beside Goridra, Mobupel and Gitasun beside Tobozen), with every part of a step priced against its roofline: flops / time against the matrix cores
+Tobozen beside Goridra, Mobupel and Gitasun beside Tobozen, Fugevik beside Gitasun), with every part of a step priced against its roofline: flops / time against the matrix cores
 for a prefill's parts, bytes / time against HBM for a decode step's. One JSON line a size."""
 import json
 import math
@@ -13,14 +13,15 @@ PROMPT, PAGE = 2048, 16
 
 # width, heads, key/value heads, head size, dense ff, experts, choices, groups, kept groups, expert ff, layers, vocabulary
 # (for Tobozen also: heads, head size, state and groups of the state-space layers; layers come in threes; for Gitasun also the rotated
-# part, the key/value latent and the query latent of its attention through latents)
+# part, the key/value latent and the query latent of its attention through latents; for Fugevik also the streams of its residual
+# and its windows)
 SIZES = {
     "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, ff=8192, experts=32, top=4, groups=4, keep=2, expert_ff=1024,
                layers=8, vocab=32000, mask=1024, ssm_heads=64, ssm_dim=64, ssm_state=128, ssm_groups=8, triples=2,
-               latent_rot=64, latent_rank=512, latent_q=1536),
+               latent_rot=64, latent_rank=512, latent_q=1536, streams=4, window=1024),
     "4k": dict(width=4096, heads=32, kv_heads=8, dim=128, ff=14336, experts=64, top=8, groups=8, keep=4, expert_ff=1024,
                layers=4, vocab=32000, mask=1024, ssm_heads=128, ssm_dim=64, ssm_state=128, ssm_groups=8, triples=1,
-               latent_rot=64, latent_rank=512, latent_q=1536),
+               latent_rot=64, latent_rank=512, latent_q=1536, streams=4, window=1024),
 }
 
 
@@ -149,6 +150,43 @@ def gitasun_work(z, T, batch, ctx):
     return pre, dec
 
 
+def fugevik_shape(z):
+    """Layers in threes: attention through latents, attention with keys and values of its own, attention that reads those; each with
+    a dense feed-forward. Every window is the same."""
+    H, G, D, W = z["heads"], z["kv_heads"], z["dim"], z["width"]
+    R, C, mask, mlp = z["latent_rot"], z["latent_rank"], dict(size=z["window"]), dict(kind="dense", ff=z["ff"])
+    layers = []
+    for l in range(0, 3 * z["triples"], 3):
+        att = dict(heads=H, kv_heads=G, dim=D, vdim=D, scale=1.0 / math.sqrt(D), softcap=50.0, mask=mask)
+        layers += [
+            dict(type="latent_attention", mixer=dict(heads=H, dim=D, rot_dim=R, vdim=D, kv_rank=C, scale=1.0 / math.sqrt(D + R),
+                                                     rot=dict(dims=R, base=10000.0), mask=mask), mlp=mlp),
+            dict(type="attention", mixer=att, mlp=mlp), dict(type="attention", mixer=dict(att, kv_from=l + 1), mlp=mlp)]
+    return dict(architecture="Fugevik", vocab=z["vocab"], width=W, streams=z["streams"], canon=dict(taps=4), norm=dict(eps=1e-6), layers=layers)
+
+
+def fugevik_work(z, T, batch, ctx):
+    """({part: flops of a prefill of T tokens}, {part: bytes of a decode step}), all layers together, bf16. The streams (their
+    update, the next sublayer's normed input and its convolution) move bytes only: in a prefill their bytes stand as the flops that
+    take as long at both peaks, so that their fraction is one of HBM's."""
+    W, H, G, D, V, n3, F = z["width"], z["heads"], z["kv_heads"], z["dim"], z["vocab"], z["triples"], z["ff"]
+    R, C, S, win = z["latent_rot"], z["latent_rank"], z["streams"], z["window"]
+    QD, KD, L = H * D, G * D, 3 * z["triples"]
+    params = {"latent_down": n3 * W * (H * (D + R) + C + R + QD), "latent_pack": n3 * H * D * C, "latent_v": n3 * H * D * C, "latent_wo": n3 * QD * W,
+              "qkv": n3 * W * (2 * QD + 2 * KD), "wo": 2 * n3 * QD * W, "up": L * F * W, "down": L * F * W, "head": V * W}
+    seen = sum(min(t + 1, win) for t in range(T))
+    streams = 2 * L * W * (4.0 * (2 * S + 1) + 2)               # bytes a token: every stream read and written, a result read, an input written
+    pre = {k: 2.0 * T * v for k, v in params.items() if k != "head"}
+    pre["latent_attn"] = n3 * 2.0 * (R + 2 * C) * H * seen
+    pre["attn"] = 2 * n3 * 4.0 * D * H * seen
+    pre["streams"] = T * streams * MFMA_PEAK / HBM_PEAK
+    dec = {k: 2.0 * v for k, v in params.items()}
+    dec["latent_attn"] = batch * min(ctx, win) * n3 * 2.0 * (R + 2 * C)
+    dec["attn"] = batch * min(ctx, win) * 2 * n3 * 2.0 * 2 * KD
+    dec["streams"] = batch * streams
+    return pre, dec
+
+
 def goridra_shape(z):
     """Layers in pairs: one with keys and values of its own and a dense feed-forward, one that reads them and has
     a mixture of experts."""
@@ -187,6 +225,8 @@ def part_work(design, z, T, batch, ctx):
         return mobupel_work(z, T, batch, ctx)
     if design == "gitasun":
         return gitasun_work(z, T, batch, ctx)
+    if design == "fugevik":
+        return fugevik_work(z, T, batch, ctx)
     W, H, G, D, L, V = z["width"], z["heads"], z["kv_heads"], z["dim"], z["layers"], z["vocab"]
     QD, KD = H * D, G * D
     if design == "qwen2":
@@ -223,9 +263,10 @@ def run(args):
     for size in (args.sizes.split(",") if args.sizes else list(SIZES)):
         z = SIZES[size]
         line = {"size": size, "dims": z, "context": context, "dtype": "bf16", "data": "synthetic"}
-        shapes = {"goridra": goridra_shape, "qwen2": qwen2_shape, "tobozen": tobozen_shape, "mobupel": mobupel_shape, "gitasun": gitasun_shape}
-        beside = {"goridra": "qwen2", "tobozen": "goridra", "mobupel": "tobozen", "gitasun": "tobozen"}[args.design]
-        if args.design in ("tobozen", "mobupel", "gitasun"):    # the same number of layers in both designs
+        shapes = {"goridra": goridra_shape, "qwen2": qwen2_shape, "tobozen": tobozen_shape, "mobupel": mobupel_shape, "gitasun": gitasun_shape,
+                  "fugevik": fugevik_shape}
+        beside = {"goridra": "qwen2", "tobozen": "goridra", "mobupel": "tobozen", "gitasun": "tobozen", "fugevik": "gitasun"}[args.design]
+        if args.design in ("tobozen", "mobupel", "gitasun", "fugevik"):    # the same number of layers in both designs
             z = dict(z, layers=3 * z["triples"])
         for design, shape in ((args.design, shapes[args.design](z)), (beside, shapes[beside](z))):
             cfg = hf_cpu_amd.config_from_dict(shape)

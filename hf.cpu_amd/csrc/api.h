@@ -219,13 +219,14 @@ int hfa_gate_mul(const void* x, int x_dtype, int ldx, const void* gate, int gate
 // latent before its norm and the rotated key part (`down`, [T, >= C + R] fp32) and the heads' queries (`q`, [T, H (D + R)]): c = down[:C] / sqrt(mean^2 +
 // eps) * w; the first rot_dim of the R rotated values are turned (pairing as in hfa_qkv_prepare); the key row [rotated: R | c] goes to
 // k_cache row slot_map[t], the value c to v_cache (transposed inside its page), and every head's rotated part to q_out, whose rows
-// hold H heads of [R | C] (their C parts are left alone: the products that fold the keys' expansion write them).
+// hold H heads of [R | C]. Their C parts are left alone (the products that fold the keys' expansion write them), or, with `fold`
+// ([H][C][D] bf16; bf16 cache, D a multiple of 16, C of 32), written by the same launch for the few rows of a decode step.
 // hfa_head_rows: out[t, h, :N] = W_h a[t, h, :K] (* sigmoid(gate[t, h, :])) for few rows t, every head with a matrix of its own
 // (w [H][N][K] bf16, a fp32 or bf16 rounded to bf16 as it is read, out bf16): one block 32 outputs of one head and 32 rows.
 // K a multiple of 16, N of 32, strides of a in 16-byte, of out in 8-byte steps.
 int hfa_latent_store(const float* down, int ld_down, const void* q, int q_dtype, int ldq, const float* w, float eps, const int* positions,
                      const float* inv_freq, int rot_dim, int pairing, void* q_out, int ld_out, void* k_cache, void* v_cache, int dtype,
-                     const int* slot_map, int page_tokens, int n_tokens, int n_heads, int dim, int rot, int latent, hipStream_t stream);
+                     const int* slot_map, int page_tokens, int n_tokens, int n_heads, int dim, int rot, int latent, const void* fold, hipStream_t stream);
 int hfa_head_rows(const void* a, int a_dtype, int lda, int a_head, const void* w, void* out, int ldo, int out_head, const float* gate,
                   int ldg, int n_rows, int n_heads, int N, int K, hipStream_t stream);
 

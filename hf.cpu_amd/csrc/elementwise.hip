@@ -324,7 +324,7 @@ extern "C" int hfa_rope_store(void* qkv, int dtype, int ld, const int* positions
     HFA_REQUIRE(n_heads + 2 * n_kv_heads <= 65535, "rope_store: too many heads for the grid");
     const int kd = n_kv_heads * head_dim;
     const size_t rows_lds = (size_t)ROPE_TOKENS * rot_dim * sizeof(float) + (size_t)ROPE_TOKENS * kd * 2 + ROPE_TOKENS * sizeof(int);
-    if (dtype == HFA_BF16 && splits == 0 && n_tokens >= ROPE_ROWS_FROM && rot_dim > 0 && rot_dim % 16 == 0 && v_head_dim == head_dim &&
+    if (dtype == HFA_BF16 && splits == 0 && n_tokens >= ROPE_ROWS_FROM && (rot_dim > 0 || (n_kv_heads > 0 && slot_map)) && rot_dim % 16 == 0 && v_head_dim == head_dim &&
         head_dim % 8 == 0 && ld % 8 == 0 && ((uintptr_t)qkv & 15) == 0 && ((uintptr_t)k_cache & 15) == 0 &&
         ((uintptr_t)v_cache & 15) == 0 && rows_lds <= 48 * 1024) {
         rope_store_rows_kernel<<<(n_tokens + ROPE_TOKENS - 1) / ROPE_TOKENS, 256, rows_lds, stream>>>(

@@ -58,6 +58,77 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
     }
 }
 
+// The same for channels in fours and NT taps, known at compile time: a thread owns four channels and walks
+// CONV_SEG4 tokens, all of whose inputs are asked for before the first is used. Sums in the same order as above.
+#define CONV_SEG4 16
+template <typename T> __device__ __forceinline__ float4 conv_load4(const T* p);
+template <> __device__ __forceinline__ float4 conv_load4<float>(const float* p) { return *reinterpret_cast<const float4*>(p); }
+template <> __device__ __forceinline__ float4 conv_load4<bf16>(const bf16* p) {
+    const uint2 u = *reinterpret_cast<const uint2*>(p);
+    return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16), __uint_as_float(u.y & 0xffff0000u));
+}
+__device__ __forceinline__ void conv_store4(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
+__device__ __forceinline__ void conv_store4(bf16* p, float4 v) {
+    *reinterpret_cast<uint2*>(p) = make_uint2((uint32_t)bf16_bits(v.x) | ((uint32_t)bf16_bits(v.y) << 16),
+                                              (uint32_t)bf16_bits(v.z) | ((uint32_t)bf16_bits(v.w) << 16));
+}
+__device__ __forceinline__ float conv_act(float v, int act) { return act == HFA_ACT_SILU ? v / (1.0f + expf(-v)) : v; }
+
+template <typename T, typename TO, int NT>
+__global__ __launch_bounds__(256) void causal_conv4_kernel(const T* __restrict__ in, int ld_in, const float* __restrict__ taps,
+                                                          const float* __restrict__ bias, int C, float* __restrict__ state,
+                                                          size_t state_ld, const int* __restrict__ q_start, const int* __restrict__ seq_slot,
+                                                          TO* __restrict__ out, int ldo, int act) {
+    constexpr int k = NT;
+    const int c = (blockIdx.x * blockDim.x + threadIdx.x) * 4, s = blockIdx.z;
+    if (c >= C) return;
+    const int q0 = q_start[s], n = q_start[s + 1] - q0, t0 = blockIdx.y * CONV_SEG4;
+    if (t0 >= n) return;
+    float* st = state + (size_t)seq_slot[s] * state_ld;
+    auto input = [&](int i) { return i >= 0 ? conv_load4<T>(in + (size_t)(q0 + i) * ld_in + c) : *reinterpret_cast<const float4*>(st + (size_t)(k - 1 + i) * C + c); };
+    // inputs t0 - (k - 1) .. t0 + CONV_SEG4 - 1 (past the request's end: its last one again, not used)
+    float4 x[k - 1 + CONV_SEG4];
+#pragma unroll
+    for (int j = 0; j < CONV_SEG4; j++) x[k - 1 + j] = conv_load4<T>(in + (size_t)(q0 + (t0 + j < n ? t0 + j : n - 1)) * ld_in + c);
+    if (t0 > 0) {                                            // uniform over the block: no load above stands under a condition
+#pragma unroll
+        for (int j = 0; j < k - 1; j++) x[j] = conv_load4<T>(in + (size_t)(q0 + t0 - (k - 1) + j) * ld_in + c);
+    } else {
+#pragma unroll
+        for (int j = 0; j < k - 1; j++) x[j] = *reinterpret_cast<const float4*>(st + (size_t)j * C + c);
+    }
+    float w[4][k];
+#pragma unroll
+    for (int j = 0; j < k; j++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) w[e][j] = taps[(size_t)(c + e) * k + j];
+    if constexpr (k > 1) {
+        if (t0 == 0) {
+            // The only thread that reads this channel's state is also the one that writes it: all reads come first.
+            float4 next[k - 1];
+#pragma unroll
+            for (int j = 0; j < k - 1; j++) next[j] = input(n - (k - 1) + j);
+#pragma unroll
+            for (int j = 0; j < k - 1; j++) *reinterpret_cast<float4*>(st + (size_t)j * C + c) = next[j];
+        }
+    }
+    const float4 b = bias ? *reinterpret_cast<const float4*>(bias + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+    for (int t = 0; t < CONV_SEG4; t++) {
+        if (t0 + t >= n) return;
+        float4 acc = b;
+#pragma unroll
+        for (int j = 0; j < k; j++) {
+            const float4 v = x[t + j];
+            acc.x = fmaf(w[0][j], v.x, acc.x);
+            acc.y = fmaf(w[1][j], v.y, acc.y);
+            acc.z = fmaf(w[2][j], v.z, acc.z);
+            acc.w = fmaf(w[3][j], v.w, acc.w);
+        }
+        conv_store4(out + (size_t)(q0 + t0 + t) * ldo + c, make_float4(conv_act(acc.x, act), conv_act(acc.y, act), conv_act(acc.z, act), conv_act(acc.w, act)));
+    }
+}
+
 extern "C" int hfa_causal_conv(const void* in, int dtype, int ld_in, const float* taps, const float* bias, int n_channels,
                                int n_taps, float* state, size_t state_ld, const int* q_start, const int* seq_slot, int n_seqs,
                                int max_q_len, void* out, int out_dtype, int ldo, int act, hipStream_t stream) {
@@ -69,6 +140,29 @@ extern "C" int hfa_causal_conv(const void* in, int dtype, int ld_in, const float
     HFA_REQUIRE(act == HFA_ACT_NONE || act == HFA_ACT_SILU, "causal_conv: the activation is silu or none");
     HFA_REQUIRE((dtype == HFA_F32 || dtype == HFA_BF16) && (out_dtype == HFA_F32 || out_dtype == HFA_BF16), "causal_conv: unknown dtype %d or %d", dtype, out_dtype);
     HFA_REQUIRE(n_seqs <= 65535 && (max_q_len + CONV_SEG - 1) / CONV_SEG <= 65535, "causal_conv: the step exceeds the grid");
+    const int in_bytes = dtype == HFA_F32 ? 16 : 8, out_bytes = out_dtype == HFA_F32 ? 16 : 8;
+    const bool fours = n_taps <= 4 && n_channels % 4 == 0 && ld_in % 4 == 0 && ldo % 4 == 0 && (n_taps == 1 || state_ld % 4 == 0) &&
+                       ((uintptr_t)in & (in_bytes - 1)) == 0 && ((uintptr_t)out & (out_bytes - 1)) == 0 && ((uintptr_t)state & 15) == 0 &&
+                       ((uintptr_t)bias & 15) == 0 && (max_q_len + CONV_SEG4 - 1) / CONV_SEG4 <= 65535;
+    if (fours) {
+        dim3 grid((n_channels / 4 + 255) / 256, (max_q_len + CONV_SEG4 - 1) / CONV_SEG4, n_seqs);
+#define CONV_GO(T, TO, NT)                                                                                                                 \
+    causal_conv4_kernel<T, TO, NT><<<grid, 256, 0, stream>>>((const T*)in, ld_in, taps, bias, n_channels, state, state_ld, q_start, \
+                                                             seq_slot, (TO*)out, ldo, act)
+#define CONV_TAPS(T, TO)                                      \
+    switch (n_taps) {                                         \
+        case 1: CONV_GO(T, TO, 1); break;                     \
+        case 2: CONV_GO(T, TO, 2); break;                     \
+        case 3: CONV_GO(T, TO, 3); break;                     \
+        default: CONV_GO(T, TO, 4); break;                    \
+    }
+        if (dtype == HFA_F32) { if (out_dtype == HFA_F32) CONV_TAPS(float, float) else CONV_TAPS(float, bf16) }
+        else { if (out_dtype == HFA_F32) CONV_TAPS(bf16, float) else CONV_TAPS(bf16, bf16) }
+#undef CONV_TAPS
+#undef CONV_GO
+        HFA_LAUNCH_CHECK("causal_conv");
+        return 0;
+    }
     dim3 grid((n_channels + 255) / 256, (max_q_len + CONV_SEG - 1) / CONV_SEG, n_seqs);
 #define CONV_GO(T, TO)                                                                                                                    \
     causal_conv_kernel<T, TO><<<grid, 256, 0, stream>>>((const T*)in, ld_in, taps, bias, n_channels, n_taps, state, state_ld, q_start, seq_slot, \

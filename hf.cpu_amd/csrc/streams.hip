@@ -68,11 +68,11 @@ __device__ __forceinline__ Vec<VW> branch_at(const float* __restrict__ y, int ld
 }
 
 // The streams at row t, columns c ..: as stored (mode 0), all equal to y (mode 1), or updated (mode 2). NS: streams at compile
-// time, 0: `S` of them.
+// time, 0: `S` of them. The weights' addresses are the same for every lane: they are read through the scalar unit.
 template <int NS, int VW>
 __device__ __forceinline__ void streams_at(Vec<VW>* nw, const float* __restrict__ x, int S, int width, int mode, const float* __restrict__ y,
-                                           int ldy, const float* __restrict__ partial, int splits, int n_rows, const float* mix_s,
-                                           const float* out_s, int t, int c) {
+                                           int ldy, const float* __restrict__ partial, int splits, int n_rows, const float* __restrict__ mix,
+                                           const float* __restrict__ out_w, int t, int c) {
     constexpr int CAP = NS ? NS : STREAMS_MAX;
     const int n = NS ? NS : S;
     if (mode == 1) {
@@ -98,81 +98,128 @@ __device__ __forceinline__ void streams_at(Vec<VW>* nw, const float* __restrict_
         if (to >= n) continue;
         Vec<VW> a;
 #pragma unroll
-        for (int e = 0; e < VW; e++) a.v[e] = out_s[to] * b.v[e];
+        for (int e = 0; e < VW; e++) a.v[e] = out_w[to] * b.v[e];
 #pragma unroll
         for (int from = 0; from < CAP; from++)
             if (from < n)
 #pragma unroll
-                for (int e = 0; e < VW; e++) a.v[e] = fmaf(mix_s[from * n + to], old[from].v[e], a.v[e]);
+                for (int e = 0; e < VW; e++) a.v[e] = fmaf(mix[from * n + to], old[from].v[e], a.v[e]);
         nw[to] = a;
     }
 }
 
-// One block a token.
-template <int NS, int VW, typename TO>
+// One block a token. ITEMS: groups of VW columns that a thread takes, held in registers between the two halves (and what the
+// second half wants from memory is asked for in the first); 0: any number, with the input in LDS.
+template <int NS, int VW, int ITEMS, typename TO>
 __global__ __launch_bounds__(1024) void stream_step_kernel(
     float* __restrict__ x, int S, int width, int mode, const float* __restrict__ y, int ldy, const float* __restrict__ partial, int splits,
     const float* __restrict__ mix, const float* __restrict__ out_w, const float* __restrict__ in_w, const float* __restrict__ norm_w,
     float eps, TO* __restrict__ out, int ldo, const float* __restrict__ taps, int K, float* __restrict__ state, size_t state_ld,
     const int* __restrict__ slots, int n_rows) {
-    constexpr int CAP = NS ? NS : STREAMS_MAX;
+    constexpr int CAP = NS ? NS : STREAMS_MAX, KEEP = ITEMS ? ITEMS : 1;
     extern __shared__ float u_s[];
     __shared__ float red[17];
-    __shared__ float mix_s[CAP * CAP], out_s[CAP], in_s[CAP];
-    const int t = blockIdx.x, n = NS ? NS : S;
-    for (int i = threadIdx.x; i < n * n; i += blockDim.x) mix_s[i] = mode == 2 ? mix[i] : 0.f;
-    for (int i = threadIdx.x; i < n; i += blockDim.x) {
-        out_s[i] = mode == 2 ? out_w[i] : 0.f;
-        in_s[i] = in_w ? in_w[i] : 0.f;
-    }
-    __syncthreads();
+    const int t = blockIdx.x, n = NS ? NS : S, stride = blockDim.x * VW, c0 = threadIdx.x * VW;
+    float* st = taps && K > 1 ? state + (size_t)slots[t] * state_ld : nullptr;
+    Vec<VW> keep[KEEP], gain[KEEP], past[KEEP];               // the input, the norm's weight, the convolution's sum over earlier inputs
+    Vec<VW> now[KEEP];                                        // the current token's taps
     float ss = 0.f;
-    for (int c = threadIdx.x * VW; c < width; c += blockDim.x * VW) {
-        Vec<VW> nw[CAP];
-        streams_at<NS, VW>(nw, x, S, width, mode, y, ldy, partial, splits, n_rows, mix_s, out_s, t, c);
-        Vec<VW> u;
+
+    // new streams and the input at columns c ..
+    auto first_half = [&](int c) {
+        Vec<VW> nw[CAP], u;
+        streams_at<NS, VW>(nw, x, S, width, mode, y, ldy, partial, splits, n_rows, mix, out_w, t, c);
 #pragma unroll
         for (int e = 0; e < VW; e++) u.v[e] = 0.f;
 #pragma unroll
         for (int s = 0; s < CAP; s++) {
             if (s >= n) continue;
             if (mode != 0) vstore<VW>(x + ((size_t)t * n + s) * width + c, nw[s]);
+            if (in_w) {
+                const float w = in_w[s];
 #pragma unroll
-            for (int e = 0; e < VW; e++) u.v[e] = fmaf(in_s[s], nw[s].v[e], u.v[e]);
+                for (int e = 0; e < VW; e++) u.v[e] = fmaf(w, nw[s].v[e], u.v[e]);
+            }
         }
-        if (in_w) {
 #pragma unroll
-            for (int e = 0; e < VW; e++) ss = fmaf(u.v[e], u.v[e], ss);
-            vstore<VW>(u_s + c, u);
+        for (int e = 0; e < VW; e++) ss = fmaf(u.v[e], u.v[e], ss);
+        return u;
+    };
+    // the request's only token of this step: the inputs before it are its state's, oldest first, which move up by one
+    auto history = [&](int c) {
+        Vec<VW> acc;
+#pragma unroll
+        for (int e = 0; e < VW; e++) acc.v[e] = 0.f;
+#pragma unroll
+        for (int j = 0; j < STREAM_TAPS_MAX - 1; j++) {
+            if (j >= K - 1) continue;
+            const Vec<VW> p = vload<VW>(st + (size_t)j * width + c);
+#pragma unroll
+            for (int e = 0; e < VW; e++) acc.v[e] = fmaf(taps[(size_t)(c + e) * K + j], p.v[e], acc.v[e]);
+            if (j > 0) vstore<VW>(st + (size_t)(j - 1) * width + c, p);
         }
-    }
-    if (!in_w) return;                                       // uniform
-    const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps);
-    float* st = taps && K > 1 ? state + (size_t)slots[t] * state_ld : nullptr;
-    for (int c = threadIdx.x * VW; c < width; c += blockDim.x * VW) {
-        Vec<VW> v = vload<VW>(u_s + c);
-        const Vec<VW> w = vload<VW>(norm_w + c);
+        return acc;
+    };
+    auto current = [&](int c) {
+        Vec<VW> r;
+#pragma unroll
+        for (int e = 0; e < VW; e++) r.v[e] = taps[(size_t)(c + e) * K + K - 1];
+        return r;
+    };
+    auto finish = [&](int c, Vec<VW> v, float inv, const Vec<VW>& w, const Vec<VW>& acc, const Vec<VW>& tap) {
 #pragma unroll
         for (int e = 0; e < VW; e++) v.v[e] = v.v[e] * inv * w.v[e];
         if (taps) {
-            // the request's only token of this step: the inputs before it are its state's, oldest first, which move up by one
-            Vec<VW> acc, last;
-#pragma unroll
-            for (int e = 0; e < VW; e++) acc.v[e] = 0.f;
-#pragma unroll
-            for (int j = 0; j < STREAM_TAPS_MAX - 1; j++) {
-                if (j >= K - 1) continue;
-                const Vec<VW> p = vload<VW>(st + (size_t)j * width + c);
-#pragma unroll
-                for (int e = 0; e < VW; e++) acc.v[e] = fmaf(taps[(size_t)(c + e) * K + j], p.v[e], acc.v[e]);
-                if (j > 0) vstore<VW>(st + (size_t)(j - 1) * width + c, p);
-            }
             if (K > 1) vstore<VW>(st + (size_t)(K - 2) * width + c, v);
 #pragma unroll
-            for (int e = 0; e < VW; e++) last.v[e] = fmaf(taps[(size_t)(c + e) * K + K - 1], v.v[e], acc.v[e]);
-            v = last;
+            for (int e = 0; e < VW; e++) v.v[e] = fmaf(tap.v[e], v.v[e], acc.v[e]);
         }
         vstore<VW>(out + (size_t)t * ldo + c, v);
+    };
+
+    if constexpr (ITEMS > 0) {
+#pragma unroll
+        for (int i = 0; i < ITEMS; i++) {
+            const int c = c0 + i * stride;
+            if (c >= width) continue;
+            if (in_w) {
+                gain[i] = vload<VW>(norm_w + c);
+                if (taps) {
+                    past[i] = history(c);
+                    now[i] = current(c);
+                }
+            }
+            keep[i] = first_half(c);
+        }
+    } else {
+        for (int c = c0; c < width; c += stride) {
+            const Vec<VW> u = first_half(c);
+            if (in_w) vstore<VW>(u_s + c, u);
+        }
+    }
+    if (!in_w) return;                                        // uniform
+    // the sum of squares over the block, in a fixed order; one barrier
+    ss = wave_sum(ss);
+    if ((threadIdx.x & (WAVE - 1)) == 0) red[threadIdx.x / WAVE] = ss;
+    __syncthreads();
+    float total = 0.f;
+    for (int i = 0; i < (int)(blockDim.x / WAVE); i++) total += red[i];
+    const float inv = 1.0f / sqrtf(total / (float)width + eps);
+    if constexpr (ITEMS > 0) {
+#pragma unroll
+        for (int i = 0; i < ITEMS; i++) {
+            const int c = c0 + i * stride;
+            if (c < width) finish(c, keep[i], inv, gain[i], past[i], now[i]);
+        }
+    } else {
+        for (int c = c0; c < width; c += stride) {
+            Vec<VW> acc, tap;
+            if (taps) {
+                acc = history(c);
+                tap = current(c);
+            }
+            finish(c, vload<VW>(u_s + c), inv, vload<VW>(norm_w + c), acc, tap);
+        }
     }
 }
 
@@ -182,15 +229,10 @@ __global__ __launch_bounds__(256) void stream_sum_kernel(const float* __restrict
                                                         const float* __restrict__ out_w, const int* __restrict__ rows, float* __restrict__ out,
                                                         int n_rows) {
     constexpr int CAP = NS ? NS : STREAMS_MAX;
-    __shared__ float mix_s[CAP * CAP], out_s[CAP];
-    const int n = NS ? NS : S;
-    for (int i = threadIdx.x; i < n * n; i += blockDim.x) mix_s[i] = mode == 2 ? mix[i] : 0.f;
-    for (int i = threadIdx.x; i < n; i += blockDim.x) out_s[i] = mode == 2 ? out_w[i] : 0.f;
-    __syncthreads();
-    const int r = blockIdx.x, t = rows ? rows[r] : r;
+    const int n = NS ? NS : S, r = blockIdx.x, t = rows ? rows[r] : r;
     for (int c = threadIdx.x * VW; c < width; c += blockDim.x * VW) {
         Vec<VW> nw[CAP], sum;
-        streams_at<NS, VW>(nw, x, S, width, mode, y, ldy, partial, splits, n_rows, mix_s, out_s, t, c);
+        streams_at<NS, VW>(nw, x, S, width, mode, y, ldy, partial, splits, n_rows, mix, out_w, t, c);
 #pragma unroll
         for (int e = 0; e < VW; e++) sum.v[e] = 0.f;
 #pragma unroll
@@ -238,24 +280,22 @@ extern "C" int hfa_stream_step(float* x, int n_streams, int width, int mode, con
     const bool vec = width % 4 == 0 && aligned16(x) && (mode == 0 || (splits > 0 ? aligned16(partial) : aligned16(y) && ldy % 4 == 0)) &&
                      (!in_w || (aligned16(norm_w) && aligned16(out) && ldo % 4 == 0)) &&
                      (!taps || n_taps == 1 || (aligned16(state) && state_ld % 4 == 0));
-    // few tokens: a block takes its token's row at once
-    const int items = (width + (vec ? 3 : 0)) / (vec ? 4 : 1);
-    int threads = n_rows < 256 ? (items + 63) / 64 * 64 : 256;
-    if (threads > 1024) threads = 1024;
-    const size_t lds = in_w ? (size_t)((width + 3) / 4 * 4) * sizeof(float) : 0;
-#define STEP_GO3(NS, VW, TO)                                                                                                          \
-    do {                                                                                                                              \
-        auto kernel = stream_step_kernel<NS, VW, TO>;                                                                                 \
-        static bool configured = false;                                                                                               \
-        if (!configured) {                                                                                                            \
-            if (hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, STREAM_WIDTH_MAX * 4) != hipSuccess) { \
-                hfa_set_error("stream_step: cannot reserve %d bytes of LDS", STREAM_WIDTH_MAX * 4);                                   \
-                return 2;                                                                                                             \
-            }                                                                                                                         \
-            configured = true;                                                                                                        \
-        }                                                                                                                             \
-        kernel<<<n_rows, threads, lds, stream>>>(x, n_streams, width, mode, y, ldy, partial, splits, mix, out_w, in_w, norm_w, eps,      \
-                                                 (TO*)out, ldo, taps, n_taps, state, state_ld, slots, n_rows);                        \
+    // few tokens: a block takes its token's row at once; many: two groups of columns a thread
+    const int groups = (width + (vec ? 3 : 0)) / (vec ? 4 : 1);
+    const bool few = n_rows < 256 && groups <= 1024;
+    int threads = ((few ? groups : (groups + 1) / 2) + 63) / 64 * 64;
+    const bool two = threads <= 1024;
+    if (!two) threads = 256;
+    const size_t lds = in_w && !few && !two ? (size_t)((width + 3) / 4 * 4) * sizeof(float) : 0;
+#define STEP_GO4(NS, VW, ITEMS, TO)                                                                                                  \
+    stream_step_kernel<NS, VW, ITEMS, TO><<<n_rows, threads, lds, stream>>>(x, n_streams, width, mode, y, ldy, partial, splits, mix, out_w, \
+                                                                           in_w, norm_w, eps, (TO*)out, ldo, taps, n_taps, state, state_ld,  \
+                                                                           slots, n_rows)
+#define STEP_GO3(NS, VW, TO)                          \
+    do {                                              \
+        if (few) STEP_GO4(NS, VW, 1, TO);             \
+        else if (two) STEP_GO4(NS, VW, 2, TO);        \
+        else STEP_GO4(NS, VW, 0, TO);                 \
     } while (0)
 #define STEP_GO(NS)                                                                 \
     do {                                                                            \
@@ -268,6 +308,7 @@ extern "C" int hfa_stream_step(float* x, int n_streams, int width, int mode, con
     STREAM_COUNTS(STEP_GO)
 #undef STEP_GO
 #undef STEP_GO3
+#undef STEP_GO4
     HFA_LAUNCH_CHECK("stream_step");
     return 0;
 }

@@ -24,7 +24,7 @@ _SIGNATURES = {
     "hfa_paged_attention": [P, I, I, P, P, I, I, P, I, P, P, P, I, I, I, P, I, I, I, I, I, I, I, I, I, F, P, I, I, F, I, P, P, P, P, P, c_size_t, I, P],
     "hfa_scale_add": [P, I, P, F, P, I, I, I, I, P],
     "hfa_gate_mul": [P, I, I, P, I, I, P, I, I, I, I, I, P],
-    "hfa_latent_store": [P, I, P, I, I, P, F, P, P, I, I, P, I, P, P, I, P, I, I, I, I, I, I, P],
+    "hfa_latent_store": [P, I, P, I, I, P, F, P, P, I, I, P, I, P, P, I, P, I, I, I, I, I, I, P, P],
     "hfa_head_rows": [P, I, I, I, P, P, I, I, P, I, I, I, I, I, P],
     "hfa_stream_step": [P, I, I, I, P, I, P, I, P, P, P, P, F, P, I, I, P, I, P, c_size_t, P, I, P],
     "hfa_stream_sum": [P, I, I, I, P, I, P, I, P, P, P, P, I, I, P],

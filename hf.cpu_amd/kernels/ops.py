@@ -607,10 +607,13 @@ class Ops:
             self._lazy_rope = LazyRope((qkv, positions, inv_freq, rot_dim, n_heads, n_kv_heads, head_dim, cache, slot_map,
                                         v_head_dim), qkv, cache)
             return
+        if rot_dim == 0 and not stores:              # nothing to turn, nothing to store
+            self.settle(qkv)
+            return
         if pend is not None and not pend.accumulate and pend.out.data_ptr() == qkv.data_ptr() \
                 and pend.out.shape == qkv.shape and qkv.shape[1] == row_width:
             self._pending = None
-            if qkv.dtype == torch.bfloat16 and qkv.shape[0] >= 512 and rot_dim > 0:
+            if qkv.dtype == torch.bfloat16 and qkv.shape[0] >= 512 and (rot_dim > 0 or stores):
                 # A prompt portion: the kernel for many tokens does not add up partial sums; finishing
                 # the product first and then taking that kernel is the quicker way.
                 self._pending = pend
@@ -1071,12 +1074,15 @@ class Ops:
                                            _rows(out, "head out"), int(out_head), None if gate is None else gate.data_ptr(),
                                            0 if gate is None else _rows(gate, "gate"), T, H, N, K, self._stream()))
 
-    def latent_store(self, down, q, weight, eps, positions, inv_freq, rot_dim, pairing, q_out, cache, slot_map, n_heads, dim, rot, latent):
+    def latent_store(self, down, q, weight, eps, positions, inv_freq, rot_dim, pairing, q_out, cache, slot_map, n_heads, dim, rot, latent,
+                     fold=None):
         """Attention through latents between the projections and ``paged_attention``, one key/value head a token (key ``[rotated
         part: rot | latent]``, value the latent): from ``down`` (fp32 [T, latent + rot]: the latent before its norm, then the key's
         part to be rotated) and ``q`` ([T, heads * (dim + rot)], a head being ``[dim | rot]``) the latent, RMS-normed with ``weight``,
         goes to the cache with the rotated key part, and the queries' rotated parts to ``q_out`` ([T, heads * (rot + latent)]), whose
-        latent parts are left alone. ``rot_dim`` of the ``rot`` values are turned, paired as in ``qkv_prepare``."""
+        latent parts are left alone, or, with ``fold`` (bf16 [heads, latent, dim], the keys' expansion transposed head by head; the few rows
+        of a decode step), written by the same launch: what ``head_rows`` gives. ``rot_dim`` of the ``rot`` values are turned, paired as in
+        ``qkv_prepare``."""
         self.settle()
         self._whole(q)
         self._scaled.pop(q_out.data_ptr(), None)
@@ -1090,13 +1096,16 @@ class Ops:
         for c, width in ((cache.k, rot + latent), (cache.v, latent)):
             if c.dim() != 2 or c.shape[1] != width or not c.is_contiguous() or c.dtype != q_out.dtype:
                 fail(EINVAL, f"latent_store: the cache must have one row of {width} values per token")
+        if fold is not None and (fold.dtype != torch.bfloat16 or tuple(fold.shape) != (n_heads, latent, dim) or not fold.is_contiguous()):
+            fail(EINVAL, "latent_store: the fold is bf16 [heads, latent, dim]")
         if rot_dim and (inv_freq is None or inv_freq.dtype != torch.float32 or inv_freq.numel() < rot_dim // 2):
             fail(EINVAL, "latent_store: a rotation needs one fp32 frequency a pair")
         self._check(self.lib.hfa_latent_store(
             down.data_ptr(), _rows(down, "latent rows"), q.data_ptr(), _code(q), _rows(q, "queries"), weight.data_ptr(), float(eps),
             None if not rot_dim else _ints(positions, "positions", T), None if not rot_dim else inv_freq.data_ptr(), int(rot_dim),
             self.PAIRINGS[pairing], q_out.data_ptr(), _rows(q_out, "queries out"), cache.k.data_ptr(), cache.v.data_ptr(), _code(q_out),
-            _ints(slot_map, "slot_map", T), cache.page_tokens, T, n_heads, dim, rot, latent, self._stream()))
+            _ints(slot_map, "slot_map", T), cache.page_tokens, T, n_heads, dim, rot, latent, None if fold is None else fold.data_ptr(),
+            self._stream()))
 
     # ---- residuals of several streams ---------------------------------------------------------------------------
     def _stream_source(self, su):

@@ -427,13 +427,12 @@ class LatentAttention(Part):
         # a head's query as attention sees it: [rotated part | the keys' expansion folded in]
         folded = ops.scratch("latent_queries", (T, H * HD), ops.act_dtype)
         with ops.section("latent_pack"):
-            if few:
-                ops.head_rows(q, self.w_uk_t, folded[:, R:], D + R, HD)
-            else:
+            if not few:
                 ops.head_products(q.view(T * H, D + R), self.w_uk_t, folded.view(T * H, HD)[:, R:], H)
             pos = self.position
             ops.latent_store(down, q, self.kv_norm_w, self.eps, step.positions, getattr(pos, "inv_freq", None), getattr(pos, "rot_dim", 0),
-                             getattr(pos, "pairing", "split_half"), folded, cache, step.group(cache.group).slot_map, H, D, R, C)
+                             getattr(pos, "pairing", "split_half"), folded, cache, step.group(cache.group).slot_map, H, D, R, C,
+                             fold=self.w_uk_t if few else None)
         att = ops.scratch("latent_att", (T, H * C), ops.act_dtype)
         with ops.section("latent_attn"):
             ops.paged_attention(folded, H, 1, HD, cache, step, self.window, self.scale, att, v_head_dim=C, sink=self.sink, sink_scores=self.sink_w)
