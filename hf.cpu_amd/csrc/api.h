@@ -233,7 +233,7 @@ int hfa_head_rows(const void* a, int a_dtype, int lda, int a_head, const void* w
 // Residuals of several streams (streams.hip). x: [n_rows][n_streams][width] fp32. mode 0: the streams as stored; 1: every stream
 // becomes y[t]; 2: new_b = sum_a mix[a * n_streams + b] old_a + out_w[b] y[t]. y is fp32 rows, or with splits > 0 the partial sums
 // ([splits][n_rows][width]) of a product that hfa_gemm deferred. hfa_stream_step writes the new streams (modes 1 and 2) and, with
-// in_w, out[t] = conv(n), n = u / sqrt(mean(u^2) + eps) * norm_w, u = sum_b in_w[b] new_b; taps ([width][n_taps], null: out = n): a
+// in_w, out[t] = conv(n), n = u / sqrt(mean(u^2) + eps) * norm_w, u = sum_b in_w[b] new_b; taps ([n_taps][width], null: out = n): a
 // causal convolution for steps in which every row is a request's only token, its earlier inputs in state row slots[t] ([n_taps - 1]
 // [width], oldest first), which moves on. hfa_stream_sum: out[r] = sum_b new_b of row rows[r] (null: r); nothing is written back.
 int hfa_stream_step(float* x, int n_streams, int width, int mode, const float* y, int ldy, const float* partial, int splits,
@@ -287,6 +287,8 @@ int hfa_moe_route(const float* logits, int ld, int n_tokens, int n_experts, int 
                   int scoring, int renorm, float out_scale, int* ids, float* weights, hipStream_t stream);
 int hfa_moe_plan(const int* ids, int n_pairs, int n_experts, int tile_rows, int* row_pair, int* tiles, int* n_tiles,
                  hipStream_t stream);
+// hfa_head_plan: the plan where every token chooses all n_heads "experts" in order (a product per head), without ids.
+int hfa_head_plan(int n_tokens, int n_heads, int tile_rows, int* row_pair, int* tiles, int* n_tiles, hipStream_t stream);
 int hfa_moe_tile_rows(int dtype, int w_dtype, int n_pairs, int n_experts, int N, int K);
 int hfa_moe_gemm(const void* a, int lda, int dtype, int a_div, const void* w, int w_dtype, const int* row_pair, const int* tiles,
                  const int* n_tiles, int max_tiles, int tile_rows, void* out, int ldo, int out_dtype, int out_by_pair,

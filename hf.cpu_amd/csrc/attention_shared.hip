@@ -326,7 +326,9 @@ int attn_shared_launch(const AttnArgs& a, int v_head_dim) {
     if (a.mask_chunk > 0 && a.mask_chunk + tpt + SH_KB < reach) reach = a.mask_chunk + tpt + SH_KB;
     if (blocks < 512 && reach > 256 && a.workspace) {
         long want = (512 + blocks - 1) / blocks;
-        const long most = (reach + 127) / 128;                // no chunk of fewer than 128 keys (64 were measured: no gain)
+        // no chunk of fewer than 128 keys (64 were measured: no gain), but where a window leaves the machine mostly empty
+        const int least = blocks * ((reach + 127) / 128) < 128 ? 64 : 128;
+        const long most = (reach + least - 1) / least;
         if (want > most) want = most;
         if (want > SH_MAX_CHUNKS) want = SH_MAX_CHUNKS;
         chunk_keys = (int)(((reach + want - 1) / want + SH_KB - 1) / SH_KB * SH_KB);

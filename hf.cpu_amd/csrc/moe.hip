@@ -168,6 +168,28 @@ extern "C" int hfa_moe_plan(const int* ids, int n_pairs, int n_experts, int tile
     return 0;
 }
 
+// The plan where every token has all E "experts" in order (the heads of a product per head): nothing to count. Row h T + t is pair
+// t E + h.
+__global__ __launch_bounds__(256) void head_plan_kernel(int T, int E, int tile_rows, int* __restrict__ row_pair, int* __restrict__ tiles,
+                                                       int* __restrict__ n_tiles) {
+    const int i = blockIdx.x * blockDim.x + threadIdx.x, per = (T + tile_rows - 1) / tile_rows;
+    if (i < T * E) row_pair[i] = i % T * E + i / T;
+    if (i < per * E) {
+        const int e = i / per, r = i % per * tile_rows;
+        tiles[3 * i] = e;
+        tiles[3 * i + 1] = e * T + r;
+        tiles[3 * i + 2] = T - r < tile_rows ? T - r : tile_rows;
+    }
+    if (i == 0) *n_tiles = per * E;
+}
+
+extern "C" int hfa_head_plan(int n_tokens, int n_heads, int tile_rows, int* row_pair, int* tiles, int* n_tiles, hipStream_t stream) {
+    HFA_REQUIRE(row_pair && tiles && n_tiles && n_tokens > 0 && n_heads > 0 && tile_rows > 0 && (long)n_tokens * n_heads < (1L << 31), "head_plan: bad arguments");
+    head_plan_kernel<<<(n_tokens * n_heads + 255) / 256, 256, 0, stream>>>(n_tokens, n_heads, tile_rows, row_pair, tiles, n_tiles);
+    HFA_LAUNCH_CHECK("head_plan");
+    return 0;
+}
+
 // ---- the experts' products ----------------------------------------------------------------
 // Gated experts (`gated` in the kernels below): the rows of an expert's matrix come in blocks of 32 gate rows, 32 up rows,
 // and a product's last lines form, from the two 32-bit sums of a pair of such blocks, g sigmoid(alpha g) (u + shift) with

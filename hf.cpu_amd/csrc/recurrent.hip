@@ -72,13 +72,13 @@ __device__ __forceinline__ void conv_store4(bf16* p, float4 v) {
     *reinterpret_cast<uint2*>(p) = make_uint2((uint32_t)bf16_bits(v.x) | ((uint32_t)bf16_bits(v.y) << 16),
                                               (uint32_t)bf16_bits(v.z) | ((uint32_t)bf16_bits(v.w) << 16));
 }
-__device__ __forceinline__ float conv_act(float v, int act) { return act == HFA_ACT_SILU ? v / (1.0f + expf(-v)) : v; }
+template <bool SILU> __device__ __forceinline__ float conv_act(float v) { return SILU ? v / (1.0f + expf(-v)) : v; }
 
-template <typename T, typename TO, int NT>
+template <typename T, typename TO, int NT, bool SILU>
 __global__ __launch_bounds__(256) void causal_conv4_kernel(const T* __restrict__ in, int ld_in, const float* __restrict__ taps,
                                                           const float* __restrict__ bias, int C, float* __restrict__ state,
                                                           size_t state_ld, const int* __restrict__ q_start, const int* __restrict__ seq_slot,
-                                                          TO* __restrict__ out, int ldo, int act) {
+                                                          TO* __restrict__ out, int ldo) {
     constexpr int k = NT;
     const int c = (blockIdx.x * blockDim.x + threadIdx.x) * 4, s = blockIdx.z;
     if (c >= C) return;
@@ -115,7 +115,6 @@ __global__ __launch_bounds__(256) void causal_conv4_kernel(const T* __restrict__
     const float4 b = bias ? *reinterpret_cast<const float4*>(bias + c) : make_float4(0.f, 0.f, 0.f, 0.f);
 #pragma unroll
     for (int t = 0; t < CONV_SEG4; t++) {
-        if (t0 + t >= n) return;
         float4 acc = b;
 #pragma unroll
         for (int j = 0; j < k; j++) {
@@ -125,7 +124,8 @@ __global__ __launch_bounds__(256) void causal_conv4_kernel(const T* __restrict__
             acc.z = fmaf(w[2][j], v.z, acc.z);
             acc.w = fmaf(w[3][j], v.w, acc.w);
         }
-        conv_store4(out + (size_t)(q0 + t0 + t) * ldo + c, make_float4(conv_act(acc.x, act), conv_act(acc.y, act), conv_act(acc.z, act), conv_act(acc.w, act)));
+        const float4 r = make_float4(conv_act<SILU>(acc.x), conv_act<SILU>(acc.y), conv_act<SILU>(acc.z), conv_act<SILU>(acc.w));
+        if (t0 + t < n) conv_store4(out + (size_t)(q0 + t0 + t) * ldo + c, r);
     }
 }
 
@@ -146,9 +146,13 @@ extern "C" int hfa_causal_conv(const void* in, int dtype, int ld_in, const float
                        ((uintptr_t)bias & 15) == 0 && (max_q_len + CONV_SEG4 - 1) / CONV_SEG4 <= 65535;
     if (fours) {
         dim3 grid((n_channels / 4 + 255) / 256, (max_q_len + CONV_SEG4 - 1) / CONV_SEG4, n_seqs);
-#define CONV_GO(T, TO, NT)                                                                                                                 \
-    causal_conv4_kernel<T, TO, NT><<<grid, 256, 0, stream>>>((const T*)in, ld_in, taps, bias, n_channels, state, state_ld, q_start, \
-                                                             seq_slot, (TO*)out, ldo, act)
+#define CONV_GO2(T, TO, NT, SILU)                                                                                                          \
+    causal_conv4_kernel<T, TO, NT, SILU><<<grid, 256, 0, stream>>>((const T*)in, ld_in, taps, bias, n_channels, state, state_ld, q_start, \
+                                                                   seq_slot, (TO*)out, ldo)
+#define CONV_GO(T, TO, NT)                                                                              \
+    do {                                                                                                \
+        if (act == HFA_ACT_SILU) CONV_GO2(T, TO, NT, true); else CONV_GO2(T, TO, NT, false);            \
+    } while (0)
 #define CONV_TAPS(T, TO)                                      \
     switch (n_taps) {                                         \
         case 1: CONV_GO(T, TO, 1); break;                     \
@@ -160,6 +164,7 @@ extern "C" int hfa_causal_conv(const void* in, int dtype, int ld_in, const float
         else { if (out_dtype == HFA_F32) CONV_TAPS(bf16, float) else CONV_TAPS(bf16, bf16) }
 #undef CONV_TAPS
 #undef CONV_GO
+#undef CONV_GO2
         HFA_LAUNCH_CHECK("causal_conv");
         return 0;
     }

@@ -151,20 +151,28 @@ __global__ __launch_bounds__(1024) void stream_step_kernel(
 #pragma unroll
         for (int e = 0; e < VW; e++) acc.v[e] = 0.f;
 #pragma unroll
-        for (int j = 0; j < STREAM_TAPS_MAX - 1; j++) {
-            if (j >= K - 1) continue;
-            const Vec<VW> p = vload<VW>(st + (size_t)j * width + c);
+        for (int j0 = 0; j0 < STREAM_TAPS_MAX - 1; j0 += 3) {
+            if (j0 >= K - 1) continue;
+            // three at a time, all asked for before the first is used (past the last one, the last one again)
+            Vec<VW> p[3], w[3];
 #pragma unroll
-            for (int e = 0; e < VW; e++) acc.v[e] = fmaf(taps[(size_t)(c + e) * K + j], p.v[e], acc.v[e]);
-            if (j > 0) vstore<VW>(st + (size_t)(j - 1) * width + c, p);
+            for (int u = 0; u < 3; u++) {
+                const int j = j0 + u < K - 1 ? j0 + u : K - 2;
+                p[u] = vload<VW>(st + (size_t)j * width + c);
+                w[u] = vload<VW>(taps + (size_t)j * width + c);
+            }
+#pragma unroll
+            for (int u = 0; u < 3; u++) {
+                if (j0 + u >= K - 1) continue;
+#pragma unroll
+                for (int e = 0; e < VW; e++) acc.v[e] = fmaf(w[u].v[e], p[u].v[e], acc.v[e]);
+                if (j0 + u > 0) vstore<VW>(st + (size_t)(j0 + u - 1) * width + c, p[u]);
+            }
         }
         return acc;
     };
     auto current = [&](int c) {
-        Vec<VW> r;
-#pragma unroll
-        for (int e = 0; e < VW; e++) r.v[e] = taps[(size_t)(c + e) * K + K - 1];
-        return r;
+        return vload<VW>(taps + (size_t)(K - 1) * width + c);
     };
     auto finish = [&](int c, Vec<VW> v, float inv, const Vec<VW>& w, const Vec<VW>& acc, const Vec<VW>& tap) {
 #pragma unroll
@@ -262,7 +270,9 @@ static bool aligned16(const void* p) { return ((uintptr_t)p & 15) == 0; }
         case 2: GO(2); break;         \
         case 3: GO(3); break;         \
         case 4: GO(4); break;         \
+        case 5: GO(5); break;         \
         case 6: GO(6); break;         \
+        case 7: GO(7); break;         \
         case 8: GO(8); break;         \
         default: GO(0); break;        \
     }
@@ -279,7 +289,7 @@ extern "C" int hfa_stream_step(float* x, int n_streams, int width, int mode, con
                 "stream_step: a convolution over 1 to %d inputs with the state of its earlier ones", STREAM_TAPS_MAX);
     const bool vec = width % 4 == 0 && aligned16(x) && (mode == 0 || (splits > 0 ? aligned16(partial) : aligned16(y) && ldy % 4 == 0)) &&
                      (!in_w || (aligned16(norm_w) && aligned16(out) && ldo % 4 == 0)) &&
-                     (!taps || n_taps == 1 || (aligned16(state) && state_ld % 4 == 0));
+                     (!taps || (aligned16(taps) && (n_taps == 1 || (aligned16(state) && state_ld % 4 == 0))));
     // few tokens: a block takes its token's row at once; many: two groups of columns a thread
     const int groups = (width + (vec ? 3 : 0)) / (vec ? 4 : 1);
     const bool few = n_rows < 256 && groups <= 1024;

@@ -50,6 +50,7 @@ _SIGNATURES = {
     "hfa_softcap": [P, I, I, I, F, P],
     "hfa_moe_route": [P, I, I, I, I, I, I, I, I, F, P, P, P],
     "hfa_moe_plan": [P, I, I, I, P, P, P, P],
+    "hfa_head_plan": [I, I, I, P, P, P, P],
     "hfa_moe_gemm": [P, I, I, I, P, I, P, P, P, I, I, P, I, I, I, P, I, I, I, I, I, F, F, F, P],
     "hfa_moe_combine": [P, P, I, I, I, P],
     "hfa_swiglu": [P, P, I, I, I, P],

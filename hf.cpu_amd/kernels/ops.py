@@ -1017,7 +1017,7 @@ class Ops:
         """``out[t * H + h, :] = w[h] @ a[t * H + h, :K]``: a product per head, every head with a matrix of its own. ``a`` is
         ``[T * H, >= K]`` (the heads' rows of all tokens, a token's heads one after the other), ``w`` ``[H, N, K]`` and ``out``
         ``[T * H, >= N]``; both are usually views of ``[T, H * width]`` matrices. The heads are the experts of the grouped product
-        that the mixture of experts runs (``hfa_moe_plan``, ``hfa_moe_gemm``): one launch for all heads, on the matrix cores
+        that the mixture of experts runs (``hfa_head_plan``, ``hfa_moe_gemm``): one launch for all heads, on the matrix cores
         where the sizes allow."""
         self.settle()
         self._whole(a)
@@ -1032,23 +1032,13 @@ class Ops:
         plain = 1 if self.force_plain_gemm or (code == BF16 and (_rows(a, "head rows") % 8 or (a.data_ptr() | w.data_ptr()) & 15)) else 0
         tile_rows = 32 if plain else int(self.lib.hfa_moe_tile_rows(code, wcode, R, H, N, K))
         max_tiles = R // tile_rows + H
-        key = ("head ids", H)
-        ids = self._shared.get(key)
-        if ids is None or ids.shape[0] * H < R:           # head h is the h-th choice of every token
-            if torch.cuda.is_current_stream_capturing():
-                fail(EINVAL, "head_products: the table of heads would have to grow while a graph is being captured")
-            rows = max(1024, 2 * (R // H))
-            if ids is not None:                           # captured graphs may still read the smaller table: it stays alive
-                self._shared[key + (ids.shape[0],)] = ids
-            ids = memory.to_device(torch.arange(H, dtype=torch.int32).repeat(rows, 1), self.device, "the heads as choices of every token")
-            self._shared[key] = ids
         # the tiles follow from these three numbers alone: one plan serves every such product of a pass
         hit = self._head_plans.get((R, H, tile_rows))
         if hit is None:
             row_pair = self.scratch(f"heads_row_pair@{H},{tile_rows}", (R,), torch.int32)
             tiles = self.scratch(f"heads_tiles@{H},{tile_rows}", (3 * max_tiles + 1,), torch.int32)
             n_tiles = tiles[3 * max_tiles:]
-            self._check(self.lib.hfa_moe_plan(ids.data_ptr(), R, H, tile_rows, row_pair.data_ptr(), tiles.data_ptr(), n_tiles.data_ptr(),
+            self._check(self.lib.hfa_head_plan(R // H, H, tile_rows, row_pair.data_ptr(), tiles.data_ptr(), n_tiles.data_ptr(),
                                               self._stream()))
             if self._stream_handle is not None:              # inside a pass
                 self._head_plans[(R, H, tile_rows)] = (row_pair, tiles, n_tiles)
@@ -1132,7 +1122,7 @@ class Ops:
         self._check(self.lib.hfa_stream_step(
             x.data_ptr(), S, E, mode, y, ldy, partial, splits, None if su is None else ptr(su.mix), None if su is None else ptr(su.out),
             ptr(in_w), ptr(weight), float(eps), ptr(out), F32 if out is None else _code(out), 0 if out is None else _rows(out, "norm out"),
-            ptr(taps), 0 if taps is None else taps.shape[1], ptr(state), 0 if state is None else state.stride(0), ptr(slots), T, self._stream()))
+            ptr(taps), 0 if taps is None else taps.shape[0], ptr(state), 0 if state is None else state.stride(0), ptr(slots), T, self._stream()))
 
     def stream_update(self, x, y, mix=None, out=None):
         """``x[t, b] <- sum_a mix[a, b] x[t, a] + out[b] y[t]`` (all from the old streams), left undone until ``stream_input`` or
@@ -1149,18 +1139,18 @@ class Ops:
         self._stream_undone = StreamUpdate(x, y, mix, out)
 
     def stream_input(self, x, in_w, weight, eps, out, taps=None, state=None, slots=None):
-        """``out[t] = rmsnorm(sum_b in_w[b] x[t, b]) * weight``, after an update of ``x`` that was left undone. ``taps`` (fp32 [width,
-        taps]): ``out`` is the causal convolution of the normed rows, for steps in which every row is a request's only token; the
+        """``out[t] = rmsnorm(sum_b in_w[b] x[t, b]) * weight``, after an update of ``x`` that was left undone. ``taps`` (fp32 [taps,
+        width]): ``out`` is the causal convolution of the normed rows, for steps in which every row is a request's only token; the
         inputs before it are rows ``slots[t]`` of ``state``, which move on (otherwise: ``causal_conv`` on ``out``)."""
         T, S, E = self._stream_check(x, "stream_input")
         if tuple(in_w.shape) != (S,) or in_w.dtype != torch.float32 or weight.dtype != torch.float32 or weight.numel() != E \
                 or not weight.is_contiguous() or not in_w.is_contiguous() or tuple(out.shape) != (T, E):
             fail(EINVAL, "stream_input: one fp32 weight a stream, a norm's weight and an output of the streams' width")
         if taps is not None:
-            K = taps.shape[1]
-            if taps.dtype != torch.float32 or not taps.is_contiguous() or taps.shape[0] != E or (K > 1 and (
+            K = taps.shape[0]
+            if taps.dtype != torch.float32 or not taps.is_contiguous() or taps.shape[1] != E or (K > 1 and (
                     state is None or state.dtype != torch.float32 or state.stride(1) != 1 or state.shape[1] < (K - 1) * E)):
-                fail(EINVAL, "stream_input: taps [width, taps] and the state of their earlier inputs, fp32")
+                fail(EINVAL, "stream_input: taps [taps, width] and the state of their earlier inputs, fp32")
             if K > 1:
                 _ints(slots, "slots", T)
         su = self._stream_undone

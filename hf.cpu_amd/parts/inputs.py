@@ -21,7 +21,7 @@ class InputConv(Part):
             fail(EINVAL, f"causal_conv: a convolution over {taps} tokens (1 to 8)")
         self.E, self.K = size, int(taps)
         self.name = prefix + weight
-        self.taps = self.no_state = None
+        self.taps = self.taps_by_age = self.no_state = None
 
     def param_specs(self):
         return [ParamSpec(self.name, (self.E, self.K), "vector", ("normal", 0.3))]
@@ -34,12 +34,13 @@ class InputConv(Part):
         memory.note(f"{self.name}, its input added")
         self.taps = params[self.name].clone().contiguous()
         self.taps[:, -1] += 1.0
+        self.taps_by_age = self.taps.t().contiguous()          # the order in which single tokens read them
         self.no_state = ops.shared("a convolution's state that is never read",
                                    lambda: memory.zeros((1, 1), torch.float32, ops.device, "a convolution's state that is never read"))
 
     def single_token(self, step, cache):
         """Keywords of ``Ops.stream_input`` for a step in which every request brings one token."""
-        return dict(taps=self.taps) if self.K == 1 else dict(taps=self.taps, state=cache.state, slots=step.token_slot)
+        return dict(taps=self.taps_by_age) if self.K == 1 else dict(taps=self.taps_by_age, state=cache.state, slots=step.token_slot)
 
     def forward(self, ops, step, n, cache, out):
         ops.causal_conv(n, self.taps, None, self.no_state if self.K == 1 else cache.state, step, out)
