@@ -1,7 +1,7 @@
 // Paged softmax attention of many query heads on ONE key/value head whose key rows are wide (up to 576 values: a latent
 // and a rotated part side by side) and whose value rows have a size of their own (up to 512: the latent), bf16 on the
 // matrix cores, for prompt portions and decoded tokens alike. This is what attention through latents comes to once the
-// keys' expansion is folded into the queries (see hfa_latent_pack): every head reads the same rows.
+// keys' expansion is folded into the queries (see hfa_latent_store): every head reads the same rows.
 //
 // A block of four waves owns a tile of 32 columns, a column being a (token, head) pair of one request (the tokens of a
 // tile are consecutive), and walks the keys of its chunk 32 at a time. The scores' chain of products over the key row is
