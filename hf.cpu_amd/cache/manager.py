@@ -15,7 +15,8 @@ src/model.c:217-230). Here pages come from shared pools:
   window ``W``, as soon as every position on the page is ``<= next_pos - W`` for the
   request's next position: no later query can see them. A group whose mixers mask by chunks gives
   back the pages that lie wholly before the current chunk's start; where other mixers read the same
-  storage (``PagedKV.readers``), a page goes back only when none of them can see it any more.
+  storage (``PagedKV.readers``), a page goes back only when none of them can see it any more. Pages that hold any
+  of the first ``PagedKV.keep_first`` positions stay until the request is released.
 * ``fork`` gives a new request the cache of another (src/model.c:271-301): whole pages are
   shared and counted, the last, partly filled page is copied, because both will write there.
   A shared page is never written: a request writes only at and beyond its own length.
@@ -68,7 +69,7 @@ class CacheManager:
         by_key = {}
         for i, need in enumerate(needs):
             if isinstance(need, PagedKV):
-                key = (need.k_width, need.v_width, need.window, need.mask_chunk, tuple(sorted(set(need.readers))))
+                key = (need.k_width, need.v_width, need.window, need.mask_chunk, tuple(sorted(set(need.readers))), need.keep_first)
                 if key not in by_key:
                     by_key[key] = len(self.groups)
                     self.groups.append(Group(len(self.groups), need.k_width, need.v_width, need.window, need))
@@ -209,10 +210,11 @@ class CacheManager:
         for g in self.groups:
             if g.need.first_kept(h.length) > 0:
                 table = h.tables[g.index]
+                start = -(-g.need.keep_first // self.page_tokens)          # whole pages from here on may go
                 stop = min(self._first_needed_block(g, h.length), len(table))
-                gone = [table[b] for b in range(stop) if table[b] >= 0]
+                gone = [table[b] for b in range(start, stop) if table[b] >= 0]
                 if gone:
-                    for b in range(stop):
+                    for b in range(start, stop):
                         table[b] = -1
                     self.pools[g.index].give_back(gone)
 

@@ -8,6 +8,7 @@ from .tobozen import TobozenConfig
 from .mobupel import MobupelConfig
 from .gitasun import GitasunConfig
 from .fugevik import FugevikConfig
+from .lurirax import LuriraxConfig
 
 
 def architecture_name(obj, origin="config.json"):
@@ -51,4 +52,4 @@ def read_config(model_dir, options=None):
     return config_from_dict(apply_model_options(read_json_file(path), options, path), path)
 
 
-__all__ = ["FugevikConfig", "GitasunConfig", "GoridraConfig", "KeyReader", "MobupelConfig", "Qwen2Config", "TobozenConfig", "architecture_name", "apply_model_options", "config_from_dict", "read_config", "read_json_file"]
+__all__ = ["FugevikConfig", "GitasunConfig", "GoridraConfig", "KeyReader", "LuriraxConfig", "MobupelConfig", "Qwen2Config", "TobozenConfig", "architecture_name", "apply_model_options", "config_from_dict", "read_config", "read_json_file"]

@@ -31,9 +31,11 @@ int hfa_rmsnorm(float* x, const float* w, void* out, int out_dtype, const int* r
 // `epilogue` 1 + k (k = HFA_ACT_GELU_ERF, HFA_ACT_GELU_TANH or HFA_ACT_RELU2; not with `accumulate`, never deferred):
 // out[m, n] = act_k(sum + bias[n]), the activation computed in fp32 in the product's last lines (on the plain path by
 // the elementwise kernel after it).
+// `epilogue` HFA_EPILOGUE_GEGLU: as 1 with the tanh form of gelu in silu's place.
 // `defer`: if K was split, leave the partial sums ([splits][M][N] fp32 at the start of the
 // workspace) for the caller's next kernel and report the number of splits in *pending_splits.
 // (src/model.c:408-424)
+#define HFA_EPILOGUE_GEGLU 17
 int hfa_gemm(const void* a, int a_dtype, int lda, const void* w, int w_dtype, int ldw, const float* bias,
              void* out, int out_dtype, int ldo, int accumulate, int epilogue, int M, int N, int K,
              void* workspace, size_t workspace_bytes, int defer, int* pending_splits, int force_plain,
@@ -47,7 +49,7 @@ int hfa_gemm_finish(const void* partial, int splits, const float* bias, void* ou
 //   HFA_ROWS_RESID   x[m, n] += sum + bias[n] (fp32, in place); ssq_out[b][m] = block b's share of sum_n x[m, n]^2
 //                    ([hfa_gemm_rows_parts()][16] floats, [..][32] from 17 rows up: give room for 32); xg[m, n] = bf16(x[m, n] * g[n]) if xg is given
 //   HFA_ROWS_SWIGLU  act[m, f] = bf16(silu(r[m] * sum_gate) * (r[m] * sum_up)), N features, w's 2 N rows in blocks of
-//                    32 gate rows, 32 up rows (src/model.c:537)
+//                    32 gate rows, 32 up rows (src/model.c:537); out_act HFA_ACT_GELU_TANH: the tanh form of gelu in silu's place
 // r[m] = rsqrt(sum over the parts_in shares ssq_in[.][m] * inv_width + eps), or 1 without ssq_in: the RMS norm of the
 // tensor whose product with the norm's weight is `a` (src/mathx.c:65-75), applied to the sums instead of the operand.
 // hfa_gemm_rows_supports says whether a shape is taken (1 to 32 rows, K a multiple of 128, strides multiples of 8).
@@ -104,13 +106,19 @@ int hfa_attention_prompt_rows(void);
 // `sink_w` (with `sink`): the extra term's score is sink_w[h] (one fp32 per query head) instead of 0. `dist_scale` and `dist_rate`
 // (one fp32 per query head each, or both null; softmax only): after scale and cap a score is lowered by dist_scale[h] ln(1 + dist_rate[h] (i - j)).
 // Sigmoid weights, caps and distance terms run on the matrix cores under the same conditions as the plain softmax.
+// `v_share`: that many neighbouring key heads read one head of values (value rows then hold n_kv_heads / v_share heads; 1: none
+// shared). `keep_first`: under a window keys 0 .. keep_first - 1 stay in sight of every later query. `rel` ([n_heads][rel_n] fp32, or
+// null): rel[h, min(i - j, rel_n - 1)] is added to a softmax's score. Head h of token t is multiplied by out_mul * sigmoid(gate[t, h])
+// (`gate`: rows of ldg values, null: by out_mul alone). `out_dtype` may be fp32 beside bf16 queries. Kept keys or a distance table
+// (one of the two), shared values, and value heads of half or twice the keys' size run on the matrix cores too (attention_masked.hip).
 int hfa_paged_attention(const void* q, int dtype, int ldq, const void* k_cache, const void* v_cache,
                         int kv_width, int v_width, const int* block_table, int max_blocks, const int* token_slot,
                         const int* positions, const int* q_start, int n_seqs, int max_q_len, int max_seq_len,
                         void* out, int ldo, int n_tokens, int n_heads, int n_kv_heads, int head_dim, int v_head_dim,
                         int page_tokens, int window, int mask_chunk, float scale, const float* slopes, int sink, int cross_values,
                         float softcap, int weights, const float* head_bias, const float* sink_w, const float* dist_scale,
-                        const float* dist_rate, void* workspace, size_t workspace_bytes, int force_plain, hipStream_t stream);
+                        const float* dist_rate, int v_share, int keep_first, const float* rel, int rel_n, const void* gate, int gate_dtype,
+                        int ldg, float out_mul, int out_dtype, void* workspace, size_t workspace_bytes, int force_plain, hipStream_t stream);
 
 // Decoded tokens (one a request) whose queries, new keys and new values are still the 32-bit rows [q | k | v] that
 // the product left (`raw`, bias added): rotation of queries and keys (cos_sin: hfa_rope_table's output for the step's
@@ -189,22 +197,31 @@ int hfa_delta_scan(const float* q, int ldq, const float* k, int ldk, int qk_head
 // Layers that norm a branch's result before it joins the stream, and what comes with them (sandwich.hip).
 // hfa_embed_pos: x[t] = table[tokens[t]] * scale + pos(positions[t]), pos[2i] = sin(p inv_freq[i]), pos[2i + 1] = cos(p inv_freq[i])
 // (positions null: no position vector).
-// hfa_rmsnorm_add: v = y[r] * sigmoid(gate[r] + gate_bias) (gate null: v = y[r]); out[r] (+)= scale * v / sqrt(mean(v^2) + eps) * w.
+// hfa_rmsnorm_add: b = [y[r], or the sum of `splits` planes of partial sums] * sigmoid(row_gate[r]) + sum_k pairs[r * top + k] (each
+// part optional), times sigmoid(gate[r] + gate_bias) element by element; out[r] (+)= scale * b / sqrt(mean(b^2) + eps) * w (w null:
+// scale * b); copy (bf16, or null) receives the new out[r]. hfa_round_rows: an fp32 matrix in bf16.
 // hfa_polynorm: out = coef[0] N(z) + coef[1] N(z^2) + coef[2] N(z^3) + coef[3], N(u) = u / sqrt(mean(u^2) + eps) over a row.
-// hfa_scale_rows: x *= s. hfa_head_norm_store: rows [q | k | v]; q and k heads RMS-normed with a weight of one head's size (null:
-// as they are), q to q_out, k and v to cache rows slot_map[t] (values transposed inside their page).
+// hfa_scale_rows: x *= s. hfa_head_norm_store: rows [q | k | v]; q and k heads RMS-normed (norm_q, norm_k) with a weight
+// of one head's size (null: 1) and turned over their first rot_dim dimensions (cos_sin: hfa_rope_table's output, null: no rotation), the
+// norm before or (norm_after) after the rotation; q to q_out, k and v to cache rows slot_map[t] (values transposed inside their page).
+// hfa_diff_mix: a [T][G][2][H / G][v_head_dim] fp32, two maps of a head: out[t, h] = c d / sqrt(mean(d^2) + eps), d = map 1 - factor[0] map 2.
 // hfa_talk_mix: out[t, h] = sigmoid(gate[t, h]) * sum_g talk[h, g] cross[t, (c(h) - c(g)) mod G, g], cross from hfa_paged_attention
 // with cross_values.
 int hfa_embed_pos(const void* table, int table_dtype, const int* tokens, const int* positions, const float* inv_freq, float* x,
                   int n_tokens, int width, int vocab, float scale, hipStream_t stream);
-int hfa_rmsnorm_add(const float* y, int ldy, const void* gate, int gate_dtype, int ldg, const float* gate_bias, const float* w,
-                    float* out, int ldo, int n_rows, int width, float eps, float scale, int accumulate, hipStream_t stream);
+int hfa_rmsnorm_add(const float* y, int ldy, const float* partial, int splits, const float* row_gate, int ld_row_gate, const float* pairs,
+                    int top, const void* gate, int gate_dtype, int ldg, const float* gate_bias, const float* w, float* out, int ldo,
+                    void* copy, int ldc, int n_rows, int width, float eps, float scale, int accumulate, hipStream_t stream);
+int hfa_round_rows(const float* x, int ldx, void* out, int ldo, int n_rows, int width, hipStream_t stream);
+int hfa_diff_mix(const float* a, int lda, const float* factor, float c, float eps, void* out, int out_dtype, int ldo, int n_tokens,
+                 int n_heads, int n_kv_heads, int v_head_dim, hipStream_t stream);
 int hfa_polynorm(const void* z, int z_dtype, int ldz, const float* coef, void* out, int out_dtype, int ldo, int n_rows, int width,
                  float eps, hipStream_t stream);
 int hfa_scale_rows(float* x, int ld, int n_rows, int width, float s, hipStream_t stream);
-int hfa_head_norm_store(const void* qkv, int in_dtype, int ld, int n_heads, int n_kv_heads, int head_dim, int v_head_dim,
-                        const float* q_w, const float* k_w, float eps, void* q_out, int ldq, void* k_cache, void* v_cache,
-                        int out_dtype, const int* slot_map, int page_tokens, int n_tokens, hipStream_t stream);
+int hfa_head_norm_store(const void* qkv, int in_dtype, int ld, int n_heads, int n_kv_heads, int head_dim, int n_v_heads, int v_head_dim,
+                        const float* q_w, const float* k_w, int norm_q, int norm_k, int norm_after, float eps, const float* cos_sin,
+                        int rot_dim, void* q_out, int ldq, void* k_cache, void* v_cache, int out_dtype, const int* slot_map,
+                        int page_tokens, int n_tokens, hipStream_t stream);
 int hfa_talk_mix(const void* cross, int cross_dtype, const float* talk, const void* gate, int gate_dtype, int ldg, void* out,
                  int out_dtype, int ldo, int n_tokens, int n_heads, int n_kv_heads, int v_head_dim, hipStream_t stream);
 
@@ -275,7 +292,8 @@ int hfa_softcap(float* x, int ld, int n_rows, int width, float cap, hipStream_t 
 // [n_tokens, top]; scoring 0 = softmax over all experts, 1 = logistic per expert, 2 = exp(logit - largest logit) (with renorm:
 // the softmax over the chosen logits alone); experts form n_groups equal runs of
 // neighbours of which the `keep` best (by their best expert) may be chosen from; weights = score (/ sum of the chosen
-// + 1e-20 if renorm) * out_scale. hfa_moe_plan puts the n_pairs = n_tokens * top pairs in expert order (row_pair) and
+// + 1e-20 if renorm) * out_scale. correction (one fp32 an expert, or null) is added to the scores for the choice alone, not for the
+// weights. hfa_moe_plan puts the n_pairs = n_tokens * top pairs in expert order (row_pair) and
 // lists tiles of at most tile_rows rows of one expert (tiles: 3 ints a tile, room for n_pairs / tile_rows + n_experts;
 // *n_tiles on the device). hfa_moe_gemm: for every row r of the plan, out[o(r), :] = act(a[s(r), :] . w[e(r)]^T)
 // (* pair_scale[pair] if given); w is [n_experts][N][K] (bf16, or fp32 beside activations of either type); s(r) = row_pair[r] / a_div if a_div > 0 else r; o(r) =
@@ -284,7 +302,7 @@ int hfa_softcap(float* x, int ld, int n_rows, int width, float cap, hipStream_t 
 // and 32 up rows, out has N / 2 columns, and with c = pair_scale of the row's pair (null: 1), g = min(c gate, limit), u = clamp(c up,
 // -limit, limit) (limit <= 0: unbounded): out = g sigmoid(alpha g) (u + shift), formed from the 32-bit sums in the product's last lines.
 int hfa_moe_route(const float* logits, int ld, int n_tokens, int n_experts, int top, int n_groups, int keep,
-                  int scoring, int renorm, float out_scale, int* ids, float* weights, hipStream_t stream);
+                  int scoring, int renorm, float out_scale, const float* correction, int* ids, float* weights, hipStream_t stream);
 int hfa_moe_plan(const int* ids, int n_pairs, int n_experts, int tile_rows, int* row_pair, int* tiles, int* n_tiles,
                  hipStream_t stream);
 // hfa_head_plan: the plan where every token chooses all n_heads "experts" in order (a product per head), without ids.
@@ -301,8 +319,8 @@ int hfa_moe_combine(const float* y, float* x, int n_tokens, int top, int width, 
 int hfa_moe_gated_act(const float* gu, int ld, const int* row_pair, const float* pair_scale, void* out, int out_dtype, int ldo,
                       int n_rows, int F, float alpha, float limit, float shift, int interleaved, hipStream_t stream);
 
-// out[t, i] = silu(gate_up[t, i]) * gate_up[t, width + i].  (src/model.c:532-538)
-int hfa_swiglu(const void* gate_up, void* out, int dtype, int n_tokens, int width, hipStream_t stream);
+// out[t, i] = act(gate_up[t, i]) * gate_up[t, width + i], act HFA_ACT_SILU or HFA_ACT_GELU_TANH.  (src/model.c:532-538)
+int hfa_swiglu(const void* gate_up, void* out, int dtype, int n_tokens, int width, int act, hipStream_t stream);
 
 // dst[idx[i]] = val[i]
 int hfa_scatter_i32(int* dst, const int* idx, const int* val, int n, hipStream_t stream);

@@ -27,6 +27,18 @@ struct AttnArgs {
     const float* sink_w;           // with sink: the extra term's score per query head (null: 0)
     const float* dist_scale;       // per query head, or null: a softmax's score is lowered by dist_scale[h] ln(1 + dist_rate[h] (i - j))
     const float* dist_rate;
+    int v_head_dim, v_width;       // a value head's size and the value rows' width (0: the keys')
+    int v_share;                   // that many neighbouring key heads read one value head (0: one)
+    int keep_first;                // > 0: under a window the keys 0 .. keep_first - 1 stay in sight
+    const float* rel; int rel_n;   // [query head][rel_n]: a number by distance (beyond rel_n - 1: the last) added to a softmax's score, or null
+    const void* gate; int gate_bf16, ldg;      // [token][query head]: a head's result is multiplied by sigmoid(gate), or null
+    float out_mul;                 // and by this number
+    int out_f32;                   // results leave in 32 bits
+};
+
+// How a call is cut: tiles of columns, chunks of keys, and for the kernel of prompt portions the pairing of long and short tiles.
+struct AttnCut {
+    int prompt, tiles, tpt, cpt, chunk_keys, n_chunks, prompt_tiles, pair_from;
 };
 
 // Whether a softmax's scores are more than a scaled product (a soft cap, a term of the distance): the matrix-core kernels
@@ -47,12 +59,8 @@ __host__ __device__ __forceinline__ int first_visible(int pos, int window, int m
     return lo;
 }
 
-int attn_generic_launch(const void* q, int dtype, int ldq, const void* k_cache, const void* v_cache, int kv_width,
-                        int v_width, const int* block_table, int max_blocks, const int* token_slot, const int* positions,
-                        void* out, int ldo, int n_tokens, int n_heads, int n_kv_heads, int head_dim, int v_head_dim,
-                        int page_tokens, int window, int mask_chunk, float scale, const float* slopes, int sink, int cross, float softcap,
-                        int weights, const float* head_bias, const float* sink_w, const float* dist_scale, const float* dist_rate,
-                        hipStream_t stream);
+// The plain kernel: any of what AttnArgs can ask for (with v_head_dim and v_width given).
+int attn_generic_launch(const AttnArgs& a, int dtype, const float* slopes, int cross);
 
 // Single tokens of a mixer that mixes its heads' weights after the softmax: every head's weights on the values of every
 // group in one pass over the cache, written in rounds of groups (see attention_cross.hip). `supports` leaves the cut
@@ -64,6 +72,14 @@ int attn_cross_launch(const AttnArgs& a, int chunk_keys, int n_chunks);
 // the matrix cores; see attention_shared.hip for what it needs.
 bool attn_shared_supports(const AttnArgs& a, int v_head_dim, int v_width);
 int attn_shared_launch(const AttnArgs& a, int v_head_dim);
+
+// Calls that take an instantiation of attention_masked.hip (whose sizes `attn_masked_sizes` names).
+inline bool attn_masked_mode(const AttnArgs& a) {
+    return a.rel != nullptr || a.keep_first > 0 || a.v_share > 1 || (a.v_head_dim > 0 && a.v_head_dim != a.head_dim) ||
+           (a.v_width > 0 && a.v_width != a.kv_width);
+}
+bool attn_masked_sizes(int head_dim, int v_head_dim);
+int attn_masked_run(const AttnArgs& a, const AttnCut& c);
 
 // bf16 on the matrix cores; see attention_mfma.hip for what it needs.
 bool attn_mfma_supports(const AttnArgs& a);

@@ -305,7 +305,7 @@ static int sh_page_shift(int page_tokens) {
 bool attn_shared_supports(const AttnArgs& a, int v_head_dim, int v_width) {
     return a.n_kv_heads == 1 && a.head_dim % 16 == 0 && a.head_dim <= 576 && v_head_dim % 32 == 0 && v_head_dim <= 512 &&
            a.kv_width == a.head_dim && v_width == v_head_dim && a.page_tokens >= 4 && sh_page_shift(a.page_tokens) >= 0 && a.scale > 0.f &&
-           a.v_rot == 0 && a.weights == 0 && !attn_shaped_scores(a) && a.q_start != nullptr &&
+           a.v_rot == 0 && a.weights == 0 && !attn_shaped_scores(a) && !a.rel && a.keep_first == 0 && a.v_share <= 1 && !a.gate && a.out_mul == 1.f && !a.out_f32 && a.q_start != nullptr &&
            a.raw == nullptr && a.ldq % 8 == 0 && a.ldo % 4 == 0 && ((uintptr_t)a.q & 15) == 0 && ((uintptr_t)a.out & 7) == 0 &&
            ((uintptr_t)a.k_cache & 15) == 0 && ((uintptr_t)a.v_cache & 15) == 0 && (size_t)a.n_tokens * a.n_heads < ((size_t)1 << 31) / 600;
 }

@@ -87,6 +87,13 @@ __device__ __forceinline__ float hfa_act_apply(int kind, float z) {
     return z;
 }
 
+// The gate's half of a gated unit, z sigmoid(z) (silu) or, `kind` HFA_ACT_GELU_TANH, the tanh form of gelu, which is z sigmoid(2 u)
+// with u = sqrt(2 / pi) (z + 0.044715 z^3): one form whose two constants the caller's `kind` chooses.
+__device__ __forceinline__ float hfa_gate_half(int kind, float z) {
+    const float a = kind == HFA_ACT_GELU_TANH ? 1.5957691216057308f : 1.0f, b = kind == HFA_ACT_GELU_TANH ? 0.071354816272600f : 0.0f;
+    return z / (1.0f + expf(-z * fmaf(b * z, z, a)));
+}
+
 // ---- error reporting of the launchers ---------------------------------------------------
 // Every extern "C" launcher returns 0, or a non-zero code after leaving a message that
 // hfa_last_error() returns. Bad shapes are refused before anything is launched.

@@ -351,27 +351,28 @@ extern "C" int hfa_rope_store(void* qkv, int dtype, int ld, const int* positions
 
 // ---- SwiGLU -----------------------------------------------------------------------------
 template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int width, size_t total) {
+__global__ void swiglu_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int width, int act, size_t total) {
     for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
          idx += (size_t)gridDim.x * blockDim.x) {
         const size_t t = idx / width;
         const int i = (int)(idx - t * width);
         const float g = to_f32(gate_up[t * 2 * width + i]);
         const float u = to_f32(gate_up[t * 2 * width + width + i]);
-        out[idx] = from_f32<T>((g / (1.0f + expf(-g))) * u);
+        out[idx] = from_f32<T>(hfa_gate_half(act, g) * u);
     }
 }
 
-extern "C" int hfa_swiglu(const void* gate_up, void* out, int dtype, int n_tokens, int width, hipStream_t stream) {
+extern "C" int hfa_swiglu(const void* gate_up, void* out, int dtype, int n_tokens, int width, int act, hipStream_t stream) {
     HFA_REQUIRE(n_tokens > 0 && width > 0, "swiglu: bad sizes tokens=%d width=%d", n_tokens, width);
+    HFA_REQUIRE(act == HFA_ACT_SILU || act == HFA_ACT_GELU_TANH, "swiglu: the gate passes silu or the tanh form of gelu, not %d", act);
     HFA_REQUIRE(dtype == HFA_F32 || dtype == HFA_BF16, "swiglu: unknown dtype %d", dtype);
     const size_t total = (size_t)n_tokens * width;
     size_t blocks = (total + 255) / 256;
     if (blocks > 65536) blocks = 65536;
     if (dtype == HFA_F32)
-        swiglu_kernel<float><<<(int)blocks, 256, 0, stream>>>((const float*)gate_up, (float*)out, width, total);
+        swiglu_kernel<float><<<(int)blocks, 256, 0, stream>>>((const float*)gate_up, (float*)out, width, act, total);
     else
-        swiglu_kernel<bf16><<<(int)blocks, 256, 0, stream>>>((const bf16*)gate_up, (bf16*)out, width, total);
+        swiglu_kernel<bf16><<<(int)blocks, 256, 0, stream>>>((const bf16*)gate_up, (bf16*)out, width, act, total);
     HFA_LAUNCH_CHECK("swiglu");
     return 0;
 }

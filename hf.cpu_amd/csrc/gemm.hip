@@ -8,6 +8,8 @@ extern "C" int hfa_gemm(const void* a, int a_dtype, int lda, const void* w, int 
                         void* workspace, size_t workspace_bytes, int defer, int* pending_splits, int force_plain,
                         hipStream_t stream) {
     HFA_REQUIRE(M > 0 && N > 0 && K > 0, "gemm: bad sizes M=%d N=%d K=%d", M, N, K);
+    const int gate_act = epilogue == HFA_EPILOGUE_GEGLU ? HFA_ACT_GELU_TANH : 0;       // a gated product whose gate is no silu
+    if (gate_act) epilogue = 1;
     HFA_REQUIRE(lda >= K && ldw >= K && ldo >= (epilogue ? N / 2 : N),
                 "gemm: a row stride is smaller than its row (lda=%d ldw=%d K=%d ldo=%d N=%d)", lda, ldw, K, ldo, N);
     HFA_REQUIRE((a_dtype == HFA_F32 || a_dtype == HFA_BF16) && (w_dtype == HFA_F32 || w_dtype == HFA_BF16) &&
@@ -22,7 +24,7 @@ extern "C" int hfa_gemm(const void* a, int a_dtype, int lda, const void* w, int 
         defer = 0;
     }
     if (pending_splits) *pending_splits = 0;
-    GemmArgs g = {a, a_dtype, lda, w, w_dtype, ldw, bias, out, out_dtype, ldo, accumulate, epilogue, M, N, K, stream, act};
+    GemmArgs g = {a, a_dtype, lda, w, w_dtype, ldw, bias, out, out_dtype, ldo, accumulate, epilogue, M, N, K, stream, gate_act ? gate_act : act};
     if (!force_plain && gemm_mfma_supports(g)) {
         if (!act || out_dtype == HFA_BF16) return gemm_mfma_launch(g, workspace, workspace_bytes, defer, pending_splits);
         g.act = 0;                            // a 32-bit output: the product, then the elementwise kernel

@@ -80,7 +80,7 @@ __device__ __forceinline__ void gemm_epilogue(floatx16 (&acc)[C::FM][C::FN], con
                     const int row = m0 + wm * C::TM + i * 32 + 8 * (r / 4) + 4 * (lane >> 5) + (r % 4);
                     if (row >= M) continue;
                     const float gt = acc[i][j][r], up = acc[i][j + 1][r];
-                    reinterpret_cast<uint16_t*>(out)[(size_t)row * ldo + f] = bf16_bits((gt / (1.0f + expf(-gt))) * up);
+                    reinterpret_cast<uint16_t*>(out)[(size_t)row * ldo + f] = bf16_bits(hfa_gate_half(act, gt) * up);
                 }
             }
         }
@@ -144,7 +144,7 @@ __device__ __forceinline__ void gemm_epilogue_rows(floatx16 (&acc)[C::FM][C::FN]
             for (int r = 0; r < 16; r++) {
                 const int row = wm * C::TM + i * 32 + 8 * (r / 4) + 4 * (lane >> 5) + (r % 4);
                 float v = acc[i][j][r] + b;
-                if constexpr (MODE == OUT_SWIGLU) v = (v / (1.0f + expf(-v))) * acc[i][j + 1][r];
+                if constexpr (MODE == OUT_SWIGLU) v = hfa_gate_half(act, v) * acc[i][j + 1][r];
                 else if constexpr (MODE == OUT_BF16_ACT) v = hfa_act_apply(act, v);
                 smem[row * O::STRIDE + col] = bf16_bits(v);
             }
@@ -485,7 +485,7 @@ __global__ void gemm_finish_kernel(const float* __restrict__ partial, int splits
         float up = 0.f;
         for (int s = 0; s < splits; s++) up += partial[(size_t)s * M * N + idx + 32];
         reinterpret_cast<uint16_t*>(out)[(size_t)row * ldo + (col / 64) * 32 + (col & 31)] =
-            bf16_bits((v / (1.0f + expf(-v))) * up);
+            bf16_bits(hfa_gate_half(act, v) * up);
     } else if (IS_BF16_OUT(MODE))
         reinterpret_cast<uint16_t*>(out)[(size_t)row * ldo + col] = bf16_bits(v);
     else if (MODE == OUT_F32)
@@ -497,7 +497,7 @@ __global__ void gemm_finish_kernel(const float* __restrict__ partial, int splits
 // The gate/up case of the above, four results a thread: 16-byte loads of every plane asked for
 // together (in batches of eight planes), added in ascending order, one 8-byte store.
 __global__ void gemm_finish_swiglu4_kernel(const float* __restrict__ partial, int splits, uint16_t* __restrict__ out,
-                                           int ldo, int M, int N) {
+                                           int ldo, int M, int N, int act) {
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;      // (row, block of 64 columns, quad)
     const int per_row = N / 8;
     if (idx >= (size_t)M * per_row) return;
@@ -520,8 +520,8 @@ __global__ void gemm_finish_swiglu4_kernel(const float* __restrict__ partial, in
         }
     }
     uint2 pk;
-    pk.x = (uint32_t)bf16_bits((g.x / (1.0f + expf(-g.x))) * u.x) | ((uint32_t)bf16_bits((g.y / (1.0f + expf(-g.y))) * u.y) << 16);
-    pk.y = (uint32_t)bf16_bits((g.z / (1.0f + expf(-g.z))) * u.z) | ((uint32_t)bf16_bits((g.w / (1.0f + expf(-g.w))) * u.w) << 16);
+    pk.x = (uint32_t)bf16_bits(hfa_gate_half(act, g.x) * u.x) | ((uint32_t)bf16_bits(hfa_gate_half(act, g.y) * u.y) << 16);
+    pk.y = (uint32_t)bf16_bits(hfa_gate_half(act, g.z) * u.z) | ((uint32_t)bf16_bits(hfa_gate_half(act, g.w) * u.w) << 16);
     *reinterpret_cast<uint2*>(out + (size_t)row * ldo + blk * 32 + quad * 4) = pk;
 }
 
@@ -616,7 +616,7 @@ int gemm_finish_launch(const float* partial, int splits, const float* bias, void
     else if (mode == OUT_F32)
         gemm_finish_kernel<OUT_F32><<<blocks, 256, 0, stream>>>(partial, splits, bias, out, ldo, M, N, act);
     else if (mode == OUT_SWIGLU && !bias && N % 64 == 0 && ldo % 4 == 0 && ((uintptr_t)out & 7) == 0 && ((uintptr_t)partial & 15) == 0)
-        gemm_finish_swiglu4_kernel<<<(int)((total / 8 + 255) / 256), 256, 0, stream>>>(partial, splits, (uint16_t*)out, ldo, M, N);
+        gemm_finish_swiglu4_kernel<<<(int)((total / 8 + 255) / 256), 256, 0, stream>>>(partial, splits, (uint16_t*)out, ldo, M, N, act);
     else if (mode == OUT_SWIGLU)
         gemm_finish_kernel<OUT_SWIGLU><<<blocks, 256, 0, stream>>>(partial, splits, bias, out, ldo, M, N, act);
     else

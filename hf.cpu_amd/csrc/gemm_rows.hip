@@ -343,7 +343,7 @@ __global__ __launch_bounds__(RG_WAVES * WAVE) void gemm_rows_kernel(const RowGem
                 const int j = i / (16 * MR), m = (i >> 4) % MR, n = i & 15, f = own0 + 16 * (tg0 / 2 + j) + n;
                 if (m < p.T && f < own1) {
                     const float gt = r_s[m] * total(2 * j, m, n), up = r_s[m] * total(2 * j + 1, m, n);
-                    p.act[(size_t)m * p.ldact + f] = rg_bf16(gt / (1.0f + __expf(-gt)) * up);        // src/mathx.c:34
+                    p.act[(size_t)m * p.ldact + f] = rg_bf16(hfa_gate_half(p.out_act, gt) * up);        // src/mathx.c:34
                 }
             }
         } else {
@@ -474,6 +474,7 @@ extern "C" int hfa_gemm_rows(int mode, const void* a, int lda, const void* w, in
         return rows_dispatch<HFA_ROWS_RESID>(p, stream);
     }
     HFA_REQUIRE(act && ldact >= N && !bias, "gemm_rows: the gate/up mode needs an output of N features and takes no bias");
-    p.act = (uint16_t*)act; p.ldact = ldact;
+    HFA_REQUIRE(out_act == 0 || out_act == HFA_ACT_GELU_TANH, "gemm_rows: the gate passes silu or the tanh form of gelu, not %d", out_act);
+    p.act = (uint16_t*)act; p.ldact = ldact; p.out_act = out_act;
     return rows_dispatch<HFA_ROWS_SWIGLU>(p, stream);
 }

@@ -32,13 +32,14 @@ __device__ __forceinline__ void wave_best(float& v, int& i) {
 // exp(logit - the largest logit), which with `renorm` makes the weights the softmax over the chosen logits alone); experts
 // form n_groups runs of neighbours, a run scores as its best expert, and only experts of the `keep` best runs can
 // be chosen; the `top` best of those are chosen, and weigh score / (sum of the chosen scores + 1e-20) if `renorm`,
-// else their score; times `out_scale`.
+// else their score; times `out_scale`. `correction` (null: none) is added to the scores for the choice, not for the weights.
 __global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict__ logits, int ld, int E, int top,
                                                         int n_groups, int keep, int scoring, int renorm, float out_scale,
-                                                        int* __restrict__ ids, float* __restrict__ weights) {
+                                                        const float* __restrict__ correction, int* __restrict__ ids, float* __restrict__ weights) {
     __shared__ float s[MOE_MAX_EXPERTS];
     __shared__ float gs[MOE_MAX_EXPERTS];
     __shared__ unsigned char open_s[MOE_MAX_EXPERTS];        // per group: may be chosen from
+    __shared__ float plain_s[MOE_MAX_EXPERTS];               // the scores without the correction
     const int t = blockIdx.x, lane = threadIdx.x;
     const float* z = logits + (size_t)t * ld;
     if (scoring == 0) {
@@ -61,6 +62,11 @@ __global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict
     } else {
         for (int e = lane; e < E; e += WAVE) s[e] = 1.0f / (1.0f + expf(-z[e]));
     }
+    if (correction)
+        for (int e = lane; e < E; e += WAVE) {               // (a lane's own experts)
+            plain_s[e] = s[e];
+            s[e] += correction[e];
+        }
     __syncthreads();
     const int per = E / n_groups;
     for (int g = lane; g < n_groups; g += WAVE) {
@@ -86,10 +92,13 @@ __global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict
         float bv = -INFINITY;
         int bi = 0x7fffffff;
         for (int e = lane; e < E; e += WAVE)
-            if (open_s[e / per] && s[e] >= 0.f) better(bv, bi, s[e], e);
+            if (open_s[e / per] && s[e] > -INFINITY) better(bv, bi, s[e], e);
         wave_best(bv, bi);
         if (bi >= E) { bi = 0; bv = 0.f; }                   // fewer open experts than choices: weight nothing
-        else if (lane == 0) s[bi] = -1.f;                    // taken
+        else {
+            if (correction) bv = plain_s[bi];
+            if (lane == 0) s[bi] = -INFINITY;                // taken
+        }
         if (lane == 0) {
             ids[(size_t)t * top + r] = bi;
             weights[(size_t)t * top + r] = bv;
@@ -104,7 +113,7 @@ __global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict
 }
 
 extern "C" int hfa_moe_route(const float* logits, int ld, int n_tokens, int n_experts, int top, int n_groups, int keep,
-                             int scoring, int renorm, float out_scale, int* ids, float* weights, hipStream_t stream) {
+                             int scoring, int renorm, float out_scale, const float* correction, int* ids, float* weights, hipStream_t stream) {
     HFA_REQUIRE(logits && ids && weights && n_tokens > 0, "moe_route: bad arguments");
     HFA_REQUIRE(n_experts > 0 && n_experts <= MOE_MAX_EXPERTS && ld >= n_experts, "moe_route: %d experts (at most %d)", n_experts,
                 MOE_MAX_EXPERTS);
@@ -112,7 +121,7 @@ extern "C" int hfa_moe_route(const float* logits, int ld, int n_tokens, int n_ex
     HFA_REQUIRE(n_groups > 0 && n_experts % n_groups == 0 && keep > 0 && keep <= n_groups,
                 "moe_route: %d experts do not form %d equal groups of which %d are kept", n_experts, n_groups, keep);
     HFA_REQUIRE(scoring >= 0 && scoring <= 2, "moe_route: unknown scoring %d", scoring);
-    moe_route_kernel<<<n_tokens, WAVE, 0, stream>>>(logits, ld, n_experts, top, n_groups, keep, scoring, renorm, out_scale, ids,
+    moe_route_kernel<<<n_tokens, WAVE, 0, stream>>>(logits, ld, n_experts, top, n_groups, keep, scoring, renorm, out_scale, correction, ids,
                                                     weights);
     HFA_LAUNCH_CHECK("moe_route");
     return 0;

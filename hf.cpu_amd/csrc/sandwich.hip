@@ -4,11 +4,13 @@
 // keys and values, and the mixing of attention outputs across heads.
 //
 //   hfa_embed_pos         x[t] = table[token] * scale + sinusoid(position)
-//   hfa_rmsnorm_add       out[r] (+)= scale * rmsnorm(y[r] * sigmoid(gate[r])) * w
+//   hfa_rmsnorm_add       out[r] (+)= scale * rmsnorm(branch[r]) * w, the branch as its last products left it; and a rounded copy of out
 //   hfa_polynorm          out = a N(z) + b N(z^2) + c N(z^3) + e, N dividing a row by its root mean square
 //   hfa_scale_rows        x *= s
-//   hfa_head_norm_store   per head: q, k <- rms or unit norm (a weight of one head's size, shared); q to a matrix, k and
-//                         v to their cache rows
+//   hfa_head_norm_store   per head: q, k <- rms norm (with a weight of one head's size, shared, or none) before or after a
+//                         rotation; q to a matrix, k and v to their cache rows
+//   hfa_diff_mix          out[t, h] = c * a / rms(a), a = map 1 of head h minus a factor times map 2
+//   hfa_round_rows        an fp32 matrix in bf16
 //   hfa_talk_mix          out[t, h] = sigmoid(gate[t, h]) * sum_g talk[h, g] * A[t, g, values of h's group]
 #include "api.h"
 #include "common.h"
@@ -49,63 +51,166 @@ extern "C" int hfa_embed_pos(const void* table, int table_dtype, const int* toke
 }
 
 // ---- the norm of a branch's result, added into the stream -----------------------------------------------------------
-// One block a row, all in fp32: v = y * sigmoid(gate) (gate null: v = y); out (+)= scale * v / sqrt(mean(v^2) + eps) * w.
-template <typename TG>
-__global__ __launch_bounds__(256) void rmsnorm_add_kernel(const float* __restrict__ y, int ldy, const TG* __restrict__ gate, int ldg,
-                                                         const float* __restrict__ gate_bias, const float* __restrict__ w,
-                                                         float* __restrict__ out, int ldo, int width, float eps, float scale,
-                                                         int accumulate) {
+// One block a row, all in fp32. The branch's value at a column is
+//   b = [ y | the sum over the planes of a product whose K was split ] * sigmoid(row_gate[r]) + sum_k pairs[r * top + k]
+// (an absent part is left out: the result of experts is `pairs`, that of a shared expert `y` with its gate), then times
+// sigmoid(gate + gate_bias) element by element; out (+)= scale * b / sqrt(mean(b^2) + eps) * w, or, w null, scale * b. `copy`
+// receives the new out in bf16: what a sublayer reads that has no norm in front of it. VW columns a thread and turn.
+#define JOIN_PLANES 8
+template <int VW>
+struct JoinVec { float v[VW]; };
+template <int VW>
+__device__ __forceinline__ JoinVec<VW> join_load(const float* p) {
+    JoinVec<VW> r;
+    if constexpr (VW == 4) {
+        const float4 u = *reinterpret_cast<const float4*>(p);
+        r.v[0] = u.x; r.v[1] = u.y; r.v[2] = u.z; r.v[3] = u.w;
+    } else {
+        r.v[0] = *p;
+    }
+    return r;
+}
+struct JoinArgs {
+    const float* y; int ldy;
+    const float* partial; int splits; size_t plane;
+    const float* row_gate; int ld_row_gate;
+    const float* pairs; int top;
+    const void* gate; int gate_bf16, ldg;
+    const float* gate_bias;
+    const float* w;
+    float* out; int ldo;
+    uint16_t* copy; int ldc;
+    int width; float eps, scale; int accumulate;
+};
+
+template <int VW>
+__global__ __launch_bounds__(1024) void rmsnorm_add_kernel(JoinArgs p) {
     __shared__ float red[17];
     const int r = blockIdx.x;
-    const float* src = y + (size_t)r * ldy;
-    const TG* gs = gate ? gate + (size_t)r * ldg : nullptr;
-    constexpr int KEEP = 8;
-    float keep[KEEP];
-    auto value = [&](int i) {
-        float v = src[i];
-        if (gs) {
-            const float z = to_f32(gs[i]) + (gate_bias ? gate_bias[i] : 0.f);
-            v *= 1.0f / (1.0f + expf(-z));
+    const float row_factor = p.row_gate ? 1.0f / (1.0f + expf(-p.row_gate[(size_t)r * p.ld_row_gate])) : 1.f;
+    constexpr int KEEP = 8 / VW * (VW == 4 ? 2 : 1);          // 16 columns a thread stay in registers (8 one at a time)
+    JoinVec<VW> keep[KEEP];
+    auto value = [&](int c) {
+        JoinVec<VW> b = {};
+        if (p.partial) {
+            const float* src = p.partial + (size_t)r * p.width + c;
+            for (int s0 = 0; s0 < p.splits; s0 += JOIN_PLANES) {          // batches of loads that do not wait for one another
+                JoinVec<VW> q[JOIN_PLANES];
+#pragma unroll
+                for (int u = 0; u < JOIN_PLANES; u++) q[u] = s0 + u < p.splits ? join_load<VW>(src + (s0 + u) * p.plane) : JoinVec<VW>{};
+#pragma unroll
+                for (int u = 0; u < JOIN_PLANES; u++)
+#pragma unroll
+                    for (int e = 0; e < VW; e++) b.v[e] += q[u].v[e];
+            }
+        } else if (p.y) {
+            b = join_load<VW>(p.y + (size_t)r * p.ldy + c);
         }
-        return v;
+#pragma unroll
+        for (int e = 0; e < VW; e++) b.v[e] *= row_factor;
+        if (p.pairs) {
+            const float* src = p.pairs + (size_t)r * p.top * p.width + c;
+            JoinVec<VW> sum = {};
+            for (int k0 = 0; k0 < p.top; k0 += 4) {
+                JoinVec<VW> q[4];
+#pragma unroll
+                for (int u = 0; u < 4; u++) q[u] = k0 + u < p.top ? join_load<VW>(src + (size_t)(k0 + u) * p.width) : JoinVec<VW>{};
+#pragma unroll
+                for (int u = 0; u < 4; u++)
+#pragma unroll
+                    for (int e = 0; e < VW; e++) sum.v[e] += q[u].v[e];
+            }
+#pragma unroll
+            for (int e = 0; e < VW; e++) b.v[e] += sum.v[e];
+        }
+        if (p.gate) {
+#pragma unroll
+            for (int e = 0; e < VW; e++) {
+                const size_t i = (size_t)r * p.ldg + c + e;
+                const float z = (p.gate_bf16 ? to_f32(((const bf16*)p.gate)[i]) : ((const float*)p.gate)[i]) + (p.gate_bias ? p.gate_bias[c + e] : 0.f);
+                b.v[e] *= 1.0f / (1.0f + expf(-z));
+            }
+        }
+        return b;
     };
+    const int stride = blockDim.x * VW, c0 = threadIdx.x * VW;
     float ss = 0.f;
 #pragma unroll
     for (int k = 0; k < KEEP; k++) {
-        const int i = threadIdx.x + k * blockDim.x;
-        keep[k] = i < width ? value(i) : 0.f;
-        ss = fmaf(keep[k], keep[k], ss);
+        const int c = c0 + k * stride;
+        keep[k] = c < p.width ? value(c) : JoinVec<VW>{};
+#pragma unroll
+        for (int e = 0; e < VW; e++) ss = fmaf(keep[k].v[e], keep[k].v[e], ss);
     }
-    for (int i = threadIdx.x + KEEP * blockDim.x; i < width; i += blockDim.x) {
-        const float v = value(i);
-        ss = fmaf(v, v, ss);
+    for (int c = c0 + KEEP * stride; c < p.width; c += stride) {
+        const JoinVec<VW> b = value(c);
+#pragma unroll
+        for (int e = 0; e < VW; e++) ss = fmaf(b.v[e], b.v[e], ss);
     }
-    const float inv = scale / sqrtf(block_sum(ss, red) / (float)width + eps);
-    float* dst = out + (size_t)r * ldo;
-    auto finish = [&](int i, float v) {
-        const float z = v * inv * w[i];
-        dst[i] = accumulate ? dst[i] + z : z;
+    const float inv = p.w ? p.scale / sqrtf(block_sum(ss, red) / (float)p.width + p.eps) : p.scale;
+    float* dst = p.out + (size_t)r * p.ldo;
+    auto finish = [&](int c, const JoinVec<VW>& b) {
+        JoinVec<VW> z, o = {};
+        if (p.accumulate) o = join_load<VW>(dst + c);
+#pragma unroll
+        for (int e = 0; e < VW; e++) z.v[e] = o.v[e] + (p.w ? b.v[e] * inv * p.w[c + e] : b.v[e] * inv);
+        if constexpr (VW == 4) {
+            *reinterpret_cast<float4*>(dst + c) = make_float4(z.v[0], z.v[1], z.v[2], z.v[3]);
+            if (p.copy)
+                *reinterpret_cast<uint2*>(p.copy + (size_t)r * p.ldc + c) =
+                    make_uint2((uint32_t)bf16_bits(z.v[0]) | ((uint32_t)bf16_bits(z.v[1]) << 16),
+                               (uint32_t)bf16_bits(z.v[2]) | ((uint32_t)bf16_bits(z.v[3]) << 16));
+        } else {
+            dst[c] = z.v[0];
+            if (p.copy) p.copy[(size_t)r * p.ldc + c] = bf16_bits(z.v[0]);
+        }
     };
 #pragma unroll
     for (int k = 0; k < KEEP; k++) {
-        const int i = threadIdx.x + k * blockDim.x;
-        if (i < width) finish(i, keep[k]);
+        const int c = c0 + k * stride;
+        if (c < p.width) finish(c, keep[k]);
     }
-    for (int i = threadIdx.x + KEEP * blockDim.x; i < width; i += blockDim.x) finish(i, value(i));
+    for (int c = c0 + KEEP * stride; c < p.width; c += stride) finish(c, value(c));
 }
 
-extern "C" int hfa_rmsnorm_add(const float* y, int ldy, const void* gate, int gate_dtype, int ldg, const float* gate_bias,
-                               const float* w, float* out, int ldo, int n_rows, int width, float eps, float scale, int accumulate,
-                               hipStream_t stream) {
-    HFA_REQUIRE(y && w && out && n_rows > 0 && width > 0 && ldy >= width && ldo >= width && (!gate || ldg >= width),
-                "rmsnorm_add: bad arguments");
+extern "C" int hfa_rmsnorm_add(const float* y, int ldy, const float* partial, int splits, const float* row_gate, int ld_row_gate,
+                               const float* pairs, int top, const void* gate, int gate_dtype, int ldg, const float* gate_bias,
+                               const float* w, float* out, int ldo, void* copy, int ldc, int n_rows, int width, float eps, float scale,
+                               int accumulate, hipStream_t stream) {
+    HFA_REQUIRE((y || partial || pairs) && out && n_rows > 0 && width > 0 && (!y || ldy >= width) && ldo >= width && (!gate || ldg >= width) &&
+                    (!copy || ldc >= width) && (!pairs || top > 0) && (!partial || splits > 0), "rmsnorm_add: bad arguments");
     HFA_REQUIRE(!gate || gate_dtype == HFA_F32 || gate_dtype == HFA_BF16, "rmsnorm_add: unknown gate dtype %d", gate_dtype);
     HFA_REQUIRE(gate || !gate_bias, "rmsnorm_add: a gate's bias without the gate");
-    if (gate && gate_dtype == HFA_BF16)
-        rmsnorm_add_kernel<bf16><<<n_rows, 256, 0, stream>>>(y, ldy, (const bf16*)gate, ldg, gate_bias, w, out, ldo, width, eps, scale, accumulate);
-    else
-        rmsnorm_add_kernel<float><<<n_rows, 256, 0, stream>>>(y, ldy, (const float*)gate, ldg, gate_bias, w, out, ldo, width, eps, scale, accumulate);
+    const JoinArgs p = {y, ldy, partial, splits, (size_t)n_rows * width, row_gate, ld_row_gate, pairs, top, gate, gate && gate_dtype == HFA_BF16,
+                        ldg, gate_bias, w, out, ldo, (uint16_t*)copy, ldc, width, eps, scale, accumulate};
+    const bool vec = width % 4 == 0 && (!y || (ldy % 4 == 0 && ((uintptr_t)y & 15) == 0)) && ((uintptr_t)partial & 15) == 0 && ((uintptr_t)pairs & 15) == 0 &&
+                     ldo % 4 == 0 && ((uintptr_t)out & 15) == 0 && (!copy || (ldc % 4 == 0 && ((uintptr_t)copy & 7) == 0));
+    if (vec) {
+        // few rows: a row's loads are shared by as many threads as it has groups of four columns
+        int threads = n_rows >= 512 ? 256 : 1024;
+        while (threads > 64 && threads / 2 * 4 >= width) threads /= 2;
+        rmsnorm_add_kernel<4><<<n_rows, threads, 0, stream>>>(p);
+    } else {
+        rmsnorm_add_kernel<1><<<n_rows, 256, 0, stream>>>(p);
+    }
     HFA_LAUNCH_CHECK("rmsnorm_add");
+    return 0;
+}
+
+// ---- an fp32 matrix in bf16 ------------------------------------------------------------------------------------------
+__global__ void round_rows_kernel(const float* __restrict__ x, int ldx, uint16_t* __restrict__ out, int ldo, int width, size_t total) {
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x) {
+        const size_t r = i / width, c = i % width;
+        out[r * ldo + c] = bf16_bits(x[r * ldx + c]);
+    }
+}
+
+extern "C" int hfa_round_rows(const float* x, int ldx, void* out, int ldo, int n_rows, int width, hipStream_t stream) {
+    HFA_REQUIRE(x && out && n_rows > 0 && width > 0 && ldx >= width && ldo >= width, "round_rows: bad arguments");
+    const size_t total = (size_t)n_rows * width;
+    const int blocks = (int)((total + 255) / 256 < 65535 ? (total + 255) / 256 : 65535);
+    round_rows_kernel<<<blocks, 256, 0, stream>>>(x, ldx, (uint16_t*)out, ldo, width, total);
+    HFA_LAUNCH_CHECK("round_rows");
     return 0;
 }
 
@@ -170,60 +275,174 @@ extern "C" int hfa_scale_rows(float* x, int ld, int n_rows, int width, float s, 
 }
 
 // ---- queries and keys normed head by head; keys and values to the cache ------------------------------------------------
-// Rows [q: H D | k: G D | v: G Dv] (fp32 or bf16): every q head and every k head is divided by sqrt(mean(head^2) + eps) and
-// multiplied by a weight of D values that all heads share (q_w, k_w; null: no norm for that part). q goes to q_out
-// ([T, H D], the cache's dtype), k to cache row slot_map[t], v to the same row with the page transposed
-// ([page][column][offset]). One wave a head, four waves a block, a block a token and four heads; the blocks of a token
-// share its values out.
-template <typename TI, typename TO>
-__global__ __launch_bounds__(256) void head_norm_store_kernel(const TI* __restrict__ qkv, int ld, int H, int G, int D, int Dv,
-                                                             const float* __restrict__ q_w, const float* __restrict__ k_w, float eps,
-                                                             TO* __restrict__ q_out, int ldq, TO* __restrict__ k_cache,
-                                                             TO* __restrict__ v_cache, const int* __restrict__ slot_map, int page_tokens) {
-    const int t = blockIdx.x, lane = threadIdx.x & (WAVE - 1), wv = threadIdx.x / WAVE, nw = blockDim.x / WAVE;
-    const TI* row = qkv + (size_t)t * ld;
-    const int QD = H * D, KD = G * D, VD = G * Dv;
-    const int slot = slot_map[t];
-    const int hs = blockIdx.y * nw + wv;
-    if (hs < H + G) {
-        const bool is_key = hs >= H;
-        const TI* src = row + hs * D;
-        const float* w = is_key ? k_w : q_w;
-        float inv = 1.f;
-        if (w) {
-            float ss = 0.f;
-            for (int i = lane; i < D; i += WAVE) { const float v = to_f32(src[i]); ss = fmaf(v, v, ss); }
-            inv = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
-        }
-        TO* dst = is_key ? k_cache + (size_t)slot * KD + (hs - H) * D : q_out + (size_t)t * ldq + hs * D;
-        for (int i = lane; i < D; i += WAVE) {
-            float v = to_f32(src[i]);
-            if (w) v = v * inv * w[i];
-            dst[i] = from_f32<TO>(v);
+// Rows [q: H D | k: G D | v: GV Dv] (fp32 or bf16). Every q head and every k head is (norm_q, norm_k) divided by sqrt(mean(head^2) +
+// eps) and multiplied by a weight of D values that all heads share (q_w, k_w; null: 1), and (cs not null) its first rot_dim
+// dimensions are turned, i with i + rot_dim / 2, by the token's angles (cs: hfa_rope_table's rows [cosines | sines]); norm_after:
+// the rotation comes first and the norm after it. q goes to q_out ([T, H D], the cache's dtype), k to cache row slot_map[t], v to
+// the same row with the page transposed ([page][column][offset]).
+struct HeadNorm {
+    int H, G, D, GV, Dv;
+    const float* q_w; const float* k_w;
+    int norm_q, norm_k, norm_after;
+    float eps;
+    const float* cs; int rot_dim;
+    const int* slot_map; int page_tokens;
+};
+
+// One head's values by S neighbouring lanes (a power of two), D <= S NE: lane l holds values l, l + S, ...
+template <typename TI, int S, int NE>
+__device__ __forceinline__ void normed_head(const TI* __restrict__ src, const HeadNorm& p, bool is_key, int t, int l, float (&v)[NE]) {
+    const int half = p.rot_dim / 2;
+    const float* cs = p.cs ? p.cs + (size_t)t * p.rot_dim : nullptr;
+    const float* w = is_key ? p.k_w : p.q_w;
+    const bool norm = is_key ? p.norm_k : p.norm_q;
+    float other[NE];
+#pragma unroll
+    for (int i = 0; i < NE; i++) {
+        const int c = l + i * S;
+        v[i] = c < p.D ? to_f32(src[c]) : 0.f;
+        other[i] = cs && c < p.rot_dim ? to_f32(src[c < half ? c + half : c - half]) : 0.f;
+    }
+    float ss = 0.f;
+    auto turn = [&](float x, float y, int c) {              // c's place in its pair decides the sign
+        return c < half ? x * cs[c] - y * cs[half + c] : x * cs[c - half] + y * cs[c];
+    };
+    if (norm && !p.norm_after) {
+#pragma unroll
+        for (int i = 0; i < NE; i++) ss = fmaf(v[i], v[i], ss);
+    } else if (cs) {
+#pragma unroll
+        for (int i = 0; i < NE; i++) {
+            const int c = l + i * S;
+            if (c < p.rot_dim) v[i] = turn(v[i], other[i], c);
         }
     }
-    for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < VD; c += gridDim.y * blockDim.x)
-        v_cache[(size_t)(slot / page_tokens) * page_tokens * VD + (size_t)c * page_tokens + slot % page_tokens] =
-            from_f32<TO>(to_f32(row[QD + KD + c]));
+    if (norm && p.norm_after) {
+#pragma unroll
+        for (int i = 0; i < NE; i++) ss = fmaf(v[i], v[i], ss);
+    }
+    if (norm) {
+#pragma unroll
+        for (int off = S / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, WAVE);
+        const float inv = 1.0f / sqrtf(ss / (float)p.D + p.eps);
+#pragma unroll
+        for (int i = 0; i < NE; i++) {
+            const int c = l + i * S;
+            if (c >= p.D) continue;
+            v[i] *= inv * (w ? w[c] : 1.f);
+            if (!p.norm_after && cs && c < p.rot_dim) {
+                const int o = c < half ? c + half : c - half;
+                v[i] = turn(v[i], other[i] * inv * (w ? w[o] : 1.f), c);
+            }
+        }
+    }
 }
 
-extern "C" int hfa_head_norm_store(const void* qkv, int in_dtype, int ld, int n_heads, int n_kv_heads, int head_dim, int v_head_dim,
-                                   const float* q_w, const float* k_w, float eps, void* q_out, int ldq, void* k_cache, void* v_cache,
-                                   int out_dtype, const int* slot_map, int page_tokens, int n_tokens, hipStream_t stream) {
+// A block of four waves a token and 4 * 64 / S heads; the blocks of a token share its values out.
+template <typename TI, typename TO, int S, int NE>
+__global__ __launch_bounds__(256) void head_norm_store_kernel(const TI* __restrict__ qkv, int ld, HeadNorm p, TO* __restrict__ q_out, int ldq,
+                                                             TO* __restrict__ k_cache, TO* __restrict__ v_cache) {
+    const int t = blockIdx.x, l = threadIdx.x % S, H = p.H, G = p.G, D = p.D;
+    const TI* row = qkv + (size_t)t * ld;
+    const int KD = G * D, VD = p.GV * p.Dv;
+    const int slot = p.slot_map[t];
+    const int hs = blockIdx.y * (256 / S) + threadIdx.x / S;
+    // (every lane of a wave takes part in the sums; lanes beyond the last head repeat it and store nothing)
+    const int hc = hs < H + G ? hs : H + G - 1;
+    float v[NE];
+    normed_head<TI, S, NE>(row + hc * D, p, hc >= H, t, l, v);
+    if (hs < H + G) {
+        TO* dst = hs >= H ? k_cache + (size_t)slot * KD + (hs - H) * D : q_out + (size_t)t * ldq + hs * D;
+#pragma unroll
+        for (int i = 0; i < NE; i++)
+            if (l + i * S < D) dst[l + i * S] = from_f32<TO>(v[i]);
+    }
+    for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < VD; c += gridDim.y * blockDim.x)
+        v_cache[(size_t)(slot / p.page_tokens) * p.page_tokens * VD + (size_t)c * p.page_tokens + slot % p.page_tokens] =
+            from_f32<TO>(to_f32(row[(H + G) * D + c]));
+}
+
+extern "C" int hfa_head_norm_store(const void* qkv, int in_dtype, int ld, int n_heads, int n_kv_heads, int head_dim, int n_v_heads, int v_head_dim,
+                                   const float* q_w, const float* k_w, int norm_q, int norm_k, int norm_after, float eps, const float* cos_sin,
+                                   int rot_dim, void* q_out, int ldq, void* k_cache, void* v_cache, int out_dtype, const int* slot_map,
+                                   int page_tokens, int n_tokens, hipStream_t stream) {
     HFA_REQUIRE(qkv && q_out && k_cache && v_cache && slot_map && n_tokens > 0 && n_heads > 0 && n_kv_heads > 0 && head_dim > 0 &&
-                    v_head_dim > 0 && page_tokens > 0, "head_norm_store: bad arguments");
-    HFA_REQUIRE(ld >= (n_heads + n_kv_heads) * head_dim + n_kv_heads * v_head_dim && ldq >= n_heads * head_dim,
+                    n_v_heads > 0 && v_head_dim > 0 && page_tokens > 0, "head_norm_store: bad arguments");
+    HFA_REQUIRE(ld >= (n_heads + n_kv_heads) * head_dim + n_v_heads * v_head_dim && ldq >= n_heads * head_dim,
                 "head_norm_store: a row is shorter than its heads");
     HFA_REQUIRE((in_dtype == HFA_F32 || in_dtype == HFA_BF16) && (out_dtype == HFA_F32 || out_dtype == HFA_BF16),
                 "head_norm_store: unknown dtype");
-#define HNS(TI, TO)                                                                                                          \
-    head_norm_store_kernel<TI, TO><<<dim3(n_tokens, (n_heads + n_kv_heads + 3) / 4), 256, 0, stream>>>((const TI*)qkv, ld, n_heads, n_kv_heads, head_dim, v_head_dim, \
-                                                                 q_w, k_w, eps, (TO*)q_out, ldq, (TO*)k_cache, (TO*)v_cache,   \
-                                                                 slot_map, page_tokens)
-    if (in_dtype == HFA_F32) { if (out_dtype == HFA_F32) HNS(float, float); else HNS(float, bf16); }
-    else { if (out_dtype == HFA_F32) HNS(bf16, float); else HNS(bf16, bf16); }
+    HFA_REQUIRE(head_dim <= 1024 && (!cos_sin || (rot_dim > 0 && rot_dim % 2 == 0 && rot_dim <= head_dim)),
+                "head_norm_store: heads of %d values (at most 1024), of which an even number within the head is turned", head_dim);
+    const HeadNorm p = {n_heads, n_kv_heads, head_dim, n_v_heads, v_head_dim, q_w, k_w, norm_q, norm_k, norm_after, eps, cos_sin,
+                        cos_sin ? rot_dim : 0, slot_map, page_tokens};
+#define HNS(TI, TO, S, NE)                                                                                                       \
+    head_norm_store_kernel<TI, TO, S, NE><<<dim3(n_tokens, (n_heads + n_kv_heads + 256 / S - 1) / (256 / S)), 256, 0, stream>>>(     \
+        (const TI*)qkv, ld, p, (TO*)q_out, ldq, (TO*)k_cache, (TO*)v_cache)
+#define HNS_SIZES(TI, TO)                            \
+    do {                                             \
+        if (head_dim <= 32) HNS(TI, TO, 16, 2);      \
+        else if (head_dim <= 64) HNS(TI, TO, 32, 2); \
+        else if (head_dim <= 128) HNS(TI, TO, 64, 2); \
+        else if (head_dim <= 256) HNS(TI, TO, 64, 4); \
+        else HNS(TI, TO, 64, 16);                    \
+    } while (0)
+    if (in_dtype == HFA_F32) { if (out_dtype == HFA_F32) HNS_SIZES(float, float); else HNS_SIZES(float, bf16); }
+    else { if (out_dtype == HFA_F32) HNS_SIZES(bf16, float); else HNS_SIZES(bf16, bf16); }
+#undef HNS_SIZES
 #undef HNS
     HFA_LAUNCH_CHECK("head_norm_store");
+    return 0;
+}
+
+// ---- two attention maps of a head as one -----------------------------------------------------------------------------
+// a [T][G][2][R][Dv] (fp32; the two maps of the R heads of each of G groups): out[t, g R + r] = c d / sqrt(mean(d^2) + eps) with
+// d = a[t, g, 0, r] - factor[0] a[t, g, 1, r]. S lanes a head, 256 / S heads a block.
+template <typename TO, int S, int NE>
+__global__ __launch_bounds__(256) void diff_mix_kernel(const float* __restrict__ a, int lda, const float* __restrict__ factor, float c, float eps,
+                                                      TO* __restrict__ out, int ldo, int H, int R, int Dv) {
+    const int t = blockIdx.x, l = threadIdx.x % S, hs = blockIdx.y * (256 / S) + threadIdx.x / S;
+    const int h = hs < H ? hs : H - 1, g = h / R, r = h % R;
+    const float* a1 = a + (size_t)t * lda + (size_t)(2 * g * R + r) * Dv;
+    const float* a2 = a1 + (size_t)R * Dv;
+    const float f = factor[0];
+    float d[NE], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NE; i++) {
+        const int x = l + i * S;
+        d[i] = x < Dv ? a1[x] - f * a2[x] : 0.f;
+        ss = fmaf(d[i], d[i], ss);
+    }
+#pragma unroll
+    for (int off = S / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, WAVE);
+    const float inv = c / sqrtf(ss / (float)Dv + eps);
+    if (hs >= H) return;
+#pragma unroll
+    for (int i = 0; i < NE; i++)
+        if (l + i * S < Dv) out[(size_t)t * ldo + (size_t)h * Dv + l + i * S] = from_f32<TO>(d[i] * inv);
+}
+
+extern "C" int hfa_diff_mix(const float* a, int lda, const float* factor, float c, float eps, void* out, int out_dtype, int ldo, int n_tokens,
+                            int n_heads, int n_kv_heads, int v_head_dim, hipStream_t stream) {
+    HFA_REQUIRE(a && factor && out && n_tokens > 0 && n_heads > 0 && n_kv_heads > 0 && n_heads % n_kv_heads == 0 && v_head_dim > 0,
+                "diff_mix: bad arguments");
+    HFA_REQUIRE(lda >= 2 * n_heads * v_head_dim && ldo >= n_heads * v_head_dim && v_head_dim <= 1024, "diff_mix: a row is shorter than its heads, "
+                "or a head has more than 1024 values");
+    HFA_REQUIRE(out_dtype == HFA_F32 || out_dtype == HFA_BF16, "diff_mix: unknown dtype %d", out_dtype);
+#define DM(TO, S, NE)                                                                                                            \
+    diff_mix_kernel<TO, S, NE><<<dim3(n_tokens, (n_heads + 256 / S - 1) / (256 / S)), 256, 0, stream>>>(a, lda, factor, c, eps, (TO*)out, ldo, \
+                                                                                                        n_heads, n_heads / n_kv_heads, v_head_dim)
+#define DM_SIZES(TO)                             \
+    do {                                         \
+        if (v_head_dim <= 64) DM(TO, 32, 2);     \
+        else if (v_head_dim <= 128) DM(TO, 64, 2); \
+        else if (v_head_dim <= 256) DM(TO, 64, 4); \
+        else DM(TO, 64, 16);                     \
+    } while (0)
+    if (out_dtype == HFA_F32) DM_SIZES(float); else DM_SIZES(bf16);
+#undef DM_SIZES
+#undef DM
+    HFA_LAUNCH_CHECK("diff_mix");
     return 0;
 }
 

@@ -21,7 +21,8 @@ _SIGNATURES = {
     "hfa_gemm_rows": [I, P, I, P, I, I, I, I, P, P, I, F, F, P, I, I, I, P, I, P, P, P, I, P, I, P],
     "hfa_gemm_rows_supports": [I, I, I, I, I, I],
     "hfa_rope_store": [P, I, I, P, P, I, I, I, I, I, P, P, P, I, I, P, I, P, P],
-    "hfa_paged_attention": [P, I, I, P, P, I, I, P, I, P, P, P, I, I, I, P, I, I, I, I, I, I, I, I, I, F, P, I, I, F, I, P, P, P, P, P, c_size_t, I, P],
+    "hfa_paged_attention": [P, I, I, P, P, I, I, P, I, P, P, P, I, I, I, P, I, I, I, I, I, I, I, I, I, F, P, I, I, F, I, P, P, P, P, I, I, P, I, P, I, I,
+                            F, I, P, c_size_t, I, P],
     "hfa_scale_add": [P, I, P, F, P, I, I, I, I, P],
     "hfa_gate_mul": [P, I, I, P, I, I, P, I, I, I, I, I, P],
     "hfa_latent_store": [P, I, P, I, I, P, F, P, P, I, I, P, I, P, P, I, P, I, I, I, I, I, I, P, P],
@@ -33,10 +34,12 @@ _SIGNATURES = {
     "hfa_group_rmsnorm": [P, I, I, P, P, I, I, P, I, I, I, F, P, I, I, I, P, P],
     "hfa_delta_scan": [P, I, P, I, I, I, P, I, I, I, P, I, P, P, P, I, F, F, P, c_size_t, P, P, I, I, P, I, P],
     "hfa_embed_pos": [P, I, P, P, P, P, I, I, I, F, P],
-    "hfa_rmsnorm_add": [P, I, P, I, I, P, P, P, I, I, I, F, F, I, P],
+    "hfa_rmsnorm_add": [P, I, P, I, P, I, P, I, P, I, I, P, P, P, I, P, I, I, I, F, F, I, P],
+    "hfa_round_rows": [P, I, P, I, I, I, P],
+    "hfa_diff_mix": [P, I, P, F, F, P, I, I, I, I, I, I, P],
     "hfa_polynorm": [P, I, I, P, P, I, I, I, I, F, P],
     "hfa_scale_rows": [P, I, I, I, F, P],
-    "hfa_head_norm_store": [P, I, I, I, I, I, I, P, P, F, P, I, P, P, I, P, I, I, P],
+    "hfa_head_norm_store": [P, I, I, I, I, I, I, I, P, P, I, I, I, F, P, I, P, I, P, P, I, P, I, I, P],
     "hfa_talk_mix": [P, I, P, P, I, I, P, I, I, I, I, I, I, P],
     "hfa_qkv_prepare": [P, I, I, P, P, I, I, I, I, I, I, P, P, F, P, P, P, P, P, P, I, I, P],
     "hfa_causal_conv": [P, I, I, P, P, I, I, P, c_size_t, P, P, I, I, P, I, I, I, P],
@@ -48,12 +51,12 @@ _SIGNATURES = {
     "hfa_layernorm": [P, P, P, P, I, P, I, I, F, P, I, P, I, P],
     "hfa_activation": [P, I, P, I, I, I, I, I, P],
     "hfa_softcap": [P, I, I, I, F, P],
-    "hfa_moe_route": [P, I, I, I, I, I, I, I, I, F, P, P, P],
+    "hfa_moe_route": [P, I, I, I, I, I, I, I, I, F, P, P, P, P],
     "hfa_moe_plan": [P, I, I, I, P, P, P, P],
     "hfa_head_plan": [I, I, I, P, P, P, P],
     "hfa_moe_gemm": [P, I, I, I, P, I, P, P, P, I, I, P, I, I, I, P, I, I, I, I, I, F, F, F, P],
     "hfa_moe_combine": [P, P, I, I, I, P],
-    "hfa_swiglu": [P, P, I, I, I, P],
+    "hfa_swiglu": [P, P, I, I, I, I, P],
     "hfa_scatter_i32": [P, P, P, I, P],
     "hfa_move_i32": [P, P, P, P, I, P],
     "hfa_argmax": [P, I, P, I, I, P, c_size_t, P],

@@ -102,6 +102,17 @@ class StreamUpdate:
     out: object
 
 
+@dataclass
+class BranchSum:
+    """A branch's result that has not been formed yet: ``out = extra * sigmoid(extra_gate) + sum over a row's pairs`` (experts and a
+    shared expert). The norm that takes it into the stream forms it on the way."""
+    out: torch.Tensor
+    pairs: torch.Tensor      # fp32 [rows * top, width], the weighted results of a row's choices one after the other
+    top: int
+    extra: object            # fp32 [rows, width] (or a product into it that is still pending), or None
+    extra_gate: object       # fp32 [rows, 1], or None
+
+
 class _NoSection:
     def __enter__(self):
         return self
@@ -156,6 +167,8 @@ class Ops:
         self._lazy = None                    # a LazyProduct
         self._lazy_rope = None               # a LazyRope
         self._stream_undone = None           # a StreamUpdate
+        self._branch = None                  # a BranchSum
+        self._rounded = {}                   # data_ptr of an fp32 tensor -> its copy in the activations' dtype
         self._head_plans = {}                # (rows, heads, tile) -> tiles of the heads' products, made once a pass
         self._rope_tables = {}               # (positions, frequencies, tokens) -> cosines and sines of a pass's angles
         self._scaled = {}                    # data_ptr of a norm's output -> Scaled
@@ -206,6 +219,7 @@ class Ops:
         self._scaled.clear()                 # what an earlier pass left in its work buffers is of no use to this one
         self._rope_tables.clear()
         self._head_plans.clear()
+        self._rounded.clear()
         try:
             yield self
         finally:
@@ -281,15 +295,28 @@ class Ops:
                                            None if positions is None else inv_freq.data_ptr(), out_x.data_ptr(), T, table.shape[1],
                                            table.shape[0], 1.0 if scale is None else float(scale), self._stream()))
 
-    def rmsnorm_add(self, y, weight, eps, out, gate=None, gate_bias=None, scale=1.0, accumulate=True):
+    def rmsnorm_add(self, y, weight, eps, out, gate=None, gate_bias=None, scale=1.0, accumulate=True, copy=False):
         """``out (+)= scale * rmsnorm(y * sigmoid(gate + gate_bias)) * weight``, all in fp32 (``gate`` None: ``y`` as it is;
-        ``accumulate`` False: ``out`` is overwritten): the norm of a branch's result on its way into the stream."""
+        ``accumulate`` False: ``out`` is overwritten; ``weight`` None: no norm): the norm of a branch's result on its way into the
+        stream. A product into ``y`` that is still pending, or a sum that ``branch_sum`` left undone, is taken along. ``copy``: the
+        same kernel leaves the new ``out`` in the activations' dtype for ``rounded(out)``."""
+        R, E = y.shape
+        br, p = self._branch, self._pending
+        if br is not None and br.out.data_ptr() == y.data_ptr() and br.out.shape == y.shape:
+            self._branch = None
+        else:
+            br = None
+        source = y if br is None else br.extra
+        partial, splits = None, 0
+        if p is not None and source is not None and p.out.data_ptr() == source.data_ptr() and p.out.shape == source.shape \
+                and not p.accumulate and p.bias is None:
+            self._pending = None
+            partial, splits = self.workspace.data_ptr(), p.splits
         self.settle()
         self._source_changes(out)
         self._scaled.pop(out.data_ptr(), None)
-        R, E = y.shape
-        if y.dtype != torch.float32 or out.dtype != torch.float32 or tuple(out.shape) != (R, E) or weight.dtype != torch.float32 \
-                or weight.numel() != E or not weight.is_contiguous():
+        if y.dtype != torch.float32 or out.dtype != torch.float32 or tuple(out.shape) != (R, E) or (weight is not None and (
+                weight.dtype != torch.float32 or weight.numel() != E or not weight.is_contiguous())):
             fail(EINVAL, "rmsnorm_add: y, out and weight must be fp32 and of one width")
         if gate is not None and (tuple(gate.shape) != (R, E) or (gate_bias is not None and (gate_bias.dtype != torch.float32
                                                                                             or gate_bias.numel() != E))):
@@ -298,10 +325,60 @@ class Ops:
             fail(EINVAL, "rmsnorm_add: a gate's bias without the gate")
         if gate is not None:
             self._whole(gate)
+        rounded = None
+        if copy and self.act_dtype != torch.float32:
+            rounded = self.scratch(f"rounded@{out.data_ptr()}", (R, E), self.act_dtype)
+            self._scaled.pop(rounded.data_ptr(), None)
+        row_gate = None if br is None else br.extra_gate
         self._check(self.lib.hfa_rmsnorm_add(
-            y.data_ptr(), _rows(y, "norm in"), None if gate is None else gate.data_ptr(), 0 if gate is None else _code(gate),
-            0 if gate is None else _rows(gate, "norm gate"), None if gate_bias is None else gate_bias.data_ptr(), weight.data_ptr(),
-            out.data_ptr(), _rows(out, "norm out"), R, E, float(eps), float(scale), 1 if accumulate else 0, self._stream()))
+            None if source is None or partial is not None else source.data_ptr(), 0 if source is None else _rows(source, "norm in"), partial,
+            splits, None if row_gate is None else row_gate.data_ptr(), 0 if row_gate is None else row_gate.stride(0),
+            None if br is None else br.pairs.data_ptr(), 0 if br is None else br.top, None if gate is None else gate.data_ptr(),
+            0 if gate is None else _code(gate), 0 if gate is None else _rows(gate, "norm gate"),
+            None if gate_bias is None else gate_bias.data_ptr(), None if weight is None else weight.data_ptr(), out.data_ptr(),
+            _rows(out, "norm out"), None if rounded is None else rounded.data_ptr(), E, R, E, float(eps), float(scale),
+            1 if accumulate else 0, self._stream()))
+        if rounded is not None:
+            self._rounded[out.data_ptr()] = rounded
+
+    def branch_sum(self, out, pairs, top, extra=None, extra_gate=None):
+        """``out[r] = sum_k pairs[r * top + k] + sigmoid(extra_gate[r]) * extra[r]`` in fp32, left undone until ``rmsnorm_add`` takes
+        ``out`` into the stream (or something else asks for it). A product into ``extra`` may still be pending."""
+        R, E = out.shape
+        if any(t.dtype != torch.float32 for t in (out, pairs)) or tuple(pairs.shape) != (R * top, E) or not pairs.is_contiguous() \
+                or (extra is not None and (extra.dtype != torch.float32 or tuple(extra.shape) != (R, E))) \
+                or (extra_gate is not None and (extra is None or extra_gate.dtype != torch.float32 or tuple(extra_gate.shape) != (R, 1))):
+            fail(EINVAL, "branch_sum: fp32 rows, their pairs' rows, and one fp32 gate a row")
+        if self._branch is not None:
+            self.settle(self._branch.out)
+        self._branch = BranchSum(out, pairs, int(top), extra, extra_gate)
+
+    def rounded(self, x):
+        """The fp32 matrix ``x`` in the activations' dtype (``x`` itself in the 32-bit engine): the copy that ``rmsnorm_add`` left beside
+        it, or one made now."""
+        if self.act_dtype == torch.float32:
+            self.settle(x)
+            return x
+        t = self._rounded.get(x.data_ptr())
+        if t is not None and t.shape == x.shape:
+            return t
+        self.settle()
+        t = self.scratch(f"rounded@{x.data_ptr()}", tuple(x.shape), self.act_dtype)
+        self._scaled.pop(t.data_ptr(), None)
+        self._check(self.lib.hfa_round_rows(x.data_ptr(), _rows(x, "rows"), t.data_ptr(), x.shape[1], x.shape[0], x.shape[1], self._stream()))
+        self._rounded[x.data_ptr()] = t
+        return t
+
+    def diff_mix(self, a, factor, c, eps, n_heads, n_kv_heads, v_head_dim, out):
+        """Two attention maps a head as one: ``a`` fp32 [T, groups, 2, heads of a group, v_head_dim]; ``d`` = map 1 - ``factor`` (one fp32
+        number on the device) map 2; ``out[t, h] = c d / sqrt(mean(d^2) + eps)`` over the head's values."""
+        self.settle()
+        self._scaled.pop(out.data_ptr(), None)
+        if a.dtype != torch.float32 or a.shape[1] != 2 * n_heads * v_head_dim or tuple(out.shape) != (a.shape[0], n_heads * v_head_dim) \
+                or factor.dtype != torch.float32 or factor.numel() != 1:
+            fail(EINVAL, "diff_mix: fp32 rows of two maps a head, one fp32 factor, rows of heads out")
+        self._check(self.lib.hfa_diff_mix(a.data_ptr(), _rows(a, "maps"), factor.data_ptr(), float(c), float(eps), out.data_ptr(), _code(out),
+                                          _rows(out, "heads"), a.shape[0], n_heads, n_kv_heads, v_head_dim, self._stream()))
 
     def polynorm(self, z, coef, eps, out):
         """``out = a N(z) + b N(z^2) + c N(z^3) + e`` row by row, ``N(u) = u / sqrt(mean(u^2) + eps)``, ``coef`` = (a, b, c, e)
@@ -322,15 +399,31 @@ class Ops:
         if x.shape[0]:
             self._check(self.lib.hfa_scale_rows(x.data_ptr(), _rows(x, "scale_rows"), x.shape[0], x.shape[1], float(s), self._stream()))
 
-    def head_norm_store(self, qkv, n_heads, n_kv_heads, head_dim, v_head_dim, q_weight, k_weight, eps, q_out, cache, slot_map):
+    def _rope_table(self, positions, inv_freq, T, rot_dim):
+        """Cosines and sines of this pass's tokens ([T, rot_dim]), made once for all its layers with these frequencies."""
+        key = (positions.data_ptr(), inv_freq.data_ptr(), T, rot_dim)
+        table = self._rope_tables.get(key)
+        if table is None:
+            table = self.scratch(f"rope_table@{inv_freq.data_ptr()}", (T, rot_dim), torch.float32)
+            self._check(self.lib.hfa_rope_table(_ints(positions, "positions", T), inv_freq.data_ptr(), rot_dim // 2,
+                                                table.data_ptr(), T, self._stream()))
+            if self._stream_handle is not None:              # inside a pass
+                self._rope_tables[key] = table
+        return table
+
+    def head_norm_store(self, qkv, n_heads, n_kv_heads, head_dim, v_head_dim, q_weight, k_weight, eps, q_out, cache, slot_map,
+                        n_v_heads=None, norm=None, after=False, positions=None, inv_freq=None, rot_dim=0):
         """Rows ``[q | k | v]`` (fp32 or bf16): every q head and every k head is RMS-normed over its ``head_dim`` values with a
-        weight of that size which all heads share (None: the part stays as it is); q goes to ``q_out`` ([T, heads * head_dim],
-        the cache's dtype), k and v to ``cache`` at the rows ``slot_map`` names (values transposed inside their page)."""
+        weight of that size which all heads share (None: the part stays as it is; with ``norm`` True it is normed without a
+        weight); q goes to ``q_out`` ([T, heads * head_dim], the cache's dtype), k and v to ``cache`` at the rows ``slot_map`` names
+        (values transposed inside their page). ``n_v_heads``: value heads, if not as many as key heads. With ``rot_dim`` the first
+        dimensions of each q and k head are turned (i with i + rot_dim/2) after the norm, or (``after``) before it."""
         self.settle()
         self._whole(qkv)
         self._scaled.pop(q_out.data_ptr(), None)
         T = qkv.shape[0]
-        QD, KD, VD = n_heads * head_dim, n_kv_heads * head_dim, n_kv_heads * v_head_dim
+        GV = n_kv_heads if n_v_heads is None else int(n_v_heads)
+        QD, KD, VD = n_heads * head_dim, n_kv_heads * head_dim, GV * v_head_dim
         for w, what in ((q_weight, "q"), (k_weight, "k")):
             if w is not None and (w.dtype != torch.float32 or w.numel() != head_dim or not w.is_contiguous()):
                 fail(EINVAL, f"head_norm_store: the {what} weight must be {head_dim} contiguous fp32 values")
@@ -339,9 +432,12 @@ class Ops:
         for c, width in ((cache.k, KD), (cache.v, VD)):
             if c.dim() != 2 or c.shape[1] != width or not c.is_contiguous():
                 fail(EINVAL, f"head_norm_store: the cache must have one row of {width} values per token")
+        table = self._rope_table(positions, inv_freq, T, rot_dim) if rot_dim else None
         self._check(self.lib.hfa_head_norm_store(
-            qkv.data_ptr(), _code(qkv), _rows(qkv, "qkv"), n_heads, n_kv_heads, head_dim, v_head_dim,
-            None if q_weight is None else q_weight.data_ptr(), None if k_weight is None else k_weight.data_ptr(), float(eps),
+            qkv.data_ptr(), _code(qkv), _rows(qkv, "qkv"), n_heads, n_kv_heads, head_dim, GV, v_head_dim,
+            None if q_weight is None else q_weight.data_ptr(), None if k_weight is None else k_weight.data_ptr(),
+            1 if norm or q_weight is not None else 0, 1 if norm or k_weight is not None else 0, 1 if after else 0, float(eps),
+            None if table is None else table.data_ptr(), int(rot_dim),
             q_out.data_ptr(), _rows(q_out, "queries"), cache.k.data_ptr(), cache.v.data_ptr(), _code(cache.k),
             _ints(slot_map, "slot_map", T), cache.page_tokens, T, self._stream()))
 
@@ -412,7 +508,9 @@ class Ops:
         self._lazy = None
         self._lazy_rope = None
         self._stream_undone = None
+        self._branch = None
         self._scaled.clear()
+        self._rounded.clear()
 
     # ---- products of few rows that finish their outputs themselves (csrc/gemm_rows.hip) -----------------------
     def _rows_mode(self, a, w, out, bias, accumulate, swiglu):
@@ -479,6 +577,7 @@ class Ops:
         """``x`` is about to change: norm outputs that were left undivided can no longer be made whole from it
         (products can still read them: x * weight and the sums of squares stay). ``keep``: one that is about to be
         overwritten is dropped."""
+        self._rounded.pop(x.data_ptr(), None)
         for key, sc in list(self._scaled.items()):
             if sc.x.data_ptr() == x.data_ptr():
                 if keep is not None and key == keep.data_ptr():
@@ -504,6 +603,9 @@ class Ops:
         if su is not None and (tensor is None or su.x.data_ptr() == tensor.data_ptr()):
             self._stream_undone = None
             self._stream_step(su, su.x)
+        br = self._branch
+        if br is not None and (tensor is None or br.out.data_ptr() == tensor.data_ptr()):
+            self.rmsnorm_add(br.out, None, 0.0, br.out, accumulate=False)      # forms the sum where it belongs
         p = self._pending
         if p is None or (tensor is not None and p.out.data_ptr() != tensor.data_ptr()):
             return
@@ -514,11 +616,11 @@ class Ops:
                                              _code(p.out), _rows(p.out, "gemm out"), 1 if p.accumulate else 0, 0,
                                              M, N, self._stream()))
 
-    def gemm(self, a, w, out, bias=None, accumulate=False, defer=False, swiglu=False, activation=None):
+    def gemm(self, a, w, out, bias=None, accumulate=False, defer=False, swiglu=False, activation=None, gate_act="silu"):
         """out (+)= a @ w.T + bias, fp32 accumulation. ``defer``: if the kernel split K, leave the
         partial sums for the next kernel that reads ``out`` (see the module's text).
         ``swiglu``: w's rows come in blocks of 32 gate, 32 up (``interleave_gate_up``) and
-        out = silu(gate) * up has half as many columns. ``activation``: ``out = act(a @ w.T + bias)`` (see ``activation``)."""
+        out = silu(gate) * up has half as many columns (``gate_act`` ``gelu_tanh``: that in silu's place). ``activation``: ``out = act(a @ w.T + bias)`` (see ``activation``)."""
         act = 0
         if activation is not None:
             if accumulate or swiglu or defer:
@@ -526,6 +628,8 @@ class Ops:
             if activation not in self.ACTIVATIONS:
                 fail(ENOTSUP, f"activation '{activation}' is not one of {', '.join(sorted(self.ACTIVATIONS))}")
             act = self.ACTIVATIONS[activation]           # the product's last lines apply it
+        if gate_act not in ("silu", "gelu_tanh"):
+            fail(ENOTSUP, f"gemm: a gate passes silu or gelu_tanh, not '{gate_act}'")
         self.settle()
         lda, ldw, ldo = _rows(a, "gemm a"), _rows(w, "gemm w"), _rows(out, "gemm out")
         M, K = a.shape
@@ -548,7 +652,8 @@ class Ops:
                     self._source_changes(out)
                     self._rows_resid(z)
             elif mode == 2:
-                self._rows_call(2, a, w, N // 2, None, scaled=scaled, act=out)
+                self._rows_call(2, a, w, N // 2, None, scaled=scaled, act=out,
+                                out_act=self.ACTIVATIONS["gelu_tanh"] if gate_act == "gelu_tanh" else 0)
             elif defer and out.dtype == torch.bfloat16 and M * N * 4 <= self.workspace.numel():
                 # 32-bit sums for the kernel that follows (the rotation of queries and keys): one plane of the workspace
                 plane = self.workspace[:M * N * 4].view(torch.float32).view(M, N)
@@ -565,7 +670,7 @@ class Ops:
         self._splits_out.value = 0
         self._check(self.lib.hfa_gemm(a.data_ptr(), _code(a), lda, w.data_ptr(), _code(w), ldw,
                                       None if bias is None else bias.data_ptr(), out.data_ptr(), _code(out), ldo,
-                                      1 if accumulate else 0, 1 + act if act else 1 if swiglu else 0, M, N, K, self.workspace.data_ptr(),
+                                      1 if accumulate else 0, 1 + act if act else 0 if not swiglu else 1 if gate_act == "silu" else self.GEGLU, M, N, K, self.workspace.data_ptr(),
                                       self.workspace.numel(), 1 if defer else 0, ctypes.byref(self._splits_out),
                                       1 if self.force_plain_gemm else 0, self._stream()))
         if self._splits_out.value:
@@ -643,7 +748,7 @@ class Ops:
 
     def paged_attention(self, q, n_heads, n_kv_heads, head_dim, cache, step, window, scale, out, slopes=None,
                         v_head_dim=None, mask_chunk=0, sink=False, cross_values=False, softcap=0.0, weights="softmax", head_bias=None,
-                        sink_scores=None, distance=None):
+                        sink_scores=None, distance=None, v_share=1, keep_first=0, rel=None, gate=None, out_scale=1.0):
         """Attention of the first ``n_heads * head_dim`` columns of ``q`` over ``cache``. ``slopes``
         (fp32, one per query head): the score of key j for the query at p gets ``slopes[h] * (j - p)``
         added, for position encodings that enter the scores; the plain kernel then runs, as it does when
@@ -656,7 +761,11 @@ class Ops:
         ``weights`` ``"sigmoid"``: no softmax; a visible key weighs ``sigmoid(score + head_bias[h])`` (``head_bias``: fp32, one per
         query head, or None), and the weights are not normalised over the keys. ``sink_scores`` (fp32, one per query head; with
         ``sink``): the extra term's score is the head's number instead of 0. ``distance`` = (a, b) (fp32, one per query head each;
-        softmax only): after scale and cap the score of key j for the query at p is lowered by ``a[h] ln(1 + b[h] (p - j))``."""
+        softmax only): after scale and cap the score of key j for the query at p is lowered by ``a[h] ln(1 + b[h] (p - j))``.
+        ``v_share``: that many neighbouring key heads read one value head. ``keep_first``: under a window the first ``keep_first`` keys of
+        a sequence stay visible. ``rel`` (fp32 [heads, n]; softmax only): ``rel[h, min(p - j, n - 1)]`` is added to the score. ``gate``
+        ([T, heads]): head h's result is multiplied by ``sigmoid(gate[t, h])``; ``out_scale`` multiplies all results. ``out`` may be
+        fp32 beside bf16 queries."""
         v_head_dim = head_dim if v_head_dim is None else int(v_head_dim)
         mask_chunk = int(mask_chunk)
         if weights not in ("softmax", "sigmoid") or (weights == "sigmoid" and (sink or cross_values)):
@@ -668,13 +777,23 @@ class Ops:
         for t, what in ((sink_scores, "sink_scores"),) + tuple((t, "distance") for t in (distance or ())):
             if t is not None and (t.dtype != torch.float32 or t.numel() != n_heads or not t.is_contiguous() or t.device != q.device):
                 fail(EINVAL, f"paged_attention: {what} is contiguous fp32 on the device, one number per query head")
+        if rel is not None and (rel.dtype != torch.float32 or rel.dim() != 2 or rel.shape[0] != n_heads or not rel.is_contiguous()
+                                or weights != "softmax" or slopes is not None):
+            fail(EINVAL, "paged_attention: a table of distance terms is contiguous fp32 [heads, distances] and goes with a softmax")
+        if gate is not None:
+            self._whole(gate)
+            if tuple(gate.shape) != (q.shape[0], n_heads):
+                fail(EINVAL, "paged_attention: the gate is one number a token and query head")
+        if n_kv_heads % int(v_share):
+            fail(EINVAL, f"paged_attention: {n_kv_heads} key heads do not share value heads by {v_share}")
+        extras = v_share != 1 or keep_first or rel is not None or gate is not None or out_scale != 1.0 or out.dtype != q.dtype
         if (sink_scores is not None and not sink) or (distance is not None and (weights != "softmax" or slopes is not None or cross_values)):
             fail(EINVAL, "paged_attention: sink_scores go with a sink term, a distance term with a softmax over a head's own values")
         dist_a, dist_b = (None, None) if distance is None else (distance[0].data_ptr(), distance[1].data_ptr())
         self._scaled.pop(out.data_ptr(), None)               # whatever `out` held, it is no norm's lazy output any more
         lr = self._lazy_rope
         if lr is not None and lr.qkv.data_ptr() == q.data_ptr() and lr.cache is cache and slopes is None and not sink \
-                and not cross_values and weights == "softmax" \
+                and not cross_values and weights == "softmax" and not extras \
                 and step.max_q_len == 1 and step.n_seqs == q.shape[0] and not self.force_plain_attention \
                 and out.dtype == torch.bfloat16 and v_head_dim == head_dim and lr.args[4] == n_heads and lr.args[6] == head_dim \
                 and lr.args[5] in (0, n_kv_heads) and cache.k.shape[1] == n_kv_heads * head_dim \
@@ -687,9 +806,9 @@ class Ops:
         T = q.shape[0]
         ldq, ldo = _rows(q, "attention q"), _rows(out, "attention out")
         g = step.group(cache.group)
-        if cache.k.dtype != q.dtype or out.dtype != q.dtype:
-            fail(EINVAL, "paged_attention: queries, cache and output must share a dtype")
-        if cache.k.shape[1] != n_kv_heads * head_dim or cache.v.shape[1] != n_kv_heads * v_head_dim:
+        if cache.k.dtype != q.dtype or out.dtype not in (q.dtype, torch.float32):
+            fail(EINVAL, "paged_attention: queries, cache and output must share a dtype (or the output is fp32)")
+        if cache.k.shape[1] != n_kv_heads * head_dim or cache.v.shape[1] != n_kv_heads // v_share * v_head_dim:
             fail(EINVAL, "paged_attention: the cache rows do not hold n_kv_heads * head_dim keys and n_kv_heads * v_head_dim values")
         _ints(step.token_slot, "token_slot", T)
         _ints(step.positions, "positions", T)
@@ -714,7 +833,10 @@ class Ops:
                 n_kv_heads, head_dim, v_head_dim, cache.page_tokens, int(window), mask_chunk, float(scale),
                 None if slopes is None else slopes.data_ptr(), 1 if sink else 0, 1 if cross_values else 0, softcap,
                 1 if weights == "sigmoid" else 0, None if head_bias is None else head_bias.data_ptr(),
-                None if sink_scores is None else sink_scores.data_ptr(), dist_a, dist_b, self.attn_workspace.data_ptr(),
+                None if sink_scores is None else sink_scores.data_ptr(), dist_a, dist_b, int(v_share), int(keep_first),
+                None if rel is None else rel.data_ptr(), 0 if rel is None else rel.shape[1],
+                None if gate is None else gate.data_ptr() + first * _rows(gate, "gate") * gate.element_size(), 0 if gate is None else _code(gate),
+                0 if gate is None else _rows(gate, "gate"), float(out_scale), _code(out), self.attn_workspace.data_ptr(),
                 self.attn_workspace.numel(), 1 if plain else 0, self._stream()))
 
         # Decoded tokens beside prompt portions: one call would send all of them to the kernel for prompt
@@ -722,7 +844,7 @@ class Ops:
         # take as long as thousands of prompt tokens). The step lays requests with few tokens first, so
         # each part is a step of its own: the first goes to the kernel that cuts the keys into chunks.
         n_short = getattr(step, "n_short_seqs", 0)
-        if not plain and v_head_dim == head_dim and q.dtype == torch.bfloat16 \
+        if not plain and (v_head_dim == head_dim or extras) and q.dtype == torch.bfloat16 \
                 and step.max_q_len >= self.prompt_rows and 0 < n_short < step.n_seqs:
             ts = step.n_short_tokens
             _ints(step.q_start_long, "q_start_long", step.n_seqs - n_short + 1)
@@ -739,13 +861,7 @@ class Ops:
         T = qkv.shape[0]
         table = None
         if rot_dim:
-            key = (positions.data_ptr(), inv_freq.data_ptr(), T, rot_dim)
-            table = self._rope_tables.get(key)
-            if table is None:                # the angles of this pass's tokens, once for all its layers
-                table = self.scratch(f"rope_table@{inv_freq.data_ptr()}", (T, rot_dim), torch.float32)
-                self._check(self.lib.hfa_rope_table(_ints(positions, "positions", T), inv_freq.data_ptr(), rot_dim // 2,
-                                                    table.data_ptr(), T, self._stream()))
-                self._rope_tables[key] = table
+            table = self._rope_table(positions, inv_freq, T, rot_dim)
         g = step.group(cache.group)
         self._lazy_rope = None
         self._pending = None                 # the 32-bit plane of q, k and v is read here
@@ -758,14 +874,17 @@ class Ops:
             self.attn_workspace.data_ptr(),
             self.attn_workspace.numel(), self._stream()))
 
-    def swiglu(self, gate_up, out):
+    GEGLU = 17                   # HFA_EPILOGUE_GEGLU
+
+    def swiglu(self, gate_up, out, gate_act="silu"):
+        """``out = act(gate) * up`` from rows ``[gate | up]``; ``gate_act`` is ``silu`` or ``gelu_tanh``."""
         self.settle()
         self._scaled.pop(out.data_ptr(), None)
         T, F2 = gate_up.shape
         if not gate_up.is_contiguous() or not out.is_contiguous() or tuple(out.shape) != (T, F2 // 2) \
                 or out.dtype != gate_up.dtype or F2 % 2:
             fail(EINVAL, "swiglu: expected contiguous [T, 2F] in and [T, F] out of one dtype")
-        self._check(self.lib.hfa_swiglu(gate_up.data_ptr(), out.data_ptr(), _code(out), T, F2 // 2, self._stream()))
+        self._check(self.lib.hfa_swiglu(gate_up.data_ptr(), out.data_ptr(), _code(out), T, F2 // 2, self.ACTIVATIONS[gate_act], self._stream()))
 
     # ---- norms in groups, queries and keys normed whole, mixers with per-request state -------------------------------
     GATES = {None: 0, "silu_before": 1, "sigmoid_after": 2, "silu_after": 3}
@@ -1229,22 +1348,24 @@ class Ops:
     # ---- mixture of experts ------------------------------------------------------------------------------------------
     SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_chosen": 2}
 
-    def moe_route(self, logits, top, n_groups, keep, scoring="softmax", renorm=True, out_scale=1.0):
+    def moe_route(self, logits, top, n_groups, keep, scoring="softmax", renorm=True, out_scale=1.0, correction=None):
         """(ids [T, top] int32, weights [T, top] fp32) from fp32 router logits [T, E]: see ``hfa_moe_route``. ``scoring``
         ``softmax_chosen``: the experts with the largest logits, weighted (with ``renorm``) by the softmax over the chosen
-        logits alone."""
+        logits alone. ``correction`` (fp32, one per expert) is added to the scores for the choice, not for the weights."""
         self.settle()
         T, E = logits.shape
+        if correction is not None and (correction.dtype != torch.float32 or correction.numel() != E or not correction.is_contiguous()):
+            fail(EINVAL, "moe_route: the correction is one fp32 number an expert")
         if logits.dtype != torch.float32 or scoring not in self.SCORINGS:
             fail(EINVAL, f"moe_route: fp32 logits and a scoring among {', '.join(self.SCORINGS)}")
         ids = self.scratch("moe_ids", (T, top), torch.int32)
         wts = self.scratch("moe_weights", (T, top), torch.float32)
         self._check(self.lib.hfa_moe_route(logits.data_ptr(), _rows(logits, "router logits"), T, E, int(top), int(n_groups), int(keep),
                                            self.SCORINGS[scoring], 1 if renorm else 0, float(out_scale),
-                                           ids.data_ptr(), wts.data_ptr(), self._stream()))
+                                           None if correction is None else correction.data_ptr(), ids.data_ptr(), wts.data_ptr(), self._stream()))
         return ids, wts
 
-    def moe_experts(self, h, ids, weights, w_up, w_down, act, x, gated=None, weight_on="input"):
+    def moe_experts(self, h, ids, weights, w_up, w_down, act, x, gated=None, weight_on="input", combine=True):
         """``x[t] += sum_k weights[t, k] * w_down[ids[t, k]] act(w_up[ids[t, k]] h[t])``: ``w_up`` is [E, F, width],
         ``w_down`` [E, width, F]. The pairs are put in expert order on the device, each expert's rows go through the
         two products in tiles, and the weighted results are added to ``x`` (fp32) choice by choice.
@@ -1256,10 +1377,12 @@ class Ops:
         unweighted; ``act`` is ignored. Interleaved, the up product's last lines form the activation from its 32-bit sums;
         otherwise the sums pass through memory and a kernel of its own forms it. ``weight_on`` ``"output"`` (gated experts only;
         experts without a gate always weigh their output): c = 1 inside the expert, and the down product's rows are multiplied
-        by the pair's weight instead."""
+        by the pair's weight instead. ``combine`` False: nothing is added to ``x``; the pairs' weighted results ([T * top, width]
+        fp32, a token's choices one after the other) are returned for ``branch_sum``."""
         self.settle()
         self._whole(h)
-        self._source_changes(x)
+        if combine:
+            self._source_changes(x)
         T, W = h.shape
         E, F, _ = w_up.shape
         if gated is not None:
@@ -1308,10 +1431,12 @@ class Ops:
                                               n_tiles.data_ptr(), max_tiles, tile_rows, y.data_ptr(), W, F32, 1,
                                               None if w_out is None else w_out.data_ptr(), 0, W, F,
                                               plain, 0, 0.0, 0.0, 0.0, self._stream()))
+        else:
+            self._plain_experts(h, code, top, w_up, w_down, wcode, row_pair, tiles, n_tiles, max_tiles, tile_rows, mid, y, weights, act, F, W,
+                                plain)
+        if combine:
             self._check(self.lib.hfa_moe_combine(y.data_ptr(), x.data_ptr(), T, top, W, self._stream()))
-            return
-        self._plain_experts(h, code, top, w_up, w_down, wcode, row_pair, tiles, n_tiles, max_tiles, tile_rows, mid, y, weights, act, F, W,
-                            plain, x, T)
+        return y
 
     def _gated_in_two(self, h, code, top, w_up, wcode, row_pair, tiles, n_tiles, max_tiles, tile_rows, mid, weights, n_pairs, F, F_up, W,
                       plain, alpha, limit, shift, interleaved):
@@ -1326,7 +1451,7 @@ class Ops:
                                                self._stream()))
 
     def _plain_experts(self, h, code, top, w_up, w_down, wcode, row_pair, tiles, n_tiles, max_tiles, tile_rows, mid, y, weights, act, F, W,
-                       plain, x, T):
+                       plain):
         """Experts without a gate: the activation in the up product's last lines, the weights in the down product's."""
         self._check(self.lib.hfa_moe_gemm(h.data_ptr(), _rows(h, "moe h"), code, top, w_up.data_ptr(), wcode, row_pair.data_ptr(),
                                           tiles.data_ptr(), n_tiles.data_ptr(), max_tiles, tile_rows, mid.data_ptr(), F, code, 0, None,
@@ -1334,7 +1459,6 @@ class Ops:
         self._check(self.lib.hfa_moe_gemm(mid.data_ptr(), F, code, 0, w_down.data_ptr(), wcode, row_pair.data_ptr(), tiles.data_ptr(),
                                           n_tiles.data_ptr(), max_tiles, tile_rows, y.data_ptr(), W, F32, 1, weights.data_ptr(), 0, W, F,
                                           plain, 0, 0.0, 0.0, 0.0, self._stream()))
-        self._check(self.lib.hfa_moe_combine(y.data_ptr(), x.data_ptr(), T, top, W, self._stream()))
 
     @staticmethod
     def interleave_experts(w_gate, w_up):

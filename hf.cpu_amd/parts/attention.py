@@ -46,8 +46,8 @@ class Attention(Part):
     are mixed after the softmax, ``weight_h <- sum_g talk[h, g] weight_g`` (tensor ``talk`` [heads, heads]), and head h applies
     its mixed weights to the values of its own group. ``out_gate``: the concatenated heads are multiplied by
     ``sigmoid(Wg h)`` (tensor ``g``) before the output projection. Any of the first three takes the mixer through a path of its
-    own (``_forward_shaped``), which knows no rotation, no ``own_kv=False`` and none of ``qk_norm``, ``sink``, ``v_mix``; an output
-    gate alone goes with every other option (its rows ride in the q/k/v product).
+    own (``_forward_shaped``), which knows no ``own_kv=False``, no ``qk_norm`` and no ``v_mix``, and with a convolution or mixed heads
+    neither rotation nor sinks; an output gate alone goes with every other option (its rows ride in the q/k/v product).
     ``forward(..., accumulate=False)`` writes ``x = ...`` instead of adding.
 
     ``softcap`` c > 0: a score becomes ``c tanh(score / c)`` after the scale. ``weights="sigmoid"``: no softmax; a visible key
@@ -55,6 +55,16 @@ class Attention(Part):
     not normalised over the keys. ``sink="learned"``: the extra term's score is one number a head (the tensor ``sink``) instead of
     0. ``distance``: after scale and cap a score is lowered by ``a_h ln(1 + b_h (i - j))`` with two numbers a head (the tensors
     ``dist_scale`` and ``dist_rate``).
+
+    Options that take the same path of their own as ``head_norm`` and go with each other, with a rotation, biases, windows, chunks,
+    caps and sinks: ``head_norm_weight=False``: the per-head norm has no weight. ``norm_after``: it comes after the rotation, not before.
+    ``out_gate="head"``: one gate a head (tensor ``g`` [heads, width]) multiplies the head's whole output. ``rel_bias`` = dict(rows=B,
+    reach=R): after scale and cap a number of the tensor ``rel`` ([B, heads]) is added to the score, its row chosen by the distance
+    (``distance_bucket``); rows 0: as many as the tensor has. ``keep_first`` n: under a window the first n keys of a sequence stay visible (their rows are kept in the
+    cache for good). ``maps=2`` with ``diff`` d: differential attention: a query head and a key head are two of ``head_dim`` values
+    ([map 1, map 2]) over the same values; with ``f = exp(lq1 . lk1) - exp(lq2 . lk2) + d`` (tensors ``lq1`` .. ``lk2``, [head_dim]) the
+    head's output is ``a = map 1 - f map 2``, divided by its root mean square (``head_norm``'s eps) and multiplied by ``1 - d``.
+    ``joins_heads`` (an attribute): ``heads(...)`` gives what the output projection reads, times ``out_scale``.
     """
     graph_safe = True
     lazy_input_ok = True
@@ -64,7 +74,8 @@ class Attention(Part):
     def __init__(self, hidden_size, n_heads, n_kv_heads, head_dim, qkv_bias, window, position,
                  scale=None, out_bias=False, v_head_dim=None, prefix="", mask_chunk=0, own_kv=True, names=None,
                  qk_norm=None, sink=False, v_mix=None, conv_taps=0, head_norm=None, talk=False, out_gate=False,
-                 softcap=None, weights="softmax", distance=False):
+                 softcap=None, weights="softmax", distance=False, head_norm_weight=True, norm_after=False, rel_bias=None,
+                 keep_first=0, maps=1, diff=0.0):
         """``v_head_dim``: the size of a value head where it is not ``head_dim`` (key rows of the cache are
         then ``n_kv_heads * head_dim`` wide, value rows ``n_kv_heads * v_head_dim``, and the output
         projection reads ``n_heads * v_head_dim`` columns; such a mixer runs the plain kernels)."""
@@ -73,7 +84,9 @@ class Attention(Part):
             fail(EINVAL, f"attention: {n_heads} heads are not a multiple of {n_kv_heads} key/value heads")
         self.E, self.H, self.G, self.D = hidden_size, n_heads, n_kv_heads, head_dim
         self.Dv = head_dim if v_head_dim is None else int(v_head_dim)
-        self.QD, self.KD = n_heads * head_dim, n_kv_heads * head_dim
+        self.maps, self.diff = int(maps), float(diff)
+        self.HQ, self.GK = n_heads * self.maps, n_kv_heads * self.maps       # query and key heads as attention counts them
+        self.QD, self.KD = self.HQ * head_dim, self.GK * head_dim
         self.VD, self.OD = n_kv_heads * self.Dv, n_heads * self.Dv
         self.qkv_bias = bool(qkv_bias)
         self.out_bias = bool(out_bias)
@@ -84,12 +97,24 @@ class Attention(Part):
         self.names.update({f"{n}_bias": f"{n}_proj.bias" for n in "qkvo"})
         self.names.update(q_norm="q_norm.weight", k_norm="k_norm.weight", v_mix="v_mix", talk="talk", g="g_proj.weight",
                           q_conv="q_conv.weight", k_conv="k_conv.weight", v_conv="v_conv.weight", head_bias="head_bias",
-                          sink="sink", dist_scale="dist_scale", dist_rate="dist_rate")
+                          sink="sink", dist_scale="dist_scale", dist_rate="dist_rate", rel="rel", lq1="lq1", lk1="lk1", lq2="lq2", lk2="lk2")
         self.names.update(names or {})
         self.conv_taps = int(conv_taps)
         self.head_norm = None if head_norm is None else float(head_norm)
-        self.talk, self.out_gate = bool(talk), bool(out_gate)
-        self.shaped = self.conv_taps >= 1 or self.head_norm is not None or self.talk
+        self.head_norm_weight, self.norm_after = bool(head_norm_weight), bool(norm_after)
+        self.talk, self.out_gate, self.head_gate = bool(talk), bool(out_gate), out_gate == "head"
+        self.gate_rows = 0 if not out_gate else n_heads if self.head_gate else self.OD
+        self.rel_bias = None if rel_bias is None else (int(rel_bias["rows"]), float(rel_bias["reach"]))
+        self.keep_first = int(keep_first)
+        # what needs the path with per-head norms but neither a convolution nor mixed heads
+        self.masked = self.head_gate or self.rel_bias is not None or self.keep_first > 0 or self.maps > 1 or self.norm_after \
+            or (head_norm is not None and not (self.conv_taps >= 1 or self.talk) and (position.kind != "none" or qkv_bias or window or mask_chunk
+                                                                                   or sink or softcap or distance))
+        self.shaped = self.conv_taps >= 1 or self.head_norm is not None or self.talk or self.masked
+        self.rel_table = self.map_factor = None
+        self.out_scale = 1.0
+        if self.maps not in (1, 2) or (self.maps == 2 and self.head_norm is None) or self.keep_first < 0:
+            fail(EINVAL, f"attention: {self.maps} maps (two need head_norm's eps), {self.keep_first} kept keys")
         self.softcap = float(softcap or 0.0)
         if weights not in ("softmax", "sigmoid") or self.softcap < 0.0 or (weights == "sigmoid" and sink):
             fail(EINVAL, f"attention: weights '{weights}' (softmax, or sigmoid without a sink term) and a soft cap of {softcap}")
@@ -101,10 +126,12 @@ class Attention(Part):
         self.dist_w = self.sink_w = None
         if self.out_gate and not own_kv:
             fail(EINVAL, "attention: an output gate goes with a mixer that has projections of its own")
-        if self.shaped and (position.kind != "none" or not own_kv or qk_norm is not None or sink or v_mix or qkv_bias or window
-                            or mask_chunk or self.softcap or weights != "softmax" or distance):
-            fail(EINVAL, "attention: a convolution, per-head norms, mixed heads and an output gate go without rotation, biases, "
-                         "windows and the other options")
+        if self.shaped and (not own_kv or qk_norm is not None or v_mix or weights != "softmax" or (self.out_gate and self.masked and not self.head_gate)):
+            fail(EINVAL, "attention: per-head norms and what goes with them need projections of the mixer's own and a softmax, and know "
+                         "gates of whole heads")
+        if (self.conv_taps >= 1 or self.talk) and (position.kind != "none" or sink or qkv_bias or window or mask_chunk or self.softcap or distance
+                                                   or self.masked):
+            fail(EINVAL, "attention: a convolution and mixed heads go without rotation, biases, windows and the other options")
         if not 0 <= self.conv_taps <= 8:
             fail(EINVAL, f"attention: a convolution over {self.conv_taps} tokens (at most 8)")
         self.taps = self.talk_w = self.no_state = None
@@ -118,10 +145,22 @@ class Attention(Part):
             fail(EINVAL, "attention: a window and a masking chunk are counted in tokens, 0 for none")
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(head_dim)   # src/model.c:507
         self.position = make_part("position", position)
+        if self.masked and (getattr(self.position, "pairing", "split_half") != "split_half" or self.position.kind not in ("none", "rotary")):
+            fail(EINVAL, "attention: per-head norms go with a rotation of split halves, or none")
+        self.joins_heads = self.shaped and self.conv_taps == 0 and not self.talk and not (self.out_gate and not self.head_gate) and not out_bias
         self.w_qkv = self.b_qkv = self.w_o = self.b_o = None
 
     def sub_parts(self):
         return [self.position]
+
+    @staticmethod
+    def distance_bucket(n, rows, reach):
+        """The row of a table of ``rows`` rows for a key n positions back: one row a distance in the lower half, logarithmic from there
+        to ``reach``, the last row beyond."""
+        half = rows // 2
+        if n < half:
+            return n
+        return min(rows - 1, half + math.floor(math.log(n / half) / math.log(reach / half) * (rows - half)))
 
     def param_specs(self):
         p, nm = self.prefix, self.names
@@ -140,12 +179,16 @@ class Attention(Part):
             specs.append(ParamSpec(p + nm["v_mix"], (), "vector", ("normal", 0.3), optional=self.v_mix == "first"))
         if self.conv_taps >= 1:
             specs += [ParamSpec(p + nm[n + "_conv"], (widths[n], self.conv_taps), "vector", ("normal", 0.3)) for n in "qkv"]
-        if self.head_norm is not None:
+        if self.head_norm is not None and self.head_norm_weight:
             specs += [ParamSpec(p + nm[n], (self.D,), "vector", ("one_plus_normal", 0.1)) for n in ("q_norm", "k_norm")]
         if self.talk:
             specs.append(ParamSpec(p + nm["talk"], (self.H, self.H), "vector", ("normal", 0.3)))
         if self.out_gate:
-            specs.append(ParamSpec(p + nm["g"], (self.OD, self.E)))
+            specs.append(ParamSpec(p + nm["g"], (self.gate_rows, self.E)))
+        if self.rel_bias is not None:
+            specs.append(ParamSpec(p + nm["rel"], (self.rel_bias[0], self.H), "vector", ("normal", 0.5)))
+        if self.maps == 2:
+            specs += [ParamSpec(p + nm[n], (self.D,), "vector", ("normal", 0.1)) for n in ("lq1", "lk1", "lq2", "lk2")]
         if self.weights == "sigmoid":
             specs.append(ParamSpec(p + nm["head_bias"], (self.H,), "vector", ("normal", 0.5)))
         if self.learned_sink:
@@ -161,27 +204,32 @@ class Attention(Part):
         if not self.own_kv:
             fail(EINVAL, f"attention '{self.prefix}' has no keys and values of its own: its schedule entry must read "
                          "another entry's cache")
-        kv = PagedKV(self.KD, self.VD, self.window, self.mask_chunk)
+        kv = PagedKV(self.KD, self.VD, self.window, self.mask_chunk, keep_first=self.keep_first)
         if self.conv_taps > 1:
             return {"kv": kv, "conv": FixedState((self.conv_taps - 1) * (self.QD + self.KD + self.VD))}
         return kv
 
     def reads_cache(self, need):
         """``need`` of the mixer whose storage this one reads, widened by what this one sees of it."""
-        return PagedKV(need.k_width, need.v_width, need.window, need.mask_chunk, need.readers + ((self.window, self.mask_chunk),))
+        return PagedKV(need.k_width, need.v_width, need.window, need.mask_chunk, need.readers + ((self.window, self.mask_chunk),),
+                       max(need.keep_first, self.keep_first))
 
     def bind(self, params, ops):
         p, nm = self.prefix, self.names
         # One matrix for the three projections that share an input: rows of q, then k, then v.
         mats = [params[p + nm[n]] for n in self._projections()]
+        if self.maps == 2:
+            mats[0] = self._maps_apart(mats[0])
         if self.out_gate:
             mats.append(params[p + nm["g"]])             # the gate reads the same input: one product for all four
         dt = torch.float32 if any(m.dtype == torch.float32 for m in mats) else mats[0].dtype
         self.w_qkv = memory.cat([m.to(dt) for m in mats], 0, f"{p}q, k and v in one matrix")
         if self.qkv_bias:
             biases = [params[p + nm[n + "_bias"]] for n in self._projections()]
+            if self.maps == 2:
+                biases[0] = self._maps_apart(biases[0])
             if self.out_gate:                            # the gate's rows have none
-                biases.append(torch.zeros(self.OD, dtype=biases[0].dtype, device=biases[0].device))
+                biases.append(torch.zeros(self.gate_rows, dtype=biases[0].dtype, device=biases[0].device))
             self.b_qkv = memory.cat(biases, 0, f"{p}q, k and v biases in one vector")
         if self.weights == "sigmoid":
             self.head_bias = params[p + nm["head_bias"]].contiguous()
@@ -201,16 +249,69 @@ class Attention(Part):
         if self.conv_taps >= 1:
             self.no_state = memory.zeros((1, 1), torch.float32, ops.device, f"{p}a convolution's state that is never read")
             self.taps = memory.cat([params[p + nm[n + "_conv"]] for n in "qkv"], 0, f"{p}taps of q, k and v in one matrix").contiguous()
-        if self.head_norm is not None:
+        if self.rel_bias is not None:
+            # the table by distance: up to the one from which the last row holds, or the farthest that the mask shows
+            rows, reach = int(params[p + nm["rel"]].shape[0]), self.rel_bias[1]
+            if rows < 2 or not reach > rows // 2:
+                fail(EINVAL, f"attention '{p}': a table of {rows} distance terms that reaches {reach:g} positions back")
+            ids, seen = [], self.mask_chunk or self.window or 1 << 30
+            while len(ids) < seen and (not ids or ids[-1] < rows - 1):
+                ids.append(self.distance_bucket(len(ids), rows, reach))
+            table = params[p + nm["rel"]].index_select(0, torch.tensor(ids, dtype=torch.int64, device=params[p + nm["rel"]].device))
+            self.rel_table = memory.to_device(table.t().contiguous(), ops.device, f"{p}distance terms")
+        if self.maps == 2:
+            a, b, c, d = (params[p + nm[n]].double() for n in ("lq1", "lk1", "lq2", "lk2"))
+            self.map_factor = memory.to_device((torch.exp((a * b).sum()) - torch.exp((c * d).sum()) + self.diff).float().reshape(1),
+                                               ops.device, f"{p}factor of the second map")
+        if self.head_norm is not None and self.head_norm_weight:
             self.q_norm_w, self.k_norm_w = params[p + nm["q_norm"]].contiguous(), params[p + nm["k_norm"]].contiguous()
         if self.talk:
             self.talk_w = params[p + nm["talk"]].contiguous()
-        elif self.out_gate and self.shaped:              # the gate rides in the kernel that mixes heads: an identity mix
+        elif self.out_gate and self.shaped and not self.masked:              # the gate rides in the kernel that mixes heads: an identity mix
             self.talk_w = memory.to_device(torch.eye(self.H, dtype=torch.float32), ops.device, f"{p}identity mix of heads")
+
+    def _maps_apart(self, rows):
+        """Rows of queries head by head, [map 1, map 2] each, in the order attention counts its heads in: for every key head the
+        first map's queries of its group, then the second's."""
+        R = self.H // self.G
+        return rows.reshape(self.G, R, 2, self.D, -1).transpose(1, 2).reshape(rows.shape)
+
+    FEW_ROWS = 64                # rows up to which the projections leave 32-bit sums for the norms
+
+    def heads(self, ops, step, h, cache, out, write_cache=True):
+        """The concatenated heads before the output projection, times ``out_scale``, into ``out`` ([T, heads * v_head_dim], rows may lie
+        apart): projections, norms, rotation and store, attention."""
+        if not write_cache:
+            fail(EINVAL, f"attention '{self.prefix}': this mixer cannot read another entry's cache")
+        T = h.shape[0]
+        C = self.QD + self.KD + self.VD
+        proj = ops.scratch("qkv", (T, self.w_qkv.shape[0]), torch.float32 if self.masked and T <= self.FEW_ROWS else ops.act_dtype)
+        with ops.section("qkv"):
+            ops.gemm(h, self.w_qkv, proj, bias=self.b_qkv)
+        pos = self.position
+        with ops.section("qkv_prepare"):
+            q = ops.scratch("q_normed", (T, self.QD), ops.act_dtype)
+            ops.head_norm_store(proj[:, :C], self.HQ, self.GK, self.D, self.Dv, self.q_norm_w, self.k_norm_w, self.head_norm or 0.0, q, cache,
+                                step.group(cache.group).slot_map, n_v_heads=self.G, norm=self.head_norm is not None, after=self.norm_after,
+                                positions=step.positions, inv_freq=getattr(pos, "inv_freq", None), rot_dim=getattr(pos, "rot_dim", 0))
+        att = out if self.maps == 1 else ops.scratch("att_maps", (T, self.HQ * self.Dv), torch.float32)
+        with ops.section("attn"):
+            ops.paged_attention(q, self.HQ, self.GK, self.D, cache, step, self.window, self.scale, att, v_head_dim=self.Dv,
+                                mask_chunk=self.mask_chunk, sink=self.sink, softcap=self.softcap, sink_scores=self.sink_w,
+                                distance=self.dist_w, v_share=self.maps, keep_first=self.keep_first, rel=self.rel_table,
+                                gate=proj[:, C:] if self.head_gate else None, out_scale=self.out_scale if self.maps == 1 else 1.0)
+            if self.maps == 2:
+                ops.diff_mix(att, self.map_factor, (1.0 - self.diff) * self.out_scale, self.head_norm, self.H, self.G, self.Dv, out)
 
     def _forward_shaped(self, ops, step, h, cache, x, accumulate):
         """The path of a mixer with a convolution, per-head norms, mixed heads or an output gate (see the class)."""
         T = h.shape[0]
+        att = ops.scratch("att", (T, self.OD), ops.act_dtype)
+        if self.joins_heads:
+            self.heads(ops, step, h, cache, att)
+            with ops.section("wo"):
+                ops.gemm(att, self.w_o, x, accumulate=accumulate, defer=True)
+            return
         C = self.QD + self.KD + self.VD
         kv = cache["kv"] if isinstance(cache, dict) else cache
         proj = ops.scratch("qkv", (T, self.w_qkv.shape[0]), ops.act_dtype)
@@ -224,13 +325,11 @@ class Attention(Part):
             q = ops.scratch("q_normed", (T, self.QD), ops.act_dtype)
             ops.head_norm_store(rows, self.H, self.G, self.D, self.Dv, self.q_norm_w, self.k_norm_w, self.head_norm or 0.0, q, kv,
                                 step.group(kv.group).slot_map)
-        att = ops.scratch("att", (T, self.OD), ops.act_dtype)
         with ops.section("attn"):
-            if self.talk_w is None:
-                ops.paged_attention(q, self.H, self.G, self.D, kv, step, 0, self.scale, att, v_head_dim=self.Dv)
-            else:
-                cross = ops.scratch("att_cross", (T, self.G * self.OD), ops.act_dtype)
-                ops.paged_attention(q, self.H, self.G, self.D, kv, step, 0, self.scale, cross, v_head_dim=self.Dv, cross_values=True)
+            cross = ops.scratch("att_cross", (T, self.G * self.OD), ops.act_dtype)
+            ops.paged_attention(q, self.H, self.G, self.D, kv, step, 0, self.scale, cross if self.talk_w is not None else att,
+                                v_head_dim=self.Dv, cross_values=self.talk_w is not None)
+            if self.talk_w is not None:
                 ops.talk_mix(cross, self.talk_w, self.H, self.G, self.Dv, att, gate=proj[:, C:] if self.out_gate else None)
         with ops.section("wo"):
             ops.gemm(att, self.w_o, x, accumulate=accumulate, defer=True)

@@ -41,15 +41,17 @@ class PagedKV:
     last ``window`` tokens only; with ``mask_chunk > 0`` only from the start of the current run of
     ``mask_chunk`` positions (counted from 0). ``readers``: the (window, mask_chunk) of every other
     mixer that reads this storage (schedule entries with ``cache_of``): a row is kept while any of
-    them, or the owner, can still see it."""
+    them, or the owner, can still see it. ``keep_first``: the rows of the first ``keep_first`` positions are kept for good."""
     k_width: int
     v_width: int
     window: int = 0
     mask_chunk: int = 0
     readers: tuple = ()
+    keep_first: int = 0
 
     def first_kept(self, next_pos):
-        """The first position that a query at ``next_pos`` or later can see, for the owner or any reader."""
+        """The first position that a query at ``next_pos`` or later can see (beside the ``keep_first`` first ones), for the owner
+        or any reader."""
         def first(window, chunk):
             lo = max(0, next_pos - window + 1) if window > 0 else 0
             return max(lo, next_pos - next_pos % chunk) if chunk > 0 else lo

@@ -165,6 +165,42 @@ class SandwichBlock(Part):
         self._sublayer(ops, step, x, h, "feed_forward", ff, parts["norm2b"], run_ff)
 
 
+@register_part("block", "postnorm")
+class PostNormBlock(Part):
+    """Norms on the sublayers' results and nowhere else: ``x += norm1(mixer(x)); x += norm2(feed_forward(x))``. The sublayers read the
+    stream itself, in the activations' dtype: the kernel that norms a result and adds it to the stream also leaves that copy for the
+    sublayer behind it (``Ops.rounded``). A sublayer's result, the norm and the sum are fp32; a product that split K, and the sum over
+    experts, are finished by the norm's kernel. The norms are parts with an ``add_into`` method (``rmsnorm``). Parts: norm1, mixer
+    and, where the layer has it, norm2, feed_forward. ``unused``: as in ``hyper``."""
+    graph_safe = True
+
+    def __init__(self, hidden_size, prefix="", unused=()):
+        super().__init__(prefix)
+        self.E, self.unused = hidden_size, tuple(unused)
+
+    def param_specs(self):
+        return [ParamSpec(self.prefix + n, tuple(shape), "vector", ("one_plus_normal", 0.1), optional=True) for n, shape in self.unused]
+
+    def _sublayer(self, ops, x, part, norm, run):
+        h = ops.rounded(x)
+        y = ops.scratch("branch", (x.shape[0], self.E), torch.float32)
+        if getattr(part, "can_overwrite", False):
+            run(h, y, dict(accumulate=False))
+        else:                                  # a part that only knows how to add: into zeros
+            ops.settle()
+            y.zero_()
+            run(h, y, {})
+        with ops.section("post_norm"):
+            norm.add_into(ops, y, x, copy=True)
+
+    def forward(self, ops, step, x, parts, caches, write_cache=True):
+        mixer, ff = parts["mixer"], parts.get("feed_forward")
+        self._sublayer(ops, x, mixer, parts["norm1"],
+                       lambda h, y, kw: mixer.forward(ops, step, h, caches.get("mixer"), y, write_cache, **kw))
+        if ff is not None:
+            self._sublayer(ops, x, ff, parts["norm2"], lambda h, y, kw: ff.forward(ops, step, h, y, **kw))
+
+
 @register_part("block", "hyper")
 class HyperBlock(Part):
     """Hyper-connections: the residual is ``streams`` streams side by side (fp32 [T, streams, width]; the plan's ``streams``).

@@ -11,17 +11,19 @@ from .base import ParamSpec, Part
 @register_part("feed_forward", "gated_mlp")
 class GatedMLP(Part):
     """``x += Wdown (act(Wgate h) * (Wup h))`` with ``act(g) = g / (1 + exp(-g))``
-    (src/model.c:612-623, src/mathx.c:34). Gate and up share their input and are held
-    as one matrix, gate rows first. ``names``: the tensors' names after ``prefix`` (keys gate, up, down)."""
+    (src/model.c:612-623, src/mathx.c:34), or ``activation`` ``gelu_tanh``. Gate and up share their input and are held
+    as one matrix, gate rows first. ``names``: the tensors' names after ``prefix`` (keys gate, up, down).
+    ``forward(..., accumulate=False)`` writes ``x = ...`` instead of adding."""
     graph_safe = True
     lazy_input_ok = True
+    can_overwrite = True
 
 
     def __init__(self, hidden_size, intermediate_size, activation="silu", prefix="", names=None):
         super().__init__(prefix)
-        if activation != "silu":
+        if activation not in ("silu", "gelu_tanh"):
             fail(ENOTSUP, f"gated_mlp: activation '{activation}' is not implemented")
-        self.E, self.F = hidden_size, intermediate_size
+        self.E, self.F, self.activation = hidden_size, intermediate_size, activation
         self.names = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
         self.names.update(names or {})
         self.w_gate_up = self.w_down = None
@@ -47,20 +49,20 @@ class GatedMLP(Part):
             self.w_gate_up = memory.cat([g.to(dt), u.to(dt)], 0, f"{p}gate and up in one matrix")
         self.w_down = params[p + nm["down"]]
 
-    def forward(self, ops, step, h, x):
+    def forward(self, ops, step, h, x, accumulate=True):
         T = h.shape[0]
         act = ops.scratch("ffn_act", (T, self.F), ops.act_dtype)
         if self.fused:
             with ops.section("gate_up"):           # the activation is the product's last step
-                ops.gemm(h, self.w_gate_up, act, swiglu=True)
+                ops.gemm(h, self.w_gate_up, act, swiglu=True, gate_act=self.activation)
         else:
             gu = ops.scratch("gate_up", (T, 2 * self.F), ops.act_dtype)
             with ops.section("gate_up"):
                 ops.gemm(h, self.w_gate_up, gu)
             with ops.section("silu"):
-                ops.swiglu(gu, act)
+                ops.swiglu(gu, act, gate_act=self.activation)
         with ops.section("down"):
-            ops.gemm(act, self.w_down, x, accumulate=True, defer=True)
+            ops.gemm(act, self.w_down, x, accumulate=accumulate, defer=True)
 
 
 @register_part("feed_forward", "mlp")

@@ -31,12 +31,17 @@ class MixtureOfExperts(Part):
 
     ``scoring="softmax_chosen"``: the ``top`` experts with the largest logits, weighted by the softmax over the chosen logits
     alone. ``router_bias``: the router's logits are ``Wrouter h + b`` (the tensor named by ``names["router_bias"]``, fp32).
-    ``shared``: the PartSpec of a feed-forward that every token passes beside its experts; its result is added."""
+    ``shared``: the PartSpec of a feed-forward that every token passes beside its experts; its result is added, with ``shared_gate``
+    times ``sigmoid(Wsg h)``, one number a token (the tensor ``names["shared_gate"]`` [1, width], a row more of the router's product).
+    ``correction``: the tensor of that name ([experts]) is added to the scores for the choice, while the weights stay the scores
+    without it. ``forward(..., accumulate=False)`` writes ``x = ...`` instead of adding, and may leave the sum over experts and shared
+    expert to the norm that reads ``x`` (``Ops.branch_sum``)."""
     graph_safe = True
+    can_overwrite = True
 
     def __init__(self, hidden_size, expert_size, n_experts, top, n_groups=1, keep_groups=1, activation="relu2",
                  scoring="softmax", renormalize=True, weight_scale=1.0, prefix="", names=None, gated=None,
-                 weight_on="output", router_bias=False, shared=None):
+                 weight_on="output", router_bias=False, shared=None, shared_gate=False, correction=False):
         super().__init__(prefix)
         if weight_on not in ("output", "input") or (weight_on == "input" and gated is None):
             fail(ENOTSUP, "moe: experts without a gate weigh their output; gated experts their input or their output")
@@ -57,11 +62,14 @@ class MixtureOfExperts(Part):
         self.renormalize, self.weight_scale = bool(renormalize), float(weight_scale)
         self.names = {"router": "router.weight", "up": "experts.{e}.up_proj.weight", "down": "experts.{e}.down_proj.weight",
                       "gate": "experts.{e}.gate_proj.weight"}
-        self.names["router_bias"] = "router.bias"
+        self.names.update(router_bias="router.bias", correction="correction", shared_gate="shared_gate.weight")
         self.names.update(names or {})
         self.router_bias = bool(router_bias)
         self.shared = None if shared is None else make_part("feed_forward", shared)
-        self.w_router = self.b_router = self.w_up = self.w_down = None
+        self.shared_gate, self.correction = bool(shared_gate), bool(correction)
+        if self.shared_gate and shared is None:
+            fail(EINVAL, "moe: a shared expert's gate without a shared expert")
+        self.w_router = self.b_router = self.w_up = self.w_down = self.correction_w = None
 
     def sub_parts(self):
         return [] if self.shared is None else [self.shared]
@@ -73,6 +81,10 @@ class MixtureOfExperts(Part):
         specs = [ParamSpec(self._name("router"), (self.n_experts, self.E))]
         if self.router_bias:
             specs.append(ParamSpec(self._name("router_bias"), (self.n_experts,), "vector", ("normal", 0.1)))
+        if self.correction:
+            specs.append(ParamSpec(self._name("correction"), (self.n_experts,), "vector", ("normal", 0.1)))
+        if self.shared_gate:
+            specs.append(ParamSpec(self._name("shared_gate"), (1, self.E)))
         for e in range(self.n_experts):
             specs += [ParamSpec(self._name("up", e), (self.F, self.E)), ParamSpec(self._name("down", e), (self.E, self.F))]
             if self.gated is not None:
@@ -82,6 +94,15 @@ class MixtureOfExperts(Part):
     def bind(self, params, ops):
         self.w_router = params[self._name("router")]
         self.b_router = params[self._name("router_bias")].contiguous() if self.router_bias else None
+        if self.correction:
+            self.correction_w = params[self._name("correction")].contiguous()
+        if self.shared_gate:                        # one row more of the router's product, without a bias
+            sg = params[self._name("shared_gate")]
+            dt = torch.float32 if torch.float32 in (sg.dtype, self.w_router.dtype) else sg.dtype
+            self.w_router = memory.cat([self.w_router.to(dt), sg.to(dt)], 0, f"{self.prefix}router and shared gate in one matrix")
+            if self.b_router is not None:
+                self.b_router = memory.cat([self.b_router, torch.zeros(1, dtype=torch.float32, device=self.b_router.device)], 0,
+                                           f"{self.prefix}router bias")
         ups = [params.pop(self._name("up", e)) for e in range(self.n_experts)]
         if self.gated is not None:                  # gate and up of an expert in one matrix: one product gives both
             gates = [params.pop(self._name("gate", e)) for e in range(self.n_experts)]
@@ -96,15 +117,37 @@ class MixtureOfExperts(Part):
         del ups
         self.w_down = memory.cat([m.to(dt).unsqueeze(0) for m in downs], 0, f"{self.prefix}down matrices of all experts")
 
-    def forward(self, ops, step, h, x):
+    def forward(self, ops, step, h, x, accumulate=True):
         T = h.shape[0]
-        logits = ops.scratch("router_logits", (T, self.n_experts), torch.float32)
+        rows = self.w_router.shape[0]
+        product = ops.scratch("router_logits", (T, rows), torch.float32)
+        logits, sg = product[:, :self.n_experts], product[:, self.n_experts:] if self.shared_gate else None
         with ops.section("router"):
-            ops.gemm(h, self.w_router, logits, bias=self.b_router)
+            ops.gemm(h, self.w_router, product, bias=self.b_router)
             ids, weights = ops.moe_route(logits, self.top, self.n_groups, self.keep_groups, self.scoring, self.renormalize,
-                                         self.weight_scale)
+                                         self.weight_scale, correction=self.correction_w)
+        if accumulate and not self.shared_gate:
+            with ops.section("experts"):
+                ops.moe_experts(h, ids, weights, self.w_up, self.w_down, self.activation, x, gated=self.gated, weight_on=self.weight_on)
+            if self.shared is not None:
+                with ops.section("shared_expert"):
+                    self.shared.forward(ops, step, h, x)
+            return
+        y = ops.scratch("moe_sum", (T, self.E), torch.float32) if accumulate else x
         with ops.section("experts"):
-            ops.moe_experts(h, ids, weights, self.w_up, self.w_down, self.activation, x, gated=self.gated, weight_on=self.weight_on)
+            pairs = ops.moe_experts(h, ids, weights, self.w_up, self.w_down, self.activation, y, gated=self.gated, weight_on=self.weight_on,
+                                    combine=False)
+        ys = None
         if self.shared is not None:
+            ys = ops.scratch("moe_shared", (T, self.E), torch.float32)
             with ops.section("shared_expert"):
-                self.shared.forward(ops, step, h, x)
+                if getattr(self.shared, "can_overwrite", False):
+                    self.shared.forward(ops, step, h, ys, accumulate=False)
+                else:
+                    ops.settle()
+                    ys.zero_()
+                    self.shared.forward(ops, step, h, ys)
+        ops.branch_sum(y, pairs, self.top, extra=ys, extra_gate=sg)
+        if accumulate:
+            with ops.section("experts"):
+                ops.rmsnorm_add(y, None, 0.0, x)

@@ -44,10 +44,10 @@ class RMSNorm(Part):
         ``out`` is read through ``ops.gemm`` alone (a part that says ``lazy_input_ok``); see ``Ops.rmsnorm``."""
         ops.rmsnorm(x, self.weight, self.eps, out, rows, lazy=lazy)
 
-    def add_into(self, ops, y, x, gate=None, gate_bias=None, scale=1.0, accumulate=True):
+    def add_into(self, ops, y, x, gate=None, gate_bias=None, scale=1.0, accumulate=True, copy=False):
         """``x (+)= scale * norm(y * sigmoid(gate + gate_bias))`` in fp32: the norm of a branch's result ``y`` (fp32) on its
-        way into the stream (``gate`` None: ``y`` as it is)."""
-        ops.rmsnorm_add(y, self.weight, self.eps, x, gate=gate, gate_bias=gate_bias, scale=scale, accumulate=accumulate)
+        way into the stream (``gate`` None: ``y`` as it is); ``copy``: see ``Ops.rmsnorm_add``."""
+        ops.rmsnorm_add(y, self.weight, self.eps, x, gate=gate, gate_bias=gate_bias, scale=scale, accumulate=accumulate, copy=copy)
 
 
 @register_part("norm", "layernorm")

@@ -1,5 +1,5 @@
 """Mixers that keep per-request state of fixed size instead of a growing cache: a state-space layer, linear
-attention with a fixed decay, a matrix memory with exponential gates, recurrences with a decay per key channel (a forget gate
+attention with a fixed decay (two forms), a matrix memory with exponential gates, recurrences with a decay per key channel (a forget gate
 that also writes; gated linear attention), and the gated delta rule. All walk a request's
 tokens in order from the state the step before left. The first three share one kernel for the recurrence
 (``Ops.linear_scan``): ``S <- a_t S + k_t (b_t v_t)^T``, ``y_t = S^T q_t + d v_t``; the delta rule, whose write depends on
@@ -148,6 +148,86 @@ class LightningAttention(Part):
             ops.group_rmsnorm(o, self.norm_w, self.eps, 1, normed, gate=gate, gate_kind="sigmoid_after")
         with ops.section("lin_wo"):
             ops.gemm(normed, self.w_o, x, accumulate=True, defer=True)
+
+
+@register_part("mixer", "retention")
+class Retention(Part):
+    """Linear attention with a fixed decay per head: ``q = Wq h`` and ``k = Wk h`` (``n_heads`` x ``head_dim``), ``v = Wv h`` (``n_heads`` x
+    ``v_head_dim``), q and k turned by ``position`` (a rotary PartSpec of split halves) and k multiplied by ``head_dim^-1/2``;
+    ``S_t = decay_h S_(t-1) + k_t v_t^T``, ``o_t = S_t^T q_t``; each head's ``o`` is divided by its root mean square (``eps``, no weight), the
+    heads together are multiplied by ``silu(Wg h)`` and projected. ``decay``: one number a head. The turned queries and keys, the
+    recurrence and the norm are fp32; the state is fp32 in the request's state row. ``names``: the tensors' names after ``prefix`` (keys
+    q, k, v, g, o). ``forward(..., accumulate=False)`` writes ``x = ...``; ``heads(...)`` gives what the output projection reads, times
+    ``out_scale`` (set before the tensors are bound)."""
+    graph_safe = True
+    can_overwrite = True
+    joins_heads = True
+    FEW_ROWS = 64                # rows up to which the gate's rows ride in the product of queries, keys and values
+
+    def __init__(self, hidden_size, n_heads, head_dim, v_head_dim, decay, eps, position, prefix="", names=None):
+        super().__init__(prefix)
+        if len(decay) != n_heads:
+            fail(EINVAL, f"retention: {len(decay)} decays for {n_heads} heads")
+        self.E, self.H, self.D, self.Dv, self.eps = hidden_size, n_heads, head_dim, v_head_dim, float(eps)
+        self.OD = n_heads * v_head_dim
+        self.decay_values = [float(d) for d in decay]
+        self.position = make_part("position", position)
+        if self.position.kind not in ("none", "rotary") or getattr(self.position, "pairing", "split_half") != "split_half":
+            fail(EINVAL, "retention: queries and keys are turned in split halves, or not at all")
+        self.names = {n: f"{n}_proj.weight" for n in "qkvgo"}
+        self.names.update(names or {})
+        self.out_scale = 1.0
+        self.w_in = self.w_o = self.norm_w = self.decay = None
+
+    def sub_parts(self):
+        return [self.position]
+
+    def param_specs(self):
+        p, nm = self.prefix, self.names
+        QD, VD = self.H * self.D, self.OD
+        return [ParamSpec(p + nm["q"], (QD, self.E)), ParamSpec(p + nm["k"], (QD, self.E)), ParamSpec(p + nm["v"], (VD, self.E)),
+                ParamSpec(p + nm["g"], (VD, self.E)), ParamSpec(p + nm["o"], (self.E, VD))]
+
+    def cache_need(self):
+        return FixedState(Ops.scan_state_floats(self.H, self.D, self.Dv))
+
+    def bind(self, params, ops):
+        p, nm = self.prefix, self.names
+        mats = [params[p + nm[n]] for n in "qkvg"]
+        dt = torch.float32 if any(m.dtype == torch.float32 for m in mats) else mats[0].dtype
+        self.w_in = memory.cat([m.to(dt) for m in mats], 0, f"{p}q, k, v and the gate in one matrix")
+        self.w_o = params[p + nm["o"]]
+        self.norm_w = memory.to_device(torch.full((self.OD,), self.out_scale, dtype=torch.float32), ops.device, f"{p}weight of the heads' norm")
+        self.decay = memory.to_device(torch.tensor(self.decay_values, dtype=torch.float64).to(torch.float32), ops.device, f"{p}decays")
+
+    def heads(self, ops, step, h, cache, out, write_cache=True):
+        if not write_cache:
+            fail(EINVAL, f"retention '{self.prefix}': a state cannot be read without being advanced")
+        T, QD, VD = h.shape[0], self.H * self.D, self.OD
+        C = 2 * QD + VD
+        few = T <= self.FEW_ROWS
+        with ops.section("ret_in"):
+            rows = ops.scratch("ret_in", (T, C + VD if few else C), torch.float32)
+            ops.gemm(h, self.w_in if few else self.w_in[:C], rows)
+            if few:
+                gate = rows[:, C:]
+            else:
+                gate = ops.scratch("ret_gate", (T, VD), ops.act_dtype)
+                ops.gemm(h, self.w_in[C:], gate)
+        o = ops.scratch("ret_o", (T, VD), torch.float32)
+        with ops.section("ret_scan"):
+            if getattr(self.position, "rot_dim", 0):
+                ops.rope_store(rows[:, :2 * QD], step.positions, self.position.inv_freq, self.position.rot_dim, 2 * self.H, 0, self.D, None, None)
+            ops.linear_scan(rows[:, :QD], rows[:, QD:2 * QD], rows[:, 2 * QD:C], self.H, self.D, self.H, self.Dv, cache.state, step, o,
+                            decay=self.decay, q_scale=self.D ** -0.5)
+        with ops.section("ret_norm"):
+            ops.group_rmsnorm(o, self.norm_w, self.eps, self.H, out, gate=gate, gate_kind="silu_after")
+
+    def forward(self, ops, step, h, cache, x, write_cache=True, accumulate=True):
+        normed = ops.scratch("ret_normed", (h.shape[0], self.OD), ops.act_dtype)
+        self.heads(ops, step, h, cache, normed, write_cache)
+        with ops.section("ret_wo"):
+            ops.gemm(normed, self.w_o, x, accumulate=accumulate, defer=True)
 
 
 @register_part("mixer", "mlstm")
@@ -458,7 +538,9 @@ class SideBySide(Part):
     over the model's width with a weight of its own (``names``: keys left_norm, right_norm, after ``prefix``) before the sum
     (``scale`` 0.5: half the sum). ``left`` and ``right`` are PartSpecs of mixers; their caches are this mixer's, by the names
     ``left`` and ``right``. The sides' results, the norms and the sum are fp32. ``normed=False``: no norms and no weights; the result
-    is the weighted sum ``left_scale * left(h) + right_scale * right(h)``."""
+    is the weighted sum ``left_scale * left(h) + right_scale * right(h)``. Two sides that can hand out their heads before the output
+    projection (``joins_heads``) then share one product: the heads side by side, each side's times its scale, on the two projections
+    side by side."""
     graph_safe = True
     can_overwrite = True
 
@@ -470,8 +552,11 @@ class SideBySide(Part):
         self.left, self.right = make_part("mixer", left), make_part("mixer", right)
         self.names = {"left_norm": "left.out", "right_norm": "right.out"}
         self.names.update(names or {})
-        self.w_left = self.w_right = None
+        self.w_left = self.w_right = self.w_joint = None
         self.short_request_rows = 0
+        self.joint = not self.normed and all(getattr(s, "joins_heads", False) for s in (self.left, self.right))
+        if self.joint:
+            self.left.out_scale, self.right.out_scale = self.side_scale["left"], self.side_scale["right"]
 
     def sub_parts(self):
         return [self.left, self.right]
@@ -487,10 +572,23 @@ class SideBySide(Part):
     def bind(self, params, ops):
         if self.normed:
             self.w_left, self.w_right = params[self.prefix + self.names["left_norm"]], params[self.prefix + self.names["right_norm"]]
+        if self.joint:
+            mats = [self.left.w_o, self.right.w_o]
+            dt = torch.float32 if any(m.dtype == torch.float32 for m in mats) else mats[0].dtype
+            self.w_joint = memory.cat([m.to(dt) for m in mats], 1, f"{self.prefix}both output projections in one matrix")
+            self.left.w_o, self.right.w_o = self.w_joint[:, :self.left.OD], self.w_joint[:, self.left.OD:]
         self.short_request_rows = max(getattr(self.left, "short_request_rows", 0), getattr(self.right, "short_request_rows", 0))
 
     def forward(self, ops, step, h, cache, x, write_cache=True, accumulate=True):
         T = h.shape[0]
+        if self.joint:
+            L = self.left.OD
+            heads = ops.scratch("side_heads", (T, L + self.right.OD), ops.act_dtype)
+            self.left.heads(ops, step, h, cache["left"], heads[:, :L], write_cache)
+            self.right.heads(ops, step, h, cache["right"], heads[:, L:], write_cache)
+            with ops.section("side_wo"):
+                ops.gemm(heads, self.w_joint, x, accumulate=accumulate, defer=True)
+            return
         for side, w, name in ((self.left, self.w_left, "left"), (self.right, self.w_right, "right")):
             y = ops.scratch("side_" + name, (T, self.E), torch.float32)
             if getattr(side, "can_overwrite", False):
