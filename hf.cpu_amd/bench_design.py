@@ -1,6 +1,6 @@
-"""``bench.py --design goridra | tobozen | mobupel | gitasun | fugevik``: prefill and decode of a design at sizes that resemble a real model's layers
+"""``bench.py --design goridra | tobozen | mobupel | gitasun | fugevik | lurirax``: prefill and decode of a design at sizes that resemble a real model's layers
 (random weights), beside the closest other design at equal width, heads and layer count (Goridra beside Qwen2 dense,
-Tobozen beside Goridra, Mobupel and Gitasun beside Tobozen, Fugevik beside Gitasun), with every part of a step priced against its roofline: flops / time against the matrix cores
+Tobozen beside Goridra, Mobupel and Gitasun beside Tobozen, Fugevik and Lurirax beside Gitasun), with every part of a step priced against its roofline: flops / time against the matrix cores
 for a prefill's parts, bytes / time against HBM for a decode step's. One JSON line a size."""
 import json
 import math
@@ -14,7 +14,7 @@ PROMPT, PAGE = 2048, 16
 # width, heads, key/value heads, head size, dense ff, experts, choices, groups, kept groups, expert ff, layers, vocabulary
 # (for Tobozen also: heads, head size, state and groups of the state-space layers; layers come in threes; for Gitasun also the rotated
 # part, the key/value latent and the query latent of its attention through latents; for Fugevik also the streams of its residual
-# and its windows)
+# and its windows; Lurirax has those windows and chunks of `mask`)
 SIZES = {
     "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, ff=8192, experts=32, top=4, groups=4, keep=2, expert_ff=1024,
                layers=8, vocab=32000, mask=1024, ssm_heads=64, ssm_dim=64, ssm_state=128, ssm_groups=8, triples=2,
@@ -187,6 +187,63 @@ def fugevik_work(z, T, batch, ctx):
     return pre, dec
 
 
+KEEP_FIRST = 64              # first tokens that stay in sight of Lurirax's differential attention
+
+
+def lurirax_shape(z):
+    """Layers in threes: windowed attention with a sink, attention in chunks beside retention, differential attention; the first layer
+    with a dense gated feed-forward, the others with a mixture of gated experts and a gated shared expert."""
+    H, G, D, W = z["heads"], z["kv_heads"], z["dim"], z["width"]
+    moe = dict(kind="moe", expert=dict(ff=z["expert_ff"]), router=dict(experts=z["experts"], top=z["top"], scale=1.0), shared=dict(ff=z["expert_ff"]))
+    scaling = dict(factor=4.0, low=1.0, high=2.0, original=8192)
+    three = [
+        dict(type="attention", mixer=dict(heads=H, kv_heads=G, dim=D, vdim=D, scale=math.sqrt(D), mask=dict(size=z["window"]),
+                                          rot=dict(dims=D, base=500000.0, scaling=scaling)), mlp=moe),
+        dict(type="parallel", mixer=dict(
+            left=dict(heads=H, kv_heads=G, dim=D, vdim=D, scale=1.0 / math.sqrt(D), bias_max=128, bias_rows=32, mask=dict(size=z["mask"])),
+            right=dict(heads=H, dim=D, vdim=D, decay=[1.0 - 2.0 ** -(3 + 8 * h // H) for h in range(H)], rot=dict(dims=D, base=500000.0)),
+            left_scale=0.5, right_scale=1.0), mlp=moe),
+        dict(type="attention_2", mixer=dict(heads=H, kv_heads=G, dim=D // 2, vdim=D, scale=1.0 / math.sqrt(D // 2), diff=0.5,
+                                            mask=dict(size=z["window"], keep_first=KEEP_FIRST)), mlp=moe)]
+    layers = three * z["triples"]
+    layers[0] = dict(layers[0], mlp=dict(kind="dense", ff=lurirax_dense(z)))
+    return dict(architecture="Lurirax", vocab=z["vocab"], width=W, embedding=dict(scale=math.sqrt(W)), norm=dict(eps=1e-6), layers=layers)
+
+
+def lurirax_dense(z):
+    return z["ff"] * 2 // 3 // 128 * 128
+
+
+def lurirax_work(z, T, batch, ctx):
+    """({part: flops of a prefill of T tokens}, {part: bytes of a decode step}), all layers together, bf16. Differential attention is two
+    maps of half-sized keys over the same values: its scores cost a head's once, its weighted values twice; retention by the products
+    of its state updates and outputs in a prefill and by its fp32 states, read and written once a request, in a decode step. Norms on
+    the way into the stream (``post_norm``) move bytes only: in a prefill their bytes stand as the flops that take as long at both
+    peaks."""
+    W, H, G, D, V, n3 = z["width"], z["heads"], z["kv_heads"], z["dim"], z["vocab"], z["triples"]
+    QD, KD, L = H * D, G * D, 3 * n3
+    E, top, F, dense = z["experts"], z["top"], z["expert_ff"], lurirax_dense(z)
+    win, chunk = z["window"], z["mask"]
+    params = {"qkv": n3 * W * (3 * (QD + 2 * KD) + H), "wo": 2 * n3 * QD * W, "ret_in": n3 * W * 4 * QD, "side_wo": n3 * 2 * QD * W,
+              "router": (L - 1) * E * W, "gate_up": 2 * W * (dense + (L - 1) * F), "down": W * (dense + (L - 1) * F), "head": V * W}
+    pre = {k: 2.0 * T * v for k, v in params.items() if k != "head"}
+    seen = sum(min(t + 1, win) for t in range(T))
+    seen_kept = sum(min(t + 1, win + min(KEEP_FIRST, max(0, t + 1 - win))) for t in range(T))
+    seen_chunk = sum(t % chunk + 1 for t in range(T))
+    pre["attn"] = n3 * H * D * (4.0 * seen + 4.0 * seen_chunk + 6.0 * seen_kept)
+    pre["ret_scan"] = n3 * T * H * 4.0 * D * D
+    pre["experts"] = (L - 1) * T * top * 6.0 * F * W
+    joint = 2 * L * W * (4.0 * 3 + 2)                # bytes a token: a result read, the stream read and written, its copy written
+    pre["post_norm"] = T * joint * MFMA_PEAK / HBM_PEAK
+    dec = {k: 2.0 * v for k, v in params.items()}
+    touched = E * (1.0 - (1.0 - top / E) ** batch)
+    dec["experts"] = (L - 1) * touched * 3 * F * W * 2.0
+    dec["attn"] = batch * n3 * 2.0 * 2 * KD * (min(ctx, win) + ctx % chunk + min(ctx, win + KEEP_FIRST))
+    dec["ret_scan"] = batch * n3 * H * D * D * 4 * 2.0
+    dec["post_norm"] = batch * joint
+    return pre, dec
+
+
 def goridra_shape(z):
     """Layers in pairs: one with keys and values of its own and a dense feed-forward, one that reads them and has
     a mixture of experts."""
@@ -227,6 +284,8 @@ def part_work(design, z, T, batch, ctx):
         return gitasun_work(z, T, batch, ctx)
     if design == "fugevik":
         return fugevik_work(z, T, batch, ctx)
+    if design == "lurirax":
+        return lurirax_work(z, T, batch, ctx)
     W, H, G, D, L, V = z["width"], z["heads"], z["kv_heads"], z["dim"], z["layers"], z["vocab"]
     QD, KD = H * D, G * D
     if design == "qwen2":
@@ -264,9 +323,10 @@ def run(args):
         z = SIZES[size]
         line = {"size": size, "dims": z, "context": context, "dtype": "bf16", "data": "synthetic"}
         shapes = {"goridra": goridra_shape, "qwen2": qwen2_shape, "tobozen": tobozen_shape, "mobupel": mobupel_shape, "gitasun": gitasun_shape,
-                  "fugevik": fugevik_shape}
-        beside = {"goridra": "qwen2", "tobozen": "goridra", "mobupel": "tobozen", "gitasun": "tobozen", "fugevik": "gitasun"}[args.design]
-        if args.design in ("tobozen", "mobupel", "gitasun", "fugevik"):    # the same number of layers in both designs
+                  "fugevik": fugevik_shape, "lurirax": lurirax_shape}
+        beside = {"goridra": "qwen2", "tobozen": "goridra", "mobupel": "tobozen", "gitasun": "tobozen", "fugevik": "gitasun",
+                  "lurirax": "gitasun"}[args.design]
+        if args.design in ("tobozen", "mobupel", "gitasun", "fugevik", "lurirax"):    # the same number of layers in both designs
             z = dict(z, layers=3 * z["triples"])
         for design, shape in ((args.design, shapes[args.design](z)), (beside, shapes[beside](z))):
             cfg = hf_cpu_amd.config_from_dict(shape)

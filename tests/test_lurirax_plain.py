@@ -1,0 +1,300 @@
+"""The plain implementation of Lurirax against second derivations, and the package's reader, plan and cache for it (no GPU)."""
+import copy
+import math
+
+import numpy as np
+import pytest
+import torch
+
+import lurirax_helpers as lh
+import plain_lurirax as pl
+
+
+def small_weights(cfg, seed=0):
+    return {k: np.asarray(v, np.float64) for k, v in lh.make_weights(cfg, seed).items()}
+
+
+# ---- the plain implementation ------------------------------------------------------------------------------------------
+
+def test_rescaled_frequencies_at_and_between_both_bounds():
+    scaling = dict(factor=4.0, low=1.0, high=4.0, original=64)
+    for f, want in ((2 * math.pi / 15.9, 1.0), (2 * math.pi / 64.1, 0.25), (2 * math.pi / 32.0, None)):
+        base = f ** -2.0                                       # frequency 1 of two pairs is base^(-1/2)
+        got = pl.rotary_frequencies(4, base, scaling)[1]
+        s = (64 / 32.0 - 1.0) / 3.0
+        assert np.isclose(got / f, want if want is not None else (1 - s) / 4.0 + s)
+    plain = pl.rotary_frequencies(6, 100.0)
+    assert np.allclose(plain, [1.0, 100.0 ** (-1 / 3), 100.0 ** (-2 / 3)])
+
+
+def test_rotation_pairs_halves_and_depends_on_distance_alone():
+    rng = np.random.default_rng(0)
+    f = pl.rotary_frequencies(6, 100.0)
+    x = rng.standard_normal((1, 1, 8))
+    turned = pl.rotate(x, [5], f)[0, 0]
+    for i in range(3):
+        assert np.allclose(turned[i] + 1j * turned[i + 3], (x[0, 0, i] + 1j * x[0, 0, i + 3]) * np.exp(5j * f[i]))
+    assert np.allclose(turned[6:], x[0, 0, 6:])
+    k = rng.standard_normal((1, 1, 8))
+
+    def score(i, j):                                           # normed after the rotation: the norm does not see the rotation
+        return float((pl.unit_rms(pl.rotate(x, [i], f), 1e-6) * pl.unit_rms(pl.rotate(k, [j], f), 1e-6)).sum())
+    assert np.isclose(score(7, 4), score(103, 100)) and not np.isclose(score(7, 4), score(7, 5))
+
+
+def test_masks_at_their_edges():
+    w = pl.sees_window(30, 5)
+    assert w[12, 8] and not w[12, 7] and w[12, 12] and not w[12, 13]
+    k = pl.sees_window(30, 5, 3)
+    assert k[20, 2] and not k[20, 3] and k[20, 16] and not k[20, 15] and not k[1, 2]
+    c = pl.sees_chunk(30, 6)
+    assert c[11, 6] and not c[12, 11] and not c[11, 5] and c[12, 12] and not c[10, 11]
+
+
+def test_distance_buckets():
+    rows, reach = 8, 64
+    got = [pl.bucket(n, rows, reach) for n in range(70)]
+    assert got[:4] == [0, 1, 2, 3] and got[4] == 4 and got[-1] == 7 and got == sorted(got)
+    for n in range(4, 64):
+        assert got[n] == min(7, 4 + math.floor(4 * math.log(n / 4) / math.log(16)))
+    table = np.arange(16.0).reshape(8, 2)
+    b = pl.distance_bias(table, 70, reach)
+    assert b.shape == (2, 70, 70) and b[1, 69, 0] == table[7, 1] and b[0, 40, 38] == table[2, 0] and b[0, 3, 9] == 0.0
+
+
+def test_bucket_of_the_part_is_the_plain_one():
+    from hf_cpu_amd.parts.attention import Attention
+    for rows, reach in ((2, 2), (8, 9), (10, 40), (32, 240), (24, 200)):
+        assert [Attention.distance_bucket(n, rows, reach) for n in range(400)] == [pl.bucket(n, rows, reach) for n in range(400)]
+
+
+def test_softmax_against_the_library_and_a_sink_that_takes_weight():
+    rng = np.random.default_rng(1)
+    T, H, G, D, P = 9, 4, 2, 6, 5
+    q, k, v = rng.standard_normal((T, H, D)), rng.standard_normal((T, G, D)), rng.standard_normal((T, G, P))
+    vis = pl.sees_window(T, 4)
+    bias = rng.standard_normal((H, T, T))
+    lib = torch.nn.functional.scaled_dot_product_attention(
+        torch.tensor(q).transpose(0, 1), torch.tensor(np.repeat(k, 2, axis=1)).transpose(0, 1), torch.tensor(np.repeat(v, 2, axis=1)).transpose(0, 1),
+        attn_mask=torch.tensor(np.where(vis[None], bias, -np.inf)), scale=0.7).transpose(0, 1).numpy()
+    assert np.allclose(pl.softmax_attention(q, k, v, 0.7, vis, bias=bias), lib)
+    sink = rng.standard_normal(H)
+    got = pl.softmax_attention(q, k, v, 0.7, vis, bias=bias, sink=sink)
+    kk = np.repeat(k, 2, axis=1)
+    for h in range(H):
+        z = sum(math.exp(q[8, h] @ kk[j, h] * 0.7 + bias[h, 8, j]) for j in range(5, 9))
+        assert np.allclose(got[8, h], lib[8, h] * z / (z + math.exp(sink[h])))
+
+
+def test_retention_against_its_sum_over_earlier_tokens():
+    rng = np.random.default_rng(2)
+    q, k, v = rng.standard_normal((7, 2, 3)), rng.standard_normal((7, 2, 3)), rng.standard_normal((7, 2, 4))
+    decay = [0.9, 0.5]
+    got = pl.fixed_decay_recurrence(q, k, v, decay)
+    for h in range(2):
+        want = sum(decay[h] ** (6 - j) * (q[6, h] @ k[j, h]) * v[j, h] for j in range(7))
+        assert np.allclose(got[6, h], want)
+
+
+def test_two_maps_and_their_factor():
+    rng = np.random.default_rng(3)
+    cfg = lh.config(20, 16, layers=[lh.layer(lh.diff(2, 1, 4, 6, 5, 2, 0.35), None)])
+    w = small_weights(cfg)
+    p, m = "l0.mix.", cfg["layers"][0]["mixer"]
+    f = pl.map_factor(w, p, 0.35)
+    assert np.isclose(f, math.exp(w[p + "lq1"] @ w[p + "lk1"]) - math.exp(w[p + "lq2"] @ w[p + "lk2"]) + 0.35)
+    h = rng.standard_normal((9, 16))
+    # both maps alike: (1 - f) times one map, which the norm makes the map itself divided by its root mean square
+    same = dict(w)
+    q, k = w[p + "q"].reshape(2, 2, 4, 16).copy(), w[p + "k"].reshape(1, 2, 4, 16).copy()
+    q[:, 1], k[:, 1] = q[:, 0], k[:, 0]
+    same[p + "q"], same[p + "k"], same[p + "o"] = q.reshape(16, 16), k.reshape(8, 16), np.eye(16)[:, :12]
+    got = pl.differential_attention(h, same, p, m, 1e-12).reshape(9, 16)[:, :12].reshape(9, 2, 6)
+    qq = pl.unit_rms((h @ q[:, 0].reshape(8, 16).T).reshape(9, 2, 4), 1e-12) * w[p + "q.norm"]
+    kk = pl.unit_rms((h @ k[:, 0].reshape(4, 16).T).reshape(9, 1, 4), 1e-12) * w[p + "k.norm"]
+    one = pl.softmax_attention(qq, kk, (h @ w[p + "v"].T).reshape(9, 1, 6), m["scale"], pl.sees_window(9, 5, 2))
+    assert np.allclose(got, pl.unit_rms(one, 1e-12) * np.sign(1.0 - f) * 0.65)
+
+
+def test_router_chooses_with_the_correction_and_weighs_without():
+    w = {"router": np.eye(4), "correction": np.array([0.0, 0.0, 10.0, -10.0])}
+    h = np.array([[2.0, 1.0, -3.0, 9.0], [0.0, 0.0, 0.0, 0.0]])
+    ids, c = pl.route(h, w, "", dict(top=2, scale=2.5))
+    assert ids.tolist() == [[2, 0], [2, 0]]                    # among equals the lower index
+    assert np.allclose(c, 2.5 * pl.sigmoid(np.array([[-3.0, 2.0], [0.0, 0.0]])))
+
+
+def test_a_shared_expert_behind_its_gate_and_the_gated_unit():
+    rng = np.random.default_rng(4)
+    cfg = lh.config(20, 8, layers=[lh.layer(lh.diff(1, 1, 4, 4, 5, 0), lh.moe(3, 3, 5, shared=4, scale=2.0))])
+    w, h = small_weights(cfg), rng.standard_normal((6, 8))
+    f, p = cfg["layers"][0]["mlp"], "l0.mlp."
+    want = np.zeros((6, 8))
+    for e in range(3):
+        g = h @ w[f"{p}e{e}.gate"].T
+        want += 2.0 * pl.sigmoid(h @ w[p + "router"][e])[:, None] * ((g * pl.sigmoid(g) * (h @ w[f"{p}e{e}.up"].T)) @ w[f"{p}e{e}.down"].T)
+    bare = pl.feed_forward(h, w, p, dict(f, shared=None))
+    assert np.allclose(bare, want)
+    g = h @ w[p + "shared.gate"].T
+    extra = (g * pl.sigmoid(g) * (h @ w[p + "shared.up"].T)) @ w[p + "shared.down"].T
+    assert np.allclose(pl.feed_forward(h, w, p, f) - bare, extra / (1.0 + np.exp(-(h @ w[p + "shared.sg"][0])))[:, None])
+    z = torch.tensor(rng.standard_normal(50) * 3)
+    assert np.allclose(pl.gelu_tanh(z.numpy()), torch.nn.functional.gelu(z, approximate="tanh").numpy())
+
+
+@pytest.mark.parametrize("name", list(lh.CONFIGS))
+def test_whole_model_properties(name):
+    """A prefix has the logits of the whole; norms of zero leave the embedding; the stream is not normed on its way in."""
+    cfg = lh.CONFIGS[name]
+    w = small_weights(cfg)
+    toks = [int(t) for t in np.random.default_rng(5).integers(0, cfg["vocab"], 40)]
+    rows = pl.forward(cfg, w, toks)
+    assert np.allclose(pl.forward(cfg, w, toks[:23]), rows[:23])
+    silent = {k: (np.zeros_like(v) if k.split(".")[-1] in ("norm1", "norm2") else v) for k, v in w.items()}
+    x = w["embed"][toks] * cfg["embedding"]["scale"]
+    assert np.allclose(pl.forward(cfg, silent, toks), pl.unit_rms(x, cfg["norm"]["eps"]) * w["final.norm"] @ w["head"].T)
+    # a sublayer's result enters at its norm's size whatever its own: ten times the output projection changes (nearly) nothing
+    louder = dict(w)
+    for l, lc in enumerate(cfg["layers"]):
+        if lc["type"] != "parallel":
+            louder[f"l{l}.mix.o"] = w[f"l{l}.mix.o"] * 10.0
+    assert np.max(np.abs(pl.forward(cfg, louder, toks) - rows)) <= 1e-2 * np.max(np.abs(rows))
+
+
+def test_tokens_leave_windows_and_chunks_but_kept_ones_stay():
+    toks = [int(t) for t in np.random.default_rng(6).integers(0, 50, 60)]
+
+    def changed(mix, at, seed=0):
+        cfg = lh.config(50, 32, layers=[lh.layer(mix, None)])
+        w = small_weights(cfg, seed)
+        other = list(toks)
+        other[at] = (toks[at] + 7) % 50
+        d = np.abs(pl.forward(cfg, w, toks) - pl.forward(cfg, w, other)).max(axis=1)
+        return [int(i) for i in np.flatnonzero(d > 1e-12)]
+    assert changed(lh.attention(2, 1, 8, 8, 6, 8), 20) == list(range(20, 26))
+    assert changed(lh.diff(2, 1, 8, 8, 6, 4), 20) == list(range(20, 26))
+    assert changed(lh.diff(2, 1, 8, 8, 6, 4), 3) == list(range(3, 60)) and changed(lh.diff(2, 1, 8, 8, 6, 4), 4) == list(range(4, 10))
+    silent_right = lh.parallel(lh.left(2, 1, 8, 8, 16, 12, 8), lh.right(1, 4, 4, 4), 1.0, 0.0)
+    assert changed(silent_right, 20) == list(range(20, 32))
+
+
+# ---- the package -------------------------------------------------------------------------------------------------------
+
+@pytest.mark.parametrize("name", list(lh.CONFIGS))
+def test_configuration_reads_every_key(name):
+    from hf_cpu_amd.config import config_from_dict
+    cfg = lh.CONFIGS[name]
+    c = config_from_dict(cfg)
+    assert (c.architecture, c.vocab, c.width, c.embedding_scale, c.norm_eps) == \
+        ("Lurirax", cfg["vocab"], cfg["width"], cfg["embedding"]["scale"], cfg["norm"]["eps"])
+    for lc, raw in zip(c.layers, cfg["layers"]):
+        m, x = raw["mixer"], lc.mixer
+        assert lc.type == raw["type"]
+        if lc.type == "parallel":
+            lt, rt = m["left"], m["right"]
+            assert (x.left.heads, x.left.kv_heads, x.left.dim, x.left.vdim, x.left.scale, x.left.chunk, x.left.bias_max) == \
+                tuple(lt[k] for k in ("heads", "kv_heads", "dim", "vdim", "scale")) + (lt["mask"]["size"], lt["bias_max"])
+            assert (x.right.heads, x.right.dim, x.right.vdim, x.right.rot.base, x.right.rot.dims, list(x.right.decay)) == \
+                (rt["heads"], rt["dim"], rt["vdim"], rt["rot"]["base"], rt["rot"]["dims"], rt["decay"])
+            assert (x.left_scale, x.right_scale) == (m["left_scale"], m["right_scale"])
+        else:
+            assert (x.heads, x.kv_heads, x.dim, x.vdim, x.scale, x.window) == tuple(m[k] for k in ("heads", "kv_heads", "dim", "vdim", "scale")) + (m["mask"]["size"],)
+            if lc.type == "attention":
+                s = m["rot"].get("scaling")
+                assert (x.rot.base, x.rot.dims) == (m["rot"]["base"], m["rot"]["dims"])
+                assert x.rot.scaling == (None if s is None else (s["factor"], s["low"], s["high"], s["original"]))
+            else:
+                assert (x.diff, x.keep_first) == (m["diff"], m["mask"]["keep_first"])
+        f = raw["mlp"]
+        if f is None:
+            assert lc.mlp is None
+        elif f["kind"] == "dense":
+            assert (lc.mlp.kind, lc.mlp.ff) == ("dense", f["ff"])
+        else:
+            assert (lc.mlp.ff, lc.mlp.experts, lc.mlp.top, lc.mlp.scale, lc.mlp.shared_ff) == \
+                (f["expert"]["ff"], f["router"]["experts"], f["router"]["top"], f["router"]["scale"], (f.get("shared") or {}).get("ff", 0))
+    assert c.to_dict() == cfg
+
+
+@pytest.mark.parametrize("change,word", [
+    (lambda c: c["layers"][0].update(type="mamba"), "mamba"),
+    (lambda c: c["layers"][0]["mixer"].update(kv_heads=4), "kv_heads"),
+    (lambda c: c["layers"][0]["mixer"].pop("diff"), "diff"),
+    (lambda c: c["layers"][1]["mixer"]["rot"].update(dims=5), "dims"),
+    (lambda c: c["layers"][1]["mixer"]["rot"].update(dims=12), "dims"),
+    (lambda c: c["layers"][1]["mixer"]["rot"]["scaling"].update(high=1.0), "high"),
+    (lambda c: c["layers"][1]["mlp"]["router"].update(top=6), "choices"),
+    (lambda c: c["layers"][2]["mixer"]["left"].update(kv_heads=3), "kv_heads"),
+    (lambda c: c["layers"][2]["mixer"]["left"].pop("bias_max"), "bias_max"),
+    (lambda c: c["layers"][2]["mixer"]["right"].update(decay=[0.5]), "decays"),
+    (lambda c: c["layers"][2]["mixer"]["right"].update(decay="0.5"), "decay"),
+    (lambda c: c["layers"][2]["mixer"].pop("left_scale"), "left_scale"),
+    (lambda c: c["layers"][2]["mlp"].update(kind="conv"), "conv"),
+    (lambda c: c["norm"].pop("eps"), "eps"),
+    (lambda c: c.pop("embedding"), "embedding"),
+    (lambda c: c.update(layers=[]), "layers"),
+])
+def test_configuration_errors_name_the_key(change, word):
+    from hf_cpu_amd.config import config_from_dict
+    from hf_cpu_amd.status import EngineError
+    cfg = copy.deepcopy(lh.SMALL)
+    change(cfg)
+    with pytest.raises(EngineError) as e:
+        config_from_dict(cfg)
+    assert word in str(e.value.msg)
+
+
+@pytest.mark.parametrize("name", list(lh.CONFIGS))
+def test_plan_declares_the_tensors_of_a_checkpoint(name):
+    from hf_cpu_amd.config import config_from_dict
+    from hf_cpu_amd.model import Model
+    cfg = lh.CONFIGS[name]
+    made = lh.make_weights(cfg, 0)
+    bare = copy.deepcopy(cfg)
+    for lc in bare["layers"]:                                  # without the optional key the table's rows are the tensor's
+        if lc["type"] == "parallel":
+            del lc["mixer"]["left"]["bias_rows"]
+    for c in (cfg, bare):
+        model = Model.from_config(config_from_dict(c))
+        declared = {s.name: s for s in model.param_specs()}
+        assert {n for n, s in declared.items() if not s.optional} == set(made)
+        for n in made:
+            assert len(declared[n].shape) == np.ndim(made[n]) and all(d in (0, e) for d, e in zip(declared[n].shape, np.shape(made[n]))), n
+        assert model.graph_safe and model.short_request_rows == 0
+    assert all(f"l{l}.norm2" in declared for l, lc in enumerate(cfg["layers"]) if lc["mlp"] is None)
+
+
+def test_first_tokens_keep_their_pages_beside_a_window():
+    from hf_cpu_amd.cache import CacheManager
+    from hf_cpu_amd.config import config_from_dict
+    from hf_cpu_amd.model import Model
+    from hf_cpu_amd.parts.base import FixedState, PagedKV
+    needs = Model.from_config(config_from_dict(lh.SMALL)).cache_needs()
+    paged = [n for n in needs if isinstance(n, PagedKV)]
+    assert [(n.k_width, n.v_width, n.window, n.mask_chunk, n.keep_first) for n in paged] == \
+        [(30, 21, 9, 0, 3), (10, 6, 7, 0, 0), (12, 18, 0, 11, 0), (24, 24, 1, 0, 0), (8, 8, 0, 33, 0), (18, 4, 13, 0, 17)]
+    assert len([n for n in needs if isinstance(n, FixedState)]) == 2
+    m = CacheManager(needs, 4, 40, 3, 96)
+    h = m.admit("a")
+    for _ in range(18):
+        m.reserve("a", 4)
+        m.commit("a", 4)
+    held = {(g.k_width, g.need.keep_first): [b for b, p in enumerate(h.tables[g.index]) if p >= 0] for g in m.groups}
+    assert held[(30, 3)] == [0, 16, 17] and held[(10, 0)] == [16, 17] and held[(12, 0)] == [16, 17] and held[(24, 0)] == []
+    assert held[(18, 17)] == [0, 1, 2, 3, 4, 15, 16, 17] and held[(8, 0)] == [16, 17]
+    m.check()
+    copies, _ = m.fork("a", "b")                               # a fork shares the kept pages and gives them back once
+    assert copies == []
+    m.release("a")
+    m.check()
+    assert [b for b, p in enumerate(m.held["b"].tables[m.entry_group[needs.index(paged[5])]]) if p >= 0] == [0, 1, 2, 3, 4, 15, 16, 17]
+    m.release("b")
+    m.check()
+    assert all(p.n_held == 0 for p in m.pools)
+    # more first tokens than the sequence has: nothing goes
+    m = CacheManager([PagedKV(4, 4, 3, keep_first=1000)], 4, 10, 1, 40)
+    m.admit("a")
+    for _ in range(10):
+        m.reserve("a", 4)
+        m.commit("a", 4)
+    assert m.pools[0].n_held == 10
