@@ -196,19 +196,21 @@ int hfa_delta_scan(const float* q, int ldq, const float* k, int ldk, int qk_head
 
 // Layers that norm a branch's result before it joins the stream, and what comes with them (sandwich.hip).
 // hfa_embed_pos: x[t] = table[tokens[t]] * scale + pos(positions[t]), pos[2i] = sin(p inv_freq[i]), pos[2i + 1] = cos(p inv_freq[i])
-// (positions null: no position vector).
+// (positions null: no position vector); copy (null: none) receives x in bf16.
 // hfa_rmsnorm_add: b = [y[r], or the sum of `splits` planes of partial sums] * sigmoid(row_gate[r]) + sum_k pairs[r * top + k] (each
 // part optional), times sigmoid(gate[r] + gate_bias) element by element; out[r] (+)= scale * b / sqrt(mean(b^2) + eps) * w (w null:
 // scale * b); copy (bf16, or null) receives the new out[r]. hfa_round_rows: an fp32 matrix in bf16.
 // hfa_polynorm: out = coef[0] N(z) + coef[1] N(z^2) + coef[2] N(z^3) + coef[3], N(u) = u / sqrt(mean(u^2) + eps) over a row.
 // hfa_scale_rows: x *= s. hfa_head_norm_store: rows [q | k | v]; q and k heads RMS-normed (norm_q, norm_k) with a weight
 // of one head's size (null: 1) and turned over their first rot_dim dimensions (cos_sin: hfa_rope_table's output, null: no rotation), the
-// norm before or (norm_after) after the rotation; q to q_out, k and v to cache rows slot_map[t] (values transposed inside their page).
+// norm before or (norm_after) after the rotation; q to q_out, k and v to cache rows slot_map[t] (values transposed inside their page); with
+// k_cache null there are no k heads and v goes to rows of v_out. Rows may be the partial sums of a deferred hfa_gemm ([splits][n_tokens]
+// [width] fp32 plus partial_bias). The n_extra columns behind v go to `extra` in fp32 (null: left alone).
 // hfa_diff_mix: a [T][G][2][H / G][v_head_dim] fp32, two maps of a head: out[t, h] = c d / sqrt(mean(d^2) + eps), d = map 1 - factor[0] map 2.
 // hfa_talk_mix: out[t, h] = sigmoid(gate[t, h]) * sum_g talk[h, g] cross[t, (c(h) - c(g)) mod G, g], cross from hfa_paged_attention
 // with cross_values.
 int hfa_embed_pos(const void* table, int table_dtype, const int* tokens, const int* positions, const float* inv_freq, float* x,
-                  int n_tokens, int width, int vocab, float scale, hipStream_t stream);
+                  int n_tokens, int width, int vocab, float scale, void* copy, hipStream_t stream);
 int hfa_rmsnorm_add(const float* y, int ldy, const float* partial, int splits, const float* row_gate, int ld_row_gate, const float* pairs,
                     int top, const void* gate, int gate_dtype, int ldg, const float* gate_bias, const float* w, float* out, int ldo,
                     void* copy, int ldc, int n_rows, int width, float eps, float scale, int accumulate, hipStream_t stream);
@@ -220,8 +222,9 @@ int hfa_polynorm(const void* z, int z_dtype, int ldz, const float* coef, void* o
 int hfa_scale_rows(float* x, int ld, int n_rows, int width, float s, hipStream_t stream);
 int hfa_head_norm_store(const void* qkv, int in_dtype, int ld, int n_heads, int n_kv_heads, int head_dim, int n_v_heads, int v_head_dim,
                         const float* q_w, const float* k_w, int norm_q, int norm_k, int norm_after, float eps, const float* cos_sin,
-                        int rot_dim, void* q_out, int ldq, void* k_cache, void* v_cache, int out_dtype, const int* slot_map,
-                        int page_tokens, int n_tokens, hipStream_t stream);
+                        int rot_dim, void* q_out, int ldq, void* k_cache, void* v_out, int ldv, int out_dtype, const int* slot_map,
+                        int page_tokens, int n_tokens, const float* partial, int splits, int width, const float* partial_bias,
+                        float* extra, int n_extra, int ld_extra, hipStream_t stream);
 int hfa_talk_mix(const void* cross, int cross_dtype, const float* talk, const void* gate, int gate_dtype, int ldg, void* out,
                  int out_dtype, int ldo, int n_tokens, int n_heads, int n_kv_heads, int v_head_dim, hipStream_t stream);
 
@@ -293,7 +296,8 @@ int hfa_softcap(float* x, int ld, int n_rows, int width, float cap, hipStream_t 
 // the softmax over the chosen logits alone); experts form n_groups equal runs of
 // neighbours of which the `keep` best (by their best expert) may be chosen from; weights = score (/ sum of the chosen
 // + 1e-20 if renorm) * out_scale. correction (one fp32 an expert, or null) is added to the scores for the choice alone, not for the
-// weights. hfa_moe_plan puts the n_pairs = n_tokens * top pairs in expert order (row_pair) and
+// weights. With splits > 0 the logits are the sums of that many planes [n_tokens][width] of a deferred hfa_gemm; columns n_experts ..
+// width - 1 then go to the logits' rows (which are written, not read). hfa_moe_plan puts the n_pairs = n_tokens * top pairs in expert order (row_pair) and
 // lists tiles of at most tile_rows rows of one expert (tiles: 3 ints a tile, room for n_pairs / tile_rows + n_experts;
 // *n_tiles on the device). hfa_moe_gemm: for every row r of the plan, out[o(r), :] = act(a[s(r), :] . w[e(r)]^T)
 // (* pair_scale[pair] if given); w is [n_experts][N][K] (bf16, or fp32 beside activations of either type); s(r) = row_pair[r] / a_div if a_div > 0 else r; o(r) =
@@ -301,8 +305,8 @@ int hfa_softcap(float* x, int ld, int n_rows, int width, float cap, hipStream_t 
 // hfa_moe_combine: x[t, :] += sum_k y[t * top + k, :]. `gated` 1 (N a multiple of 64, act 0): w's rows come in blocks of 32 gate rows
 // and 32 up rows, out has N / 2 columns, and with c = pair_scale of the row's pair (null: 1), g = min(c gate, limit), u = clamp(c up,
 // -limit, limit) (limit <= 0: unbounded): out = g sigmoid(alpha g) (u + shift), formed from the 32-bit sums in the product's last lines.
-int hfa_moe_route(const float* logits, int ld, int n_tokens, int n_experts, int top, int n_groups, int keep,
-                  int scoring, int renorm, float out_scale, const float* correction, int* ids, float* weights, hipStream_t stream);
+int hfa_moe_route(float* logits, int ld, int n_tokens, int n_experts, int top, int n_groups, int keep,
+                  int scoring, int renorm, float out_scale, const float* correction, const float* partial, int splits, int width, int* ids, float* weights, hipStream_t stream);
 int hfa_moe_plan(const int* ids, int n_pairs, int n_experts, int tile_rows, int* row_pair, int* tiles, int* n_tiles,
                  hipStream_t stream);
 // hfa_head_plan: the plan where every token chooses all n_heads "experts" in order (a product per head), without ids.

@@ -33,15 +33,63 @@ __device__ __forceinline__ void wave_best(float& v, int& i) {
 // form n_groups runs of neighbours, a run scores as its best expert, and only experts of the `keep` best runs can
 // be chosen; the `top` best of those are chosen, and weigh score / (sum of the chosen scores + 1e-20) if `renorm`,
 // else their score; times `out_scale`. `correction` (null: none) is added to the scores for the choice, not for the weights.
-__global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict__ logits, int ld, int E, int top,
+// With `splits` > 0 the logits lie in that many planes of partial sums (`partial`, rows of `width` columns), added in ascending
+// order here; the columns behind the experts' go to the rows of `logits`.
+__global__ __launch_bounds__(WAVE) void moe_route_kernel(float* __restrict__ logits, int ld, int E, int top,
                                                         int n_groups, int keep, int scoring, int renorm, float out_scale,
-                                                        const float* __restrict__ correction, int* __restrict__ ids, float* __restrict__ weights) {
+                                                        const float* __restrict__ correction, const float* __restrict__ partial, int splits,
+                                                        int width, int* __restrict__ ids, float* __restrict__ weights) {
     __shared__ float s[MOE_MAX_EXPERTS];
     __shared__ float gs[MOE_MAX_EXPERTS];
     __shared__ unsigned char open_s[MOE_MAX_EXPERTS];        // per group: may be chosen from
     __shared__ float plain_s[MOE_MAX_EXPERTS];               // the scores without the correction
     const int t = blockIdx.x, lane = threadIdx.x;
-    const float* z = logits + (size_t)t * ld;
+    float* z = logits + (size_t)t * ld;
+    if (splits > 0) {                                        // finish the product's sums (a lane reads back what it wrote)
+        const float* src = partial + (size_t)t * width;
+        const size_t plane = (size_t)gridDim.x * width;
+        for (int e = lane; e < width; e += WAVE) {
+            float v = 0.f;
+            for (int s0 = 0; s0 < splits; s0 += 8) {
+                float q[8];
+#pragma unroll
+                for (int u = 0; u < 8; u++) q[u] = s0 + u < splits ? src[(s0 + u) * plane + e] : 0.f;
+#pragma unroll
+                for (int u = 0; u < 8; u++) v += q[u];
+            }
+            z[e] = v;
+        }
+    }
+    if (E <= WAVE && keep >= n_groups) {                     // an expert a lane: nothing leaves the registers
+        const bool mine = lane < E;
+        const float zl = mine ? z[lane] : -INFINITY;
+        float sc;
+        if (scoring == 1) {
+            sc = 1.0f / (1.0f + expf(-zl));
+        } else {
+            const float m = wave_max(zl);
+            sc = mine ? expf(zl - m) : 0.f;
+            if (scoring == 0) sc = sc / wave_sum(sc);
+        }
+        float rank = !mine ? -INFINITY : correction ? sc + correction[lane] : sc;
+        float chosen = 0.f, my_w = 0.f;
+        int my_id = 0;
+        for (int r = 0; r < top; r++) {
+            float bv = rank > -INFINITY ? rank : -INFINITY;  // (a score that is no number is never chosen)
+            int bi = bv > -INFINITY ? lane : 0x7fffffff;
+            wave_best(bv, bi);
+            const bool none = bi >= E;                       // fewer experts than choices: weight nothing
+            const float wv = none ? 0.f : __shfl(sc, none ? 0 : bi, WAVE);
+            if (lane == bi) rank = -INFINITY;                // taken
+            if (lane == r) { my_w = wv; my_id = none ? 0 : bi; }
+            chosen += wv;
+        }
+        if (lane < top) {
+            ids[(size_t)t * top + lane] = my_id;
+            weights[(size_t)t * top + lane] = (renorm ? my_w / (chosen + 1e-20f) : my_w) * out_scale;
+        }
+        return;
+    }
     if (scoring == 0) {
         float m = -INFINITY;
         for (int e = lane; e < E; e += WAVE) m = fmaxf(m, z[e]);
@@ -112,16 +160,19 @@ __global__ __launch_bounds__(WAVE) void moe_route_kernel(const float* __restrict
     }
 }
 
-extern "C" int hfa_moe_route(const float* logits, int ld, int n_tokens, int n_experts, int top, int n_groups, int keep,
-                             int scoring, int renorm, float out_scale, const float* correction, int* ids, float* weights, hipStream_t stream) {
+extern "C" int hfa_moe_route(float* logits, int ld, int n_tokens, int n_experts, int top, int n_groups, int keep,
+                             int scoring, int renorm, float out_scale, const float* correction, const float* partial, int splits,
+                             int width, int* ids, float* weights, hipStream_t stream) {
     HFA_REQUIRE(logits && ids && weights && n_tokens > 0, "moe_route: bad arguments");
     HFA_REQUIRE(n_experts > 0 && n_experts <= MOE_MAX_EXPERTS && ld >= n_experts, "moe_route: %d experts (at most %d)", n_experts,
                 MOE_MAX_EXPERTS);
     HFA_REQUIRE(top > 0 && top <= WAVE && top <= n_experts, "moe_route: %d choices of %d experts (at most %d)", top, n_experts, WAVE);
     HFA_REQUIRE(n_groups > 0 && n_experts % n_groups == 0 && keep > 0 && keep <= n_groups,
                 "moe_route: %d experts do not form %d equal groups of which %d are kept", n_experts, n_groups, keep);
+    HFA_REQUIRE(splits >= 0 && (splits == 0 || (partial && width >= n_experts && ld >= width)), "moe_route: partial sums of rows shorter than the experts");
     HFA_REQUIRE(scoring >= 0 && scoring <= 2, "moe_route: unknown scoring %d", scoring);
-    moe_route_kernel<<<n_tokens, WAVE, 0, stream>>>(logits, ld, n_experts, top, n_groups, keep, scoring, renorm, out_scale, correction, ids,
+    moe_route_kernel<<<n_tokens, WAVE, 0, stream>>>(logits, ld, n_experts, top, n_groups, keep, scoring, renorm, out_scale, correction,
+                                                    partial, splits, width, ids,
                                                     weights);
     HFA_LAUNCH_CHECK("moe_route");
     return 0;

@@ -8,7 +8,7 @@
 //   hfa_polynorm          out = a N(z) + b N(z^2) + c N(z^3) + e, N dividing a row by its root mean square
 //   hfa_scale_rows        x *= s
 //   hfa_head_norm_store   per head: q, k <- rms norm (with a weight of one head's size, shared, or none) before or after a
-//                         rotation; q to a matrix, k and v to their cache rows
+//                         rotation; q to a matrix, k and v to their cache rows (or, without keys, v to a matrix)
 //   hfa_diff_mix          out[t, h] = c * a / rms(a), a = map 1 of head h minus a factor times map 2
 //   hfa_round_rows        an fp32 matrix in bf16
 //   hfa_talk_mix          out[t, h] = sigmoid(gate[t, h]) * sum_g talk[h, g] * A[t, g, values of h's group]
@@ -20,7 +20,8 @@
 // from 64-bit on the host); the angle is one fp32 product.
 template <typename T>
 __global__ void embed_pos_kernel(const T* __restrict__ table, const int* __restrict__ tokens, const int* __restrict__ positions,
-                                 const float* __restrict__ inv_freq, float* __restrict__ x, int width, int vocab, float scale) {
+                                 const float* __restrict__ inv_freq, float* __restrict__ x, int width, int vocab, float scale,
+                                 uint16_t* __restrict__ copy) {
     const int t = blockIdx.x;
     int tok = tokens[t];
     tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);
@@ -34,18 +35,19 @@ __global__ void embed_pos_kernel(const T* __restrict__ table, const int* __restr
             v += (i & 1) ? cosf(ang) : sinf(ang);
         }
         dst[i] = v;
+        if (copy) copy[(size_t)t * width + i] = bf16_bits(v);
     }
 }
 
 extern "C" int hfa_embed_pos(const void* table, int table_dtype, const int* tokens, const int* positions, const float* inv_freq,
-                             float* x, int n_tokens, int width, int vocab, float scale, hipStream_t stream) {
+                             float* x, int n_tokens, int width, int vocab, float scale, void* copy, hipStream_t stream) {
     HFA_REQUIRE(table && tokens && x && n_tokens > 0 && width > 0 && vocab > 0, "embed_pos: bad arguments");
     HFA_REQUIRE(!positions || inv_freq, "embed_pos: positions come with their frequencies");
     HFA_REQUIRE(table_dtype == HFA_F32 || table_dtype == HFA_BF16, "embed_pos: unknown dtype %d", table_dtype);
     if (table_dtype == HFA_F32)
-        embed_pos_kernel<float><<<n_tokens, 256, 0, stream>>>((const float*)table, tokens, positions, inv_freq, x, width, vocab, scale);
+        embed_pos_kernel<float><<<n_tokens, 256, 0, stream>>>((const float*)table, tokens, positions, inv_freq, x, width, vocab, scale, (uint16_t*)copy);
     else
-        embed_pos_kernel<bf16><<<n_tokens, 256, 0, stream>>>((const bf16*)table, tokens, positions, inv_freq, x, width, vocab, scale);
+        embed_pos_kernel<bf16><<<n_tokens, 256, 0, stream>>>((const bf16*)table, tokens, positions, inv_freq, x, width, vocab, scale, (uint16_t*)copy);
     HFA_LAUNCH_CHECK("embed_pos");
     return 0;
 }
@@ -134,6 +136,15 @@ __global__ __launch_bounds__(1024) void rmsnorm_add_kernel(JoinArgs p) {
         return b;
     };
     const int stride = blockDim.x * VW, c0 = threadIdx.x * VW;
+    float* dst = p.out + (size_t)r * p.ldo;
+    // what the last lines need from memory is asked for with the branch, so that no trip waits behind the block's sum
+    JoinVec<VW> old[KEEP], wv[KEEP];
+#pragma unroll
+    for (int k = 0; k < KEEP; k++) {
+        const int c = c0 + k * stride;
+        old[k] = p.accumulate && c < p.width ? join_load<VW>(dst + c) : JoinVec<VW>{};
+        wv[k] = p.w && c < p.width ? join_load<VW>(p.w + c) : JoinVec<VW>{};
+    }
     float ss = 0.f;
 #pragma unroll
     for (int k = 0; k < KEEP; k++) {
@@ -148,12 +159,10 @@ __global__ __launch_bounds__(1024) void rmsnorm_add_kernel(JoinArgs p) {
         for (int e = 0; e < VW; e++) ss = fmaf(b.v[e], b.v[e], ss);
     }
     const float inv = p.w ? p.scale / sqrtf(block_sum(ss, red) / (float)p.width + p.eps) : p.scale;
-    float* dst = p.out + (size_t)r * p.ldo;
-    auto finish = [&](int c, const JoinVec<VW>& b) {
-        JoinVec<VW> z, o = {};
-        if (p.accumulate) o = join_load<VW>(dst + c);
+    auto finish = [&](int c, const JoinVec<VW>& b, const JoinVec<VW>& o, const JoinVec<VW>& w) {
+        JoinVec<VW> z;
 #pragma unroll
-        for (int e = 0; e < VW; e++) z.v[e] = o.v[e] + (p.w ? b.v[e] * inv * p.w[c + e] : b.v[e] * inv);
+        for (int e = 0; e < VW; e++) z.v[e] = o.v[e] + (p.w ? b.v[e] * inv * w.v[e] : b.v[e] * inv);
         if constexpr (VW == 4) {
             *reinterpret_cast<float4*>(dst + c) = make_float4(z.v[0], z.v[1], z.v[2], z.v[3]);
             if (p.copy)
@@ -168,9 +177,10 @@ __global__ __launch_bounds__(1024) void rmsnorm_add_kernel(JoinArgs p) {
 #pragma unroll
     for (int k = 0; k < KEEP; k++) {
         const int c = c0 + k * stride;
-        if (c < p.width) finish(c, keep[k]);
+        if (c < p.width) finish(c, keep[k], old[k], wv[k]);
     }
-    for (int c = c0 + KEEP * stride; c < p.width; c += stride) finish(c, value(c));
+    for (int c = c0 + KEEP * stride; c < p.width; c += stride)
+        finish(c, value(c), p.accumulate ? join_load<VW>(dst + c) : JoinVec<VW>{}, p.w ? join_load<VW>(p.w + c) : JoinVec<VW>{});
 }
 
 extern "C" int hfa_rmsnorm_add(const float* y, int ldy, const float* partial, int splits, const float* row_gate, int ld_row_gate,
@@ -183,7 +193,7 @@ extern "C" int hfa_rmsnorm_add(const float* y, int ldy, const float* partial, in
     HFA_REQUIRE(gate || !gate_bias, "rmsnorm_add: a gate's bias without the gate");
     const JoinArgs p = {y, ldy, partial, splits, (size_t)n_rows * width, row_gate, ld_row_gate, pairs, top, gate, gate && gate_dtype == HFA_BF16,
                         ldg, gate_bias, w, out, ldo, (uint16_t*)copy, ldc, width, eps, scale, accumulate};
-    const bool vec = width % 4 == 0 && (!y || (ldy % 4 == 0 && ((uintptr_t)y & 15) == 0)) && ((uintptr_t)partial & 15) == 0 && ((uintptr_t)pairs & 15) == 0 &&
+    const bool vec = width % 4 == 0 && ((uintptr_t)w & 15) == 0 && (!y || (ldy % 4 == 0 && ((uintptr_t)y & 15) == 0)) && ((uintptr_t)partial & 15) == 0 && ((uintptr_t)pairs & 15) == 0 &&
                      ldo % 4 == 0 && ((uintptr_t)out & 15) == 0 && (!copy || (ldc % 4 == 0 && ((uintptr_t)copy & 7) == 0));
     if (vec) {
         // few rows: a row's loads are shared by as many threads as it has groups of four columns
@@ -275,11 +285,12 @@ extern "C" int hfa_scale_rows(float* x, int ld, int n_rows, int width, float s, 
 }
 
 // ---- queries and keys normed head by head; keys and values to the cache ------------------------------------------------
-// Rows [q: H D | k: G D | v: GV Dv] (fp32 or bf16). Every q head and every k head is (norm_q, norm_k) divided by sqrt(mean(head^2) +
-// eps) and multiplied by a weight of D values that all heads share (q_w, k_w; null: 1), and (cs not null) its first rot_dim
-// dimensions are turned, i with i + rot_dim / 2, by the token's angles (cs: hfa_rope_table's rows [cosines | sines]); norm_after:
-// the rotation comes first and the norm after it. q goes to q_out ([T, H D], the cache's dtype), k to cache row slot_map[t], v to
-// the same row with the page transposed ([page][column][offset]).
+// Rows [q: H D | k: G D | v: GV Dv | extra] (fp32, bf16, or the partial sums of a product whose K was split, plus its bias). Every q
+// head and every k head is (norm_q, norm_k) divided by sqrt(mean(head^2) + eps) and multiplied by a weight of D values that all heads
+// share (q_w, k_w; null: 1), and (cs not null) its first rot_dim dimensions are turned, i with i + rot_dim / 2, by the token's angles
+// (cs: hfa_rope_table's rows [cosines | sines]); norm_after: the rotation comes first and the norm after it. q goes to q_out ([T, H D]),
+// k to cache row slot_map[t], v to the same row with the page transposed ([page][column][offset]); without a cache (k_cache null) there
+// are no k heads and v goes to v_rows ([T, GV Dv]). The extra columns go to `extra` in fp32 (null: they are left alone).
 struct HeadNorm {
     int H, G, D, GV, Dv;
     const float* q_w; const float* k_w;
@@ -287,11 +298,64 @@ struct HeadNorm {
     float eps;
     const float* cs; int rot_dim;
     const int* slot_map; int page_tokens;
+    const float* partial; int splits, width; size_t plane;       // partial sums: [splits][T][width], or null
+    const float* bias;                                           // [width], with partial sums
+    float* extra; int n_extra, ld_extra;
+    int ldv;                                                     // of v_rows
 };
+
+template <typename TI>
+struct HeadRow {
+    const TI* row;
+    const float* sums;               // the token's row of the first plane, or null
+    const HeadNorm* p;
+    __device__ __forceinline__ float at(int c) const {
+        if (!sums) return to_f32(row[c]);
+        if (p->splits == 1) return p->bias ? sums[c] + p->bias[c] : sums[c];
+        float v = 0.f;
+        for (int s0 = 0; s0 < p->splits; s0 += JOIN_PLANES) {    // batches of loads that do not wait for one another
+            float q[JOIN_PLANES];
+#pragma unroll
+            for (int u = 0; u < JOIN_PLANES; u++) q[u] = s0 + u < p->splits ? sums[(s0 + u) * p->plane + c] : 0.f;
+#pragma unroll
+            for (int u = 0; u < JOIN_PLANES; u++) v += q[u];
+        }
+        return p->bias ? v + p->bias[c] : v;
+    }
+    // eight neighbouring columns (c a multiple of 8, operands on 16 bytes)
+    __device__ __forceinline__ void at8(int c, float (&v)[8]) const {
+        if (sums) {
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[e] = p->bias ? p->bias[c + e] : 0.f;
+            for (int s = 0; s < p->splits; s++) {
+                const float4 a = *reinterpret_cast<const float4*>(sums + s * p->plane + c);
+                const float4 b = *reinterpret_cast<const float4*>(sums + s * p->plane + c + 4);
+                v[0] += a.x; v[1] += a.y; v[2] += a.z; v[3] += a.w;
+                v[4] += b.x; v[5] += b.y; v[6] += b.z; v[7] += b.w;
+            }
+        } else if constexpr (sizeof(TI) == 2) {
+            const uint4 u = *reinterpret_cast<const uint4*>(row + c);
+            const uint32_t w[4] = {u.x, u.y, u.z, u.w};
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                v[2 * e] = __uint_as_float(w[e] << 16);
+                v[2 * e + 1] = __uint_as_float(w[e] & 0xffff0000u);
+            }
+        } else {
+            const float4 a = *reinterpret_cast<const float4*>(row + c), b = *reinterpret_cast<const float4*>(row + c + 4);
+            v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+            v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+        }
+    }
+};
+template <typename TI>
+__device__ __forceinline__ HeadRow<TI> head_row(const TI* qkv, int ld, const HeadNorm& p, int t) {
+    return {qkv + (size_t)t * ld, p.partial ? p.partial + (size_t)t * p.width : nullptr, &p};
+}
 
 // One head's values by S neighbouring lanes (a power of two), D <= S NE: lane l holds values l, l + S, ...
 template <typename TI, int S, int NE>
-__device__ __forceinline__ void normed_head(const TI* __restrict__ src, const HeadNorm& p, bool is_key, int t, int l, float (&v)[NE]) {
+__device__ __forceinline__ void normed_head(const HeadRow<TI>& src, int first, const HeadNorm& p, bool is_key, int t, int l, float (&v)[NE]) {
     const int half = p.rot_dim / 2;
     const float* cs = p.cs ? p.cs + (size_t)t * p.rot_dim : nullptr;
     const float* w = is_key ? p.k_w : p.q_w;
@@ -300,8 +364,8 @@ __device__ __forceinline__ void normed_head(const TI* __restrict__ src, const He
 #pragma unroll
     for (int i = 0; i < NE; i++) {
         const int c = l + i * S;
-        v[i] = c < p.D ? to_f32(src[c]) : 0.f;
-        other[i] = cs && c < p.rot_dim ? to_f32(src[c < half ? c + half : c - half]) : 0.f;
+        v[i] = c < p.D ? src.at(first + c) : 0.f;
+        other[i] = cs && c < p.rot_dim ? src.at(first + (c < half ? c + half : c - half)) : 0.f;
     }
     float ss = 0.f;
     auto turn = [&](float x, float y, int c) {              // c's place in its pair decides the sign
@@ -338,50 +402,191 @@ __device__ __forceinline__ void normed_head(const TI* __restrict__ src, const He
     }
 }
 
-// A block of four waves a token and 4 * 64 / S heads; the blocks of a token share its values out.
+// A block of four waves a token and 4 * 64 / S heads; the blocks of a token share its values and extra columns out.
 template <typename TI, typename TO, int S, int NE>
 __global__ __launch_bounds__(256) void head_norm_store_kernel(const TI* __restrict__ qkv, int ld, HeadNorm p, TO* __restrict__ q_out, int ldq,
-                                                             TO* __restrict__ k_cache, TO* __restrict__ v_cache) {
+                                                             TO* __restrict__ k_cache, TO* __restrict__ v_out) {
     const int t = blockIdx.x, l = threadIdx.x % S, H = p.H, G = p.G, D = p.D;
-    const TI* row = qkv + (size_t)t * ld;
+    const HeadRow<TI> row = head_row(qkv, ld, p, t);
     const int KD = G * D, VD = p.GV * p.Dv;
-    const int slot = p.slot_map[t];
+    const int slot = p.slot_map ? p.slot_map[t] : 0;
     const int hs = blockIdx.y * (256 / S) + threadIdx.x / S;
     // (every lane of a wave takes part in the sums; lanes beyond the last head repeat it and store nothing)
     const int hc = hs < H + G ? hs : H + G - 1;
     float v[NE];
-    normed_head<TI, S, NE>(row + hc * D, p, hc >= H, t, l, v);
+    normed_head<TI, S, NE>(row, hc * D, p, hc >= H, t, l, v);
     if (hs < H + G) {
         TO* dst = hs >= H ? k_cache + (size_t)slot * KD + (hs - H) * D : q_out + (size_t)t * ldq + hs * D;
 #pragma unroll
         for (int i = 0; i < NE; i++)
             if (l + i * S < D) dst[l + i * S] = from_f32<TO>(v[i]);
     }
-    for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < VD; c += gridDim.y * blockDim.x)
-        v_cache[(size_t)(slot / p.page_tokens) * p.page_tokens * VD + (size_t)c * p.page_tokens + slot % p.page_tokens] =
-            from_f32<TO>(to_f32(row[(H + G) * D + c]));
+    const int v0 = (H + G) * D;
+    for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < VD; c += gridDim.y * blockDim.x) {
+        const size_t at = k_cache ? (size_t)(slot / p.page_tokens) * p.page_tokens * VD + (size_t)c * p.page_tokens + slot % p.page_tokens
+                                  : (size_t)t * p.ldv + c;
+        v_out[at] = from_f32<TO>(row.at(v0 + c));
+    }
+    if (p.extra)
+        for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < p.n_extra; c += gridDim.y * blockDim.x)
+            p.extra[(size_t)t * p.ld_extra + c] = row.at(v0 + VD + c);
+}
+
+// The same for prompt portions: HEAD_SHARES blocks take eight consecutive tokens, a share of the heads and of the values each; a head lies over L = D / 8 neighbouring lanes (4, 8 or 16) with
+// eight values each, the other halves of its pairs come from the lanes that hold them, and the values of the eight tokens go
+// through LDS, so that where the tokens' cache rows are neighbours on one page every value column is one 16-byte store.
+#define HEAD_TOKENS 8
+#define HEAD_SHARES 4
+template <typename TO>
+__device__ __forceinline__ void store8(TO* dst, const float (&v)[8]) {
+    if constexpr (sizeof(TO) == 2) {
+        uint32_t w[4];
+#pragma unroll
+        for (int e = 0; e < 4; e++) w[e] = (uint32_t)bf16_bits(v[2 * e]) | ((uint32_t)bf16_bits(v[2 * e + 1]) << 16);
+        *reinterpret_cast<uint4*>(dst) = make_uint4(w[0], w[1], w[2], w[3]);
+    } else {
+        *reinterpret_cast<float4*>(dst) = make_float4(v[0], v[1], v[2], v[3]);
+        *reinterpret_cast<float4*>(dst + 4) = make_float4(v[4], v[5], v[6], v[7]);
+    }
+}
+
+template <typename TI, typename TO, int L>
+__global__ __launch_bounds__(256) void head_norm_rows_kernel(const TI* __restrict__ qkv, int ld, HeadNorm p, TO* __restrict__ q_out, int ldq,
+                                                            TO* __restrict__ k_cache, TO* __restrict__ v_out, int n_tokens) {
+    extern __shared__ __attribute__((aligned(16))) uint16_t head_vt[];               // [HEAD_TOKENS][this block's values]
+    constexpr int D = 8 * L, PER = 256 / L;
+    const int t0 = blockIdx.x * HEAD_TOKENS, nt = n_tokens - t0 < HEAD_TOKENS ? n_tokens - t0 : HEAD_TOKENS;
+    const int tid = threadIdx.x, l = tid % L, H = p.H, G = p.G, KD = G * D, VD = p.GV * p.Dv, v0 = (H + G) * D;
+    const int half = p.rot_dim / 2, lanes_half = half / 8;                           // (half is a multiple of 8)
+    const int heads = H + G, n_items = nt * heads;
+    const bool turns = p.cs != nullptr && 8 * l < p.rot_dim, low = l < lanes_half;
+    const int partner = low ? l + lanes_half : l - lanes_half;
+    for (int i0 = blockIdx.y * PER; i0 < n_items; i0 += PER * HEAD_SHARES) {                                      // (uniform: every lane takes part in the exchanges)
+        const int item = i0 + tid / L, it = item < n_items ? item : n_items - 1;
+        const int t = t0 + it / heads, hs = it % heads;
+        const bool is_key = hs >= H;
+        const float* w = is_key ? p.k_w : p.q_w;
+        const bool norm = is_key ? p.norm_k : p.norm_q;
+        float v[8];
+        head_row(qkv, ld, p, t).at8(hs * D + 8 * l, v);
+        auto turn = [&]() {
+            float o[8];
+#pragma unroll
+            for (int e = 0; e < 8; e++) o[e] = __shfl(v[e], turns ? partner : l, L);
+            if (turns) {
+                const float* cs = p.cs + (size_t)t * p.rot_dim + 8 * (low ? l : l - lanes_half);
+                float cv[8], sv[8];
+#pragma unroll
+                for (int u = 0; u < 2; u++) {
+                    *reinterpret_cast<float4*>(cv + 4 * u) = *reinterpret_cast<const float4*>(cs + 4 * u);
+                    *reinterpret_cast<float4*>(sv + 4 * u) = *reinterpret_cast<const float4*>(cs + half + 4 * u);
+                }
+#pragma unroll
+                for (int e = 0; e < 8; e++) v[e] = low ? v[e] * cv[e] - o[e] * sv[e] : v[e] * cv[e] + o[e] * sv[e];
+            }
+        };
+        if (p.cs && (p.norm_after || !norm)) turn();
+        if (norm) {
+            float ss = 0.f;
+#pragma unroll
+            for (int e = 0; e < 8; e++) ss = fmaf(v[e], v[e], ss);
+#pragma unroll
+            for (int off = L / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, L);
+            const float inv = 1.0f / sqrtf(ss / (float)D + p.eps);
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[e] *= inv * (w ? w[8 * l + e] : 1.f);
+            if (p.cs && !p.norm_after) turn();
+        }
+        if (item < n_items) {
+            TO* dst = is_key ? k_cache + (size_t)p.slot_map[t] * KD + (hs - H) * D : q_out + (size_t)t * ldq + hs * D;
+            store8(dst + 8 * l, v);
+        }
+    }
+    if (p.extra)
+        for (int i = blockIdx.y * 256 + tid; i < nt * p.n_extra; i += 256 * HEAD_SHARES)
+            p.extra[(size_t)(t0 + i / p.n_extra) * p.ld_extra + i % p.n_extra] = head_row(qkv, ld, p, t0 + i / p.n_extra).at(v0 + VD + i % p.n_extra);
+    // this block's columns of the values: v8 groups of eight from cv on
+    const int all8 = VD / 8, share8 = (all8 + HEAD_SHARES - 1) / HEAD_SHARES, cv = (int)blockIdx.y * share8 * 8;
+    const int v8 = all8 - cv / 8 < share8 ? all8 - cv / 8 : share8;
+    if (v8 <= 0) return;                                                             // (uniform over the block)
+    if (!k_cache) {
+        for (int i = tid; i < nt * v8; i += 256) {
+            const int t = t0 + i / v8, c = cv + i % v8 * 8;
+            float v[8];
+            head_row(qkv, ld, p, t).at8(v0 + c, v);
+            store8(v_out + (size_t)t * p.ldv + c, v);
+        }
+        return;
+    }
+    if constexpr (sizeof(TO) == 2) {                                                 // (values into a cache: 16 bits only, see the launcher)
+        for (int i = tid; i < nt * v8; i += 256) {
+            float v[8];
+            head_row(qkv, ld, p, t0 + i / v8).at8(v0 + cv + i % v8 * 8, v);
+            store8(reinterpret_cast<TO*>(head_vt) + i / v8 * (8 * share8) + i % v8 * 8, v);
+        }
+        __shared__ int slots[HEAD_TOKENS];
+        if (tid < HEAD_TOKENS) slots[tid] = tid < nt ? p.slot_map[t0 + tid] : -1;
+        __syncthreads();
+        const int P = p.page_tokens;
+        bool run = nt == HEAD_TOKENS && P % 8 == 0 && slots[0] % 8 == 0;
+        for (int t = 1; run && t < HEAD_TOKENS; t++) run = slots[t] == slots[0] + t;
+        uint16_t* vc = reinterpret_cast<uint16_t*>(v_out);
+        if (run) {
+            uint16_t* page = vc + (size_t)(slots[0] / P) * P * VD + (size_t)cv * P + slots[0] % P;
+            for (int c = tid; c < 8 * v8; c += 256) {
+                uint16_t x[HEAD_TOKENS];
+#pragma unroll
+                for (int t = 0; t < HEAD_TOKENS; t++) x[t] = head_vt[t * 8 * share8 + c];
+                *reinterpret_cast<uint4*>(page + (size_t)c * P) =
+                    make_uint4(x[0] | ((uint32_t)x[1] << 16), x[2] | ((uint32_t)x[3] << 16), x[4] | ((uint32_t)x[5] << 16), x[6] | ((uint32_t)x[7] << 16));
+            }
+        } else {
+            for (int i = tid; i < nt * 8 * v8; i += 256) {
+                const int t = i / (8 * v8), c = i % (8 * v8), slot = slots[t];
+                vc[(size_t)(slot / P) * P * VD + (size_t)(cv + c) * P + slot % P] = head_vt[t * 8 * share8 + c];
+            }
+        }
+    }
 }
 
 extern "C" int hfa_head_norm_store(const void* qkv, int in_dtype, int ld, int n_heads, int n_kv_heads, int head_dim, int n_v_heads, int v_head_dim,
                                    const float* q_w, const float* k_w, int norm_q, int norm_k, int norm_after, float eps, const float* cos_sin,
-                                   int rot_dim, void* q_out, int ldq, void* k_cache, void* v_cache, int out_dtype, const int* slot_map,
-                                   int page_tokens, int n_tokens, hipStream_t stream) {
-    HFA_REQUIRE(qkv && q_out && k_cache && v_cache && slot_map && n_tokens > 0 && n_heads > 0 && n_kv_heads > 0 && head_dim > 0 &&
-                    n_v_heads > 0 && v_head_dim > 0 && page_tokens > 0, "head_norm_store: bad arguments");
-    HFA_REQUIRE(ld >= (n_heads + n_kv_heads) * head_dim + n_v_heads * v_head_dim && ldq >= n_heads * head_dim,
-                "head_norm_store: a row is shorter than its heads");
+                                   int rot_dim, void* q_out, int ldq, void* k_cache, void* v_out, int ldv, int out_dtype, const int* slot_map,
+                                   int page_tokens, int n_tokens, const float* partial, int splits, int width, const float* partial_bias,
+                                   float* extra, int n_extra, int ld_extra, hipStream_t stream) {
+    HFA_REQUIRE(qkv && q_out && v_out && n_tokens > 0 && n_heads > 0 && head_dim > 0 && n_v_heads > 0 && v_head_dim > 0, "head_norm_store: bad arguments");
+    HFA_REQUIRE(k_cache ? n_kv_heads > 0 && slot_map && page_tokens > 0 : n_kv_heads == 0 && ldv >= n_v_heads * v_head_dim,
+                "head_norm_store: keys need a cache and its rows; without a cache there are none, and the values' rows have a stride");
+    const int used = (n_heads + n_kv_heads) * head_dim + n_v_heads * v_head_dim + (extra ? n_extra : 0);
+    HFA_REQUIRE(ld >= used && ldq >= n_heads * head_dim && (!extra || (n_extra > 0 && ld_extra >= n_extra)), "head_norm_store: a row is shorter than its heads");
+    HFA_REQUIRE(!partial || (splits > 0 && width >= used), "head_norm_store: partial sums of rows shorter than their heads");
     HFA_REQUIRE((in_dtype == HFA_F32 || in_dtype == HFA_BF16) && (out_dtype == HFA_F32 || out_dtype == HFA_BF16),
                 "head_norm_store: unknown dtype");
     HFA_REQUIRE(head_dim <= 1024 && (!cos_sin || (rot_dim > 0 && rot_dim % 2 == 0 && rot_dim <= head_dim)),
                 "head_norm_store: heads of %d values (at most 1024), of which an even number within the head is turned", head_dim);
+    const int vd = n_v_heads * v_head_dim;
     const HeadNorm p = {n_heads, n_kv_heads, head_dim, n_v_heads, v_head_dim, q_w, k_w, norm_q, norm_k, norm_after, eps, cos_sin,
-                        cos_sin ? rot_dim : 0, slot_map, page_tokens};
+                        cos_sin ? rot_dim : 0, slot_map, page_tokens > 0 ? page_tokens : 1, partial, splits, width, (size_t)n_tokens * width, partial_bias,
+                        extra, n_extra, ld_extra, ldv};
+    // eight tokens a block: prompt-sized calls whose rows are made of 16-byte pieces
+    const int in_step = in_dtype == HFA_F32 ? 4 : 8, out_step = out_dtype == HFA_F32 ? 4 : 8;
+    const bool rows = n_tokens >= 512 && (head_dim == 32 || head_dim == 64 || head_dim == 128) && v_head_dim * n_v_heads % 8 == 0 && p.rot_dim % 16 == 0 &&
+                      (k_cache == nullptr || (out_dtype == HFA_BF16 && (vd / 8 + HEAD_SHARES - 1) / HEAD_SHARES * 8 * HEAD_TOKENS * 2 <= (48 << 10))) &&
+                      (partial ? width % 4 == 0 && ((uintptr_t)partial & 15) == 0 : ld % in_step == 0 && ((uintptr_t)qkv & 15) == 0) &&
+                      ldq % out_step == 0 && (k_cache || ldv % out_step == 0) && (((uintptr_t)q_out | (uintptr_t)k_cache | (uintptr_t)v_out | (uintptr_t)cos_sin) & 15) == 0;
+#define HNR(TI, TO, L)                                                                                                                \
+    head_norm_rows_kernel<TI, TO, L><<<dim3((n_tokens + HEAD_TOKENS - 1) / HEAD_TOKENS, HEAD_SHARES), 256,                          \
+                                           k_cache ? (vd / 8 + HEAD_SHARES - 1) / HEAD_SHARES * 8 * HEAD_TOKENS * 2 : 0, stream>>>(   \
+        (const TI*)qkv, ld, p, (TO*)q_out, ldq, (TO*)k_cache, (TO*)v_out, n_tokens)
 #define HNS(TI, TO, S, NE)                                                                                                       \
     head_norm_store_kernel<TI, TO, S, NE><<<dim3(n_tokens, (n_heads + n_kv_heads + 256 / S - 1) / (256 / S)), 256, 0, stream>>>(     \
-        (const TI*)qkv, ld, p, (TO*)q_out, ldq, (TO*)k_cache, (TO*)v_cache)
+        (const TI*)qkv, ld, p, (TO*)q_out, ldq, (TO*)k_cache, (TO*)v_out)
 #define HNS_SIZES(TI, TO)                            \
     do {                                             \
-        if (head_dim <= 32) HNS(TI, TO, 16, 2);      \
+        if (rows && head_dim == 32) HNR(TI, TO, 4);  \
+        else if (rows && head_dim == 64) HNR(TI, TO, 8); \
+        else if (rows) HNR(TI, TO, 16);              \
+        else if (head_dim <= 32) HNS(TI, TO, 16, 2); \
         else if (head_dim <= 64) HNS(TI, TO, 32, 2); \
         else if (head_dim <= 128) HNS(TI, TO, 64, 2); \
         else if (head_dim <= 256) HNS(TI, TO, 64, 4); \
@@ -391,6 +596,7 @@ extern "C" int hfa_head_norm_store(const void* qkv, int in_dtype, int ld, int n_
     else { if (out_dtype == HFA_F32) HNS_SIZES(bf16, float); else HNS_SIZES(bf16, bf16); }
 #undef HNS_SIZES
 #undef HNS
+#undef HNR
     HFA_LAUNCH_CHECK("head_norm_store");
     return 0;
 }

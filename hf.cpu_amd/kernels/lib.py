@@ -33,13 +33,13 @@ _SIGNATURES = {
     "hfa_channel_decay": [P, I, I, P, I, P, F, P, I, I, I, P],
     "hfa_group_rmsnorm": [P, I, I, P, P, I, I, P, I, I, I, F, P, I, I, I, P, P],
     "hfa_delta_scan": [P, I, P, I, I, I, P, I, I, I, P, I, P, P, P, I, F, F, P, c_size_t, P, P, I, I, P, I, P],
-    "hfa_embed_pos": [P, I, P, P, P, P, I, I, I, F, P],
+    "hfa_embed_pos": [P, I, P, P, P, P, I, I, I, F, P, P],
     "hfa_rmsnorm_add": [P, I, P, I, P, I, P, I, P, I, I, P, P, P, I, P, I, I, I, F, F, I, P],
     "hfa_round_rows": [P, I, P, I, I, I, P],
     "hfa_diff_mix": [P, I, P, F, F, P, I, I, I, I, I, I, P],
     "hfa_polynorm": [P, I, I, P, P, I, I, I, I, F, P],
     "hfa_scale_rows": [P, I, I, I, F, P],
-    "hfa_head_norm_store": [P, I, I, I, I, I, I, I, P, P, I, I, I, F, P, I, P, I, P, P, I, P, I, I, P],
+    "hfa_head_norm_store": [P, I, I, I, I, I, I, I, P, P, I, I, I, F, P, I, P, I, P, P, I, I, P, I, I, P, I, I, P, P, I, I, P],
     "hfa_talk_mix": [P, I, P, P, I, I, P, I, I, I, I, I, I, P],
     "hfa_qkv_prepare": [P, I, I, P, P, I, I, I, I, I, I, P, P, F, P, P, P, P, P, P, I, I, P],
     "hfa_causal_conv": [P, I, I, P, P, I, I, P, c_size_t, P, P, I, I, P, I, I, I, P],
@@ -51,7 +51,7 @@ _SIGNATURES = {
     "hfa_layernorm": [P, P, P, P, I, P, I, I, F, P, I, P, I, P],
     "hfa_activation": [P, I, P, I, I, I, I, I, P],
     "hfa_softcap": [P, I, I, I, F, P],
-    "hfa_moe_route": [P, I, I, I, I, I, I, I, I, F, P, P, P, P],
+    "hfa_moe_route": [P, I, I, I, I, I, I, I, I, F, P, P, I, I, P, P, P],
     "hfa_moe_plan": [P, I, I, I, P, P, P, P],
     "hfa_head_plan": [I, I, I, P, P, P, P],
     "hfa_moe_gemm": [P, I, I, I, P, I, P, P, P, I, I, P, I, I, I, P, I, I, I, I, I, F, F, F, P],

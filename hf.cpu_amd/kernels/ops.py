@@ -273,17 +273,18 @@ class Ops:
         return view
 
     # ---- kernels -----------------------------------------------------------
-    def embed(self, table, tokens, out_x, scale=None, positions=None, inv_freq=None):
+    def embed(self, table, tokens, out_x, scale=None, positions=None, inv_freq=None, copy=False):
         """``out_x[t] = table[tokens[t]]``; with ``scale`` the row is multiplied by it, and with ``positions`` and
         ``inv_freq`` (fp32, one per pair of columns) a sinusoidal vector is added: column 2i gets ``sin(p inv_freq[i])``,
-        column 2i + 1 the cosine."""
+        column 2i + 1 the cosine. ``copy``: the same kernel leaves the rows in the activations' dtype for ``rounded(out_x)``."""
         self.settle()
         self._source_changes(out_x)
         T = out_x.shape[0]
         if out_x.dtype != torch.float32 or not out_x.is_contiguous() or not table.is_contiguous() \
                 or table.shape[1] != out_x.shape[1]:
             fail(EINVAL, "embed: the output must be contiguous fp32 with the table's width")
-        if scale is None and positions is None:
+        copy = copy and self.act_dtype != torch.float32
+        if scale is None and positions is None and not copy:
             self._check(self.lib.hfa_embed(table.data_ptr(), _code(table), _ints(tokens, "embed tokens", T),
                                            out_x.data_ptr(), T, table.shape[1], table.shape[0], self._stream()))
             return
@@ -293,7 +294,8 @@ class Ops:
         self._check(self.lib.hfa_embed_pos(table.data_ptr(), _code(table), _ints(tokens, "embed tokens", T),
                                            None if positions is None else _ints(positions, "positions", T),
                                            None if positions is None else inv_freq.data_ptr(), out_x.data_ptr(), T, table.shape[1],
-                                           table.shape[0], 1.0 if scale is None else float(scale), self._stream()))
+                                           table.shape[0], 1.0 if scale is None else float(scale),
+                                           self._rounded_buffer(out_x) if copy else None, self._stream()))
 
     def rmsnorm_add(self, y, weight, eps, out, gate=None, gate_bias=None, scale=1.0, accumulate=True, copy=False):
         """``out (+)= scale * rmsnorm(y * sigmoid(gate + gate_bias)) * weight``, all in fp32 (``gate`` None: ``y`` as it is;
@@ -325,10 +327,7 @@ class Ops:
             fail(EINVAL, "rmsnorm_add: a gate's bias without the gate")
         if gate is not None:
             self._whole(gate)
-        rounded = None
-        if copy and self.act_dtype != torch.float32:
-            rounded = self.scratch(f"rounded@{out.data_ptr()}", (R, E), self.act_dtype)
-            self._scaled.pop(rounded.data_ptr(), None)
+        rounded = self._rounded_buffer(out) if copy and self.act_dtype != torch.float32 else None
         row_gate = None if br is None else br.extra_gate
         self._check(self.lib.hfa_rmsnorm_add(
             None if source is None or partial is not None else source.data_ptr(), 0 if source is None else _rows(source, "norm in"), partial,
@@ -336,10 +335,8 @@ class Ops:
             None if br is None else br.pairs.data_ptr(), 0 if br is None else br.top, None if gate is None else gate.data_ptr(),
             0 if gate is None else _code(gate), 0 if gate is None else _rows(gate, "norm gate"),
             None if gate_bias is None else gate_bias.data_ptr(), None if weight is None else weight.data_ptr(), out.data_ptr(),
-            _rows(out, "norm out"), None if rounded is None else rounded.data_ptr(), E, R, E, float(eps), float(scale),
+            _rows(out, "norm out"), rounded, E, R, E, float(eps), float(scale),
             1 if accumulate else 0, self._stream()))
-        if rounded is not None:
-            self._rounded[out.data_ptr()] = rounded
 
     def branch_sum(self, out, pairs, top, extra=None, extra_gate=None):
         """``out[r] = sum_k pairs[r * top + k] + sigmoid(extra_gate[r]) * extra[r]`` in fp32, left undone until ``rmsnorm_add`` takes
@@ -353,6 +350,13 @@ class Ops:
             self.settle(self._branch.out)
         self._branch = BranchSum(out, pairs, int(top), extra, extra_gate)
 
+    def _rounded_buffer(self, x):
+        """The place for x's copy in the activations' dtype, which the caller's kernel writes beside x (its address)."""
+        t = self.scratch(f"rounded@{x.data_ptr()}", tuple(x.shape), self.act_dtype)
+        self._scaled.pop(t.data_ptr(), None)
+        self._rounded[x.data_ptr()] = t
+        return t.data_ptr()
+
     def rounded(self, x):
         """The fp32 matrix ``x`` in the activations' dtype (``x`` itself in the 32-bit engine): the copy that ``rmsnorm_add`` left beside
         it, or one made now."""
@@ -363,11 +367,9 @@ class Ops:
         if t is not None and t.shape == x.shape:
             return t
         self.settle()
-        t = self.scratch(f"rounded@{x.data_ptr()}", tuple(x.shape), self.act_dtype)
-        self._scaled.pop(t.data_ptr(), None)
-        self._check(self.lib.hfa_round_rows(x.data_ptr(), _rows(x, "rows"), t.data_ptr(), x.shape[1], x.shape[0], x.shape[1], self._stream()))
-        self._rounded[x.data_ptr()] = t
-        return t
+        self._check(self.lib.hfa_round_rows(x.data_ptr(), _rows(x, "rows"), self._rounded_buffer(x), x.shape[1], x.shape[0], x.shape[1],
+                                            self._stream()))
+        return self._rounded[x.data_ptr()]
 
     def diff_mix(self, a, factor, c, eps, n_heads, n_kv_heads, v_head_dim, out):
         """Two attention maps a head as one: ``a`` fp32 [T, groups, 2, heads of a group, v_head_dim]; ``d`` = map 1 - ``factor`` (one fp32
@@ -412,34 +414,55 @@ class Ops:
         return table
 
     def head_norm_store(self, qkv, n_heads, n_kv_heads, head_dim, v_head_dim, q_weight, k_weight, eps, q_out, cache, slot_map,
-                        n_v_heads=None, norm=None, after=False, positions=None, inv_freq=None, rot_dim=0):
-        """Rows ``[q | k | v]`` (fp32 or bf16): every q head and every k head is RMS-normed over its ``head_dim`` values with a
-        weight of that size which all heads share (None: the part stays as it is; with ``norm`` True it is normed without a
-        weight); q goes to ``q_out`` ([T, heads * head_dim], the cache's dtype), k and v to ``cache`` at the rows ``slot_map`` names
-        (values transposed inside their page). ``n_v_heads``: value heads, if not as many as key heads. With ``rot_dim`` the first
-        dimensions of each q and k head are turned (i with i + rot_dim/2) after the norm, or (``after``) before it."""
-        self.settle()
-        self._whole(qkv)
-        self._scaled.pop(q_out.data_ptr(), None)
+                        n_v_heads=None, norm=None, after=False, positions=None, inv_freq=None, rot_dim=0, v_rows=None, extra=None):
+        """Rows ``[q | k | v | more]`` (fp32, bf16, or a product that is still pending: the kernel adds up its partial sums): every q head
+        and every k head is RMS-normed over its ``head_dim`` values with a weight of that size which all heads share (None: the part
+        stays as it is; with ``norm`` True it is normed without a weight); q goes to ``q_out`` ([T, heads * head_dim]), k and v to
+        ``cache`` at the rows ``slot_map`` names (values transposed inside their page). ``n_v_heads``: value heads, if not as many as key
+        heads. With ``rot_dim`` the first dimensions of each q and k head are turned (i with i + rot_dim/2) after the norm, or
+        (``after``) before it. ``v_rows`` ([T, values]): no cache and no key heads, the values go there. ``extra``: the name of a work
+        buffer for the columns behind the values, if the product was pending; returns those columns, from there or from ``qkv``."""
         T = qkv.shape[0]
         GV = n_kv_heads if n_v_heads is None else int(n_v_heads)
         QD, KD, VD = n_heads * head_dim, n_kv_heads * head_dim, GV * v_head_dim
+        C = QD + KD + VD
+        p = self._pending
+        if p is not None and p.out.data_ptr() == qkv.data_ptr() and p.out.shape == qkv.shape and not p.accumulate:
+            self._pending = None                 # (its sums stay in the workspace until the next product)
+        else:
+            p = None
+        self.settle()
+        self._whole(qkv)
+        self._scaled.pop(q_out.data_ptr(), None)
         for w, what in ((q_weight, "q"), (k_weight, "k")):
             if w is not None and (w.dtype != torch.float32 or w.numel() != head_dim or not w.is_contiguous()):
                 fail(EINVAL, f"head_norm_store: the {what} weight must be {head_dim} contiguous fp32 values")
-        if qkv.shape[1] < QD + KD + VD or tuple(q_out.shape) != (T, QD) or q_out.dtype != cache.k.dtype:
-            fail(EINVAL, "head_norm_store: rows of q, k and v in; queries of the cache's dtype out")
-        for c, width in ((cache.k, KD), (cache.v, VD)):
-            if c.dim() != 2 or c.shape[1] != width or not c.is_contiguous():
-                fail(EINVAL, f"head_norm_store: the cache must have one row of {width} values per token")
+        out = cache.k if v_rows is None else v_rows
+        if qkv.shape[1] < C or tuple(q_out.shape) != (T, QD) or q_out.dtype != out.dtype:
+            fail(EINVAL, "head_norm_store: rows of q, k and v in; queries of the cache's (or the values') dtype out")
+        if v_rows is None:
+            for c, width in ((cache.k, KD), (cache.v, VD)):
+                if c.dim() != 2 or c.shape[1] != width or not c.is_contiguous():
+                    fail(EINVAL, f"head_norm_store: the cache must have one row of {width} values per token")
+        elif n_kv_heads or tuple(v_rows.shape) != (T, VD):
+            fail(EINVAL, "head_norm_store: without a cache there are no key heads, and the values have rows of their own")
         table = self._rope_table(positions, inv_freq, T, rot_dim) if rot_dim else None
+        more = None
+        if extra is not None:
+            more = qkv[:, C:] if p is None else self.scratch(extra, (T, qkv.shape[1] - C), torch.float32)
+
+        def ptr(t):
+            return None if t is None else t.data_ptr()
+        finish = more is not None and p is not None
         self._check(self.lib.hfa_head_norm_store(
-            qkv.data_ptr(), _code(qkv), _rows(qkv, "qkv"), n_heads, n_kv_heads, head_dim, GV, v_head_dim,
-            None if q_weight is None else q_weight.data_ptr(), None if k_weight is None else k_weight.data_ptr(),
+            qkv.data_ptr(), _code(qkv), _rows(qkv, "qkv"), n_heads, n_kv_heads, head_dim, GV, v_head_dim, ptr(q_weight), ptr(k_weight),
             1 if norm or q_weight is not None else 0, 1 if norm or k_weight is not None else 0, 1 if after else 0, float(eps),
-            None if table is None else table.data_ptr(), int(rot_dim),
-            q_out.data_ptr(), _rows(q_out, "queries"), cache.k.data_ptr(), cache.v.data_ptr(), _code(cache.k),
-            _ints(slot_map, "slot_map", T), cache.page_tokens, T, self._stream()))
+            ptr(table), int(rot_dim), q_out.data_ptr(), _rows(q_out, "queries"), None if v_rows is not None else cache.k.data_ptr(),
+            cache.v.data_ptr() if v_rows is None else v_rows.data_ptr(), 0 if v_rows is None else _rows(v_rows, "values"), _code(out),
+            None if v_rows is not None else _ints(slot_map, "slot_map", T), 0 if v_rows is not None else cache.page_tokens, T,
+            None if p is None else self.workspace.data_ptr(), 0 if p is None else p.splits, qkv.shape[1], None if p is None else ptr(p.bias),
+            ptr(more) if finish else None, more.shape[1] if finish else 0, more.stride(0) if finish else 0, self._stream()))
+        return more
 
     def talk_mix(self, cross, talk, n_heads, n_kv_heads, v_head_dim, out, gate=None):
         """``out[t, h] = sigmoid(gate[t, h]) * sum_g talk[h, g] A[t, g, group of h]``: the heads' attention weights mixed after
@@ -1348,10 +1371,17 @@ class Ops:
     # ---- mixture of experts ------------------------------------------------------------------------------------------
     SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_chosen": 2}
 
-    def moe_route(self, logits, top, n_groups, keep, scoring="softmax", renorm=True, out_scale=1.0, correction=None):
+    def moe_route(self, logits, top, n_groups, keep, scoring="softmax", renorm=True, out_scale=1.0, correction=None, product=None):
         """(ids [T, top] int32, weights [T, top] fp32) from fp32 router logits [T, E]: see ``hfa_moe_route``. ``scoring``
         ``softmax_chosen``: the experts with the largest logits, weighted (with ``renorm``) by the softmax over the chosen
-        logits alone. ``correction`` (fp32, one per expert) is added to the scores for the choice, not for the weights."""
+        logits alone. ``correction`` (fp32, one per expert) is added to the scores for the choice, not for the weights. ``product``: the
+        contiguous matrix whose first columns ``logits`` is; if its product is still pending, this kernel finishes it."""
+        p = self._pending
+        if p is not None and product is not None and p.out.data_ptr() == product.data_ptr() == logits.data_ptr() and p.out.shape == product.shape \
+                and not p.accumulate and p.bias is None:
+            self._pending = None
+        else:
+            p = None
         self.settle()
         T, E = logits.shape
         if correction is not None and (correction.dtype != torch.float32 or correction.numel() != E or not correction.is_contiguous()):
@@ -1362,7 +1392,8 @@ class Ops:
         wts = self.scratch("moe_weights", (T, top), torch.float32)
         self._check(self.lib.hfa_moe_route(logits.data_ptr(), _rows(logits, "router logits"), T, E, int(top), int(n_groups), int(keep),
                                            self.SCORINGS[scoring], 1 if renorm else 0, float(out_scale),
-                                           None if correction is None else correction.data_ptr(), ids.data_ptr(), wts.data_ptr(), self._stream()))
+                                           None if correction is None else correction.data_ptr(), None if p is None else self.workspace.data_ptr(),
+                                           0 if p is None else p.splits, E if product is None else product.shape[1], ids.data_ptr(), wts.data_ptr(), self._stream()))
         return ids, wts
 
     def moe_experts(self, h, ids, weights, w_up, w_down, act, x, gated=None, weight_on="input", combine=True):

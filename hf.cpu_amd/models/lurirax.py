@@ -83,7 +83,7 @@ def lurirax_plan(cfg):
         schedule.append(ScheduleEntry(l))
     return ModelPlan(
         hidden_size=E, vocab_size=cfg.vocab,
-        embedding=PartSpec("lookup", dict(vocab_size=cfg.vocab, hidden_size=E, prefix="", weight="embed", scale=cfg.embedding_scale)),
+        embedding=PartSpec("lookup", dict(vocab_size=cfg.vocab, hidden_size=E, prefix="", weight="embed", scale=cfg.embedding_scale, copy=True)),
         layers=tuple(layers), schedule=tuple(schedule), final_norm=_norm(cfg, "final.norm"),
         head=PartSpec("linear", dict(vocab_size=cfg.vocab, hidden_size=E, tied=False, prefix="", weight="head")),
     ).check()

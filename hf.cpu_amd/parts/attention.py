@@ -276,30 +276,28 @@ class Attention(Part):
         R = self.H // self.G
         return rows.reshape(self.G, R, 2, self.D, -1).transpose(1, 2).reshape(rows.shape)
 
-    FEW_ROWS = 64                # rows up to which the projections leave 32-bit sums for the norms
-
     def heads(self, ops, step, h, cache, out, write_cache=True):
         """The concatenated heads before the output projection, times ``out_scale``, into ``out`` ([T, heads * v_head_dim], rows may lie
         apart): projections, norms, rotation and store, attention."""
         if not write_cache:
             fail(EINVAL, f"attention '{self.prefix}': this mixer cannot read another entry's cache")
         T = h.shape[0]
-        C = self.QD + self.KD + self.VD
-        proj = ops.scratch("qkv", (T, self.w_qkv.shape[0]), torch.float32 if self.masked and T <= self.FEW_ROWS else ops.act_dtype)
-        with ops.section("qkv"):
-            ops.gemm(h, self.w_qkv, proj, bias=self.b_qkv)
+        proj = ops.scratch("qkv", (T, self.w_qkv.shape[0]), ops.act_dtype)
+        with ops.section("qkv"):                # (sums of a product that split K, or of few rows, are finished by the next kernel)
+            ops.gemm(h, self.w_qkv, proj, bias=self.b_qkv, defer=True)
         pos = self.position
         with ops.section("qkv_prepare"):
             q = ops.scratch("q_normed", (T, self.QD), ops.act_dtype)
-            ops.head_norm_store(proj[:, :C], self.HQ, self.GK, self.D, self.Dv, self.q_norm_w, self.k_norm_w, self.head_norm or 0.0, q, cache,
+            gate = ops.head_norm_store(proj, self.HQ, self.GK, self.D, self.Dv, self.q_norm_w, self.k_norm_w, self.head_norm or 0.0, q, cache,
                                 step.group(cache.group).slot_map, n_v_heads=self.G, norm=self.head_norm is not None, after=self.norm_after,
-                                positions=step.positions, inv_freq=getattr(pos, "inv_freq", None), rot_dim=getattr(pos, "rot_dim", 0))
+                                positions=step.positions, inv_freq=getattr(pos, "inv_freq", None), rot_dim=getattr(pos, "rot_dim", 0),
+                                extra="head_gate" if self.head_gate else None)
         att = out if self.maps == 1 else ops.scratch("att_maps", (T, self.HQ * self.Dv), torch.float32)
         with ops.section("attn"):
             ops.paged_attention(q, self.HQ, self.GK, self.D, cache, step, self.window, self.scale, att, v_head_dim=self.Dv,
                                 mask_chunk=self.mask_chunk, sink=self.sink, softcap=self.softcap, sink_scores=self.sink_w,
                                 distance=self.dist_w, v_share=self.maps, keep_first=self.keep_first, rel=self.rel_table,
-                                gate=proj[:, C:] if self.head_gate else None, out_scale=self.out_scale if self.maps == 1 else 1.0)
+                                gate=gate, out_scale=self.out_scale if self.maps == 1 else 1.0)
             if self.maps == 2:
                 ops.diff_mix(att, self.map_factor, (1.0 - self.diff) * self.out_scale, self.head_norm, self.H, self.G, self.Dv, out)
 

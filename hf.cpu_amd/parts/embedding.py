@@ -15,10 +15,11 @@ class Embedding(Part):
     graph_safe = True
 
 
-    def __init__(self, vocab_size, hidden_size, prefix="", weight="weight", scale=None, sinusoid_base=None):
-        """The table is the tensor ``prefix + weight``."""
+    def __init__(self, vocab_size, hidden_size, prefix="", weight="weight", scale=None, sinusoid_base=None, copy=False):
+        """The table is the tensor ``prefix + weight``. ``copy``: the rows are left in the activations' dtype too (``Ops.rounded``),
+        for a first layer that reads the stream itself."""
         super().__init__(prefix)
-        self.V, self.E = vocab_size, hidden_size
+        self.V, self.E, self.copy = vocab_size, hidden_size, bool(copy)
         self.name = prefix + weight
         self.scale = None if scale is None else float(scale)
         self.sinusoid_base = None if sinusoid_base is None else float(sinusoid_base)
@@ -39,9 +40,9 @@ class Embedding(Part):
     def forward(self, ops, step, out_x):
         with ops.section("embed"):
             if self.inv_freq is not None:
-                ops.embed(self.table, step.tokens, out_x, scale=self.scale, positions=step.positions, inv_freq=self.inv_freq)
+                ops.embed(self.table, step.tokens, out_x, scale=self.scale, positions=step.positions, inv_freq=self.inv_freq, copy=self.copy)
             else:
-                ops.embed(self.table, step.tokens, out_x, scale=self.scale)
+                ops.embed(self.table, step.tokens, out_x, scale=self.scale, copy=self.copy)
 
 
 @register_part("head", "linear")

@@ -123,9 +123,9 @@ class MixtureOfExperts(Part):
         product = ops.scratch("router_logits", (T, rows), torch.float32)
         logits, sg = product[:, :self.n_experts], product[:, self.n_experts:] if self.shared_gate else None
         with ops.section("router"):
-            ops.gemm(h, self.w_router, product, bias=self.b_router)
+            ops.gemm(h, self.w_router, product, bias=self.b_router, defer=self.b_router is None)
             ids, weights = ops.moe_route(logits, self.top, self.n_groups, self.keep_groups, self.scoring, self.renormalize,
-                                         self.weight_scale, correction=self.correction_w)
+                                         self.weight_scale, correction=self.correction_w, product=product)
         if accumulate and not self.shared_gate:
             with ops.section("experts"):
                 ops.moe_experts(h, ids, weights, self.w_up, self.w_down, self.activation, x, gated=self.gated, weight_on=self.weight_on)

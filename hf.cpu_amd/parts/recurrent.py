@@ -162,7 +162,6 @@ class Retention(Part):
     graph_safe = True
     can_overwrite = True
     joins_heads = True
-    FEW_ROWS = 64                # rows up to which the gate's rows ride in the product of queries, keys and values
 
     def __init__(self, hidden_size, n_heads, head_dim, v_head_dim, decay, eps, position, prefix="", names=None):
         super().__init__(prefix)
@@ -204,21 +203,18 @@ class Retention(Part):
         if not write_cache:
             fail(EINVAL, f"retention '{self.prefix}': a state cannot be read without being advanced")
         T, QD, VD = h.shape[0], self.H * self.D, self.OD
-        C = 2 * QD + VD
-        few = T <= self.FEW_ROWS
+        proj = ops.scratch("ret_in", (T, 2 * QD + 2 * VD), ops.act_dtype)
         with ops.section("ret_in"):
-            rows = ops.scratch("ret_in", (T, C + VD if few else C), torch.float32)
-            ops.gemm(h, self.w_in if few else self.w_in[:C], rows)
-            if few:
-                gate = rows[:, C:]
-            else:
-                gate = ops.scratch("ret_gate", (T, VD), ops.act_dtype)
-                ops.gemm(h, self.w_in[C:], gate)
+            ops.gemm(h, self.w_in, proj, defer=True)
+        pos = self.position
+        rows = ops.scratch("ret_rows", (T, 2 * QD + VD), torch.float32)
+        with ops.section("ret_prepare"):        # queries and keys are both turned: as attention's queries, 2 H of them
+            gate = ops.head_norm_store(proj, 2 * self.H, 0, self.D, self.Dv, None, None, 0.0, rows[:, :2 * QD], None, None, n_v_heads=self.H,
+                                       positions=step.positions, inv_freq=getattr(pos, "inv_freq", None), rot_dim=getattr(pos, "rot_dim", 0),
+                                       v_rows=rows[:, 2 * QD:], extra="ret_gate")
         o = ops.scratch("ret_o", (T, VD), torch.float32)
         with ops.section("ret_scan"):
-            if getattr(self.position, "rot_dim", 0):
-                ops.rope_store(rows[:, :2 * QD], step.positions, self.position.inv_freq, self.position.rot_dim, 2 * self.H, 0, self.D, None, None)
-            ops.linear_scan(rows[:, :QD], rows[:, QD:2 * QD], rows[:, 2 * QD:C], self.H, self.D, self.H, self.Dv, cache.state, step, o,
+            ops.linear_scan(rows[:, :QD], rows[:, QD:2 * QD], rows[:, 2 * QD:], self.H, self.D, self.H, self.Dv, cache.state, step, o,
                             decay=self.decay, q_scale=self.D ** -0.5)
         with ops.section("ret_norm"):
             ops.group_rmsnorm(o, self.norm_w, self.eps, self.H, out, gate=gate, gate_kind="silu_after")

@@ -202,7 +202,7 @@ def random_config(rng, big):
             rows = pick(2, 8, 32, 24)
             lt = left(H, G, D, P, pick(1, 7, 16, 50, 300), rows // 2 + pick(1, 5, 30, 200), rows)
             rh, rd = pick(1, 2, 4), pick(32, 64, 128) if big else pick(4, 8, 18, 24)
-            rt = right(rh, rd, pick(32, 64) if big else pick(4, 5, 12, 20), pick(rd, rd // 2), base=pick(100.0, 10000.0))
+            rt = right(rh, rd, pick(32, 64) if big else pick(4, 5, 12, 20), pick(rd, rd // 2 - (rd // 2) % 2), base=pick(100.0, 10000.0))
             mix = parallel(lt, rt, pick(1.0, 0.55, -0.4), pick(1.0, 1.15, 0.3))
         X = pick(2, 5, 8)
         ff = pick(None, dense(pick(32, 64, 96) if big else pick(4, 10, 24)),

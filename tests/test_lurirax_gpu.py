@@ -120,6 +120,42 @@ def test_heads_normed_before_or_after_a_rotation_and_stored(ops32, ops16, in_dty
             assert np.array_equal(v[slots], rounded(x[:, (H + G) * D:], out_dtype))
             untouched = np.setdiff1d(np.arange(n_pages * page), slots)
             assert (cache.k.float().cpu().numpy()[untouched] == 7.0).all() and (v[untouched] == 7.0).all()
+            # without a cache: queries and values to rows
+            q2, v2 = (torch.empty((T, n), dtype=out_dtype, device="cuda") for n in (H * D, GV * Dv))
+            ops.head_norm_store(dev(np.concatenate([rows[:, :H * D], rows[:, (H + G) * D:]], axis=1), in_dtype), H, 0, D, Dv, dev(weights[0]) if weighted else None,
+                                None, 1e-5, q2, None, None, n_v_heads=GV, norm=True, after=after, positions=ints(positions),
+                                inv_freq=dev(freqs) if rot else None, rot_dim=rot, v_rows=v2)
+            assert float((q2.float() - q.float()).abs().max()) <= tol and np.array_equal(v2.float().cpu().numpy(), rounded(x[:, (H + G) * D:], out_dtype))
+
+
+@pytest.mark.parametrize("T,E,H,G,D,GV,Dv,rot,n_extra", [(3, 256, 4, 2, 64, 2, 64, 32, 4), (20, 2048, 8, 2, 128, 2, 128, 128, 8), (48, 512, 4, 4, 32, 2, 64, 0, 2),
+                                                        (600, 2048, 8, 2, 64, 2, 64, 64, 8), (700, 512, 4, 2, 128, 2, 64, 32, 5), (130, 1024, 6, 2, 40, 2, 24, 8, 3)])
+def test_heads_from_a_product_that_is_still_pending(ops16, T, E, H, G, D, GV, Dv, rot, n_extra):
+    """Projections with a bias, their sums finished by the kernel that norms, turns and stores, which also hands out the columns
+    behind the values: as from the finished product, and as in fp64."""
+    rng = np.random.default_rng(T + E)
+    N = (H + G) * D + GV * Dv + n_extra
+    a, w = dev(rng.standard_normal((T, E)), torch.bfloat16), dev(rng.standard_normal((N, E)) / math.sqrt(E), torch.bfloat16)
+    bias = rng.standard_normal(N).astype(np.float32) * 0.3
+    rows = a.double().cpu().numpy() @ w.double().cpu().numpy().T + bias
+    positions, freqs, page = np.arange(T), pl.rotary_frequencies(rot, 500.0) if rot else None, 16
+    n_pages = T // page + 2
+    slots = np.arange(T, dtype=np.int32) + page
+    for defer in (True, False):
+        cache = FakeCache(group=0, k=torch.zeros((n_pages * page, G * D), dtype=torch.bfloat16, device="cuda"),
+                          v=torch.zeros((n_pages * page, GV * Dv), dtype=torch.bfloat16, device="cuda"), page_tokens=page, window=0)
+        proj, q = torch.empty((T, N), dtype=torch.bfloat16, device="cuda"), torch.empty((T, H * D), dtype=torch.bfloat16, device="cuda")
+        b = dev(bias)
+        ops16.gemm(a, w, proj, bias=b, defer=defer)
+        more = ops16.head_norm_store(proj, H, G, D, Dv, None, None, 1e-5, q, cache, ints(slots), n_v_heads=GV, norm=True, after=True, positions=ints(positions),
+                                     inv_freq=dev(freqs) if rot else None, rot_dim=rot, extra="a test's columns")
+        for got, first, heads in ((q, 0, H), (cache.k[page:page + T], H * D, G)):
+            ref = rows[:, first:first + heads * D].reshape(T, heads, D)
+            ref = pl.unit_rms(pl.rotate(ref, positions, freqs) if rot else ref, 1e-5).reshape(T, -1)
+            assert np.max(np.abs(got.float().cpu().numpy() - ref)) <= 6e-2, defer
+        v = from_value_layout(cache.v.float().cpu().numpy(), page)[slots]
+        assert np.max(np.abs(v - rows[:, (H + G) * D:N - n_extra])) <= 3e-2
+        assert np.max(np.abs(more.float().cpu().numpy() - rows[:, N - n_extra:])) <= 3e-2
 
 
 def masked_case(rng, H, G, share, D, Dv, page, window, chunk, keep, rel_n, lengths, q_lens, dtype, gate_dtype):
